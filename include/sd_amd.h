@@ -436,6 +436,11 @@ typedef enum {
 int sd_linear(const void* W, const float* w_scale, const void* x, int64_t ldx,
               const void* bias, const void* residual, void* out, int64_t ldo,
               int M, int N, int K, int epilogue, sd_stream_t stream);
+/* Two matrices of equal input width stacked in one tiled weight, with an input each: output columns
+ * below n_first (a multiple of 16) are products with x, the others with x2 (both [M, K] bf16, row
+ * stride ldx).  out f32 [M, N].                                                             */
+int sd_linear_two_inputs(const void* W, const void* x, const void* x2, int64_t ldx, int n_first,
+                         float* out, int64_t ldo, int M, int N, int K, sd_stream_t stream);
 
 /* The same linear layers at up to 256 token rows (batched draft passes, batched
  * verify; replaces the batch-expanded target pass of
@@ -1346,6 +1351,95 @@ int sd_residual_norm_scaled(float* x, const float* a, int n_a, const void* a_bia
                             const void* add, const void* w_next, int w_f32, float eps,
                             float* x_copy, float* h, void* h_bf16, int n_rows, int W,
                             sd_stream_t stream);
+/* sd_multimap_softmax_attention whose scores, scaled and capped, lose dist1[unit] * ln(1 +
+ * dist2[unit] * (i - j)) with the distance of key j from the row's position i (dist1, dist2 f32
+ * [H*maps], or both NULL), and whose output rows are ldo elements apart (out f32 and out_bf16
+ * alike; either may be NULL).                                                              */
+int sd_distance_softmax_attention(const float* q, int64_t ldq, const void* k_cache,
+                                  const void* v_cache, int cache_f32, const int32_t* row_pos,
+                                  const int32_t* row_slot, const int32_t* block_tables,
+                                  int max_blocks, int page, int n_rows, int H, int G, int maps, int dk,
+                                  int dv, int window, int keep_first, int chunk, float scale,
+                                  float softcap, const float* sinks, const float* dist1,
+                                  const float* dist2, float* out, void* out_bf16, int64_t ldo,
+                                  void* scratch, size_t scratch_bytes, sd_stream_t stream);
+/* Residual update with the layer norms of both sublayers that read the result, per row:
+ *   x[r] += a[r] + a_bias                                 (a != NULL; a_bias [W] or NULL)
+ *   x_copy[r] = x[r]                                      (x_copy != NULL)
+ *   h1[r] = LN(x[r]) * w1, h2[r] = LN(x[r]) * w2          (w1 != NULL; w2 may be NULL)
+ * LN(x) = (x - mean) / sqrt(mean((x - mean)^2) + eps); h1_bf16 / h2_bf16 the same as bf16, every
+ * output may be NULL.  rows (int32 [n_rows], or NULL): output row i comes from x and a of row
+ * rows[i], and x is left as it is.  conv_w ([W, taps] or NULL): h1 is replaced by h1 + conv(h1), a
+ * causal convolution per channel over the sequence; every row must then be alone in its entry (a
+ * decoding step): its predecessors are in conv_state f32 [slots, taps-1, W] (oldest first; what
+ * lies before position 0 counts as zero), which is moved on.  Weights in the model's element type. */
+int sd_joint_residual(float* x, const int32_t* rows, const float* a, const void* a_bias,
+                      float* x_copy, const void* w1, const void* w2, int w_f32, float eps, float* h1,
+                      void* h1_bf16, float* h2, void* h2_bf16, const void* conv_w, int taps,
+                      float* conv_state, const int32_t* row_pos, const int32_t* row_slot, int n_rows,
+                      int W, sd_stream_t stream);
+/* out[r] = x[r] + sum_j w[:, j] * x(r - taps + 1 + j): a causal convolution per channel (w [C, taps])
+ * added to its input, over each entry's rows, the sequence's state and zeros before its start;
+ * then conv_state is moved on (sd_conv_tail).  entries as in sd_seq_batch.                  */
+int sd_conv_add_rows(const float* x, int64_t ldx, const void* w, int w_f32, float* conv_state,
+                     const int32_t* row_pos, const int32_t* row_slot, const int32_t* entries,
+                     int n_entries, float* out, void* out_bf16, int64_t ldo, int n_rows, int C,
+                     int taps, sd_stream_t stream);
+/* Every entry's last taps - 1 rows of x (+ bias [C], or NULL) become its slot's conv_state.  */
+int sd_conv_tail(const float* x, int64_t ldx, const void* bias, int w_f32, float* conv_state,
+                 const int32_t* entries, int n_entries, int C, int taps, sd_stream_t stream);
+/* An activation of normed powers: with z the row + bias ([n] in the model's element type, or NULL),
+ * out = coef[0] N(z) + coef[1] N(z^2) + coef[2] N(z^3) + coef[3], N(y) = y / sqrt(mean(y^2) + eps)
+ * over the row's n values; coef f32 [4] on the device.  sd_poly_norm: the same as a part of
+ * another launch (out / out_bf16: row stride ldo, either may be NULL).                      */
+int sd_poly_norm_rows(const float* z, int64_t ldz, const void* bias, int w_f32, const float* coef,
+                      float eps, float* out, void* out_bf16, int64_t ldo, int n_rows, int n,
+                      sd_stream_t stream);
+typedef struct {
+  const float* z;
+  int64_t ldz;
+  const void* bias;
+  const float* coef;
+  float* out;
+  void* out_bf16;
+  int64_t ldo;
+  int n;
+} sd_poly_norm;
+/* Grouped-query attention's preparation where q, k and v pass a causal convolution each.  proj
+ * [rows, ld] f32 stacks q [H*dk], k [G*dk], v [G*dv] (shared: q alone, the layer reads keys and
+ * values another layer appended), C channels in all; bias [C] (or NULL) is added before the
+ * convolution conv_w [C, taps] (conv_state f32 [slots, taps-1, C], moved on).  q and k are then
+ * RMS-normed per head (weights [dk]); q is multiplied by 1 + temp_coef * ln(floor((p + 1) /
+ * temp_every) + 1) at position p (temp_every 0: not) and written to q_out [rows, H*dk]; k and v
+ * go to the caches as sd_cache_append puts them.  act (or NULL): an activation computed in the
+ * same launch.                                                                             */
+int sd_conv_attn_prep(const float* proj, int64_t ld, const void* bias, const void* conv_w, int taps,
+                      float* conv_state, int H, int G, int dk, int dv, int shared,
+                      const void* q_norm_w, const void* k_norm_w, int w_f32, float eps,
+                      float temp_coef, int temp_every, float* q_out, void* k_cache, void* v_cache,
+                      const int32_t* row_pos, const int32_t* row_slot, const int32_t* entries,
+                      int n_entries, const int32_t* block_tables, int max_blocks, int page, int n_rows,
+                      const sd_poly_norm* act, sd_stream_t stream);
+/* A matrix memory with exponential gates, token by token per (entry, head): log gates
+ * i = cap tanh((zi + bi) / cap), f = logsigmoid(cap tanh((zf + bf) / cap)); m' = max(f + m, i);
+ * S <- e^(f+m-m') S + e^(i-m') k v^T; n <- e^(f+m-m') n + e^(i-m') k; m <- m'.  q (times q_scale), k
+ * [rows, H*dk], v [rows, H*dv], zi, zf [rows, H], all ld floats per row; bi, bf f32 [H]; S f32
+ * [slots, H, dk, dv], n_state f32 [slots, H, dk], m_state f32 [slots, H] (an entry that starts at
+ * position 0 starts from zero).  num f32 [rows, H, dv + 1]: S^T q, then n . q; m_rows f32 [rows, H]: m.
+ * S and n_state are moved on; m_state is left to sd_mlstm_read.                             */
+int sd_mlstm_scan(const float* q, const float* k, const float* v, const float* zi, const float* zf,
+                  int64_t ld, const float* bi, const float* bf, float cap, float q_scale, float* S,
+                  float* n_state, const float* m_state, const int32_t* entries, int n_entries,
+                  float* num, float* m_rows, int H, int dk, int dv, sd_stream_t stream);
+/* What the memory's read-out becomes: o = num / (max(|n . q|, e^-m) + 1e-6) per head, divided by
+ * its root mean square over the head's dv channels (eps inside the root), times w [H*dv], times
+ * sigmoid(gate [rows, H*dv]); y / y_bf16 [rows, H*dv] (row stride ldy, either may be NULL).  The
+ * last row of every entry leaves its m in m_state.  act (or NULL): an activation computed in the
+ * same launch, with act->ldo == ldy.                                                       */
+int sd_mlstm_read(const float* num, const float* m_rows, float* m_state, const int32_t* row_slot,
+                  const float* gate, int64_t ldg, const void* w, int w_f32, float eps, float* y,
+                  void* y_bf16, int64_t ldy, int n_rows, int H, int dv, const sd_poly_norm* act,
+                  sd_stream_t stream);
 /* x[r, c] *= s                                                                             */
 int sd_scale_rows(float* x, int64_t ld, float s, int n_rows, int n_cols, sd_stream_t stream);
 
@@ -1355,13 +1449,15 @@ typedef enum {
   SD_MIX_WINDOW_POOL = 2,   /* sd_window_pool_attention */
   SD_MIX_LATENT = 3,        /* softmax window attention over latent keys / values */
   SD_MIX_SOFTMAX_SSD = 4,   /* softmax window attention and a state-space recurrence side by side */
-  SD_MIX_SOFTMAX = 5        /* grouped-query softmax attention (sd_masked_softmax_attention), no rotation */
+  SD_MIX_SOFTMAX = 5,       /* grouped-query softmax attention (sd_masked_softmax_attention), no rotation */
+  SD_MIX_MLSTM = 6          /* matrix memory with exponential gates (sd_mlstm_scan) */
 } sd_mixer_kind;
 
 typedef enum {
   SD_BLOCK_GATED = 0,       /* h = norm(x); x += sigmoid(r1) mixer(h) + sigmoid(r2) ff(h) */
   SD_BLOCK_POSTNORM = 1,    /* x += norm1(mixer(x)); x += norm2(ff(x)) */
-  SD_BLOCK_SANDWICH = 2     /* x += post_norm(mixer(norm(x))); x += post_norm2(ff(norm2(x))) */
+  SD_BLOCK_SANDWICH = 2,    /* x += post_norm(mixer(norm(x))); x += post_norm2(ff(norm2(x))) */
+  SD_BLOCK_JOINT = 3        /* x += mixer(u + conv(u)) + ff(LN2(x)), u = LN1(x): layer norms */
 } sd_block_kind;
 
 /* One layer: h = norm(x); x += sigmoid(r1) * mixer(h) + sigmoid(r2) * ff(h).  w_in stacks every
@@ -1480,6 +1576,29 @@ typedef struct {
   const void* w_o_bias;     /* [width] or NULL */
   const float* router_bias; /* f32 [n_experts] or NULL */
   float residual_mult;      /* factor of both residual updates; 0: 1 */
+  /* ---- SD_BLOCK_JOINT layers (all zero otherwise).  w_in [mix_rows + ff, width] stacks two matrices
+   * with an input each: the mixer's rows (padded with zero rows to mix_rows, a multiple of 16), which
+   * read u + conv(u), and the feed-forward's up rows, which read LN2(x).  Mixer rows: SD_MIX_SOFTMAX
+   * as above; SD_MIX_MLSTM: q [heads*dim], k [heads*dim], v [heads*vdim], g [heads*vdim], i [heads],
+   * f [heads].  w_o [width, heads*vdim + ff] puts the mixer's output matrix and the feed-forward's
+   * down matrix side by side: one product adds both sublayers.  w_o_bias: the down matrix's bias. */
+  int mix_rows;
+  const void* in_conv_w;    /* [width, in_taps] the mixer's input convolution, or NULL */
+  int in_taps;
+  float* in_conv_state;     /* [slots, in_taps-1, width] */
+  /* attention: conv_w [channels of q, k, v, s_taps] with conv_state; q_norm_w / k_norm_w [dim] */
+  float q_temp_coef;
+  int q_temp_every;         /* 0: no position factor of the query */
+  const float* dist1;       /* [heads] or NULL: sd_distance_softmax_attention */
+  const float* dist2;
+  /* matrix memory: state [slots, heads, dim, vdim], s_norm_w [heads*vdim] */
+  float* n_state;           /* [slots, heads, dim] */
+  float* m_state;           /* [slots, heads] */
+  const float* gate_bias;   /* [2*heads]: input gates', then forget gates' */
+  float gate_cap;
+  /* feed-forward (ff > 0): an activation of normed powers */
+  const void* ff_bias;      /* [ff] the up matrix's bias, or NULL */
+  const float* ff_coef;     /* [4] */
 } sd_seq_layer;
 
 typedef struct {

@@ -102,7 +102,17 @@ class SeqLayer(C.Structure):
                 ("w_shared_down", vp), ("w_shared_down_tiled", vp), ("w_shared_gate", vp),
                 ("maps", i32), ("diff_lambda", C.c_float), ("diff_scale", C.c_float), ("qk_full_norm", i32),
                 ("value_from_key", i32), ("kv_shared", i32), ("w_in_bias", vp), ("w_o_bias", vp),
-                ("router_bias", vp), ("residual_mult", C.c_float)]
+                ("router_bias", vp), ("residual_mult", C.c_float),
+                ("mix_rows", i32), ("in_conv_w", vp), ("in_taps", i32), ("in_conv_state", vp),
+                ("q_temp_coef", C.c_float), ("q_temp_every", i32), ("dist1", vp), ("dist2", vp),
+                ("n_state", vp), ("m_state", vp), ("gate_bias", vp), ("gate_cap", C.c_float),
+                ("ff_bias", vp), ("ff_coef", vp)]
+
+
+class PolyNorm(C.Structure):
+    """sd_poly_norm"""
+    _fields_ = [("z", vp), ("ldz", i64), ("bias", vp), ("coef", vp), ("out", vp), ("out_bf16", vp), ("ldo", i64),
+                ("n", i32)]
 
 
 class SeqModelDesc(C.Structure):
@@ -287,6 +297,21 @@ SIGNATURES = {
                                        C.c_float, vp, i32, vp, vp]),
     "sd_residual_norm_scaled": (i32, [vp, vp, i32, vp, vp, vp, i64, vp, C.c_float, vp, vp, i32, C.c_float, vp, vp,
                                       vp, i32, i32, vp]),
+    "sd_linear_two_inputs": (i32, [vp, vp, vp, i64, i32, vp, i64, i32, i32, i32, vp]),
+    "sd_distance_softmax_attention": (i32, [vp, i64, vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32,
+                                            i32, i32, i32, C.c_float, C.c_float, vp, vp, vp, vp, vp, i64, vp,
+                                            C.c_size_t, vp]),
+    "sd_joint_residual": (i32, [vp, vp, vp, vp, vp, vp, vp, i32, C.c_float, vp, vp, vp, vp, vp, i32, vp, vp, vp, i32,
+                                i32, vp]),
+    "sd_conv_add_rows": (i32, [vp, i64, vp, i32, vp, vp, vp, vp, i32, vp, vp, i64, i32, i32, i32, vp]),
+    "sd_conv_tail": (i32, [vp, i64, vp, i32, vp, vp, i32, i32, i32, vp]),
+    "sd_poly_norm_rows": (i32, [vp, i64, vp, i32, vp, C.c_float, vp, vp, i64, i32, i32, vp]),
+    "sd_conv_attn_prep": (i32, [vp, i64, vp, vp, i32, vp, i32, i32, i32, i32, i32, vp, vp, i32, C.c_float, C.c_float,
+                                i32, vp, vp, vp, vp, vp, vp, i32, vp, i32, i32, i32, C.POINTER(PolyNorm), vp]),
+    "sd_mlstm_scan": (i32, [vp, vp, vp, vp, vp, i64, vp, vp, C.c_float, C.c_float, vp, vp, vp, vp, i32, vp, vp, i32,
+                            i32, i32, vp]),
+    "sd_mlstm_read": (i32, [vp, vp, vp, vp, vp, i64, vp, i32, C.c_float, vp, vp, i64, i32, i32, i32,
+                            C.POINTER(PolyNorm), vp]),
     "sd_seq_model_create": (vp, [C.POINTER(SeqModelDesc)]),
     "sd_seq_model_destroy": (None, [vp]),
     "sd_seq_model_workspace_bytes": (C.c_size_t, [vp, i32, i32, i32]),

@@ -210,7 +210,7 @@ def rope_table(cfg: ModelConfig, device="cpu") -> torch.Tensor:
 
 # ---------------------------------------------------------------------------------------------
 # Decoders described layer by layer (recurrent and windowed mixers); served by seq_engine.SeqEngine.
-MIXER_KINDS = ("retention", "gla", "attention", "latent_attention", "parallel", "softmax_attention")
+MIXER_KINDS = ("retention", "gla", "attention", "latent_attention", "parallel", "softmax_attention", "mlstm")
 
 
 @dataclass
@@ -300,7 +300,14 @@ class MixerSpec:
     k over the whole projection (qk_full_norm); add biases to the q, k and output projections
     (proj_bias); take its values from the keys as projected (value_is_key: no value matrix); keep
     one term of score 0 in the softmax's denominator (unit_sink); read the keys and values that
-    layer kv_from cached instead of projecting its own."""
+    layer kv_from cached instead of projecting its own; add biases to the q, k and v projections
+    (qkv_bias) and pass each through a causal convolution of conv_taps taps before its norm; multiply
+    q by 1 + q_temp_coef * ln(floor((p + 1) / q_temp_every) + 1) at position p; take r1 * ln(1 + r2 *
+    distance) off a head's scores (distance_bias).  "mlstm": a matrix memory per head,
+    S <- e^(f+m-m') S + e^(i-m') k v^T with log gates from the input capped at gate_cap (i = cap
+    tanh(z/cap), f = logsigmoid of the same), m' = max(f + m, i), read as S^T q over
+    max(|n . q|, e^-m') with n the same memory of k alone, each head divided by its root mean square,
+    gated by a sigmoid."""
     kind: str
     heads: int
     dim: int
@@ -335,6 +342,18 @@ class MixerSpec:
     value_is_key: bool = False     # values are the keys as projected
     unit_sink: bool = False        # one term exp(0) in the softmax's denominator
     kv_from: int = -1              # the layer whose cached keys and values this one reads (-1: its own)
+    qkv_bias: bool = False         # biases on the q, k and v projections
+    conv_taps: int = 0             # a causal convolution on each of q, k and v (0: none)
+    q_temp_coef: float = 0.0       # q grows with the logarithm of its position
+    q_temp_every: int = 0          # (0: it does not)
+    distance_bias: bool = False    # two learned numbers per head: a logarithm of the distance off the score
+    gate_cap: float = 0.0          # mlstm: bound of the gates' logits
+
+    @property
+    def conv_channels(self) -> int:
+        """Channels of q, k and v that a layer of its own keys convolves (q alone: shared keys)."""
+        own = 0 if self.kv_from >= 0 else self.kv_heads * (self.dim + self.vdim)
+        return self.heads * self.dim + own
 
     def validate(self) -> None:
         if self.kind not in MIXER_KINDS:
@@ -353,7 +372,13 @@ class MixerSpec:
             if self.kv_rank > 512 or self.kv_heads != self.heads:
                 raise ValueError("latent attention: kv_rank above 512, or kv_heads given")
             return
+        if self.kind == "mlstm":
+            if not self.gate_cap > 0 or self.dim > 256 or self.vdim > 512 or self.kv_heads != self.heads:
+                raise ValueError("mlstm needs gate_cap > 0, dim <= 256, vdim <= 512 and one key head per query head")
+            return
         if self.kind == "softmax_attention":
+            if self.conv_taps < 0 or self.q_temp_every < 0:
+                raise ValueError("softmax attention needs conv_taps >= 0 and q_temp_every >= 0")
             if self.window < 0 or self.chunk < 0 or self.softcap < 0 or self.vdim > 512:
                 raise ValueError("softmax attention needs window >= 0, chunk >= 0, softcap >= 0, vdim <= 512")
             if self.rot_dims < 0 or self.rot_dims % 2 or self.rot_dims > self.dim:
@@ -417,7 +442,10 @@ class SeqLayerSpec:
     mixer: MixerSpec
     ff: int = 0                    # width of the gated feed-forward beside the mixer; 0: none
     experts: Optional[ExpertsSpec] = None   # routed experts as the feed-forward
-    ff_act: str = "relu"           # the gated feed-forward's activation: "relu" or "silu"
+    ff_act: str = "relu"           # the gated feed-forward's activation: "relu" or "silu"; "joint" models:
+                                   # "polynorm", an ungated feed-forward with biases and the activation
+                                   # a N(z) + b N(z^2) + c N(z^3) + e, N(y) = y / rms(y), of four learned numbers
+    in_taps: int = 0               # "joint" models: taps of the mixer's input convolution (0: none)
 
 
 @dataclass
@@ -435,6 +463,8 @@ class SeqModelConfig:
     # weights, the sublayers read x itself; the feed-forward is a set of routed experts or absent.
     # "sandwich": x += norm1b(mixer(norm1(x))); x += norm2b(ff(norm2(x))), plain norm weights; the
     # feed-forward is gated, a set of routed experts (with or without a shared one), or absent.
+    # "joint": x += mixer(u + conv(u)) + ff(norm2(x)), u = norm1(x): both sublayers read the same x;
+    # layer norms with a weight and no bias, a causal convolution of the mixer's input.
     block: str = "gated"
     embed_scale: float = 1.0
     bigram: Optional[dict] = None  # {buckets, mul_prev, mul_cur}: a hashed table of token pairs added to the embedding
@@ -467,6 +497,9 @@ class SeqModelConfig:
                 raise ValueError(f"mixer {l.mixer.kind!r} does not belong to a 'sandwich' model")
             if l.mixer.kind == "latent_attention" and l.mixer.q_rank:
                 raise ValueError("a 'sandwich' model's latent attention projects its queries straight from the input")
+            if l.mixer.conv_taps or l.mixer.qkv_bias or l.mixer.q_temp_every or l.mixer.distance_bias or l.in_taps:
+                raise ValueError("convolved inputs, biases on q, k and v, a position factor of the query and a distance "
+                                 "bias belong to 'joint' models")
             src = l.mixer.kv_from
             if src >= 0:
                 if self.loop is not None or l.mixer.kind != "softmax_attention" or not src < i:
@@ -487,11 +520,36 @@ class SeqModelConfig:
             if not 0 <= a < b <= len(self.layers) or t < 1:
                 raise ValueError(f"loop {self.loop}: needs 0 <= start < stop <= layers and times >= 1")
 
+    def _validate_joint(self) -> None:
+        if self.loop is not None or self.bigram is not None or self.width > 16384:
+            raise ValueError("a 'joint' model has no repeated span, no bigram table and a width of at most 16384")
+        for i, l in enumerate(self.layers):
+            m = l.mixer
+            m.validate()
+            if m.kind not in ("softmax_attention", "mlstm"):
+                raise ValueError(f"mixer {m.kind!r} does not belong to a 'joint' model")
+            if l.ff < 0 or l.experts is not None or l.in_taps < 0 or (l.ff and l.ff_act != "polynorm"):
+                raise ValueError("a 'joint' layer's feed-forward is dense with the 'polynorm' activation, or absent")
+            if m.kind != "softmax_attention":
+                continue
+            if m.conv_taps < 1 or not m.qk_head_norm or m.dim > 512 or m.maps != 1 or m.rot_dims or m.value_is_key \
+                    or m.sink or m.unit_sink or m.chunk or m.proj_bias:
+                raise ValueError("a 'joint' model's attention convolves q, k and v, norms q and k per head (dim <= 512), "
+                                 "and has one score map, no rotation, no sink and no chunks")
+            if m.kv_from >= 0:
+                b = self.layers[m.kv_from].mixer if m.kv_from < i else None
+                same = ("kind", "heads", "kv_heads", "dim", "vdim")
+                if b is None or b.kv_from >= 0 or any(getattr(m, k) != getattr(b, k) for k in same):
+                    raise ValueError(f"layer {i}: layer {m.kv_from} must be an earlier attention layer that projects "
+                                     "keys and values of its own, with this layer's head counts and sizes")
+
     def validate(self) -> None:
         if self.width < 1 or self.vocab < 1 or not self.layers:
             raise ValueError("a model needs width, vocab and at least one layer")
-        if self.block not in ("gated", "postnorm", "sandwich"):
+        if self.block not in ("gated", "postnorm", "sandwich", "joint"):
             raise ValueError(f"unknown block {self.block!r}")
+        if self.block == "joint":
+            return self._validate_joint()
         if self.block == "sandwich":
             if self.bigram is not None:
                 raise ValueError("a 'sandwich' model has no bigram table")
@@ -528,6 +586,15 @@ class SeqModelConfig:
             n += int(self.loop["times"]) * W
         for l in self.layers:
             m = l.mixer
+            if self.block == "joint":
+                n += W + l.in_taps * W + m.heads * m.vdim * W
+                if m.kind == "mlstm":
+                    n += W * (2 * m.heads * (m.dim + m.vdim + 1)) + 2 * m.heads + m.heads * m.vdim
+                else:
+                    n += m.conv_channels * (W + m.conv_taps + (1 if m.qkv_bias else 0))
+                    n += m.dim * (1 if m.kv_from >= 0 else 2) + (2 * m.heads if m.distance_bias else 0)
+                n += W + 2 * l.ff * W + l.ff + W + 4 if l.ff else 0
+                continue
             if self.block == "sandwich":
                 n += 2 * W + (2 * W if (l.ff or l.experts) else 0) + m.heads * m.vdim * W
                 if m.kind == "latent_attention":
@@ -573,6 +640,12 @@ class SeqModelConfig:
                 n += 4 * (m.ssd.heads * m.ssd.state * m.ssd.vdim + (m.ssd.taps - 1) * m.ssd.conv_channels)
             elif m.kind in ("retention", "gla"):
                 n += 4 * m.heads * m.dim * m.vdim
+            elif m.kind == "mlstm":
+                n += 4 * m.heads * (m.dim * (m.vdim + 1) + 1)
+            elif m.conv_taps > 1:
+                n += 4 * (m.conv_taps - 1) * m.conv_channels
+            if l.in_taps > 1:
+                n += 4 * (l.in_taps - 1) * self.width
         return n
 
 
@@ -757,9 +830,49 @@ def zopupel_config(cfg: dict, tensor_shapes: Optional[dict] = None, **overrides)
     return out
 
 
+def gufasun_config(cfg: dict, tensor_shapes: Optional[dict] = None, **overrides) -> SeqModelConfig:
+    """A Gufasun config.json: both sublayers of a layer read the same residual through a layer norm
+    each, the mixer's input passes a causal convolution first.  "attention": grouped-query softmax
+    attention over a sliding window without rotation, q, k and v with biases and a convolution each,
+    q and k normed per head, a query that grows with the logarithm of its position, capped scores
+    less a logarithm of the distance; it may read an earlier layer's cached keys and values
+    (kv_from).  "mlstm": a matrix memory with exponential gates.  A dense feed-forward with biases
+    whose activation mixes normed powers, or none; a scaled embedding and an untied head."""
+    taps = int((cfg.get("canon") or {}).get("taps") or 0)
+    layers = []
+    for i, l in enumerate(cfg["layers"]):
+        m, kind = l["mixer"], l["type"]
+        if kind == "attention":
+            mask, qt, src = m.get("mask") or {}, m.get("q_temp") or {}, m.get("kv_from")
+            spec = MixerSpec(kind="softmax_attention", heads=int(m["heads"]), kv_heads=int(m.get("kv_heads") or 0),
+                             dim=int(m["dim"]), vdim=int(m["vdim"]), scale=float(m["scale"]),
+                             window=int(mask.get("size") or 0), softcap=float(m.get("softcap") or 0.0),
+                             qk_head_norm=True, qkv_bias=True, conv_taps=int(m["conv"]), distance_bias=True,
+                             q_temp_coef=float(qt.get("coef", 0.0)), q_temp_every=int(qt.get("every", 0)),
+                             kv_from=-1 if src is None else int(src))
+        elif kind == "mlstm":
+            spec = MixerSpec(kind="mlstm", heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                             gate_cap=float(m["gate_cap"]))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+        mlp = l.get("mlp")
+        if mlp and mlp.get("kind", "dense") != "dense":
+            raise ValueError(f"layer {i}: feed-forward kind {mlp.get('kind')!r} is not supported")
+        layers.append(SeqLayerSpec(spec, int(mlp["ff"]) if mlp else 0, ff_act="polynorm", in_taps=taps))
+    out = SeqModelConfig(arch="gufasun", width=int(cfg["width"]), vocab=int(cfg["vocab"]), layers=layers,
+                         norm_eps=float(cfg["norm"]["eps"]), name=cfg.get("architecture", "Gufasun"), block="joint",
+                         embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), tied_head=False)
+    for k, v in overrides.items():
+        if not hasattr(out, k):
+            raise ValueError(f"Unknown config parameter: {k}")
+        setattr(out, k, v)
+    out.validate()
+    return out
+
+
 # config.json "architecture" -> builder of a layer-list config
 SEQ_ARCHITECTURES = {"Puguzen": puguzen_config, "Naburax": naburax_config, "Fepopel": fepopel_config,
-                     "Zopupel": zopupel_config}
+                     "Zopupel": zopupel_config, "Gufasun": gufasun_config}
 
 
 def safetensors_shapes(path: str) -> dict:

@@ -83,6 +83,8 @@ struct LinArgs {
   int64_t ld_add;
   bf16_t* x_out;           // NORM_RMS_ADD: [M][ldx] bf16 = x + add, or NULL
   int32_t* part_idx;       // EPI_ARGMAX: [M][SD_ARGMAX_PARTS] beside out = part_val (f32)
+  const bf16_t* x2;        // SD_EPI_F32 without a norm: tiles from tile2 on read x2 (same ldx) instead of x
+  int tile2;
 };
 
 // HALF: a work unit is 8 of a tile's 16 rows (lanes of the other 8 rows load nothing and
@@ -127,6 +129,10 @@ __global__ __launch_bounds__(kLinThreads) void linear_kernel(LinArgs a) {
   const int xc = lane & 15, xq = lane >> 4;
   const bf16_t* xrow = xs + (size_t)(xc < M ? xc : M) * LDX + 8 * xq;           // LDS
   const bf16_t* xglob = a.x + (size_t)(xc < M ? xc : 0) * a.ldx + 8 * xq;        // DIRECT
+  // two stacked matrices with an input each: the second one's tiles read x2
+  constexpr bool TWO = DIRECT && EPI == SD_EPI_F32 && !W8;
+  const bf16_t* xglob2 = TWO && a.x2 ? a.x2 + (size_t)(xc < M ? xc : 0) * a.ldx + 8 * xq : xglob;
+  auto x_of = [&](int tile) { return TWO && a.x2 && tile >= a.tile2 ? xglob2 : xglob; };
   // the grid is even in HALF mode, so a workgroup keeps one row half for all its units
   const int row_half = HALF ? (int)(blockIdx.x & 1) : 0;
   // Lanes whose output nobody reads (HALF: the other 8 rows of the tile; DIRECT: token
@@ -146,7 +152,7 @@ __global__ __launch_bounds__(kLinThreads) void linear_kernel(LinArgs a) {
   };
   auto load_whole_seg = [&](int tile, int seg) {  // all of the segment's k-steps exist
     const bf16_t* p = seg_ptr(tile, seg);
-    const bf16_t* q = xglob + (size_t)seg * kSeg * 32;
+    const bf16_t* q = x_of(tile) + (size_t)seg * kSeg * 32;
 #pragma unroll
     for (int j = 0; j < kWLoads; ++j)
       nxt[j] = __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(p + (size_t)j * 512));
@@ -161,7 +167,7 @@ __global__ __launch_bounds__(kLinThreads) void linear_kernel(LinArgs a) {
       load_whole_seg(tile, seg);
     } else {
       const bf16_t* p = seg_ptr(tile, seg);
-      const bf16_t* q = xglob + (size_t)seg * kSeg * 32;
+      const bf16_t* q = x_of(tile) + (size_t)seg * kSeg * 32;
 #pragma unroll
       for (int j = 0; j < kWLoads; ++j) {
         bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
@@ -1019,6 +1025,19 @@ extern "C" int sd_linear(const void* W, const float* w_scale, const void* x, int
   a.w_scale = w_scale;
   a.n_tiles = tiles_for(N, epilogue);
   return linear_common(a, epilogue, NORM_NONE, (hipStream_t)stream);
+}
+
+extern "C" int sd_linear_two_inputs(const void* W, const void* x, const void* x2, int64_t ldx, int n_first, float* out,
+                                    int64_t ldo, int M, int N, int K, sd_stream_t stream) {
+  SD_REQUIRE(x2 && sd_aligned16(x2) && n_first >= 16 && n_first % 16 == 0 && n_first < N, SD_ERR_INVALID,
+             "sd_linear_two_inputs: the second matrix must start at a multiple of 16 rows below N (%d of %d)", n_first, N);
+  SD_REQUIRE(ldo >= N, SD_ERR_INVALID, "sd_linear_two_inputs: ldo < N");
+  LinArgs a{};
+  a.W = (const bf16_t*)W; a.x = (const bf16_t*)x; a.ldx = ldx; a.out = out; a.ldo = ldo; a.M = M; a.N = N; a.K = K;
+  a.n_tiles = tiles_for(N, SD_EPI_F32);
+  a.x2 = (const bf16_t*)x2;
+  a.tile2 = n_first / 16;
+  return linear_common(a, SD_EPI_F32, NORM_NONE, (hipStream_t)stream);
 }
 
 extern "C" int sd_linear_attn_merge(const void* W, const float* w_scale, const void* workspace,

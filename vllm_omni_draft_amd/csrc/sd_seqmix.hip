@@ -1000,6 +1000,7 @@ struct SeqWs {
   size_t sg;   // a shared expert's gate per row
   // layers normed on their output
   size_t pq, qe, cqb, conv, step, decay, rlog, sel_e, sel_w, dn, moe, moe_bytes;
+  size_t hc, h2b;   // layers whose sublayers read norms of their own
 };
 // column offsets inside the fused input projection of a layer normed on its output
 struct PnCols {
@@ -1023,6 +1024,31 @@ SwCols sw_cols(const sd_seq_layer& l) {
     c.v = at; at += l.kv_shared || l.value_from_key ? 0 : l.kv_heads * l.vdim;
   }
   c.total = at;
+  return c;
+}
+// column offsets inside the input projections of a layer whose sublayers read the same residual: the
+// mixer's columns, then (from mix on, a multiple of 16) the feed-forward's
+struct JtCols {
+  int q, k, v, g, i, f, used, mix, ff, total;
+};
+JtCols jt_cols(const sd_seq_layer& l) {
+  JtCols c = {};
+  int at = 0;
+  c.q = at; at += l.heads * l.dim;
+  if (l.kind == SD_MIX_MLSTM) {
+    c.k = at; at += l.heads * l.dim;
+    c.v = at; at += l.heads * l.vdim;
+    c.g = at; at += l.heads * l.vdim;
+    c.i = at; at += l.heads;
+    c.f = at; at += l.heads;
+  } else if (!l.kv_shared) {
+    c.k = at; at += l.kv_heads * l.dim;
+    c.v = at; at += l.kv_heads * l.vdim;
+  }
+  c.used = at;
+  c.mix = (at + 15) / 16 * 16;
+  c.ff = l.ff;
+  c.total = c.mix + l.ff;
   return c;
 }
 // whether a grouped-query softmax layer needs the general preparation (sd_attn_prep) rather than
@@ -1054,7 +1080,7 @@ PnCols pn_cols(const sd_seq_layer& l) {
 SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
   const int W = m.d.width;
   size_t proj = 0, hk = 0, hv = 0, ff = 0, wide = 0, attn = 0;
-  size_t pq = 0, qe = 0, cq = 0, conv = 0, sh = 0, ne = 0, top = 0, moe = 0;
+  size_t pq = 0, qe = 0, cq = 0, conv = 0, sh = 0, ne = 0, top = 0, moe = 0, joint = 0;
   const int wr = rows < kWideRows ? rows : kWideRows;
   auto up = [](size_t& a, size_t b) { a = b > a ? b : a; };
   auto need = [&](const void* tiled, int M, int N, int K) {
@@ -1063,6 +1089,24 @@ SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
     wide = n > wide ? n : wide;
   };
   for (const sd_seq_layer& l : m.layers) {
+    if (l.block == SD_BLOCK_JOINT) {
+      const JtCols c = jt_cols(l);
+      const int K = l.heads * l.vdim + l.ff;
+      joint = (size_t)W;
+      up(proj, (size_t)c.total);
+      up(hv, (size_t)K);
+      need(l.w_in_tiled, wr, c.mix, W);
+      if (l.ff > 0) need(l.w_in_tiled, wr, l.ff, W);
+      need(l.w_o_tiled, wr, W, K);
+      if (l.kind == SD_MIX_MLSTM) {
+        up(hv, (size_t)l.heads * (l.vdim + 1));
+        up(sh, (size_t)l.heads);
+      } else {
+        up(pq, (size_t)l.heads * l.dim);
+        up(attn, sd_multimap_softmax_attention_scratch_bytes(rows, l.heads, 1, l.vdim, l.window, 0, 0, max_ctx));
+      }
+      continue;
+    }
     if (l.block == SD_BLOCK_SANDWICH) {
       const SwCols c = sw_cols(l);
       up(proj, (size_t)c.total);
@@ -1172,6 +1216,8 @@ SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
   w.moe_bytes = moe;
   w.moe = off;   off += al(moe ? moe : 16);
   w.sg = off;    off += al(R * f);
+  w.hc = off;    off += al(R * joint * f);
+  w.h2b = off;   off += al(R * joint * 2);
   w.total = off;
   return w;
 }
@@ -1207,6 +1253,24 @@ extern "C" sd_seq_model* sd_seq_model_create(const sd_seq_model_desc* desc) {
   for (int i = 0; i < desc->n_layers; ++i) {
     const sd_seq_layer& l = m->layers[i];
     const char* bad = nullptr;
+    if (l.block == SD_BLOCK_JOINT) {
+      const bool f32 = desc->weights_f32;
+      if (l.kind != SD_MIX_SOFTMAX && l.kind != SD_MIX_MLSTM) bad = "a layer whose sublayers read the same residual takes grouped-query softmax attention or a matrix memory";
+      else if (i > 0 && m->layers[i - 1].block != SD_BLOCK_JOINT) bad = "it follows a layer of another kind";
+      else if (l.heads < 1 || l.dim < 1 || l.vdim < 1 || l.dim > 512 || l.vdim > 512 || l.ff < 0 || l.mix_rows != jt_cols(l).mix) bad = "head counts / sizes / rows of the stacked input matrix";
+      else if (!l.norm_w || !(l.w_in || l.w_in_tiled) || !(l.w_o || l.w_o_tiled)) bad = "a null weight";
+      else if ((l.w_in_tiled || l.w_o_tiled) && f32) bad = "tiled matrices are bf16";
+      else if ((l.w_in_tiled && desc->width % 32) || (l.w_o_tiled && (l.heads * l.vdim + l.ff) % 32)) bad = "a tiled matrix needs an input width that is a multiple of 32";
+      else if (l.in_conv_w && (l.in_taps < 1 || (l.in_taps > 1 && !l.in_conv_state))) bad = "the input convolution needs taps and a state";
+      else if (l.ff > 0 && (!l.norm2_w || !l.ff_coef)) bad = "a feed-forward needs its norm and its activation's factors";
+      else if (desc->width > 16384) bad = "a width above 16384";
+      else if (l.kind == SD_MIX_MLSTM) {
+        if (l.dim > 256 || !l.state || !l.n_state || !l.m_state || !l.gate_bias || !(l.gate_cap > 0.f) || !l.s_norm_w) bad = "a matrix memory needs dim <= 256, its states, gate biases, a cap and its norm";
+      } else if (l.kv_heads < 1 || l.heads % l.kv_heads || l.window < 1 || l.softcap < 0.f || !l.k_cache || !l.v_cache ||
+                 l.maps > 1 || l.rot_dims || l.value_from_key || (l.kv_shared && i == 0)) bad = "attention needs kv heads that divide the heads, a window, caches, one score map and no rotation";
+      else if (!l.conv_w || l.s_taps < 1 || (l.s_taps > 1 && !l.conv_state) || !l.q_norm_w || (!l.kv_shared && !l.k_norm_w) ||
+               l.q_temp_every < 0 || !l.dist1 != !l.dist2) bad = "attention needs its convolutions, norms per head and both distance factors or none";
+    } else
     if (l.block == SD_BLOCK_SANDWICH) {
       if (l.kind != SD_MIX_LATENT && l.kind != SD_MIX_SOFTMAX) bad = "a layer normed before and after its sublayers takes latent or grouped-query softmax attention";
       else if (i > 0 && m->layers[i - 1].block != SD_BLOCK_SANDWICH) bad = "it follows a layer of another kind";
@@ -1501,6 +1565,89 @@ int sandwich_layer(const sd_seq_model& m, const sd_seq_layer& l, const sd_seq_la
   return sd_residual_norm_scaled(x, dn, l.top, nullptr, l.shared_ff > 0 ? ffo : nullptr, gated_shared ? sg : nullptr, 1,
                                  l.post_norm2_w, mult, next_add, next_norm, f32, eps, x_copy, h, hb, R, W, stream);
 }
+
+// What both sublayers of a joint layer read, into the workspace: x += a + a_bias, then u + conv(u) of
+// u = LN1(x) (hc, or its bf16 copy hb) and LN2(x) (ffo, or h2b).  A decoding step does it in one
+// launch, otherwise the convolution follows in its own.
+int joint_inputs(const sd_seq_model& m, const sd_seq_layer& l, const float* a, const void* a_bias, float* x_copy,
+                 const sd_seq_batch& b, char* base, const SeqWs& w, sd_stream_t stream) {
+  const int W = m.d.width, R = b.n_rows, f32 = m.d.weights_f32;
+  float* x = (float*)(base + w.x);
+  float* h = (float*)(base + w.h);
+  float* hc = (float*)(base + w.hc);
+  float* h2 = (float*)(base + w.ffo);
+  const bool tiled = l.w_in_tiled, single = R == b.n_entries, conv = l.in_conv_w != nullptr;
+  void* hcb = tiled ? base + w.hb : nullptr;
+  void* h2b = tiled ? base + w.h2b : nullptr;
+  const void* w2 = l.ff > 0 ? l.norm2_w : nullptr;
+  if (single || !conv)
+    return sd_joint_residual(x, nullptr, a, a_bias, x_copy, l.norm_w, w2, f32, m.d.norm_eps, tiled ? nullptr : hc, hcb,
+                             tiled ? nullptr : h2, h2b, l.in_conv_w, l.in_taps, l.in_conv_state, b.row_pos, b.row_slot,
+                             R, W, stream);
+  SQ_TRY(sd_joint_residual(x, nullptr, a, a_bias, x_copy, l.norm_w, w2, f32, m.d.norm_eps, h, nullptr,
+                           tiled ? nullptr : h2, h2b, nullptr, 0, nullptr, nullptr, nullptr, R, W, stream));
+  return sd_conv_add_rows(h, W, l.in_conv_w, f32, l.in_conv_state, b.row_pos, b.row_slot, b.entries, b.n_entries,
+                          tiled ? nullptr : hc, hcb, W, R, W, l.in_taps, stream);
+}
+
+// One layer whose sublayers read the same residual.  On entry its inputs are ready (joint_inputs);
+// on return mix [R, W] holds what is to be added to x, without the down matrix's bias.
+int joint_layer(const sd_seq_model& m, const sd_seq_layer& l, const sd_seq_batch& b, char* base, const SeqWs& w,
+                sd_stream_t stream) {
+  const sd_seq_model_desc& d = m.d;
+  const int W = d.width, R = b.n_rows, f32 = d.weights_f32;
+  const size_t es = f32 ? sizeof(float) : sizeof(bf16_t);
+  float* proj = (float*)(base + w.proj);
+  float* o = (float*)(base + w.o);
+  float* hc = (float*)(base + w.hc);
+  float* h2 = (float*)(base + w.ffo);
+  bf16_t* hcb = (bf16_t*)(base + w.hb);
+  bf16_t* h2b = (bf16_t*)(base + w.h2b);
+  void* wide_ws = base + w.wide;
+  const JtCols c = jt_cols(l);
+  const int64_t ld = c.total;
+  const int H = l.heads, dk = l.dim, dv = l.vdim, K = H * dv + l.ff;
+  float* y = l.w_o_tiled ? nullptr : (float*)(base + w.y);
+  bf16_t* yb = l.w_o_tiled ? (bf16_t*)(base + w.yb) : nullptr;
+  if (l.w_in_tiled && l.ff > 0 && R <= 16) {
+    SQ_TRY(sd_linear_two_inputs(l.w_in_tiled, hcb, h2b, W, c.mix, proj, ld, R, c.total, W, stream));
+  } else {
+    SQ_TRY(seq_linear(l.w_in, l.w_in_tiled, f32, hc, nullptr, W, hcb, W, nullptr, proj, ld, R, c.mix, W, wide_ws,
+                      w.wide_bytes, stream));
+    if (l.ff > 0) {
+      const size_t at = (size_t)c.mix * W;
+      SQ_TRY(seq_linear(l.w_in ? (const char*)l.w_in + at * es : nullptr,
+                        l.w_in_tiled ? (const char*)l.w_in_tiled + at * sizeof(bf16_t) : nullptr, f32, h2, nullptr, W,
+                        h2b, W, nullptr, proj + c.mix, ld, R, l.ff, W, wide_ws, w.wide_bytes, stream));
+    }
+  }
+  // the feed-forward's activation rides along with a launch of the mixer, into its place beside the
+  // mixer's output
+  sd_poly_norm act = {proj + c.mix, ld, l.ff_bias, l.ff_coef, y ? y + H * dv : nullptr,
+                      yb ? (void*)(yb + H * dv) : nullptr, K, l.ff};
+  const sd_poly_norm* pact = l.ff > 0 ? &act : nullptr;
+  if (l.kind == SD_MIX_MLSTM) {
+    float* m_rows = (float*)(base + w.step);
+    SQ_TRY(sd_mlstm_scan(proj + c.q, proj + c.k, proj + c.v, proj + c.i, proj + c.f, ld, l.gate_bias, l.gate_bias + H,
+                         l.gate_cap, l.q_scale, l.state, l.n_state, l.m_state, b.entries, b.n_entries, o, m_rows, H, dk,
+                         dv, stream));
+    SQ_TRY(sd_mlstm_read(o, m_rows, l.m_state, b.row_slot, proj + c.g, ld, l.s_norm_w, f32, d.norm_eps, y, yb, K, R, H,
+                         dv, pact, stream));
+  } else {
+    float* q = (float*)(base + w.pq);
+    SQ_TRY(sd_conv_attn_prep(proj, ld, l.w_in_bias, l.conv_w, l.s_taps, l.conv_state, H, l.kv_heads, dk, dv, l.kv_shared,
+                             l.q_norm_w, l.k_norm_w, f32, d.norm_eps, l.q_temp_coef, l.q_temp_every, q, l.k_cache,
+                             l.v_cache, b.row_pos, b.row_slot, b.entries, b.n_entries, b.block_tables, b.max_blocks,
+                             b.page, R, pact, stream));
+    SQ_TRY(sd_distance_softmax_attention(q, (int64_t)H * dk, l.k_cache, l.v_cache, f32, b.row_pos, b.row_slot,
+                                         b.block_tables, b.max_blocks, b.page, R, H, l.kv_heads, 1, dk, dv, l.window, 0,
+                                         0, l.score_scale, l.softcap, nullptr, l.dist1, l.dist2, y, yb, K,
+                                         base + w.attn, w.attn_bytes, stream));
+  }
+  // both sublayers' last matrices side by side: one product adds them
+  return seq_linear(l.w_o, l.w_o_tiled, f32, y, nullptr, K, yb, K, nullptr, (float*)(base + w.mix), W, R, W, K, wide_ws,
+                    w.wide_bytes, stream);
+}
 }  // namespace
 
 extern "C" int sd_seq_model_forward(sd_seq_model* m, const sd_seq_batch* b, void* workspace,
@@ -1547,6 +1694,17 @@ extern "C" int sd_seq_model_forward(sd_seq_model* m, const sd_seq_batch* b, void
 
   for (int li = 0; li < d.n_layers; ++li) {
     const sd_seq_layer& l = m->layers[li];
+    if (l.block == SD_BLOCK_JOINT) {
+      if (li == 0) SQ_TRY(joint_inputs(*m, l, nullptr, nullptr, nullptr, *b, base, w, stream));
+      SQ_TRY(joint_layer(*m, l, *b, base, w, stream));
+      float* copy = b->layer_out ? b->layer_out + (size_t)li * R * W : nullptr;
+      if (li + 1 < d.n_layers)
+        SQ_TRY(joint_inputs(*m, m->layers[li + 1], mix, l.w_o_bias, copy, *b, base, w, stream));
+      else if (copy)   // (otherwise the final norm adds the last layer's update to the rows it reads)
+        SQ_TRY(sd_joint_residual(x, nullptr, mix, l.w_o_bias, copy, nullptr, nullptr, f32, d.norm_eps, nullptr, nullptr,
+                                 nullptr, nullptr, nullptr, 0, nullptr, nullptr, nullptr, R, W, stream));
+      continue;
+    }
     if (l.block == SD_BLOCK_SANDWICH) {
       if (li == 0)   // the first layer's input: what is added before it, then its norm
         SQ_TRY(sd_residual_norm(x, nullptr, 0, nullptr, nullptr, 0, nullptr, l.pre_add, l.norm_w, f32, d.norm_eps,
@@ -1626,6 +1784,12 @@ extern "C" int sd_seq_model_forward(sd_seq_model* m, const sd_seq_batch* b, void
     }
   }
   if (b->n_out > 0) {
+    const sd_seq_layer& last = m->layers[d.n_layers - 1];
+    if (last.block == SD_BLOCK_JOINT)
+      SQ_TRY(sd_joint_residual(x, b->out_rows, b->layer_out ? nullptr : mix, b->layer_out ? nullptr : last.w_o_bias,
+                               nullptr, d.final_norm_w, nullptr, f32, d.norm_eps, hout, d.head_tiled ? houtb : nullptr,
+                               nullptr, nullptr, nullptr, 0, nullptr, nullptr, nullptr, b->n_out, W, stream));
+    else
     SQ_TRY(sd_rmsnorm_rows(x, b->out_rows, d.final_norm_w, f32, d.plain_norm ? 0.f : 1.f, d.norm_eps, hout,
                            d.head_tiled ? houtb : nullptr, b->n_out, W, stream));
     SQ_TRY(seq_linear(d.head ? d.head : d.embed, d.head_tiled, f32, hout, nullptr, W, houtb, W, nullptr, b->logits,

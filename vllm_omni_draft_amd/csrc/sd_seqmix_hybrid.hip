@@ -198,6 +198,7 @@ __device__ __forceinline__ void score_key(const KT_* __restrict__ kr, const floa
 // n_splits > 1 (few rows): workgroup (.., .., z) takes tile z / n_hgroups of the row's keys only
 // and leaves its maximum, its sum of weights and its unnormalised weighted values in part_ml /
 // part_acc; softmax_merge_kernel puts a row's tiles together in tile order.
+// dist1 / dist2 (per unit, or nullptr): a score, capped already, loses dist1 ln(1 + dist2 (i - j)).
 // maps > 1: a head holds `maps` queries of dk channels (unit h * maps + m of a row of q), the key
 // cache `maps` key rows per kv head (cache head g * maps + m), and every map reads the kv head's
 // one value row; blockIdx.y counts key heads, and out / sinks count units.
@@ -208,7 +209,8 @@ __global__ __launch_bounds__(256) void window_softmax_attn_kernel(
     const int32_t* __restrict__ block_tables, int max_blocks, int page, int H, int G, int dk, int dv, int window,
     int keep_first, float scale, float* __restrict__ out, bf16_t* __restrict__ out_b, int n_hgroups, int n_splits,
     float* __restrict__ part_acc, float* __restrict__ part_ml, int chunk, float softcap,
-    const float* __restrict__ sinks, int maps) {
+    const float* __restrict__ sinks, int maps, const float* __restrict__ dist1, const float* __restrict__ dist2,
+    int64_t ldo) {
   extern __shared__ float lds[];
   constexpr int nthr = 256, nw = 4, PARTS = nthr / KT, KW = KT / 64;
   unsigned long long* vat = reinterpret_cast<unsigned long long*>(lds);  // [KT] cache row of the key
@@ -250,6 +252,12 @@ __global__ __launch_bounds__(256) void window_softmax_attn_kernel(
   const int c_lo = (part * per < units ? part * per : units) * unit;
   const int c_hi = ((part + 1) * per < units ? (part + 1) * per : units) * unit;
   const int wave = tid >> 6, lane = tid & 63;
+  // what a score loses with the key's distance: dist1[unit] ln(1 + dist2[unit] (i - j))
+  auto away = [&](int hq, int idx) {
+    if (!dist1) return 0.f;
+    const int j = idx < n_kept ? idx : t_first + (idx - n_kept);
+    return dist1[h0 + hq * maps] * log1pf(dist2[h0 + hq * maps] * (float)(i - j));
+  };
   float acc[NH][NC];
 #pragma unroll
   for (int hq = 0; hq < NH; ++hq)
@@ -271,7 +279,7 @@ __global__ __launch_bounds__(256) void window_softmax_attn_kernel(
       if constexpr (PARTS == 1) {
 #pragma unroll
         for (int hq = 0; hq < NH; ++hq)
-          if (hq < nh) wt[hq * KT + key] = idx < key_hi ? cap_score(s[hq] * scale, softcap) : -INFINITY;
+          if (hq < nh) wt[hq * KT + key] = idx < key_hi ? cap_score(s[hq] * scale, softcap) - away(hq, idx) : -INFINITY;
       } else {
 #pragma unroll
         for (int hq = 0; hq < NH; ++hq)
@@ -284,7 +292,7 @@ __global__ __launch_bounds__(256) void window_softmax_attn_kernel(
               float sum = ps[hq * KT + key];
 #pragma unroll
               for (int pp = 1; pp < PARTS; ++pp) sum += ps[(pp * NH + hq) * KT + key];
-              wt[hq * KT + key] = idx < key_hi ? cap_score(sum * scale, softcap) : -INFINITY;
+              wt[hq * KT + key] = idx < key_hi ? cap_score(sum * scale, softcap) - away(hq, idx) : -INFINITY;
             }
         }
       }
@@ -372,8 +380,8 @@ __global__ __launch_bounds__(256) void window_softmax_attn_kernel(
         if (n_splits > 1) {
           part_acc[(((size_t)split * R + r) * HM + h0 + hq * maps) * dv + c] = o;
         } else {
-          const size_t at = (size_t)r * HM * dv + (size_t)(h0 + hq * maps) * dv + c;
-          out[at] = o;
+          const size_t at = (size_t)r * ldo + (size_t)(h0 + hq * maps) * dv + c;
+          if (out) out[at] = o;
           if (out_b) out_b[at] = (bf16_t)o;
         }
       }
@@ -392,7 +400,8 @@ __global__ __launch_bounds__(256) void window_softmax_attn_kernel(
 // tile's factor in LDS; then a thread per column adds the tiles' rows in tile order, eight loads
 // in flight.
 __global__ void softmax_merge_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
-                                     int n_splits, float* __restrict__ out, bf16_t* __restrict__ out_b, int H, int dv) {
+                                     int n_splits, float* __restrict__ out, bf16_t* __restrict__ out_b, int H, int dv,
+                                     int64_t ldo) {
   extern __shared__ float fac[];   // [n_splits]
   __shared__ float inv_l;
   const int r = blockIdx.x, h = blockIdx.y, R = gridDim.x, tid = threadIdx.x;
@@ -428,8 +437,8 @@ __global__ void softmax_merge_kernel(const float* __restrict__ part_acc, const f
         if (s0 + u < n_splits && fac[s0 + u] != 0.f) o = fmaf(v[u], fac[s0 + u], o);
     }
     o *= inv_l;
-    const size_t at = at0 * dv + c;
-    out[at] = o;
+    const size_t at = (size_t)r * ldo + (size_t)h * dv + c;
+    if (out) out[at] = o;
     if (out_b) out_b[at] = (bf16_t)o;
   }
 }
@@ -442,13 +451,14 @@ void launch_softmax_nc(dim3 grid, int kt, size_t lds, hipStream_t st, int nc, co
                        const void* kc, const void* vc, int v_row, const int32_t* row_pos, const int32_t* row_slot,
                        const int32_t* bt, int max_blocks, int page, int H, int G, int dk, int dv, int window,
                        int keep_first, float scale, float* out, bf16_t* out_b, int n_hgroups, int n_splits,
-                       float* part_acc, float* part_ml, int chunk, float softcap, const float* sinks, int maps) {
+                       float* part_acc, float* part_ml, int chunk, float softcap, const float* sinks, int maps,
+                       const float* dist1, const float* dist2, int64_t ldo) {
 #define SD_GO2(NC, KT)                                                                                               \
   window_softmax_attn_kernel<T, NH, NC, KT><<<grid, 256, lds, st>>>(q, ldq, (const T*)kc, (const T*)vc, v_row, row_pos, \
                                                                     row_slot, bt, max_blocks, page, H, G, dk, dv,       \
                                                                     window, keep_first, scale, out, out_b, n_hgroups,   \
                                                                     n_splits, part_acc, part_ml, chunk, softcap, sinks, \
-                                                                    maps)
+                                                                    maps, dist1, dist2, ldo)
 #define SD_GO(NC)                                          \
   do {                                                     \
     if constexpr (NH <= 4) {                               \
@@ -1954,8 +1964,23 @@ extern "C" int sd_multimap_softmax_attention(const float* q, int64_t ldq, const 
                                              int G, int maps, int dk, int dv, int window, int keep_first, int chunk,
                                              float scale, float softcap, const float* sinks, float* out,
                                              void* out_bf16, void* scratch, size_t scratch_bytes, sd_stream_t stream) {
-  SD_REQUIRE(q && k_cache && row_pos && row_slot && block_tables && out, SD_ERR_INVALID,
+  SD_REQUIRE(out, SD_ERR_INVALID, "sd_masked_softmax_attention: null argument");
+  return sd_distance_softmax_attention(q, ldq, k_cache, v_cache, cache_f32, row_pos, row_slot, block_tables, max_blocks,
+                                       page, n_rows, H, G, maps, dk, dv, window, keep_first, chunk, scale, softcap, sinks,
+                                       nullptr, nullptr, out, out_bf16, (int64_t)H * maps * dv, scratch, scratch_bytes,
+                                       stream);
+}
+
+extern "C" int sd_distance_softmax_attention(const float* q, int64_t ldq, const void* k_cache, const void* v_cache,
+                                             int cache_f32, const int32_t* row_pos, const int32_t* row_slot,
+                                             const int32_t* block_tables, int max_blocks, int page, int n_rows, int H,
+                                             int G, int maps, int dk, int dv, int window, int keep_first, int chunk,
+                                             float scale, float softcap, const float* sinks, const float* dist1,
+                                             const float* dist2, float* out, void* out_bf16, int64_t ldo, void* scratch,
+                                             size_t scratch_bytes, sd_stream_t stream) {
+  SD_REQUIRE(q && k_cache && row_pos && row_slot && block_tables && (out || out_bf16) && !dist1 == !dist2, SD_ERR_INVALID,
              "sd_masked_softmax_attention: null argument");
+  SD_REQUIRE(ldo >= (int64_t)H * maps * dv, SD_ERR_INVALID, "sd_masked_softmax_attention: output rows too short");
   SD_REQUIRE(n_rows >= 1 && H >= 1 && G >= 1 && H % G == 0 && dk >= 1 && window >= 1 && keep_first >= 0 && page >= 1 &&
                  chunk >= 0 && softcap >= 0.f && maps >= 1 && (maps == 1 || v_cache) &&
                  ldq >= (int64_t)H * maps * dk,
@@ -1988,7 +2013,7 @@ extern "C" int sd_multimap_softmax_attention(const float* q, int64_t ldq, const 
 #define SD_NH(T, N)                                                                                                  \
   launch_softmax_nc<T, N>(grid, kt, lds, st, nc, q, ldq, k_cache, vc, v_row, row_pos, row_slot, block_tables,      \
                           max_blocks, page, H, G, dk, dv, window, keep_first, scale, out, (bf16_t*)out_bf16, n_hgroups, \
-                          n_splits, part_acc, part_ml, chunk, softcap, sinks, maps)
+                          n_splits, part_acc, part_ml, chunk, softcap, sinks, maps, dist1, dist2, ldo)
 #define SD_T(T)                      \
   do {                               \
     if (NH == 1) SD_NH(T, 1);        \
@@ -2003,7 +2028,7 @@ extern "C" int sd_multimap_softmax_attention(const float* q, int64_t ldq, const 
   SD_CHECK_LAUNCH("sd_masked_softmax_attention");
   if (split) {
     softmax_merge_kernel<<<dim3(n_rows, HM), dv <= 64 ? 64 : (dv <= 128 ? 128 : 256), sizeof(float) * n_splits, st>>>(
-        part_acc, part_ml, n_splits, out, (bf16_t*)out_bf16, HM, dv);
+        part_acc, part_ml, n_splits, out, (bf16_t*)out_bf16, HM, dv, ldo);
     SD_CHECK_LAUNCH("sd_masked_softmax_attention (merge)");
   }
   return SD_OK;

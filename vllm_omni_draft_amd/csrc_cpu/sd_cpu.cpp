@@ -1588,6 +1588,48 @@ extern "C" int sd_residual_norm_scaled(float*, const float*, int, const void*, c
                                        int, int, sd_stream_t) {
   UNSUPPORTED("sd_residual_norm_scaled");
 }
+extern "C" int sd_linear_two_inputs(const void*, const void*, const void*, int64_t, int, float*, int64_t, int, int,
+                                    int, sd_stream_t) {
+  UNSUPPORTED("sd_linear_two_inputs");
+}
+extern "C" int sd_distance_softmax_attention(const float*, int64_t, const void*, const void*, int, const int32_t*,
+                                             const int32_t*, const int32_t*, int, int, int, int, int, int, int, int,
+                                             int, int, int, float, float, const float*, const float*, const float*,
+                                             float*, void*, int64_t, void*, size_t, sd_stream_t) {
+  UNSUPPORTED("sd_distance_softmax_attention");
+}
+extern "C" int sd_joint_residual(float*, const int32_t*, const float*, const void*, float*, const void*, const void*,
+                                 int, float, float*, void*, float*, void*, const void*, int, float*, const int32_t*,
+                                 const int32_t*, int, int, sd_stream_t) {
+  UNSUPPORTED("sd_joint_residual");
+}
+extern "C" int sd_conv_add_rows(const float*, int64_t, const void*, int, float*, const int32_t*, const int32_t*,
+                                const int32_t*, int, float*, void*, int64_t, int, int, int, sd_stream_t) {
+  UNSUPPORTED("sd_conv_add_rows");
+}
+extern "C" int sd_conv_tail(const float*, int64_t, const void*, int, float*, const int32_t*, int, int, int,
+                            sd_stream_t) {
+  UNSUPPORTED("sd_conv_tail");
+}
+extern "C" int sd_poly_norm_rows(const float*, int64_t, const void*, int, const float*, float, float*, void*,
+                                 int64_t, int, int, sd_stream_t) {
+  UNSUPPORTED("sd_poly_norm_rows");
+}
+extern "C" int sd_conv_attn_prep(const float*, int64_t, const void*, const void*, int, float*, int, int, int, int,
+                                 int, const void*, const void*, int, float, float, int, float*, void*, void*,
+                                 const int32_t*, const int32_t*, const int32_t*, int, const int32_t*, int, int, int,
+                                 const sd_poly_norm*, sd_stream_t) {
+  UNSUPPORTED("sd_conv_attn_prep");
+}
+extern "C" int sd_mlstm_scan(const float*, const float*, const float*, const float*, const float*, int64_t,
+                             const float*, const float*, float, float, float*, float*, const float*, const int32_t*,
+                             int, float*, float*, int, int, int, sd_stream_t) {
+  UNSUPPORTED("sd_mlstm_scan");
+}
+extern "C" int sd_mlstm_read(const float*, const float*, float*, const int32_t*, const float*, int64_t, const void*,
+                             int, float, float*, void*, int64_t, int, int, int, const sd_poly_norm*, sd_stream_t) {
+  UNSUPPORTED("sd_mlstm_read");
+}
 extern "C" int sd_scale_rows(float*, int64_t, float, int, int, sd_stream_t) { UNSUPPORTED("sd_scale_rows"); }
 extern "C" sd_seq_model* sd_seq_model_create(const sd_seq_model_desc*) {
   set_error("sd_seq_model_create: not provided by the CPU build of the library");

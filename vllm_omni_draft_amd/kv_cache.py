@@ -152,8 +152,11 @@ class SeqCache:
     keyed by the layer's place in the order of running (cfg.runs): a layer that runs several
     times over keeps a cache for every pass.  A softmax attention with several score maps per head
     keeps that many key rows per kv head and token (cache head = kv head * maps + map) and one value
-    row; a layer that reads another layer's keys and values owns no tensors: kv_source names the
-    run whose tensors it reads."""
+    row; a layer that reads another layer's keys and values owns no key and value tensors: kv_source
+    names the run whose tensors it reads.  Convolutions keep their last inputs, f32: of q, k and v in
+    conv[layer] [slots, taps - 1, channels], of a mixer's input in in_conv[layer] [slots, taps - 1,
+    width].  A matrix memory with exponential gates keeps state[layer], its normalizer
+    nstate[layer] [slots, heads, dim] and its running maximum mstate[layer] [slots, heads]."""
 
     def __init__(self, cfg, dtype: torch.dtype, max_seqs: int, num_pages: int, max_seq_len: int,
                  device="cuda"):
@@ -171,11 +174,21 @@ class SeqCache:
         self.pk: Dict[int, torch.Tensor] = {}
         self.pv: Dict[int, torch.Tensor] = {}
         self.conv: Dict[int, torch.Tensor] = {}
+        self.in_conv: Dict[int, torch.Tensor] = {}
+        self.nstate: Dict[int, torch.Tensor] = {}
+        self.mstate: Dict[int, torch.Tensor] = {}
+
+        def f32(*shape):
+            return torch.zeros(*shape, dtype=torch.float32, device=device)
         self.kv_source: Dict[int, int] = {}
         self.has_pages = False
         run_of = {li: i for i, (li, _) in enumerate(cfg.runs)}   # (a layer others read runs once)
         for i, (li, _) in enumerate(cfg.runs):
             m = cfg.layers[li].mixer
+            if cfg.layers[li].in_taps > 1:
+                self.in_conv[i] = f32(max_seqs, cfg.layers[li].in_taps - 1, cfg.width)
+            if m.conv_taps > 1:
+                self.conv[i] = f32(max_seqs, m.conv_taps - 1, m.conv_channels)
             if m.kv_from >= 0:
                 self.has_pages = True
                 self.kv_source[i] = run_of[m.kv_from]
@@ -204,7 +217,9 @@ class SeqCache:
                 self.pk[i] = torch.zeros(num_pages, m.kv_heads, ps, m.dim, dtype=torch.float32, device=device)
                 self.pv[i] = torch.zeros(num_pages, m.kv_heads, ps, m.vdim, dtype=torch.float32, device=device)
             else:
-                self.state[i] = torch.zeros(max_seqs, m.heads, m.dim, m.vdim, dtype=torch.float32, device=device)
+                self.state[i] = f32(max_seqs, m.heads, m.dim, m.vdim)
+                if m.kind == "mlstm":
+                    self.nstate[i], self.mstate[i] = f32(max_seqs, m.heads, m.dim), f32(max_seqs, m.heads)
 
     def keys_of(self, run: int):
         """The key cache run `run` reads: its own, or the one of the run it shares with."""
@@ -240,5 +255,6 @@ class SeqCache:
         self.slots.free(slot)
 
     def nbytes(self) -> int:
-        return sum(t.numel() * t.element_size() for d in (self.state, self.k, self.v, self.pk, self.pv, self.conv)
+        return sum(t.numel() * t.element_size() for d in (self.state, self.k, self.v, self.pk, self.pv, self.conv,
+                                                                  self.in_conv, self.nstate, self.mstate)
                    for t in d.values())

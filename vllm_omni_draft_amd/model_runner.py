@@ -201,7 +201,8 @@ class DecoderModel:
 
 
 # ---------------------------------------------------------------------------------------------
-_MIX_KIND = {"retention": 0, "gla": 1, "attention": 2, "latent_attention": 3, "parallel": 4, "softmax_attention": 5}
+_MIX_KIND = {"retention": 0, "gla": 1, "attention": 2, "latent_attention": 3, "parallel": 4, "softmax_attention": 5,
+             "mlstm": 6}
 
 
 class SeqModel:
@@ -266,6 +267,22 @@ class SeqModel:
                     w_shared_in=rm(t.w_shared_in), w_shared_in_tiled=tl(t.w_shared_in),
                     w_shared_down=rm(t.w_shared_down), w_shared_down_tiled=tl(t.w_shared_down),
                     w_shared_gate=_ptr(t.w_shared_gate))
+                continue
+            if cfg.block == "joint":
+                layers[i] = _lib.SeqLayer(
+                    kind=_MIX_KIND[m.kind], block=3, heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim,
+                    ff=spec.ff, q_scale=m.dim ** -0.5 if m.kind == "mlstm" else 1.0, score_scale=m.scale,
+                    window=m.window or 0x7fffffff, softcap=m.softcap, norm_w=_ptr(t.norm_w), norm2_w=_ptr(t.norm2_w),
+                    w_in=rm(t.w_in), w_in_tiled=tl(t.w_in), w_o=rm(t.w_o), w_o_tiled=tl(t.w_o),
+                    w_in_bias=_ptr(t.w_in_bias), w_o_bias=_ptr(t.w_o_bias), mix_rows=t.mix_rows,
+                    in_conv_w=_ptr(t.in_conv_w), in_taps=spec.in_taps, in_conv_state=_ptr(cache.in_conv.get(i)),
+                    conv_w=_ptr(t.conv_w), s_taps=m.conv_taps, conv_state=_ptr(cache.conv.get(i)),
+                    q_norm_w=_ptr(t.q_norm_w), k_norm_w=_ptr(t.k_norm_w), kv_shared=int(m.kv_from >= 0),
+                    q_temp_coef=m.q_temp_coef, q_temp_every=m.q_temp_every, dist1=_ptr(t.dist1), dist2=_ptr(t.dist2),
+                    k_cache=_ptr(cache.keys_of(i)), v_cache=_ptr(cache.values_of(i)),
+                    state=_ptr(cache.state.get(i)), n_state=_ptr(cache.nstate.get(i)), m_state=_ptr(cache.mstate.get(i)),
+                    gate_bias=_ptr(t.gate_bias), gate_cap=m.gate_cap, s_norm_w=_ptr(t.s_norm_w),
+                    ff_bias=_ptr(t.ff_bias), ff_coef=_ptr(t.ff_coef))
                 continue
             if cfg.block == "postnorm":
                 sd, ex = m.ssd, spec.experts

@@ -366,6 +366,15 @@ class SeqLayerTensors:
     w_o_bias: Optional[torch.Tensor] = None    # [width]
     router_bias: Optional[torch.Tensor] = None  # f32 [experts]
     diff_lambda: float = 0.0                   # differential attention: the second map's factor
+    # layers whose sublayers read the same residual: w_in [mixer rows, padded to mix_rows | ff up rows],
+    # w_o [width, mixer output | ff] (the mixer's output matrix and the feed-forward's down matrix)
+    mix_rows: int = 0
+    in_conv_w: Optional[torch.Tensor] = None   # [width, taps]: the mixer's input convolution
+    dist1: Optional[torch.Tensor] = None       # f32 [heads]
+    dist2: Optional[torch.Tensor] = None
+    gate_bias: Optional[torch.Tensor] = None   # f32 [2*heads]: input gates', then forget gates'
+    ff_bias: Optional[torch.Tensor] = None     # [ff]
+    ff_coef: Optional[torch.Tensor] = None     # f32 [4]
 
 
 @dataclass
@@ -426,8 +435,9 @@ def seq_from_state_dict(cfg, state: Dict[str, torch.Tensor], device="cuda",
             return ops.tile_weights(d, ops.TILE_PLAIN)
         return d
 
-    if cfg.block == "sandwich":
-        layers = [_sandwich_layer(cfg, i, get, dev, mat) for i in range(cfg.n_layers)]
+    if cfg.block in ("sandwich", "joint"):
+        one = _sandwich_layer if cfg.block == "sandwich" else _joint_layer
+        layers = [one(cfg, i, get, dev, mat) for i in range(cfg.n_layers)]
         head = mat(get("head", (cfg.vocab, W)))
         return SeqModelWeights(cfg, dtype, dev(get("embed", (cfg.vocab, W))), dev(get("final.norm", (W,))), layers,
                                head if isinstance(head, ops.TiledWeight) else None, dev(get("head", (cfg.vocab, W))),
@@ -596,6 +606,47 @@ def _sandwich_layer(cfg, i: int, get, dev, mat) -> SeqLayerTensors:
     return lt
 
 
+def _joint_layer(cfg, i: int, get, dev, mat) -> SeqLayerTensors:
+    """Layer i of a model whose sublayers read the same residual: the matrices that read the mixer's
+    input stacked, padded with zero rows to a multiple of 16 and followed by the feed-forward's up
+    matrix; the mixer's output matrix and the down matrix side by side, so that one product adds
+    both sublayers; the convolutions of q, k and v as one over the stacked channels."""
+    l, p, W = cfg.layers[i], f"l{i}.", cfg.width
+    m = l.mixer
+    H, G, dk, dv, F = m.heads, m.kv_heads, m.dim, m.vdim, l.ff
+    if m.kind == "mlstm":
+        names = [("q", H * dk), ("k", H * dk), ("v", H * dv), ("g", H * dv), ("i", H), ("f", H)]
+    else:
+        names = [("q", H * dk)] + ([("k", G * dk), ("v", G * dv)] if m.kv_from < 0 else [])
+    parts = [get(p + "mix." + n, (rows, W)).float() for n, rows in names]
+    used = sum(rows for _, rows in names)
+    mix_rows = -(-used // 16) * 16
+    parts.append(torch.zeros(mix_rows - used, W))
+    out = [get(p + "mix.o", (W, H * dv)).float()]
+    if F:
+        parts.append(get(p + "mlp.up", (F, W)).float())
+        out.append(get(p + "mlp.down", (W, F)).float())
+    lt = SeqLayerTensors(norm_w=dev(get(p + "norm1", (W,))), w_in=mat(torch.cat(parts)), w_o=mat(torch.cat(out, dim=1)),
+                         r1_bias=None, mix_rows=mix_rows)
+    if l.in_taps:
+        lt.in_conv_w = dev(get(p + "canon1", (W, l.in_taps)))
+    if m.kind == "mlstm":
+        lt.gate_bias = dev(torch.cat([get(p + "mix.i.b", (H,)).float(), get(p + "mix.f.b", (H,)).float()]), torch.float32)
+        lt.s_norm_w = dev(get(p + "mix.norm", (H * dv,)))
+    else:
+        lt.conv_w = dev(torch.cat([get(p + f"mix.{n}.conv", (rows, m.conv_taps)) for n, rows in names]))
+        if m.qkv_bias:
+            lt.w_in_bias = dev(torch.cat([get(p + f"mix.{n}.b", (rows,)) for n, rows in names]))
+        lt.q_norm_w = dev(get(p + "mix.q.norm", (dk,)))
+        lt.k_norm_w = dev(get(p + "mix.k.norm", (dk,))) if m.kv_from < 0 else None
+        if m.distance_bias:
+            lt.dist1, lt.dist2 = dev(get(p + "mix.r1", (H,)), torch.float32), dev(get(p + "mix.r2", (H,)), torch.float32)
+    if F:
+        lt.norm2_w, lt.ff_bias = dev(get(p + "norm2", (W,))), dev(get(p + "mlp.up.b", (F,)))
+        lt.w_o_bias, lt.ff_coef = dev(get(p + "mlp.down.b", (W,))), dev(get(p + "mlp.act", (4,)), torch.float32)
+    return lt
+
+
 def seq_from_safetensors_dir(cfg, model_dir: str, device="cuda",
                              dtype: torch.dtype = torch.bfloat16) -> SeqModelWeights:
     from safetensors import safe_open
@@ -624,6 +675,8 @@ def seq_random_state(cfg, seed: int = 0) -> Dict[str, torch.Tensor]:
         return _postnorm_random_state(cfg, rn)
     if cfg.block == "sandwich":
         return _sandwich_random_state(cfg, rn)
+    if cfg.block == "joint":
+        return _joint_random_state(cfg, rn)
     st = {"embed": rn(cfg.vocab, W, s=1.0), "final.norm": rn(W, s=0.1)}
     for i, l in enumerate(cfg.layers):
         m, p = l.mixer, f"l{i}."
@@ -739,6 +792,36 @@ def _sandwich_random_state(cfg, rn) -> Dict[str, torch.Tensor]:
                 st[p + f"mlp.{nm}.up"], st[p + f"mlp.{nm}.down"] = rn(F, W, s=W ** -0.5), rn(W, F, s=F ** -0.5)
             if ex.shared_ff and ex.shared_gate:
                 st[p + "mlp.shared.sg"] = rn(1, W, s=W ** -0.5)
+    return st
+
+
+def _joint_random_state(cfg, rn) -> Dict[str, torch.Tensor]:
+    W = cfg.width
+    st = {"embed": rn(cfg.vocab, W, s=1.0), "final.norm": 1 + rn(W, s=0.1), "head": rn(cfg.vocab, W, s=W ** -0.5)}
+    for i, l in enumerate(cfg.layers):
+        m, p = l.mixer, f"l{i}."
+        H, G, dk, dv = m.heads, m.kv_heads, m.dim, m.vdim
+        st[p + "norm1"] = 1 + rn(W, s=0.1)
+        if l.in_taps:
+            st[p + "canon1"] = rn(W, l.in_taps, s=0.3)
+        if m.kind == "mlstm":
+            for n, rows in (("q", H * dk), ("k", H * dk), ("v", H * dv), ("g", H * dv), ("i", H), ("f", H)):
+                st[p + "mix." + n] = rn(rows, W, s=W ** -0.5)
+            st[p + "mix.i.b"], st[p + "mix.f.b"], st[p + "mix.norm"] = rn(H, s=1.0), rn(H, s=1.0) + 3.0, 1 + rn(H * dv, s=0.1)
+        else:
+            for n, rows in [("q", H * dk)] + ([("k", G * dk), ("v", G * dv)] if m.kv_from < 0 else []):
+                st[p + "mix." + n], st[p + f"mix.{n}.conv"] = rn(rows, W, s=W ** -0.5), rn(rows, m.conv_taps, s=0.6)
+                if m.qkv_bias:
+                    st[p + f"mix.{n}.b"] = rn(rows, s=0.2)
+                if n != "v":
+                    st[p + f"mix.{n}.norm"] = 1 + rn(dk, s=0.1)
+            if m.distance_bias:
+                st[p + "mix.r1"], st[p + "mix.r2"] = rn(H, s=0.5).abs(), rn(H, s=0.5).abs()
+        st[p + "mix.o"] = rn(W, H * dv, s=(H * dv) ** -0.5)
+        if l.ff:
+            st[p + "norm2"], st[p + "mlp.act"] = 1 + rn(W, s=0.1), rn(4, s=0.5)
+            st[p + "mlp.up"], st[p + "mlp.up.b"] = rn(l.ff, W, s=W ** -0.5), rn(l.ff, s=0.2)
+            st[p + "mlp.down"], st[p + "mlp.down.b"] = rn(W, l.ff, s=l.ff ** -0.5), rn(W, s=0.2)
     return st
 
 
