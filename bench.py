@@ -102,7 +102,7 @@ def parse():
     ap.add_argument("--tp-draft", choices=["replicated", "sharded"], default="replicated",
                     help="the draft whole on every rank (no exchange in its passes), or sharded "
                          "like the target with a vocabulary-parallel head")
-    ap.add_argument("--family", choices=["spec", "puguzen", "naburax", "fepopel", "zopupel"], default="spec",
+    ap.add_argument("--family", choices=["spec", "puguzen", "naburax", "fepopel", "zopupel", "gufasun"], default="spec",
                     help="spec: the headline speculative-decoding workload (default).  puguzen: prefill and "
                          "decode throughput of the Puguzen decoder family (recurrent and windowed layers) at "
                          "layer sizes of real models, beside a Llama-style decoder of equal size, with the "
@@ -114,9 +114,12 @@ def parse():
                          "layers), beside the Naburax family at equal size.  zopupel: the same for the "
                          "Zopupel family (differential attention with shared keys and values, attention whose "
                          "values are its keys, gated experts with a router bias beside a shared one), beside "
-                         "the Fepopel family at equal size")
+                         "the Fepopel family at equal size.  gufasun: the same for the Gufasun family (both "
+                         "sublayers on one residual, convolved window attention with a distance bias, matrix "
+                         "memories with exponential gates), beside the Puguzen family at equal size and the "
+                         "Naburax family's like kernels")
     ap.add_argument("--seq-sizes", default="w1024,w2048,w4096",
-                    help="--family puguzen / naburax / fepopel / zopupel: sizes to run")
+                    help="--family puguzen / naburax / fepopel / zopupel / gufasun: sizes to run")
     return ap.parse_args()
 
 
@@ -1228,8 +1231,126 @@ def main_zop_family(args):
                       "data": "synthetic", "n_gpus": 1, "steps": steps, "warmup": warm, "sizes": results}))
 
 
+# --family gufasun
+GUF_TAPS, GUF_CAP = 4, 15.0
+
+
+def _guf_config(sz):
+    """Four layers as the Puguzen bench model has: window attention and matrix memories in turn, the
+    second attention layer reading the first one's keys and values."""
+    from vllm_omni_draft_amd.config import MixerSpec, SeqLayerSpec, SeqModelConfig
+    H, G, D = sz["heads"], sz["kv_heads"], SEQ_HEAD
+    att = dict(kind="softmax_attention", heads=H, dim=D, vdim=D, kv_heads=G, scale=D ** -0.5, window=SEQ_WINDOW,
+               softcap=50.0, qk_head_norm=True, qkv_bias=True, conv_taps=GUF_TAPS, q_temp_coef=0.1, q_temp_every=1024,
+               distance_bias=True)
+    mem = MixerSpec("mlstm", H, D, D, gate_cap=GUF_CAP)
+    mixers = [MixerSpec(**att), mem, MixerSpec(kv_from=0, **att), mem]
+    cfg = SeqModelConfig("gufasun", sz["width"], SEQ_VOCAB,
+                         [SeqLayerSpec(m, sz["ff"], ff_act="polynorm", in_taps=GUF_TAPS) for m in mixers],
+                         name="gufasun-bench", block="joint", embed_scale=sz["width"] ** 0.5, tied_head=False)
+    cfg.validate()
+    return cfg
+
+
+def guf_kernel_rooflines(cfg, device, ctx, rows):
+    """The family's own kernels alone at `rows` token rows of one sequence that ends at position
+    ctx, as fep_kernel_rooflines reports them; `like` names the kernel of another family each is
+    set beside."""
+    from vllm_omni_draft_amd import ops
+    att, mem = cfg.layers[0].mixer, cfg.layers[1].mixer
+    W, F = cfg.width, cfg.layers[0].ff
+    g = torch.Generator(device="cpu").manual_seed(0)
+    rn = lambda *s: torch.randn(*s, generator=g).to(device)
+    bf = lambda *s: torch.randn(*s, generator=g).to(torch.bfloat16).to(device)
+    pages = -(-ctx // ops.PAGE)
+    tables = torch.arange(pages, dtype=torch.int32, device=device).view(1, -1)
+    pos_l = list(range(ctx - rows, ctx))
+    pos = torch.tensor(pos_l, dtype=torch.int32, device=device)
+    slot = torch.zeros(rows, dtype=torch.int32, device=device)
+    ent = torch.tensor([[0, 0, rows, ctx - rows]], dtype=torch.int32, device=device)
+    keys = sum(min(p + 1, att.window) for p in pos_l)
+    span = min(ctx, att.window + rows - 1)
+    H, G, D, taps = att.heads, att.kv_heads, att.dim, att.conv_taps
+    out = []
+    kc, vc, q = bf(pages, G, ops.PAGE, D), bf(pages, G, ops.PAGE, D), rn(rows, H * D)
+    d1, d2 = rn(H).abs(), rn(H).abs()
+    us = _events(lambda: ops.distance_softmax_attention(q, kc, vc, pos, slot, tables, H, G, D, D, att.scale, att.window,
+                                                        att.softcap, d1, d2, bf16_only=True), 5)
+    # (matrix-core work where rows share their keys: priced at the f32 vector peak, like the kernel beside it)
+    out.append(("distance_softmax_attention", "window_softmax_attention (grouped heads)", us,
+                G * 2 * D * 2 * span + rows * H * D * 6, 2.0 * keys * H * 2 * D, F32_VALU_PEAK_TFLOPS))
+    Cq = (H + 2 * G) * D
+    proj, cw, cst, cb = rn(rows, Cq), bf(Cq, taps), torch.zeros(1, taps - 1, Cq, device=device), bf(Cq)
+    qw, kw = bf(D), bf(D)
+    us = _events(lambda: ops.conv_attn_prep(proj, cw, cst, H, G, D, D, qw, kw, 1e-5, kc, vc, pos, slot, ent, tables, bias=cb,
+                                            temp=(0.1, 1024)), 5)
+    out.append(("conv_attn_prep", "qk_head_norm_append", us, rows * (4 * Cq + 4 * H * D + 2 * 2 * G * D) + 2 * Cq * (taps + 1),
+                0.0, F32_VALU_PEAK_TFLOPS))
+    Hm, dk, dv = mem.heads, mem.dim, mem.vdim
+    qm, km, vm, zi, zf = rn(rows, Hm * dk), rn(rows, Hm * dk), rn(rows, Hm * dv), rn(rows, Hm), rn(rows, Hm) + 3
+    S, N_, M_ = (torch.zeros(1, Hm, *s, device=device) for s in ((dk, dv), (dk,), ()))
+    bi, bff, buf = rn(Hm), rn(Hm), torch.cat([qm, km, vm, zi, zf], 1).contiguous()
+    num, mr = torch.empty(rows, Hm, dv + 1, device=device), torch.empty(rows, Hm, device=device)
+    us = _events(lambda: ops.mlstm_scan_packed(buf, bi, bff, mem.gate_cap, S, N_, M_, ent, num, mr, dk ** -0.5), 5)
+    out.append(("mlstm_scan", "decay_scan_rows", us,
+                4 * (rows * (2 * Hm * dk + 2 * Hm * dv + 4 * Hm) + 2 * Hm * dk * (dv + 1)),
+                rows * Hm * dk * (dv + 1) * 5.0, F32_VALU_PEAK_TFLOPS))
+    gate, w = rn(rows, Hm * dv), bf(Hm * dv)
+    us = _events(lambda: ops.mlstm_read(num, mr, M_, slot, gate, w, 1e-5), 5)
+    out.append(("mlstm_read", "head_post", us, rows * Hm * dv * 12, 0.0, F32_VALU_PEAK_TFLOPS))
+    z, zb, coef = rn(rows, F), bf(F), rn(4)
+    us = _events(lambda: ops.poly_norm_rows(z, coef, 1e-5, bias=zb, bf16=True), 5)
+    out.append(("poly_norm_rows", "act_rows / relu_mul_rows", us, rows * F * 6, 0.0, F32_VALU_PEAK_TFLOPS))
+    x, a, ab, w1, w2 = rn(rows, W), rn(rows, W), bf(W), bf(W), bf(W)
+    icw, ics = bf(W, GUF_TAPS), torch.zeros(1, GUF_TAPS - 1, W, device=device)
+    if rows == 1:
+        us = _events(lambda: ops.joint_residual(x, a, ab, w1, w2, bf16=True, conv_w=icw, conv_state=ics, row_pos=pos,
+                                                row_slot=slot), 5)
+        out.append(("joint_residual (with the convolution)", "gated_residual_norm", us, rows * W * 16, 0.0,
+                    F32_VALU_PEAK_TFLOPS))
+    else:
+        us = _events(lambda: ops.joint_residual(x, a, ab, w1, w2), 5)
+        out.append(("joint_residual", "gated_residual_norm", us, rows * W * 20, 0.0, F32_VALU_PEAK_TFLOPS))
+        us = _events(lambda: ops.conv_add_rows(x, icw, ics, pos, slot, ent, bf16=True), 5)
+        out.append(("conv_add_rows", "causal_conv_rows", us, rows * W * 6, 0.0, F32_VALU_PEAK_TFLOPS))
+    res = []
+    for name, like, us, nbytes, flops, peak in out:
+        floor_us = max(nbytes / (HBM_PEAK_GBS * 1e3), flops / (peak * 1e6))
+        res.append({"kernel": name, "like": like, "rows": rows, "ctx": ctx, "avg_us": round(us, 2),
+                    "min_bytes": int(nbytes), "flops": int(flops), "achieved_gbs": round(nbytes / us * 1e-3, 1),
+                    "achieved_tflops": round(flops / us * 1e-6, 2), "roofline_us": round(floor_us, 2),
+                    "times_roofline": round(us / floor_us, 1)})
+    return res
+
+
+def main_guf_family(args):
+    """Prefill and decode throughput of the Gufasun family beside the Puguzen family at equal
+    width, heads, window and feed-forward width (both bf16, seeded random weights), with the like
+    kernels of the Naburax family, one JSON line."""
+    if not torch.cuda.is_available():
+        raise SystemExit("bench.py needs a GPU (there is no CPU path)")
+    device = torch.device("cuda", 0)
+    P, B, steps, warm = args.prompt_len, 4, args.steps, args.warmup
+    results = []
+    for name in args.seq_sizes.split(","):
+        sz = SEQ_SIZES[name]
+        cfg, pcfg, ncfg = _guf_config(sz), _seq_config(sz), _nab_config(NAB_SIZES[name])
+        mine = _run_seq_engine(cfg, device, P, B, steps, warm)
+        kern = guf_kernel_rooflines(cfg, device, P, 1) + guf_kernel_rooflines(cfg, device, P, min(P, 1024))
+        other = _run_seq_engine(pcfg, device, P, B, steps, warm)
+        like = nab_kernel_rooflines(ncfg, device, P, 1) + nab_kernel_rooflines(ncfg, device, P, min(P, 1024))
+        results.append({"size": name, **sz, "layers": [l.mixer.kind for l in cfg.layers], "head_dim": SEQ_HEAD,
+                        "window": SEQ_WINDOW, "taps": GUF_TAPS, "prompt_len": P, "decode_batch": B, "gufasun": mine,
+                        "puguzen_equal_size": other, "kernels": kern, "naburax_kernels": like})
+    print(json.dumps({"metric": "gufasun_family_throughput", "unit": "tokens/s", "dtype": "bf16",
+                      "data": "synthetic", "n_gpus": 1, "steps": steps, "warmup": warm, "sizes": results}))
+
+
 def main():
     args = parse()
+    if args.family == "gufasun":
+        main_guf_family(args)
+        return
     if args.family == "zopupel":
         main_zop_family(args)
         return

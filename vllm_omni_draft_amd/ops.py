@@ -1444,6 +1444,146 @@ def residual_norm_scaled(x, a, w_post, mult, n_a=1, a_bias=None, b=None, w_next=
     return h
 
 
+def linear_two_inputs(W: "TiledWeight", x, x2, n_first: int) -> torch.Tensor:
+    """One tiled weight that stacks two matrices: x bf16 [M <= 16, K] times its first n_first (a
+    multiple of 16) rows, x2 (same shape) times the others -> f32 [M, N]."""
+    if x.dtype != torch.bfloat16 or x2.dtype != torch.bfloat16 or x.shape != x2.shape or x.stride() != x2.stride() \
+            or x.shape[1] != W.K:
+        raise _lib.SdError("linear_two_inputs: two bfloat16 inputs of one shape, as wide as the weight")
+    out = torch.empty(x.shape[0], W.N, dtype=torch.float32, device=x.device)
+    _lib.check(_lib.load().sd_linear_two_inputs(W.data.data_ptr(), x.data_ptr(), x2.data_ptr(), x.stride(0), int(n_first),
+                                                _p(out), W.N, x.shape[0], W.N, W.K, _stream()), "sd_linear_two_inputs")
+    return out
+
+
+def distance_softmax_attention(q, k_cache, v_cache, row_pos, row_slot, block_tables, H, G, dk, dv, scale, window=0,
+                               softcap=0.0, dist1=None, dist2=None, split=True, ldo=0, bf16_only=False):
+    """Grouped-query softmax attention over a sliding window (0: every earlier token) whose capped
+    scores lose dist1[h] * ln(1 + dist2[h] * distance); q f32 [rows, H*dk] -> f32 [rows, H*dv], or, with
+    ldo > H*dv, a view of rows that far apart; bf16_only: bfloat16 instead."""
+    _f32(q, "q")
+    window, ldo = int(window) or 0x7fffffff, int(ldo) or H * dv
+    dt = torch.bfloat16 if bf16_only else torch.float32
+    out = torch.zeros(q.shape[0], ldo, dtype=dt, device=q.device)
+    lib = _lib.load()
+    n = int(lib.sd_multimap_softmax_attention_scratch_bytes(q.shape[0], H, 1, dv, window, 0, 0,
+                                                            block_tables.shape[1] * PAGE)) if split else 0
+    scratch = torch.empty(n, dtype=torch.uint8, device=q.device) if n else None
+    _lib.check(lib.sd_distance_softmax_attention(
+        _p(q), q.shape[1], _p(k_cache), _p(v_cache), int(k_cache.dtype == torch.float32), _p(row_pos), _p(row_slot),
+        _p(block_tables), block_tables.shape[1], PAGE, q.shape[0], H, G, 1, dk, dv, window, 0, 0, float(scale),
+        float(softcap), None, _p(dist1), _p(dist2), None if bf16_only else _p(out), _p(out) if bf16_only else None, ldo,
+        _p(scratch), n, _stream()), "sd_distance_softmax_attention")
+    return out[:, :H * dv]
+
+
+def joint_residual(x, a=None, a_bias=None, w1=None, w2=None, eps=1e-5, rows=None, x_copy=False, bf16=False, conv_w=None,
+                   conv_state=None, row_pos=None, row_slot=None):
+    """sd_joint_residual, in place on x f32 [rows, W] (rows given: x is only read).  Returns (h1, h2,
+    copy): the two layer norms (bf16: as bfloat16), h1 with its convolution added when conv_w
+    [W, taps] is given (rows alone in their entries; conv_state moves on), and the row before them."""
+    _f32(x, "x")
+    n, W = (rows.numel() if rows is not None else x.shape[0]), x.shape[1]
+    dt = torch.bfloat16 if bf16 else torch.float32
+    h1 = torch.empty(n, W, dtype=dt, device=x.device) if w1 is not None else None
+    h2 = torch.empty(n, W, dtype=dt, device=x.device) if w2 is not None else None
+    copy = torch.empty(n, W, dtype=torch.float32, device=x.device) if x_copy else None
+    typed = next((t for t in (w1, a_bias, conv_w) if t is not None), None)
+    f32p, b16p = (lambda t: None if bf16 else _p(t)), (lambda t: _p(t) if bf16 else None)
+    _lib.check(_lib.load().sd_joint_residual(
+        _p(x), _p(rows), _p(a), _p(a_bias), _p(copy), _p(w1), _p(w2), 1 if typed is None else _wkind(typed, "weights"),
+        float(eps), f32p(h1), b16p(h1), f32p(h2), b16p(h2), _p(conv_w), conv_w.shape[1] if conv_w is not None else 0,
+        _p(conv_state), _p(row_pos), _p(row_slot), n, W, _stream()), "sd_joint_residual")
+    return h1, h2, copy
+
+
+def conv_add_rows(x, w, conv_state, row_pos, row_slot, entries, bf16=False) -> torch.Tensor:
+    """x f32 [rows, C] + its causal convolution with w [C, taps] over each entry; conv_state f32
+    [slots, taps-1, C] (None with one tap) moves on."""
+    _f32(x, "x")
+    out = torch.empty(x.shape, dtype=torch.bfloat16 if bf16 else torch.float32, device=x.device)
+    _lib.check(_lib.load().sd_conv_add_rows(_p(x), x.shape[1], _p(w), _wkind(w, "w"), _p(conv_state), _p(row_pos),
+                                            _p(row_slot), _p(entries), entries.shape[0], None if bf16 else _p(out),
+                                            _p(out) if bf16 else None, x.shape[1], x.shape[0], x.shape[1], w.shape[1],
+                                            _stream()), "sd_conv_add_rows")
+    return out
+
+
+def poly_norm_rows(z, coef, eps, bias=None, bf16=False) -> torch.Tensor:
+    """coef[0] N(z) + coef[1] N(z^2) + coef[2] N(z^3) + coef[3] of z f32 [rows, n] (+ bias), N(y) = y / rms(y)."""
+    _f32(z, "z")
+    _f32(coef, "coef")
+    out = torch.empty(z.shape, dtype=torch.bfloat16 if bf16 else torch.float32, device=z.device)
+    n = z.shape[1]
+    _lib.check(_lib.load().sd_poly_norm_rows(_p(z), n, _p(bias), 1 if bias is None else _wkind(bias, "bias"), _p(coef),
+                                             float(eps), None if bf16 else _p(out), _p(out) if bf16 else None, n,
+                                             z.shape[0], n, _stream()), "sd_poly_norm_rows")
+    return out
+
+
+def _poly_norm_part(z, coef, bias, out):
+    """The sd_poly_norm of an activation computed inside another launch, into f32 out [rows, n]."""
+    return _lib.PolyNorm(z=z.data_ptr(), ldz=z.stride(0), bias=_p(bias), coef=coef.data_ptr(), out=out.data_ptr(),
+                         out_bf16=None, ldo=out.stride(0), n=z.shape[1])
+
+
+def conv_attn_prep(proj, conv_w, conv_state, H, G, dk, dv, q_norm_w, k_norm_w, eps, k_cache, v_cache, row_pos, row_slot,
+                   entries, block_tables, bias=None, temp=(0.0, 0), act=None) -> torch.Tensor:
+    """sd_conv_attn_prep on proj f32 [rows, channels] (q | k | v; q alone when k_cache is None): returns
+    the prepared q f32 [rows, H*dk]; keys and values are appended, conv_state moves on.  act (or
+    None): (z, coef, bias or None, out), an activation of the same rows computed in the launch."""
+    _f32(proj, "proj")
+    q = torch.empty(proj.shape[0], H * dk, dtype=torch.float32, device=proj.device)
+    part = _poly_norm_part(*act) if act is not None else None
+    _lib.check(_lib.load().sd_conv_attn_prep(
+        _p(proj), proj.shape[1], _p(bias), _p(conv_w), conv_w.shape[1], _p(conv_state), H, G, dk, dv,
+        int(k_cache is None), _p(q_norm_w), _p(k_norm_w), _wkind(conv_w, "conv_w"), float(eps), float(temp[0]),
+        int(temp[1]), _p(q), _p(k_cache), _p(v_cache), _p(row_pos), _p(row_slot), _p(entries), entries.shape[0],
+        _p(block_tables), block_tables.shape[1] if block_tables is not None else 0, PAGE, proj.shape[0],
+        C.byref(part) if part is not None else None, _stream()), "sd_conv_attn_prep")
+    return q
+
+
+def mlstm_scan_packed(buf, bi, bf, cap, state, n_state, m_state, entries, num, m_rows, q_scale=1.0) -> None:
+    """sd_mlstm_scan on rows buf f32 [rows, q | k | v | zi | zf] (zi, zf the last 2*H columns) into num
+    [rows, H, dv + 1] and m_rows [rows, H]; state [slots, H, dk, dv] and n_state [slots, H, dk] move on."""
+    _f32(buf, "buf")
+    H, dk, dv = state.shape[1:]
+    ptr, at = [], 0
+    for cols in (H * dk, H * dk, H * dv):
+        ptr.append(buf.data_ptr() + 4 * at)
+        at += cols
+    ptr += [buf.data_ptr() + 4 * (buf.shape[1] - 2 * H), buf.data_ptr() + 4 * (buf.shape[1] - H)]
+    _lib.check(_lib.load().sd_mlstm_scan(*ptr, buf.shape[1], _p(bi), _p(bf), float(cap), float(q_scale), _p(state),
+                                         _p(n_state), _p(m_state), _p(entries), entries.shape[0], _p(num), _p(m_rows), H,
+                                         dk, dv, _stream()), "sd_mlstm_scan")
+
+
+def mlstm_scan(q, k, v, zi, zf, bi, bf, cap, state, n_state, m_state, entries, q_scale=1.0):
+    """mlstm_scan_packed on separate q, k [rows, H*dk], v [rows, H*dv], zi, zf [rows, H]: (num, m_rows)."""
+    buf = torch.cat([q, k, v, zi, zf], dim=1).contiguous()
+    n, H, dv = q.shape[0], state.shape[1], state.shape[3]
+    num = torch.empty(n, H, dv + 1, dtype=torch.float32, device=q.device)
+    m_rows = torch.empty(n, H, dtype=torch.float32, device=q.device)
+    mlstm_scan_packed(buf, bi, bf, cap, state, n_state, m_state, entries, num, m_rows, q_scale)
+    return num, m_rows
+
+
+def mlstm_read(num, m_rows, m_state, row_slot, gate, w, eps, act=None) -> torch.Tensor:
+    """The gated, per-head normed read-out f32 [rows, H*dv] of mlstm_scan's results; m_state [slots, H]
+    moves on.  act as conv_attn_prep's, with rows as far apart as the result's (a part of one buffer)."""
+    n, H, dv = num.shape[0], num.shape[1], num.shape[2] - 1
+    F = act[0].shape[1] if act is not None else 0
+    buf = torch.empty(n, H * dv + F, dtype=torch.float32, device=num.device)
+    part = _poly_norm_part(act[0], act[1], act[2], buf[:, H * dv:]) if act is not None else None
+    _lib.check(_lib.load().sd_mlstm_read(_p(num), _p(m_rows), _p(m_state), _p(row_slot), _p(gate), gate.shape[1], _p(w),
+                                         _wkind(w, "w"), float(eps), _p(buf), None, H * dv + F, n, H, dv,
+                                         C.byref(part) if part is not None else None, _stream()), "sd_mlstm_read")
+    if act is None:
+        return buf
+    return buf[:, :H * dv], buf[:, H * dv:]
+
+
 def matmul_rows_batched(x, w) -> torch.Tensor:
     """x f32 [M, B, K], w [B, N, K] -> f32 [M, B, N]: product b uses w[b]."""
     _f32(x, "x")
