@@ -1275,7 +1275,7 @@ def guf_kernel_rooflines(cfg, device, ctx, rows):
     kc, vc, q = bf(pages, G, ops.PAGE, D), bf(pages, G, ops.PAGE, D), rn(rows, H * D)
     d1, d2 = rn(H).abs(), rn(H).abs()
     us = _events(lambda: ops.distance_softmax_attention(q, kc, vc, pos, slot, tables, H, G, D, D, att.scale, att.window,
-                                                        att.softcap, d1, d2, bf16_only=True), 5)
+                                                        att.softcap, d1, d2, bf16_only=True, entries=ent), 5)
     # (matrix-core work where rows share their keys: priced at the f32 vector peak, like the kernel beside it)
     out.append(("distance_softmax_attention", "window_softmax_attention (grouped heads)", us,
                 G * 2 * D * 2 * span + rows * H * D * 6, 2.0 * keys * H * 2 * D, F32_VALU_PEAK_TFLOPS))
@@ -1291,7 +1291,8 @@ def guf_kernel_rooflines(cfg, device, ctx, rows):
     S, N_, M_ = (torch.zeros(1, Hm, *s, device=device) for s in ((dk, dv), (dk,), ()))
     bi, bff, buf = rn(Hm), rn(Hm), torch.cat([qm, km, vm, zi, zf], 1).contiguous()
     num, mr = torch.empty(rows, Hm, dv + 1, device=device), torch.empty(rows, Hm, device=device)
-    us = _events(lambda: ops.mlstm_scan_packed(buf, bi, bff, mem.gate_cap, S, N_, M_, ent, num, mr, dk ** -0.5), 5)
+    scr = ops.mlstm_scratch(rows, 1, Hm, dk, dv, device)
+    us = _events(lambda: ops.mlstm_scan_packed(buf, bi, bff, mem.gate_cap, S, N_, M_, ent, num, mr, dk ** -0.5, scr), 5)
     out.append(("mlstm_scan", "decay_scan_rows", us,
                 4 * (rows * (2 * Hm * dk + 2 * Hm * dv + 4 * Hm) + 2 * Hm * dk * (dv + 1)),
                 rows * Hm * dk * (dv + 1) * 5.0, F32_VALU_PEAK_TFLOPS))

@@ -1354,15 +1354,18 @@ int sd_residual_norm_scaled(float* x, const float* a, int n_a, const void* a_bia
 /* sd_multimap_softmax_attention whose scores, scaled and capped, lose dist1[unit] * ln(1 +
  * dist2[unit] * (i - j)) with the distance of key j from the row's position i (dist1, dist2 f32
  * [H*maps], or both NULL), and whose output rows are ldo elements apart (out f32 and out_bf16
- * alike; either may be NULL).                                                              */
+ * alike; either may be NULL).  entries (as in sd_seq_batch, or NULL): the rows' portions.  With it,
+ * many rows over bf16 caches (one map, no sinks, no kept tokens, no chunks, dk and dv multiples of 8
+ * up to 128, page 16) run tiled on the matrix cores: queries and weights as sums of two bf16 parts
+ * each against the cache's bf16 rows, f32 accumulation and softmax.                         */
 int sd_distance_softmax_attention(const float* q, int64_t ldq, const void* k_cache,
                                   const void* v_cache, int cache_f32, const int32_t* row_pos,
                                   const int32_t* row_slot, const int32_t* block_tables,
                                   int max_blocks, int page, int n_rows, int H, int G, int maps, int dk,
                                   int dv, int window, int keep_first, int chunk, float scale,
                                   float softcap, const float* sinks, const float* dist1,
-                                  const float* dist2, float* out, void* out_bf16, int64_t ldo,
-                                  void* scratch, size_t scratch_bytes, sd_stream_t stream);
+                                  const float* dist2, const int32_t* entries, int n_entries,
+                                  float* out, void* out_bf16, int64_t ldo, void* scratch, size_t scratch_bytes, sd_stream_t stream);
 /* Residual update with the layer norms of both sublayers that read the result, per row:
  *   x[r] += a[r] + a_bias                                 (a != NULL; a_bias [W] or NULL)
  *   x_copy[r] = x[r]                                      (x_copy != NULL)
@@ -1426,11 +1429,16 @@ int sd_conv_attn_prep(const float* proj, int64_t ld, const void* bias, const voi
  * [rows, H*dk], v [rows, H*dv], zi, zf [rows, H], all ld floats per row; bi, bf f32 [H]; S f32
  * [slots, H, dk, dv], n_state f32 [slots, H, dk], m_state f32 [slots, H] (an entry that starts at
  * position 0 starts from zero).  num f32 [rows, H, dv + 1]: S^T q, then n . q; m_rows f32 [rows, H]: m.
- * S and n_state are moved on; m_state is left to sd_mlstm_read.                             */
+ * S and n_state are moved on; m_state is left to sd_mlstm_read.  With scratch (f32 [], of
+ * sd_mlstm_scratch_bytes, 0: none needed) long portions run in chunks of 64 tokens on the f32 matrix
+ * instruction, every chunk beside the others: the chunks' own sums, a scan over the chunks, then
+ * the tokens' results; otherwise token by token.                                           */
+size_t sd_mlstm_scratch_bytes(int n_rows, int n_entries, int H, int dk, int dv);
 int sd_mlstm_scan(const float* q, const float* k, const float* v, const float* zi, const float* zf,
                   int64_t ld, const float* bi, const float* bf, float cap, float q_scale, float* S,
                   float* n_state, const float* m_state, const int32_t* entries, int n_entries,
-                  float* num, float* m_rows, int H, int dk, int dv, sd_stream_t stream);
+                  int n_rows, float* num, float* m_rows, int H, int dk, int dv, void* scratch,
+                  size_t scratch_bytes, sd_stream_t stream);
 /* What the memory's read-out becomes: o = num / (max(|n . q|, e^-m) + 1e-6) per head, divided by
  * its root mean square over the head's dv channels (eps inside the root), times w [H*dv], times
  * sigmoid(gate [rows, H*dv]); y / y_bf16 [rows, H*dv] (row stride ldy, either may be NULL).  The

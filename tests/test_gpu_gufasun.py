@@ -141,8 +141,10 @@ def test_distance_attention_random(H, Gk, dk, dv, window, cap, cdt):
         a, b = (r1, r2) if dist else (torch.zeros(H), torch.zeros(H))
         want = plain_attention(q, k, v, torch.arange(n), H, Gk, 0.3, cap, a, b, window)
         for rows in (list(range(n)), list(range(17, 90)), [n - 1], [0, 15, 16, 17, 31, 32, 44]):   # prompts, decoded rows
-            for split in (True, False):
+            for split in (True, False):                       # (split: with the rows' portion, where they are one)
                 kw = dict(dist1=dev(a), dist2=dev(b)) if dist else {}
+                if split and len(rows) > 64:
+                    kw["entries"] = i32([[0, 0, len(rows), rows[0]]])
                 got = ops.distance_softmax_attention(dev(q[rows]), kc, vc, i32(rows), i32([0] * len(rows)), bt, H, Gk, dk, dv,
                                                      0.3, window, cap, split=split, ldo=H * dv + 7, **kw)
                 assert rel(got, want[rows]) < 5e-6, (len(rows), split, dist)
@@ -165,7 +167,8 @@ def test_window_visibility_with_one_hot_values():
             r1, r2 = torch.tensor([0.5, 0.0]), torch.tensor([1.5, 2.0])
             for rows in (list(range(n)), [n - 1], [30, 31, 32]):
                 got = ops.distance_softmax_attention(torch.zeros(len(rows), 2 * dk, device=DEV), kc, vc, i32(rows),
-                                                     i32([0] * len(rows)), bt, 2, 1, dk, 128, 1.0, window, 7.0, dev(r1), dev(r2))
+                                                     i32([0] * len(rows)), bt, 2, 1, dk, 128, 1.0, window, 7.0, dev(r1), dev(r2),
+                                                     entries=i32([[0, 0, n, 0]]) if len(rows) == n else None)
                 got = got.double().cpu().view(len(rows), 2, 128)
                 for a, i in enumerate(rows):
                     for h in range(2):
@@ -189,15 +192,49 @@ def test_a_far_key_among_hundreds(cdt):
     v = torch.randn(n, dv, generator=g).to(cdt)
     pages = list(range(44))[::-1]
     kc, vc, bt = fill_pages(k, 1, pages), fill_pages(v, 1, pages), table(pages)
-    rows = list(range(655, 700))
+    rows = list(range(600, 700))
     r1, r2 = torch.tensor([1.5, 0.3]), torch.tensor([0.7, 5.0])
     q = torch.cat([60.0 * k[3].float(), 60.0 * k[650].float()]).repeat(len(rows), 1) + 0.1 * torch.randn(len(rows), 2 * dk, generator=g)
     want = plain_attention(q, k, v, torch.tensor(rows), H, 1, 1.0, 50.0, r1, r2, 0)
-    for sel in (slice(None), slice(44, 45), slice(0, 3)):
+    for sel in (slice(None), slice(99, 100), slice(0, 3), slice(7, 93)):
         got = ops.distance_softmax_attention(dev(q[sel]), kc, vc, i32(rows[sel]), i32([0] * len(rows[sel])), bt, H, 1, dk, dv,
-                                             1.0, 0, 50.0, dev(r1), dev(r2))
-        assert rel(got, want[sel]) < 5e-6
+                                             1.0, 0, 50.0, dev(r1), dev(r2), entries=i32([[0, 0, len(rows[sel]), rows[sel][0]]]))
+        assert rel(got, want[sel]) < 2e-5 if cdt == torch.bfloat16 else 5e-6
         assert rel(got[:, :dv], v[3].float().expand(len(rows[sel]), dv)) < 1e-3
+
+
+@pytest.mark.parametrize("H,Gk,dk,dv", [(4, 1, 128, 128), (3, 3, 40, 64), (6, 2, 64, 104), (4, 2, 128, 56)])
+def test_portions_of_several_sequences_on_the_matrix_cores(H, Gk, dk, dv):
+    """One launch over portions of four sequences: a long one, single tokens, two tokens, one that
+    starts at its first token; each row against the plain attention over its own sequence."""
+    from vllm_omni_draft_amd import ops
+    g = torch.Generator().manual_seed(dk + dv)
+    n, window = 300, 61
+    k, v = torch.randn(4, n, Gk * dk, generator=g).to(torch.bfloat16), torch.randn(4, n, Gk * dv, generator=g).to(torch.bfloat16)
+    order = torch.randperm(76, generator=g).view(4, 19).tolist()
+    kc = torch.zeros(76, Gk, PAGE, dk, dtype=torch.bfloat16, device=DEV)
+    vc = torch.zeros(76, Gk, PAGE, dv, dtype=torch.bfloat16, device=DEV)
+    for s in range(4):
+        for j in range(n):
+            kc[order[s][j // PAGE], :, j % PAGE] = k[s, j].view(Gk, dk).to(DEV)
+            vc[order[s][j // PAGE], :, j % PAGE] = v[s, j].view(Gk, dv).to(DEV)
+    bt = i32(order)
+    portions = [(2, 190, 70), (0, 299, 1), (3, 0, 33), (1, 17, 2)]        # slot, first position, rows
+    q = torch.randn(sum(p[2] for p in portions), H * dk, generator=g)
+    r1, r2 = torch.rand(H, generator=g), torch.rand(H, generator=g) * 3
+    ents, pos, slots, want, at = [], [], [], [], 0
+    for s, p0, m in portions:
+        ents.append([s, at, m, p0])
+        pos += range(p0, p0 + m)
+        slots += [s] * m
+        want.append(plain_attention(q[at:at + m], k[s, :p0 + m], v[s, :p0 + m], torch.arange(p0, p0 + m), H, Gk, 0.2, 4.0, r1,
+                                    r2, window))
+        at += m
+    got = ops.distance_softmax_attention(dev(q), kc, vc, i32(pos), i32(slots), bt, H, Gk, dk, dv, 0.2, window, 4.0, dev(r1),
+                                         dev(r2), entries=i32(ents))
+    assert rel(got, torch.cat(want)) < 5e-6
+    for (s, p0, m), (_, a, _, _), w in zip(portions, ents, want):
+        assert rel(got[a:a + m], w) < 5e-6, (s, p0, m)
 
 
 @pytest.mark.parametrize("W,taps", [(5, 1), (72, 3), (1000, 2), (2048, 4), (4100, 6), (6002, 3)])
@@ -309,8 +346,9 @@ def test_convolved_preparation(H, Gk, dk, dv, taps, temp, shared, wdt):
 
 @pytest.mark.parametrize("H,dk,dv", [(2, 16, 24), (3, 21, 37), (1, 1, 1), (2, 130, 72), (4, 256, 260), (1, 5, 400), (2, 128, 128),
                                      (2, 64, 192), (3, 32, 64), (1, 96, 40)])
-def test_matrix_memory(H, dk, dv):
-    """Scan and read-out in portions of two interleaved sequences (down to single tokens), from slots
+@pytest.mark.parametrize("chunks", [True, False])
+def test_matrix_memory(H, dk, dv, chunks):
+    """Scan (in chunks, and token by token) and read-out in portions of two interleaved sequences (down to single tokens), from slots
     an earlier request left full, against the plain recurrence; the activation that rides along."""
     from vllm_omni_draft_amd import ops
     g = torch.Generator().manual_seed(H * 1000 + dk)
@@ -327,7 +365,7 @@ def test_matrix_memory(H, dk, dv):
         n = hi - lo
         cat = lambda t: dev(torch.cat([t[0, lo:hi], t[1, lo:hi]]))
         num, mr = ops.mlstm_scan(cat(q), cat(k), cat(v), cat(zi), cat(zf), dev(bi), dev(bf), cap, S, N, M,
-                                 i32([[2, 0, n, lo], [0, n, n, lo]]), q_scale=dk ** -0.5)
+                                 i32([[2, 0, n, lo], [0, n, n, lo]]), q_scale=dk ** -0.5, chunks=chunks)
         y, a = ops.mlstm_read(num, mr, M, i32([2] * n + [0] * n), cat(gate), dev(w), eps, act=(cat(z), dev(coef), None))
         for s in range(2):
             got[s].append(y[s * n:(s + 1) * n])

@@ -299,7 +299,7 @@ SIGNATURES = {
                                       vp, i32, i32, vp]),
     "sd_linear_two_inputs": (i32, [vp, vp, vp, i64, i32, vp, i64, i32, i32, i32, vp]),
     "sd_distance_softmax_attention": (i32, [vp, i64, vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32,
-                                            i32, i32, i32, C.c_float, C.c_float, vp, vp, vp, vp, vp, i64, vp,
+                                            i32, i32, i32, C.c_float, C.c_float, vp, vp, vp, vp, i32, vp, vp, i64, vp,
                                             C.c_size_t, vp]),
     "sd_joint_residual": (i32, [vp, vp, vp, vp, vp, vp, vp, i32, C.c_float, vp, vp, vp, vp, vp, i32, vp, vp, vp, i32,
                                 i32, vp]),
@@ -308,8 +308,9 @@ SIGNATURES = {
     "sd_poly_norm_rows": (i32, [vp, i64, vp, i32, vp, C.c_float, vp, vp, i64, i32, i32, vp]),
     "sd_conv_attn_prep": (i32, [vp, i64, vp, vp, i32, vp, i32, i32, i32, i32, i32, vp, vp, i32, C.c_float, C.c_float,
                                 i32, vp, vp, vp, vp, vp, vp, i32, vp, i32, i32, i32, C.POINTER(PolyNorm), vp]),
-    "sd_mlstm_scan": (i32, [vp, vp, vp, vp, vp, i64, vp, vp, C.c_float, C.c_float, vp, vp, vp, vp, i32, vp, vp, i32,
-                            i32, i32, vp]),
+    "sd_mlstm_scratch_bytes": (C.c_size_t, [i32, i32, i32, i32, i32]),
+    "sd_mlstm_scan": (i32, [vp, vp, vp, vp, vp, i64, vp, vp, C.c_float, C.c_float, vp, vp, vp, vp, i32, i32, vp, vp, i32,
+                            i32, i32, vp, C.c_size_t, vp]),
     "sd_mlstm_read": (i32, [vp, vp, vp, vp, vp, i64, vp, i32, C.c_float, vp, vp, i64, i32, i32, i32,
                             C.POINTER(PolyNorm), vp]),
     "sd_seq_model_create": (vp, [C.POINTER(SeqModelDesc)]),

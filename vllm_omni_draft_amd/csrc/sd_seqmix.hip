@@ -994,13 +994,14 @@ InCols in_cols(const sd_seq_layer& l, int W) {
   return c;
 }
 inline size_t al(size_t v) { return (v + 255) & ~(size_t)255; }
+constexpr int kPlanEntries = 64;  // portions of one pass that the matrix memories' scratch is planned for
 constexpr int kWideRows = 256;  // rows one call of the many-row linear family takes
 struct SeqWs {
   size_t x, h, proj, dec, o, y, mix, ffo, hout, hb, yb, actb, houtb, wide, wide_bytes, attn, attn_bytes, total;
   size_t sg;   // a shared expert's gate per row
   // layers normed on their output
   size_t pq, qe, cqb, conv, step, decay, rlog, sel_e, sel_w, dn, moe, moe_bytes;
-  size_t hc, h2b;   // layers whose sublayers read norms of their own
+  size_t hc, h2b, mem, mem_bytes;   // layers whose sublayers read norms of their own
 };
 // column offsets inside the fused input projection of a layer normed on its output
 struct PnCols {
@@ -1080,7 +1081,7 @@ PnCols pn_cols(const sd_seq_layer& l) {
 SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
   const int W = m.d.width;
   size_t proj = 0, hk = 0, hv = 0, ff = 0, wide = 0, attn = 0;
-  size_t pq = 0, qe = 0, cq = 0, conv = 0, sh = 0, ne = 0, top = 0, moe = 0, joint = 0;
+  size_t pq = 0, qe = 0, cq = 0, conv = 0, sh = 0, ne = 0, top = 0, moe = 0, joint = 0, mem = 0;
   const int wr = rows < kWideRows ? rows : kWideRows;
   auto up = [](size_t& a, size_t b) { a = b > a ? b : a; };
   auto need = [&](const void* tiled, int M, int N, int K) {
@@ -1101,6 +1102,7 @@ SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
       if (l.kind == SD_MIX_MLSTM) {
         up(hv, (size_t)l.heads * (l.vdim + 1));
         up(sh, (size_t)l.heads);
+        up(mem, sd_mlstm_scratch_bytes(rows, rows < kPlanEntries ? rows : kPlanEntries, l.heads, l.dim, l.vdim));
       } else {
         up(pq, (size_t)l.heads * l.dim);
         up(attn, sd_multimap_softmax_attention_scratch_bytes(rows, l.heads, 1, l.vdim, l.window, 0, 0, max_ctx));
@@ -1218,6 +1220,8 @@ SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
   w.sg = off;    off += al(R * f);
   w.hc = off;    off += al(R * joint * f);
   w.h2b = off;   off += al(R * joint * 2);
+  w.mem_bytes = mem;
+  w.mem = off;   off += al(mem ? mem : 16);
   w.total = off;
   return w;
 }
@@ -1629,8 +1633,8 @@ int joint_layer(const sd_seq_model& m, const sd_seq_layer& l, const sd_seq_batch
   if (l.kind == SD_MIX_MLSTM) {
     float* m_rows = (float*)(base + w.step);
     SQ_TRY(sd_mlstm_scan(proj + c.q, proj + c.k, proj + c.v, proj + c.i, proj + c.f, ld, l.gate_bias, l.gate_bias + H,
-                         l.gate_cap, l.q_scale, l.state, l.n_state, l.m_state, b.entries, b.n_entries, o, m_rows, H, dk,
-                         dv, stream));
+                         l.gate_cap, l.q_scale, l.state, l.n_state, l.m_state, b.entries, b.n_entries, R, o, m_rows, H,
+                         dk, dv, base + w.mem, w.mem_bytes, stream));
     SQ_TRY(sd_mlstm_read(o, m_rows, l.m_state, b.row_slot, proj + c.g, ld, l.s_norm_w, f32, d.norm_eps, y, yb, K, R, H,
                          dv, pact, stream));
   } else {
@@ -1641,8 +1645,8 @@ int joint_layer(const sd_seq_model& m, const sd_seq_layer& l, const sd_seq_batch
                              b.page, R, pact, stream));
     SQ_TRY(sd_distance_softmax_attention(q, (int64_t)H * dk, l.k_cache, l.v_cache, f32, b.row_pos, b.row_slot,
                                          b.block_tables, b.max_blocks, b.page, R, H, l.kv_heads, 1, dk, dv, l.window, 0,
-                                         0, l.score_scale, l.softcap, nullptr, l.dist1, l.dist2, y, yb, K,
-                                         base + w.attn, w.attn_bytes, stream));
+                                         0, l.score_scale, l.softcap, nullptr, l.dist1, l.dist2, b.entries,
+                                         b.n_entries, y, yb, K, base + w.attn, w.attn_bytes, stream));
   }
   // both sublayers' last matrices side by side: one product adds them
   return seq_linear(l.w_o, l.w_o_tiled, f32, y, nullptr, K, yb, K, nullptr, (float*)(base + w.mix), W, R, W, K, wide_ws,

@@ -1967,8 +1967,8 @@ extern "C" int sd_multimap_softmax_attention(const float* q, int64_t ldq, const 
   SD_REQUIRE(out, SD_ERR_INVALID, "sd_masked_softmax_attention: null argument");
   return sd_distance_softmax_attention(q, ldq, k_cache, v_cache, cache_f32, row_pos, row_slot, block_tables, max_blocks,
                                        page, n_rows, H, G, maps, dk, dv, window, keep_first, chunk, scale, softcap, sinks,
-                                       nullptr, nullptr, out, out_bf16, (int64_t)H * maps * dv, scratch, scratch_bytes,
-                                       stream);
+                                       nullptr, nullptr, nullptr, 0, out, out_bf16, (int64_t)H * maps * dv, scratch,
+                                       scratch_bytes, stream);
 }
 
 extern "C" int sd_distance_softmax_attention(const float* q, int64_t ldq, const void* k_cache, const void* v_cache,
@@ -1976,8 +1976,9 @@ extern "C" int sd_distance_softmax_attention(const float* q, int64_t ldq, const 
                                              const int32_t* block_tables, int max_blocks, int page, int n_rows, int H,
                                              int G, int maps, int dk, int dv, int window, int keep_first, int chunk,
                                              float scale, float softcap, const float* sinks, const float* dist1,
-                                             const float* dist2, float* out, void* out_bf16, int64_t ldo, void* scratch,
-                                             size_t scratch_bytes, sd_stream_t stream) {
+                                             const float* dist2, const int32_t* entries, int n_entries, float* out,
+                                             void* out_bf16, int64_t ldo, void* scratch, size_t scratch_bytes,
+                                             sd_stream_t stream) {
   SD_REQUIRE(q && k_cache && row_pos && row_slot && block_tables && (out || out_bf16) && !dist1 == !dist2, SD_ERR_INVALID,
              "sd_masked_softmax_attention: null argument");
   SD_REQUIRE(ldo >= (int64_t)H * maps * dv, SD_ERR_INVALID, "sd_masked_softmax_attention: output rows too short");
@@ -1988,6 +1989,12 @@ extern "C" int sd_distance_softmax_attention(const float* q, int64_t ldq, const 
   SD_REQUIRE(dv >= 1 && dv <= 512 && (v_cache || dv <= dk), SD_ERR_UNSUPPORTED,
              "sd_masked_softmax_attention: value size %d outside 1..512 (or above the key row it is part of)", dv);
   hipStream_t st = (hipStream_t)stream;
+  if (entries && !cache_f32 && n_rows > kSplitRows && maps == 1 && !sinks && keep_first == 0 && chunk == 0 && v_cache) {
+    const int rc = sd_tiled_window_attention_(q, ldq, k_cache, v_cache, row_pos, block_tables, max_blocks, page, n_rows,
+                                              H, G, dk, dv, window, scale, softcap, dist1, dist2, entries, n_entries, out,
+                                              out_bf16, ldo, stream);
+    if (rc != SD_ERR_UNSUPPORTED) return rc;
+  }
   const int qh = H / G;
   const int HM = H * maps;
   const size_t need = sd_multimap_softmax_attention_scratch_bytes(n_rows, H, maps, dv, window, keep_first, chunk,

@@ -16,6 +16,8 @@
 // entry's other rows still read the old state.
 #include <math.h>
 
+#include <mutex>
+
 #include "sd_common.h"
 
 namespace {
@@ -237,67 +239,85 @@ __global__ void conv_tail_kernel(const float* __restrict__ x, int64_t ldx, const
 
 // ------------------------------------------------------------------ an activation of normed powers
 // out = k0 N(z) + k1 N(z^2) + k2 N(z^3) + k3, z the row + bias, N(y) = y / sqrt(mean(y^2) + eps) over
-// the row's F values.  By a whole workgroup.
-template <typename T>
-__device__ __forceinline__ void poly_norm_row(const float* __restrict__ z, const T* __restrict__ bias,
-                                              const float* __restrict__ coef, float eps, int F,
-                                              float* __restrict__ out, bf16_t* __restrict__ out_b, float* red) {
-  constexpr int U = 8;
-  const int nthr = blockDim.x;
-  float s1 = 0.f, s2 = 0.f, s3 = 0.f;
-  for (int c0 = threadIdx.x; c0 < F; c0 += U * nthr) {
-    float v[U];
+// the row's F values.  By a whole workgroup of 256 threads; pieces of V values, the first kPolyRegs
+// of a thread held in registers between the sums and the result.
+constexpr int kPolyRegs = 8;
+template <typename T, int V>
+__device__ __forceinline__ void poly_norm_pieces(const float* __restrict__ z, const T* __restrict__ bias,
+                                                 const float* __restrict__ coef, float eps, int F,
+                                                 float* __restrict__ out, bf16_t* __restrict__ out_b, float* red) {
+  const int np = F / V;
+  auto piece = [&](int i) {
+    Pack<V> v = ld_pack<V>(z + (size_t)i * V);
+    if (bias) {
+      const Pack<V> b = ld_pack<V>(bias + (size_t)i * V);
 #pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const int c = c0 + u * nthr < F ? c0 + u * nthr : F - 1;
-      v[u] = z[c] + (bias ? ld_f(bias + c) : 0.f);
+      for (int e = 0; e < V; ++e) v.v[e] += b.v[e];
     }
+    return v;
+  };
+  float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+  auto add = [&](const Pack<V>& v) {
 #pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const float q = c0 + u * nthr < F ? v[u] * v[u] : 0.f;
+    for (int e = 0; e < V; ++e) {
+      const float q = v.v[e] * v.v[e];
       s1 += q;
       s2 = fmaf(q, q, s2);
       s3 = fmaf(q * q, q, s3);
     }
+  };
+  Pack<V> keep[kPolyRegs];
+#pragma unroll
+  for (int u = 0; u < kPolyRegs; ++u) {   // (on a piece clamped into the row: every load is issued)
+    const int i = threadIdx.x + 256 * u;
+    keep[u] = piece(i < np ? i : np - 1);
   }
+#pragma unroll
+  for (int u = 0; u < kPolyRegs; ++u)
+    if ((int)threadIdx.x + 256 * u < np) add(keep[u]);
+  for (int i = threadIdx.x + 256 * kPolyRegs; i < np; i += 256) add(piece(i));
   s1 = wave_sum(s1);
   s2 = wave_sum(s2);
   s3 = wave_sum(s3);
-  const int wave = threadIdx.x >> 6, nw = (nthr + 63) >> 6;
+  const int wave = threadIdx.x >> 6;
   if ((threadIdx.x & 63) == 0) {
     red[wave] = s1;
-    red[nw + wave] = s2;
-    red[2 * nw + wave] = s3;
+    red[4 + wave] = s2;
+    red[8 + wave] = s3;
   }
   __syncthreads();
   s1 = red[0];
-  s2 = red[nw];
-  s3 = red[2 * nw];
-  for (int w = 1; w < nw; ++w) {
+  s2 = red[4];
+  s3 = red[8];
+  for (int w = 1; w < 4; ++w) {
     s1 += red[w];
-    s2 += red[nw + w];
-    s3 += red[2 * nw + w];
+    s2 += red[4 + w];
+    s3 += red[8 + w];
   }
   const float n = (float)F;
   const float f1 = coef[0] / sqrtf(s1 / n + eps), f2 = coef[1] / sqrtf(s2 / n + eps),
               f3 = coef[2] / sqrtf(s3 / n + eps), f0 = coef[3];
-  for (int c0 = threadIdx.x; c0 < F; c0 += U * nthr) {
-    float v[U];
+  auto write = [&](int i, const Pack<V>& v) {
+    Pack<V> o;
 #pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const int c = c0 + u * nthr < F ? c0 + u * nthr : F - 1;
-      v[u] = z[c] + (bias ? ld_f(bias + c) : 0.f);
-    }
+    for (int e = 0; e < V; ++e) o.v[e] = fmaf(v.v[e], fmaf(v.v[e], fmaf(v.v[e], f3, f2), f1), f0);
+    if (out) st_pack<V>(out + (size_t)i * V, o);
+    if (out_b) st_pack<V>(out_b + (size_t)i * V, o);
+  };
 #pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const int c = c0 + u * nthr;
-      if (c < F) {
-        const float o = fmaf(v[u], fmaf(v[u], fmaf(v[u], f3, f2), f1), f0);
-        if (out) out[c] = o;
-        if (out_b) out_b[c] = (bf16_t)o;
-      }
-    }
-  }
+  for (int u = 0; u < kPolyRegs; ++u)
+    if ((int)threadIdx.x + 256 * u < np) write(threadIdx.x + 256 * u, keep[u]);
+  for (int i = threadIdx.x + 256 * kPolyRegs; i < np; i += 256) write(i, piece(i));
+}
+template <typename T>
+__device__ __forceinline__ void poly_norm_row(const float* __restrict__ z, const T* __restrict__ bias,
+                                              const float* __restrict__ coef, float eps, int F,
+                                              float* __restrict__ out, bf16_t* __restrict__ out_b, float* red) {
+  const uintptr_t at = reinterpret_cast<uintptr_t>(z) | reinterpret_cast<uintptr_t>(out) |
+                       (reinterpret_cast<uintptr_t>(bias) * (16 / (4 * sizeof(T)))) |
+                       (reinterpret_cast<uintptr_t>(out_b) * 2);
+  if (F % 4 == 0 && (at & 15) == 0) poly_norm_pieces<T, 4>(z, bias, coef, eps, F, out, out_b, red);
+  else poly_norm_pieces<T, 1>(z, bias, coef, eps, F, out, out_b, red);
 }
 template <typename T>
 __global__ __launch_bounds__(256) void poly_norm_kernel(const float* __restrict__ z, int64_t ldz,
@@ -625,6 +645,570 @@ __global__ __launch_bounds__(256) void mlstm_post_kernel(MlstmPostArgs g) {
   if (lane == 0 && (r + 1 == (int)gridDim.x || g.row_slot[r + 1] != slot)) g.m[(size_t)slot * g.H + h] = m;
 }
 
+// ------------------------------------------------------------------ window attention on the matrix cores
+// Many rows over bf16 caches.  A workgroup of four waves takes one kv head and a tile of query rows
+// of one portion: wh query heads of the kv head x (4 / wh) groups of 16 rows, a wave each, which
+// share the tiles of 64 keys that are staged in LDS (keys as rows, values transposed).  A wave
+// computes S^T = K Q^T, so that a query's scores sit in one column of the accumulator and are, as
+// they are, the right operand of O^T = V^T P^T (the keys of an MFMA step in the order the
+// accumulators hold them).  Queries and weights enter as the sum of two bf16 parts, keys and values
+// are the cache's bf16 values: products carry 2^-17 of their operands, sums, softmax, cap and
+// distance are f32.  The distance's logarithm is formed once per distinct distance of a tile.
+struct TiledAttnArgs {
+  const float* q;
+  int64_t ldq;
+  const bf16_t* k_cache;
+  const bf16_t* v_cache;
+  const int32_t* block_tables;
+  const int32_t* entries;
+  const float* dist1;      // or nullptr
+  const float* dist2;
+  float* out;
+  bf16_t* out_b;
+  int64_t ldo;
+  float scale, softcap;
+  int n_entries, max_blocks, H, G, dk, dv, window, wh, n_hgroups;
+};
+constexpr int kTileKeys = 64;
+constexpr int kPage = 16;
+constexpr float kLog2e = 1.4426950408889634f;
+
+// The portion and the first row (inside it) of the n-th group of `per` rows over all portions.
+__device__ __forceinline__ bool nth_group(const int32_t* entries, int n_entries, int per, int n, int* e, int* first) {
+  int i = 0;
+  for (; i < n_entries; ++i) {
+    const int groups = (entries[4 * i + 2] + per - 1) / per;
+    if (n < groups) break;
+    n -= groups;
+  }
+  *e = i;
+  *first = n * per;
+  return i < n_entries;
+}
+
+template <int KS, int VT>   // heads of up to 32 * KS key and 16 * VT value channels
+__global__ __launch_bounds__(256) void tiled_window_attn_kernel(TiledAttnArgs g) {
+  constexpr int KLD = 32 * KS + 8, VLD = kTileKeys + 4, NV = VT / 4;
+  __shared__ __attribute__((aligned(16))) bf16_t ks[kTileKeys * KLD];
+  __shared__ __attribute__((aligned(16))) bf16_t vs[16 * VT * VLD];
+  __shared__ float away[4][80];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, quad = lane >> 4;
+  const int kvh = blockIdx.y, hgroup = blockIdx.z, qh = g.H / g.G, dk = g.dk, dv = g.dv;
+  const int n_sub = 4 / g.wh, tq = 16 * n_sub;
+  int e, first;
+  if (!nth_group(g.entries, g.n_entries, tq, blockIdx.x, &e, &first)) return;
+  const int slot = g.entries[4 * e], row0 = g.entries[4 * e + 1], len = g.entries[4 * e + 2], pos0 = g.entries[4 * e + 3];
+  const int hw = hgroup * g.wh + wave % g.wh, sub = first + 16 * (wave / g.wh);
+  const int n_rows = len - sub < 16 ? len - sub : 16;        // this wave's rows (<= 0: none)
+  const bool works = hw < qh && n_rows > 0;
+  const int h = kvh * qh + (hw < qh ? hw : qh - 1);
+  const int p = pos0 + sub + col;                            // this lane's query
+  const int32_t* tbl = g.block_tables + (size_t)slot * g.max_blocks;
+  const int last = pos0 + (len < first + tq ? len : first + tq) - 1;   // the workgroup's last position
+  int base = pos0 + first - g.window + 1;
+  base = base > 0 ? base & ~(kPage - 1) : 0;
+  const float r1 = g.dist1 ? g.dist1[h] : 0.f, r2 = g.dist1 ? g.dist2[h] : 0.f;
+
+  bf16x8 qa[KS], qb[KS];                                     // the query's two parts
+  {
+    const int r = row0 + (works ? sub + (col < n_rows ? col : n_rows - 1) : 0);
+    const float* qr = g.q + (size_t)r * g.ldq + (size_t)h * dk;
+#pragma unroll
+    for (int s = 0; s < KS; ++s) {
+      const int c = 32 * s + 8 * quad;
+      float f[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) f[i] = 0.f;
+      if (c < dk) {
+        const f32x4 a = *reinterpret_cast<const f32x4*>(qr + c), b = *reinterpret_cast<const f32x4*>(qr + c + 4);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          f[i] = a[i] * g.scale;
+          f[4 + i] = b[i] * g.scale;
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        qa[s][i] = (bf16_t)f[i];
+        qb[s][i] = (bf16_t)(f[i] - (float)qa[s][i]);
+      }
+    }
+  }
+  // a thread's pieces of a key tile: KS of 8 channels; of a value tile: NV of 8 channels of two keys
+  const u32x4 zero = {0, 0, 0, 0};
+  u32x4 kr[KS], vr[NV][2];
+  int kpg[KS], vpg[NV];
+  auto pages = [&](int b0) {     // the pages of the tile at b0 (clamped: rows behind `last` are zeroed)
+#pragma unroll
+    for (int i = 0; i < KS; ++i) {
+      const int j = b0 + (tid + 256 * i) / (4 * KS);
+      kpg[i] = tbl[(j < last ? j : last) / kPage];
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int j = b0 + 2 * ((tid + 256 * i) / (2 * VT));
+      vpg[i] = tbl[(j < last ? j : last) / kPage];
+    }
+  };
+  auto fetch = [&](int b0) {
+#pragma unroll
+    for (int i = 0; i < KS; ++i) {
+      const int idx = tid + 256 * i, j = b0 + idx / (4 * KS), c = 8 * (idx % (4 * KS));
+      kr[i] = zero;
+      if (j <= last && c < dk)
+        kr[i] = *reinterpret_cast<const u32x4*>(g.k_cache + (((size_t)kpg[i] * g.G + kvh) * kPage + j % kPage) * dk + c);
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int idx = tid + 256 * i, j = b0 + 2 * (idx / (2 * VT)), c = 8 * (idx % (2 * VT));
+      const bf16_t* v = g.v_cache + (((size_t)vpg[i] * g.G + kvh) * kPage + j % kPage) * dv + c;
+      vr[i][0] = vr[i][1] = zero;
+      if (j <= last && c < dv) vr[i][0] = *reinterpret_cast<const u32x4*>(v);
+      if (j + 1 <= last && c < dv) vr[i][1] = *reinterpret_cast<const u32x4*>(v + dv);
+    }
+  };
+  f32x4 o[VT];
+#pragma unroll
+  for (int t = 0; t < VT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m_run = -INFINITY, l_run = 0.f;
+  const float cap = g.softcap, cap_in = cap > 0.f ? 2.f * kLog2e / cap : 0.f;
+
+  pages(base);
+  fetch(base);
+  pages(base + kTileKeys);
+  for (; base <= last; base += kTileKeys) {
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < KS; ++i) {
+      const int idx = tid + 256 * i;
+      *reinterpret_cast<u32x4*>(ks + (idx / (4 * KS)) * KLD + 8 * (idx % (4 * KS))) = kr[i];
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int idx = tid + 256 * i, c = 8 * (idx % (2 * VT)), j = 2 * (idx / (2 * VT));
+      const bf16x8 a = __builtin_bit_cast(bf16x8, vr[i][0]), b = __builtin_bit_cast(bf16x8, vr[i][1]);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) *reinterpret_cast<bf16x2*>(vs + (c + u) * VLD + j) = bf16x2{a[u], b[u]};
+    }
+    if (g.dist1) {   // entry n: distance pos0 + sub - base - 63 + n
+      const int d0 = pos0 + sub - base - (kTileKeys - 1);
+      away[wave][lane] = r1 * log1pf(r2 * (float)(d0 + lane > 0 ? d0 + lane : 0));
+      if (lane < 16) away[wave][64 + lane] = r1 * log1pf(r2 * (float)(d0 + 64 + lane > 0 ? d0 + 64 + lane : 0));
+    }
+    __syncthreads();
+    if (base + kTileKeys <= last) {
+      fetch(base + kTileKeys);
+      pages(base + 2 * kTileKeys);
+    }
+    if (!works || base > pos0 + sub + n_rows - 1) continue;   // (keys behind this wave's last query)
+    f32x4 sc[4];
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      sc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < KS; ++s) {
+        const bf16x8 a = *reinterpret_cast<const bf16x8*>(ks + (16 * t + col) * KLD + 32 * s + 8 * quad);
+        sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qa[s], sc[t], 0, 0, 0);
+        sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qb[s], sc[t], 0, 0, 0);
+      }
+    }
+    float mx = m_run;
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int kk = 16 * t + 4 * quad + i, d = p - (base + kk);
+        float v = sc[t][i];
+        // cap tanh(v / cap) = cap - 2 cap / (e^(2 v / cap) + 1)
+        if (cap > 0.f) v = fmaf(-2.f * cap, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(v * cap_in) + 1.f), cap);
+        if (g.dist1) v -= away[wave][col + kTileKeys - 1 - kk];
+        v = d >= 0 && d < g.window ? v : -INFINITY;
+        sc[t][i] = v;
+        mx = fmaxf(mx, v);
+      }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, SD_WAVE));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, SD_WAVE));
+    const float ref = mx == -INFINITY ? 0.f : mx;            // (no key seen yet)
+    const float corr = __builtin_amdgcn_exp2f((m_run - ref) * kLog2e);
+    m_run = mx;
+    float sum = 0.f;
+    bf16x8 pa[2], pb[2];
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float w = __builtin_amdgcn_exp2f((sc[t][i] - ref) * kLog2e);
+        sum += w;
+        const bf16_t a = (bf16_t)w;
+        pa[t >> 1][4 * (t & 1) + i] = a;
+        pb[t >> 1][4 * (t & 1) + i] = (bf16_t)(w - (float)a);
+      }
+    l_run = fmaf(l_run, corr, sum);
+    if (__any(corr != 1.f)) {
+#pragma unroll
+      for (int t = 0; t < VT; ++t) o[t] *= corr;
+    }
+#pragma unroll
+    for (int t = 0; t < VT; ++t)
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        const bf16_t* vrow = vs + (16 * t + col) * VLD + 32 * u + 4 * quad;
+        const bf16x4 a0 = *reinterpret_cast<const bf16x4*>(vrow), a1 = *reinterpret_cast<const bf16x4*>(vrow + 16);
+        const bf16x8 a = {a0[0], a0[1], a0[2], a0[3], a1[0], a1[1], a1[2], a1[3]};
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pa[u], o[t], 0, 0, 0);
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb[u], o[t], 0, 0, 0);
+      }
+  }
+  l_run += __shfl_xor(l_run, 16, SD_WAVE);
+  l_run += __shfl_xor(l_run, 32, SD_WAVE);
+  if (!works || col >= n_rows) return;
+  const float inv = 1.f / l_run;
+  const size_t at = (size_t)(row0 + sub + col) * g.ldo + (size_t)h * dv;
+  const bool quads = g.ldo % 4 == 0;
+#pragma unroll
+  for (int t = 0; t < VT; ++t) {
+    const int c = 16 * t + 4 * quad;
+    if (c >= dv) continue;
+    const Pack<4> v = {{o[t][0] * inv, o[t][1] * inv, o[t][2] * inv, o[t][3] * inv}};
+    if (quads) {
+      if (g.out) st_pack<4>(g.out + at + c, v);
+      if (g.out_b) st_pack<4>(g.out_b + at + c, v);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        if (g.out) g.out[at + c + i] = v.v[i];
+        if (g.out_b) g.out_b[at + c + i] = (bf16_t)v.v[i];
+      }
+    }
+  }
+}
+
+// ------------------------------------------------------------------ the matrix memory in chunks
+// The recurrence of mlstm_scan_kernel over chunks of 64 tokens, on the f32 matrix instruction (no
+// reduced precision).  With D(t, s) the sum of the log forget gates of s+1 .. t and b_t = D(t, -1):
+//   num_t = e^(b_t + m0 - m_t) q_t S0 + sum_{s <= t} e^(D(t, s) + i_s - m_t) (q_t . k_s) v_s,
+// S0, m0 the memory and its running maximum at the chunk's start.  Three launches: every chunk's own
+// sum of e^(D(63, s) + i_s - mu) k_s v_s^T with a maximum mu of its own (chunk_sums), the memories at
+// the chunks' starts (chunk_carry, chunk after chunk), the tokens' results (chunk_reads).  A maximum
+// only scales numbers, so mu and m_t need not be the ones another cut of the tokens would give.
+struct MlstmChunkArgs {
+  MlstmArgs a;
+  int n_entries;
+  float* cs;               // [chunks, H, dk, dv]: own sums, then the memory at the chunk's start
+  float* cn;               // [chunks, H, dk]: the same of k alone
+  float* sc;               // [chunks, H, 4]: b of the last token, mu, m at the start, m at the end
+};
+constexpr int kChunk = 64;
+
+// log gates of the chunk's token `lane` (a token behind the chunk's end adds nothing)
+__device__ __forceinline__ void chunk_gates(const MlstmArgs& a, int row, int h, bool in, float* li, float* lf) {
+  const float zi = a.zi[(size_t)row * a.ld + h] + a.bi[h], zf = a.zf[(size_t)row * a.ld + h] + a.bf[h];
+  *li = in ? a.cap * tanhf(zi / a.cap) : -INFINITY;
+  *lf = in ? log_sigmoid_f(a.cap * tanhf(zf / a.cap)) : 0.f;
+}
+
+typedef __attribute__((ext_vector_type(16))) float acc32_t;
+// row of register i of a 32x32 accumulator
+__device__ __forceinline__ int acc_row(int i, int half) { return 8 * (i >> 2) + 4 * half + (i & 3); }
+
+constexpr int kChunkCols = 128;   // value columns per workgroup
+__global__ __launch_bounds__(256) void mlstm_chunk_sums_kernel(MlstmChunkArgs g) {
+  extern __shared__ float lds[];
+  const MlstmArgs& a = g.a;
+  const int dk = a.dk, dv = a.dv, H = a.H, nkt = (dk + 31) / 32, dkp = 32 * nkt;
+  float* ks = lds;                   // [64][dkp], times the token's weight
+  float* vs = ks + kChunk * dkp;     // [64][128]
+  float* wt = vs + kChunk * kChunkCols;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l31 = lane & 31, half = lane >> 5;
+  const int h = blockIdx.y, c0 = blockIdx.z * kChunkCols;
+  int e, first;
+  if (!nth_group(a.entries, g.n_entries, kChunk, blockIdx.x, &e, &first)) return;
+  const int row0 = a.entries[4 * e + 1] + first, left = a.entries[4 * e + 2] - first, nt = left < kChunk ? left : kChunk;
+  const size_t at = (size_t)blockIdx.x * H + h;
+  if (wave == 0) {
+    float li, lf;
+    chunk_gates(a, row0 + (lane < nt ? lane : nt - 1), h, lane < nt, &li, &lf);
+    float d = __shfl_down(lf, 1, SD_WAVE);        // sum of the gates behind this token
+    if (lane == 63) d = 0.f;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float n = __shfl_down(d, o, SD_WAVE);
+      if (lane + o < 64) d += n;
+    }
+    const float mu = wave_max(d + li);
+    wt[lane] = expf(d + li - mu);
+    if (lane == 0 && blockIdx.z == 0) {
+      g.sc[at * 4] = d + lf;
+      g.sc[at * 4 + 1] = mu;
+    }
+  }
+  // (four rows of k and of v in flight per thread and turn; loads on clamped addresses)
+  __syncthreads();
+  for (int i = tid; i < kChunk * dkp; i += 256 * 8) {
+    float v[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int idx = i + 256 * u, t = idx / dkp < nt ? idx / dkp : nt - 1, c = idx % dkp;
+      v[u] = a.k[(size_t)(row0 + t) * a.ld + (size_t)h * dk + (c < dk ? c : dk - 1)];
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int idx = i + 256 * u;
+      if (idx < kChunk * dkp) ks[idx] = idx / dkp < nt && idx % dkp < dk ? v[u] * wt[idx / dkp] : 0.f;
+    }
+  }
+  for (int i = tid; i < kChunk * kChunkCols; i += 256 * 8) {
+    float v[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int idx = i + 256 * u, t = idx / kChunkCols < nt ? idx / kChunkCols : nt - 1, c = c0 + idx % kChunkCols;
+      v[u] = a.v[(size_t)(row0 + t) * a.ld + (size_t)h * dv + (c < dv ? c : dv - 1)];
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int idx = i + 256 * u;
+      vs[idx] = idx / kChunkCols < nt && c0 + idx % kChunkCols < dv ? v[u] : 0.f;
+    }
+  }
+  __syncthreads();
+  const int cols = dv - c0 < kChunkCols ? dv - c0 : kChunkCols, nct = (cols + 31) / 32;
+  float* cs = g.cs + at * dk * dv + c0;
+  for (int p = wave; p < nkt * nct; p += 4) {
+    const int kt = p % nkt, ct = p / nkt;
+    acc32_t acc;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) acc[i] = 0.f;
+#pragma unroll 8
+    for (int s = 0; s < kChunk; s += 2)
+      acc = __builtin_amdgcn_mfma_f32_32x32x2f32(ks[(s + half) * dkp + 32 * kt + l31],
+                                                 vs[(s + half) * kChunkCols + 32 * ct + l31], acc, 0, 0, 0);
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const int r = 32 * kt + acc_row(i, half);
+      if (r < dk && 32 * ct + l31 < cols) cs[(size_t)r * dv + 32 * ct + l31] = acc[i];
+    }
+  }
+  if (blockIdx.z == 0 && tid < dk) {
+    float n = 0.f;
+    for (int s = 0; s < kChunk; ++s) n += ks[s * dkp + tid];
+    g.cn[at * dk + tid] = n;
+  }
+}
+
+// One element of a head's memory (or normalizer) through the chunks of its portion.
+__global__ __launch_bounds__(256) void mlstm_chunk_carry_kernel(MlstmChunkArgs g) {
+  const MlstmArgs& a = g.a;
+  const int dk = a.dk, dv = a.dv, H = a.H, h = blockIdx.y, e = blockIdx.z;
+  const int x = blockIdx.x * 256 + threadIdx.x;
+  const int slot = a.entries[4 * e], len = a.entries[4 * e + 2], pos0 = a.entries[4 * e + 3];
+  int c0 = 0;
+  for (int i = 0; i < e; ++i) c0 += (a.entries[4 * i + 2] + kChunk - 1) / kChunk;
+  const int nc = (len + kChunk - 1) / kChunk;
+  const bool is_n = x >= dk * dv;
+  if (x >= dk * dv + dk) return;
+  float* st = is_n ? a.nrm + ((size_t)slot * H + h) * dk + (x - dk * dv) : a.S + ((size_t)slot * H + h) * dk * dv + x;
+  float* own = is_n ? g.cn + ((size_t)c0 * H + h) * dk + (x - dk * dv) : g.cs + ((size_t)c0 * H + h) * dk * dv + x;
+  const size_t step = is_n ? (size_t)H * dk : (size_t)H * dk * dv;
+  float* sc = g.sc + ((size_t)c0 * H + h) * 4;
+  float val = pos0 > 0 ? *st : 0.f, m = pos0 > 0 ? a.m[(size_t)slot * H + h] : 0.f;
+  constexpr int U = 8;
+  for (int i = 0; i < nc; i += U) {
+    float v[U], b[U], mu[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int c = i + u < nc ? i + u : nc - 1;
+      v[u] = own[c * step];
+      b[u] = sc[(size_t)c * H * 4];
+      mu[u] = sc[(size_t)c * H * 4 + 1];
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      if (i + u >= nc) break;
+      const float m_new = fmaxf(b[u] + m, mu[u]);
+      own[(i + u) * step] = val;
+      val = fmaf(expf(b[u] + m - m_new), val, expf(mu[u] - m_new) * v[u]);
+      if (x == 0) {
+        sc[(size_t)(i + u) * H * 4 + 2] = m;
+        sc[(size_t)(i + u) * H * 4 + 3] = m_new;
+      }
+      m = m_new;
+    }
+  }
+  *st = val;
+}
+
+constexpr int kChunkSteps = 64;   // dk <= 128: pairs of key channels
+__global__ __launch_bounds__(256) void mlstm_chunk_reads_kernel(MlstmChunkArgs g) {
+  extern __shared__ float lds[];
+  const MlstmArgs& a = g.a;
+  const int dk = a.dk, dv = a.dv, H = a.H, dkp = (dk + 31) / 32 * 32, ldk = dkp + 1;
+  constexpr int kLdA = kChunk + 1;
+  float* qs = lds;                     // [64][ldk]
+  float* ks = qs + kChunk * ldk;       // [64][ldk]
+  float* vs = ks + kChunk * ldk;       // [64][128]
+  float* as = vs + kChunk * kChunkCols;  // [64][65] weighted scores
+  float* lis = as + kChunk * kLdA;     // [64] each
+  float* lfs = lis + kChunk;
+  float* ms = lfs + kChunk;
+  float* carry = ms + kChunk;
+  float* ns = carry + kChunk;          // [dkp]
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l31 = lane & 31, half = lane >> 5;
+  const int h = blockIdx.y, c0 = blockIdx.z * kChunkCols;
+  int e, first;
+  if (!nth_group(a.entries, g.n_entries, kChunk, blockIdx.x, &e, &first)) return;
+  const int row0 = a.entries[4 * e + 1] + first, left = a.entries[4 * e + 2] - first, nt = left < kChunk ? left : kChunk;
+  const size_t at = (size_t)blockIdx.x * H + h;
+  // the memory at the chunk's start: this wave's 32 columns, rows 2 j + half, asked for first
+  const int wcol = 32 * wave + l31;
+  const bool col_in = c0 + wcol < dv;
+  float S[kChunkSteps];
+  {
+    const float* s0 = g.cs + at * dk * dv + (col_in ? c0 + wcol : 0);
+#pragma unroll
+    for (int j = 0; j < kChunkSteps; ++j) {
+      S[j] = 0.f;
+      if (2 * j < dkp) {
+        const int r = 2 * j + half;
+        const float v = s0[(size_t)(r < dk ? r : dk - 1) * dv];
+        S[j] = r < dk && col_in ? v : 0.f;
+      }
+    }
+  }
+  if (wave == 0) {
+    float li, lf;
+    chunk_gates(a, row0 + (lane < nt ? lane : nt - 1), h, lane < nt, &li, &lf);
+    const float m0 = g.sc[at * 4 + 2], m1 = g.sc[at * 4 + 3];
+    float F = lf, I = li;              // (F, I): m = max(F + m0, I), composed over the tokens so far
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float fp = __shfl_up(F, o, SD_WAVE), ip = __shfl_up(I, o, SD_WAVE);
+      if (lane >= o) {
+        I = fmaxf(ip + F, I);
+        F += fp;
+      }
+    }
+    float m = fmaxf(F + m0, I);
+    if (lane == nt - 1) m = m1;        // the maximum the carried memory was scaled with
+    lis[lane] = li;
+    lfs[lane] = lf;
+    ms[lane] = m;
+    carry[lane] = expf(F + m0 - m);
+    if (blockIdx.z == 0 && lane < nt) a.m_rows[(size_t)(row0 + lane) * H + h] = m;
+  } else {
+    for (int c = tid - 64; c < dkp; c += 192) ns[c] = c < dk ? g.cn[at * dk + c] : 0.f;
+  }
+  for (int i = tid; i < kChunk * dkp; i += 256 * 8) {
+    float vq[8], vk[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int idx = i + 256 * u, t = idx / dkp < nt ? idx / dkp : nt - 1, c = idx % dkp;
+      const size_t from = (size_t)(row0 + t) * a.ld + (size_t)h * dk + (c < dk ? c : dk - 1);
+      vq[u] = a.q[from];
+      vk[u] = a.k[from];
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int idx = i + 256 * u, t = idx / dkp, c = idx % dkp;
+      if (idx < kChunk * dkp) {
+        qs[t * ldk + c] = t < nt && c < dk ? vq[u] * a.q_scale : 0.f;
+        ks[t * ldk + c] = t < nt && c < dk ? vk[u] : 0.f;
+      }
+    }
+  }
+  for (int i = tid; i < kChunk * kChunkCols; i += 256 * 8) {
+    float v[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int idx = i + 256 * u, t = idx / kChunkCols < nt ? idx / kChunkCols : nt - 1, c = c0 + idx % kChunkCols;
+      v[u] = a.v[(size_t)(row0 + t) * a.ld + (size_t)h * dv + (c < dv ? c : dv - 1)];
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int idx = i + 256 * u;
+      vs[idx] = idx / kChunkCols < nt && c0 + idx % kChunkCols < dv ? v[u] : 0.f;
+    }
+  }
+  __syncthreads();
+  {
+    // the tokens' weights: lane s, sixteen tokens t per wave; D(t, s) is summed from s on, so that a
+    // long stretch of forgetting before s costs nothing of its precision
+    const float li = lis[lane];
+    float d = 0.f;
+    const int t0 = 16 * wave;
+    for (int t = 0; t < t0; ++t) d += t > lane ? lfs[t] : 0.f;
+#pragma unroll
+    for (int t = t0; t < t0 + 16; ++t) {
+      d += t > lane ? lfs[t] : 0.f;
+      as[t * kLdA + lane] = t >= lane ? expf(d + li - ms[t]) : 0.f;
+    }
+  }
+  acc32_t acc[2];
+  {
+    const int tt = wave >> 1, ss = wave & 1;    // q k^T, a 32 x 32 part per wave
+#pragma unroll
+    for (int i = 0; i < 16; ++i) acc[0][i] = 0.f;
+    const float* qa = qs + (32 * tt + l31) * ldk + half;
+    const float* kb = ks + (32 * ss + l31) * ldk + half;
+    if (tt >= ss) {
+#pragma unroll 8
+      for (int c = 0; c < dkp; c += 2) acc[0] = __builtin_amdgcn_mfma_f32_32x32x2f32(qa[c], kb[c], acc[0], 0, 0, 0);
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 16; ++i) as[(32 * tt + acc_row(i, half)) * kLdA + 32 * ss + l31] *= acc[0][i];
+  }
+#pragma unroll
+  for (int u = 0; u < 2; ++u)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) acc[u][i] = 0.f;
+#pragma unroll
+  for (int j = 0; j < kChunkSteps; ++j) {
+    if (2 * j < dkp) {
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+        acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(qs[(32 * u + l31) * ldk + 2 * j + half], S[j], acc[u], 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int u = 0; u < 2; ++u)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) acc[u][i] *= carry[32 * u + acc_row(i, half)];
+  __syncthreads();
+#pragma unroll
+  for (int s = 0; s < kChunk; s += 2) {
+    const float b = vs[(s + half) * kChunkCols + wcol];
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+      if (s < 32 * (u + 1)) acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(as[(32 * u + l31) * kLdA + s + half], b, acc[u], 0, 0, 0);
+  }
+  if (col_in) {
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int t = 32 * u + acc_row(i, half);
+        if (t < nt) a.num[((size_t)(row0 + t) * H + h) * (dv + 1) + c0 + wcol] = acc[u][i];
+      }
+  }
+  if (blockIdx.z == 0) {   // n . q, four threads a token
+    const int t = tid >> 2, part = tid & 3;
+    float n = 0.f, o = 0.f;
+    for (int c = part; c < dkp; c += 4) n = fmaf(qs[t * ldk + c], ns[c], n);
+    for (int s = part; s < kChunk; s += 4) o += as[t * kLdA + s];
+    n = fmaf(n, carry[t], o);
+    n += __shfl_xor(n, 1, SD_WAVE);
+    n += __shfl_xor(n, 2, SD_WAVE);
+    if (part == 0 && t < nt) a.num[((size_t)(row0 + t) * H + h) * (dv + 1) + dv] = n;
+  }
+}
+
+inline size_t chunk_reads_lds(int dk) {
+  const size_t dkp = (dk + 31) / 32 * 32;
+  return sizeof(float) * (2 * kChunk * (dkp + 1) + (size_t)kChunk * kChunkCols + kChunk * (kChunk + 1) + 4 * kChunk + dkp);
+}
+// chunks that n_entries portions of n_rows rows in all may have
+inline size_t max_chunks(int n_rows, int n_entries) { return (size_t)n_rows / kChunk + n_entries; }
+
 template <typename T>
 void launch_joint(const JointArgs& g, int n, hipStream_t st) {
   const bool quad = g.W % 4 == 0;
@@ -741,14 +1325,49 @@ extern "C" int sd_conv_attn_prep(const float* proj, int64_t ld, const void* bias
   return sd_conv_tail(proj, ld, bias, w_f32, conv_state, entries, n_entries, g.C, taps, stream);
 }
 
+extern "C" size_t sd_mlstm_scratch_bytes(int n_rows, int n_entries, int H, int dk, int dv) {
+  // (a few rows beyond one per portion do not fill chunks: token by token is as fast)
+  if (n_rows < 1 || n_entries < 1 || n_rows - n_entries < kChunk / 2 || H < 1 || dk < 1 || dk > 128 || dv < 1) return 0;
+  return sizeof(float) * max_chunks(n_rows, n_entries) * H * ((size_t)dk * dv + dk + 4);
+}
+
 extern "C" int sd_mlstm_scan(const float* q, const float* k, const float* v, const float* zi, const float* zf,
                              int64_t ld, const float* bi, const float* bf, float cap, float q_scale, float* S,
-                             float* n_state, const float* m_state, const int32_t* entries, int n_entries, float* num,
-                             float* m_rows, int H, int dk, int dv, sd_stream_t stream) {
+                             float* n_state, const float* m_state, const int32_t* entries, int n_entries, int n_rows,
+                             float* num, float* m_rows, int H, int dk, int dv, void* scratch, size_t scratch_bytes,
+                             sd_stream_t stream) {
   SD_REQUIRE(q && k && v && zi && zf && bi && bf && S && n_state && m_state && entries && num && m_rows &&
-                 n_entries >= 1 && H >= 1 && dv >= 1 && cap > 0.f,
+                 n_entries >= 1 && n_rows >= n_entries && H >= 1 && dv >= 1 && cap > 0.f,
              SD_ERR_INVALID, "sd_mlstm_scan: bad argument");
   SD_REQUIRE(dk >= 1 && dk <= 256, SD_ERR_UNSUPPORTED, "sd_mlstm_scan: key size %d outside 1..256", dk);
+  hipStream_t st = (hipStream_t)stream;
+  MlstmArgs g{q, k, v, zi, zf, ld, bi, bf, cap, q_scale, S, n_state, const_cast<float*>(m_state), entries, num, m_rows, H, dk, dv};
+  const size_t need = sd_mlstm_scratch_bytes(n_rows, n_entries, H, dk, dv);
+  if (need > 0 && scratch && scratch_bytes >= need && sd_aligned16(scratch)) {
+    static std::once_flag once;
+    static hipError_t err = hipSuccess;
+    std::call_once(once, [] {
+      err = hipFuncSetAttribute(reinterpret_cast<const void*>(mlstm_chunk_sums_kernel),
+                                hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+      if (err == hipSuccess)
+        err = hipFuncSetAttribute(reinterpret_cast<const void*>(mlstm_chunk_reads_kernel),
+                                  hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    });
+    SD_REQUIRE(err == hipSuccess, SD_ERR_HIP, "sd_mlstm_scan: hipFuncSetAttribute failed: %s", hipGetErrorString(err));
+    const size_t nc = max_chunks(n_rows, n_entries);
+    MlstmChunkArgs c{g, n_entries, (float*)scratch, nullptr, nullptr};
+    c.cn = c.cs + nc * H * dk * dv;
+    c.sc = c.cn + nc * H * dk;
+    const int dkp = (dk + 31) / 32 * 32, zs = (dv + kChunkCols - 1) / kChunkCols;
+    const size_t lds = sizeof(float) * ((size_t)kChunk * dkp + (size_t)kChunk * kChunkCols + kChunk);
+    mlstm_chunk_sums_kernel<<<dim3((unsigned)nc, H, zs), 256, lds, st>>>(c);
+    SD_CHECK_LAUNCH("sd_mlstm_scan (chunk sums)");
+    mlstm_chunk_carry_kernel<<<dim3((dk * dv + dk + 255) / 256, H, n_entries), 256, 0, st>>>(c);
+    SD_CHECK_LAUNCH("sd_mlstm_scan (carry)");
+    mlstm_chunk_reads_kernel<<<dim3((unsigned)nc, H, zs), 256, chunk_reads_lds(dk), st>>>(c);
+    SD_CHECK_LAUNCH("sd_mlstm_scan (reads)");
+    return SD_OK;
+  }
   const int NS = (dk + kStrip - 1) / kStrip, cols = dv + 1;
   int CT = 256 / NS;
   if (CT > cols) CT = cols;
@@ -760,9 +1379,33 @@ extern "C" int sd_mlstm_scan(const float* q, const float* k, const float* v, con
   SD_REQUIRE(CH >= 1 && CH * CT <= kScanLoadsV * CT * NS, SD_ERR_UNSUPPORTED,
              "sd_mlstm_scan: key size %d with value size %d leaves no chunk", dk, dv);
   const size_t lds = sizeof(float) * ((size_t)2 * CH * dkp + (size_t)CH * CT + 2 * CH + (size_t)CH * NS * CT);
-  MlstmArgs g{q, k, v, zi, zf, ld, bi, bf, cap, q_scale, S, n_state, const_cast<float*>(m_state), entries, num, m_rows, H, dk, dv};
-  mlstm_scan_kernel<<<dim3((cols + CT - 1) / CT, H, n_entries), CT * NS, lds, (hipStream_t)stream>>>(g, CT, NS, CH);
+  mlstm_scan_kernel<<<dim3((cols + CT - 1) / CT, H, n_entries), CT * NS, lds, st>>>(g, CT, NS, CH);
   SD_CHECK_LAUNCH("sd_mlstm_scan");
+  return SD_OK;
+}
+
+int sd_tiled_window_attention_(const float* q, int64_t ldq, const void* k_cache, const void* v_cache,
+                               const int32_t* row_pos, const int32_t* block_tables, int max_blocks, int page, int n_rows,
+                               int H, int G, int dk, int dv, int window, float scale, float softcap, const float* dist1,
+                               const float* dist2, const int32_t* entries, int n_entries, float* out, void* out_bf16,
+                               int64_t ldo, sd_stream_t stream) {
+  (void)row_pos;
+  if (page != kPage || dk % 8 || dv % 8 || dk > 128 || dv > 128 || ldq % 4 || !sd_aligned16(q) || !sd_aligned16(k_cache) ||
+      !sd_aligned16(v_cache) || !(ldo % 4 || (sd_aligned16(out) && sd_aligned16(out_bf16))))
+    return SD_ERR_UNSUPPORTED;
+  const int qh = H / G;
+  TiledAttnArgs g{q, ldq, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, entries, dist1, dist2, out,
+                  (bf16_t*)out_bf16, ldo, scale, softcap, n_entries, max_blocks, H, G, dk, dv, window, 0, 0};
+  g.wh = qh >= 4 ? 4 : (qh >= 2 ? 2 : 1);
+  g.n_hgroups = (qh + g.wh - 1) / g.wh;
+  const int tq = 16 * (4 / g.wh);
+  dim3 grid(n_rows / tq + n_entries, G, g.n_hgroups);
+  hipStream_t st = (hipStream_t)stream;
+  if (dk <= 64 && dv <= 64) tiled_window_attn_kernel<2, 4><<<grid, 256, 0, st>>>(g);
+  else if (dk <= 64) tiled_window_attn_kernel<2, 8><<<grid, 256, 0, st>>>(g);
+  else if (dv <= 64) tiled_window_attn_kernel<4, 4><<<grid, 256, 0, st>>>(g);
+  else tiled_window_attn_kernel<4, 8><<<grid, 256, 0, st>>>(g);
+  SD_CHECK_LAUNCH("sd_distance_softmax_attention (tiled)");
   return SD_OK;
 }
 

@@ -1595,7 +1595,7 @@ extern "C" int sd_linear_two_inputs(const void*, const void*, const void*, int64
 extern "C" int sd_distance_softmax_attention(const float*, int64_t, const void*, const void*, int, const int32_t*,
                                              const int32_t*, const int32_t*, int, int, int, int, int, int, int, int,
                                              int, int, int, float, float, const float*, const float*, const float*,
-                                             float*, void*, int64_t, void*, size_t, sd_stream_t) {
+                                             const int32_t*, int, float*, void*, int64_t, void*, size_t, sd_stream_t) {
   UNSUPPORTED("sd_distance_softmax_attention");
 }
 extern "C" int sd_joint_residual(float*, const int32_t*, const float*, const void*, float*, const void*, const void*,
@@ -1621,9 +1621,10 @@ extern "C" int sd_conv_attn_prep(const float*, int64_t, const void*, const void*
                                  const sd_poly_norm*, sd_stream_t) {
   UNSUPPORTED("sd_conv_attn_prep");
 }
+extern "C" size_t sd_mlstm_scratch_bytes(int, int, int, int, int) { return 0; }
 extern "C" int sd_mlstm_scan(const float*, const float*, const float*, const float*, const float*, int64_t,
                              const float*, const float*, float, float, float*, float*, const float*, const int32_t*,
-                             int, float*, float*, int, int, int, sd_stream_t) {
+                             int, int, float*, float*, int, int, int, void*, size_t, sd_stream_t) {
   UNSUPPORTED("sd_mlstm_scan");
 }
 extern "C" int sd_mlstm_read(const float*, const float*, float*, const int32_t*, const float*, int64_t, const void*,

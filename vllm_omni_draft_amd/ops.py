@@ -1457,10 +1457,11 @@ def linear_two_inputs(W: "TiledWeight", x, x2, n_first: int) -> torch.Tensor:
 
 
 def distance_softmax_attention(q, k_cache, v_cache, row_pos, row_slot, block_tables, H, G, dk, dv, scale, window=0,
-                               softcap=0.0, dist1=None, dist2=None, split=True, ldo=0, bf16_only=False):
+                               softcap=0.0, dist1=None, dist2=None, split=True, ldo=0, bf16_only=False, entries=None):
     """Grouped-query softmax attention over a sliding window (0: every earlier token) whose capped
     scores lose dist1[h] * ln(1 + dist2[h] * distance); q f32 [rows, H*dk] -> f32 [rows, H*dv], or, with
-    ldo > H*dv, a view of rows that far apart; bf16_only: bfloat16 instead."""
+    ldo > H*dv, a view of rows that far apart; bf16_only: bfloat16 instead.  entries int32 [n, 4] (or
+    None): the rows' portions, with which many rows over bfloat16 caches run on the matrix cores."""
     _f32(q, "q")
     window, ldo = int(window) or 0x7fffffff, int(ldo) or H * dv
     dt = torch.bfloat16 if bf16_only else torch.float32
@@ -1472,8 +1473,9 @@ def distance_softmax_attention(q, k_cache, v_cache, row_pos, row_slot, block_tab
     _lib.check(lib.sd_distance_softmax_attention(
         _p(q), q.shape[1], _p(k_cache), _p(v_cache), int(k_cache.dtype == torch.float32), _p(row_pos), _p(row_slot),
         _p(block_tables), block_tables.shape[1], PAGE, q.shape[0], H, G, 1, dk, dv, window, 0, 0, float(scale),
-        float(softcap), None, _p(dist1), _p(dist2), None if bf16_only else _p(out), _p(out) if bf16_only else None, ldo,
-        _p(scratch), n, _stream()), "sd_distance_softmax_attention")
+        float(softcap), None, _p(dist1), _p(dist2), _p(entries), entries.shape[0] if entries is not None else 0,
+        None if bf16_only else _p(out), _p(out) if bf16_only else None, ldo, _p(scratch), n, _stream()),
+        "sd_distance_softmax_attention")
     return out[:, :H * dv]
 
 
@@ -1544,9 +1546,11 @@ def conv_attn_prep(proj, conv_w, conv_state, H, G, dk, dv, q_norm_w, k_norm_w, e
     return q
 
 
-def mlstm_scan_packed(buf, bi, bf, cap, state, n_state, m_state, entries, num, m_rows, q_scale=1.0) -> None:
+def mlstm_scan_packed(buf, bi, bf, cap, state, n_state, m_state, entries, num, m_rows, q_scale=1.0,
+                      scratch=None) -> None:
     """sd_mlstm_scan on rows buf f32 [rows, q | k | v | zi | zf] (zi, zf the last 2*H columns) into num
-    [rows, H, dv + 1] and m_rows [rows, H]; state [slots, H, dk, dv] and n_state [slots, H, dk] move on."""
+    [rows, H, dv + 1] and m_rows [rows, H]; state [slots, H, dk, dv] and n_state [slots, H, dk] move on.
+    scratch (uint8, of mlstm_scratch's size): long portions in chunks."""
     _f32(buf, "buf")
     H, dk, dv = state.shape[1:]
     ptr, at = [], 0
@@ -1555,17 +1559,26 @@ def mlstm_scan_packed(buf, bi, bf, cap, state, n_state, m_state, entries, num, m
         at += cols
     ptr += [buf.data_ptr() + 4 * (buf.shape[1] - 2 * H), buf.data_ptr() + 4 * (buf.shape[1] - H)]
     _lib.check(_lib.load().sd_mlstm_scan(*ptr, buf.shape[1], _p(bi), _p(bf), float(cap), float(q_scale), _p(state),
-                                         _p(n_state), _p(m_state), _p(entries), entries.shape[0], _p(num), _p(m_rows), H,
-                                         dk, dv, _stream()), "sd_mlstm_scan")
+                                         _p(n_state), _p(m_state), _p(entries), entries.shape[0], buf.shape[0], _p(num),
+                                         _p(m_rows), H, dk, dv, _p(scratch), scratch.numel() if scratch is not None else 0,
+                                         _stream()), "sd_mlstm_scan")
 
 
-def mlstm_scan(q, k, v, zi, zf, bi, bf, cap, state, n_state, m_state, entries, q_scale=1.0):
-    """mlstm_scan_packed on separate q, k [rows, H*dk], v [rows, H*dv], zi, zf [rows, H]: (num, m_rows)."""
+def mlstm_scratch(n_rows, n_entries, H, dk, dv, device="cuda"):
+    """The scratch of mlstm_scan's chunked form, or None where it needs none."""
+    n = int(_lib.load().sd_mlstm_scratch_bytes(n_rows, n_entries, H, dk, dv))
+    return torch.empty(n, dtype=torch.uint8, device=device) if n else None
+
+
+def mlstm_scan(q, k, v, zi, zf, bi, bf, cap, state, n_state, m_state, entries, q_scale=1.0, chunks=True):
+    """mlstm_scan_packed on separate q, k [rows, H*dk], v [rows, H*dv], zi, zf [rows, H]: (num, m_rows).
+    chunks=False: token by token, whatever the portions' lengths."""
     buf = torch.cat([q, k, v, zi, zf], dim=1).contiguous()
     n, H, dv = q.shape[0], state.shape[1], state.shape[3]
     num = torch.empty(n, H, dv + 1, dtype=torch.float32, device=q.device)
     m_rows = torch.empty(n, H, dtype=torch.float32, device=q.device)
-    mlstm_scan_packed(buf, bi, bf, cap, state, n_state, m_state, entries, num, m_rows, q_scale)
+    scratch = mlstm_scratch(n, entries.shape[0], *state.shape[1:], device=q.device) if chunks else None
+    mlstm_scan_packed(buf, bi, bf, cap, state, n_state, m_state, entries, num, m_rows, q_scale, scratch)
     return num, m_rows
 
 
