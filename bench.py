@@ -1280,7 +1280,7 @@ def guf_kernel_rooflines(cfg, device, ctx, rows):
     out.append(("distance_softmax_attention", "window_softmax_attention (grouped heads)", us,
                 G * 2 * D * 2 * span + rows * H * D * 6, 2.0 * keys * H * 2 * D, F32_VALU_PEAK_TFLOPS))
     Cq = (H + 2 * G) * D
-    proj, cw, cst, cb = rn(rows, Cq), bf(Cq, taps), torch.zeros(1, taps - 1, Cq, device=device), bf(Cq)
+    proj, cw, cst, cb = rn(rows, Cq), bf(taps, Cq), torch.zeros(1, taps - 1, Cq, device=device), bf(Cq)
     qw, kw = bf(D), bf(D)
     us = _events(lambda: ops.conv_attn_prep(proj, cw, cst, H, G, D, D, qw, kw, 1e-5, kc, vc, pos, slot, ent, tables, bias=cb,
                                             temp=(0.1, 1024)), 5)
@@ -1303,7 +1303,7 @@ def guf_kernel_rooflines(cfg, device, ctx, rows):
     us = _events(lambda: ops.poly_norm_rows(z, coef, 1e-5, bias=zb, bf16=True), 5)
     out.append(("poly_norm_rows", "act_rows / relu_mul_rows", us, rows * F * 6, 0.0, F32_VALU_PEAK_TFLOPS))
     x, a, ab, w1, w2 = rn(rows, W), rn(rows, W), bf(W), bf(W), bf(W)
-    icw, ics = bf(W, GUF_TAPS), torch.zeros(1, GUF_TAPS - 1, W, device=device)
+    icw, ics = bf(GUF_TAPS, W), torch.zeros(1, GUF_TAPS - 1, W, device=device)
     if rows == 1:
         us = _events(lambda: ops.joint_residual(x, a, ab, w1, w2, bf16=True, conv_w=icw, conv_state=ics, row_pos=pos,
                                                 row_slot=slot), 5)

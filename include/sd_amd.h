@@ -1372,7 +1372,7 @@ int sd_distance_softmax_attention(const float* q, int64_t ldq, const void* k_cac
  *   h1[r] = LN(x[r]) * w1, h2[r] = LN(x[r]) * w2          (w1 != NULL; w2 may be NULL)
  * LN(x) = (x - mean) / sqrt(mean((x - mean)^2) + eps); h1_bf16 / h2_bf16 the same as bf16, every
  * output may be NULL.  rows (int32 [n_rows], or NULL): output row i comes from x and a of row
- * rows[i], and x is left as it is.  conv_w ([W, taps] or NULL): h1 is replaced by h1 + conv(h1), a
+ * rows[i], and x is left as it is.  conv_w ([taps, W] or NULL): h1 is replaced by h1 + conv(h1), a
  * causal convolution per channel over the sequence; every row must then be alone in its entry (a
  * decoding step): its predecessors are in conv_state f32 [slots, taps-1, W] (oldest first; what
  * lies before position 0 counts as zero), which is moved on.  Weights in the model's element type. */
@@ -1381,7 +1381,7 @@ int sd_joint_residual(float* x, const int32_t* rows, const float* a, const void*
                       void* h1_bf16, float* h2, void* h2_bf16, const void* conv_w, int taps,
                       float* conv_state, const int32_t* row_pos, const int32_t* row_slot, int n_rows,
                       int W, sd_stream_t stream);
-/* out[r] = x[r] + sum_j w[:, j] * x(r - taps + 1 + j): a causal convolution per channel (w [C, taps])
+/* out[r] = x[r] + sum_j w[j] * x(r - taps + 1 + j): a causal convolution per channel (w [taps, C])
  * added to its input, over each entry's rows, the sequence's state and zeros before its start;
  * then conv_state is moved on (sd_conv_tail).  entries as in sd_seq_batch.                  */
 int sd_conv_add_rows(const float* x, int64_t ldx, const void* w, int w_f32, float* conv_state,
@@ -1411,7 +1411,7 @@ typedef struct {
 /* Grouped-query attention's preparation where q, k and v pass a causal convolution each.  proj
  * [rows, ld] f32 stacks q [H*dk], k [G*dk], v [G*dv] (shared: q alone, the layer reads keys and
  * values another layer appended), C channels in all; bias [C] (or NULL) is added before the
- * convolution conv_w [C, taps] (conv_state f32 [slots, taps-1, C], moved on).  q and k are then
+ * convolution conv_w [taps, C] (conv_state f32 [slots, taps-1, C], moved on).  q and k are then
  * RMS-normed per head (weights [dk]); q is multiplied by 1 + temp_coef * ln(floor((p + 1) /
  * temp_every) + 1) at position p (temp_every 0: not) and written to q_out [rows, H*dk]; k and v
  * go to the caches as sd_cache_append puts them.  act (or NULL): an activation computed in the
@@ -1429,10 +1429,10 @@ int sd_conv_attn_prep(const float* proj, int64_t ld, const void* bias, const voi
  * [rows, H*dk], v [rows, H*dv], zi, zf [rows, H], all ld floats per row; bi, bf f32 [H]; S f32
  * [slots, H, dk, dv], n_state f32 [slots, H, dk], m_state f32 [slots, H] (an entry that starts at
  * position 0 starts from zero).  num f32 [rows, H, dv + 1]: S^T q, then n . q; m_rows f32 [rows, H]: m.
- * S and n_state are moved on; m_state is left to sd_mlstm_read.  With scratch (f32 [], of
- * sd_mlstm_scratch_bytes, 0: none needed) long portions run in chunks of 64 tokens on the f32 matrix
- * instruction, every chunk beside the others: the chunks' own sums, a scan over the chunks, then
- * the tokens' results; otherwise token by token.                                           */
+ * S and n_state are moved on; m_state is left to sd_mlstm_read.  With scratch of
+ * sd_mlstm_scratch_bytes bytes (0: few rows, or sizes that take none) long portions run in chunks of
+ * 64 tokens on the f32 matrix instruction, every chunk beside the others: the chunks' own sums, a
+ * scan over the chunks, then the tokens' results; otherwise token by token.                 */
 size_t sd_mlstm_scratch_bytes(int n_rows, int n_entries, int H, int dk, int dv);
 int sd_mlstm_scan(const float* q, const float* k, const float* v, const float* zi, const float* zf,
                   int64_t ld, const float* bi, const float* bf, float cap, float q_scale, float* S,
@@ -1447,6 +1447,14 @@ int sd_mlstm_scan(const float* q, const float* k, const float* v, const float* z
 int sd_mlstm_read(const float* num, const float* m_rows, float* m_state, const int32_t* row_slot,
                   const float* gate, int64_t ldg, const void* w, int w_f32, float eps, float* y,
                   void* y_bf16, int64_t ldy, int n_rows, int H, int dv, const sd_poly_norm* act,
+                  sd_stream_t stream);
+/* sd_mlstm_scan and sd_mlstm_read in one launch for rows that are alone in their entries (a decoding
+ * step): row_pos and row_slot give every row's position and slot; all three states are moved on. */
+int sd_mlstm_step(const float* q, const float* k, const float* v, const float* zi, const float* zf,
+                  int64_t ld, const float* bi, const float* bf, float cap, float q_scale, float* S,
+                  float* n_state, float* m_state, const int32_t* row_pos, const int32_t* row_slot,
+                  const float* gate, const void* w, int w_f32, float eps, float* y, void* y_bf16,
+                  int64_t ldy, int n_rows, int H, int dk, int dv, const sd_poly_norm* act,
                   sd_stream_t stream);
 /* x[r, c] *= s                                                                             */
 int sd_scale_rows(float* x, int64_t ld, float s, int n_rows, int n_cols, sd_stream_t stream);
@@ -1591,10 +1599,10 @@ typedef struct {
    * f [heads].  w_o [width, heads*vdim + ff] puts the mixer's output matrix and the feed-forward's
    * down matrix side by side: one product adds both sublayers.  w_o_bias: the down matrix's bias. */
   int mix_rows;
-  const void* in_conv_w;    /* [width, in_taps] the mixer's input convolution, or NULL */
+  const void* in_conv_w;    /* [in_taps, width] the mixer's input convolution, or NULL */
   int in_taps;
   float* in_conv_state;     /* [slots, in_taps-1, width] */
-  /* attention: conv_w [channels of q, k, v, s_taps] with conv_state; q_norm_w / k_norm_w [dim] */
+  /* attention: conv_w [s_taps, channels of q, k, v] with conv_state; q_norm_w / k_norm_w [dim] */
   float q_temp_coef;
   int q_temp_every;         /* 0: no position factor of the query */
   const float* dist1;       /* [heads] or NULL: sd_distance_softmax_attention */

@@ -255,7 +255,7 @@ def test_residual_update_with_two_norms(W, taps, wdt):
     st = torch.full((3, max(taps - 1, 1), W), 7.0, device=DEV)          # (what an earlier request left)
     for t in range(T):
         x = dev(xs[:, t].clone())
-        g1, g2, cp = ops.joint_residual(x, dev(a[:, t]), dev(ab), dev(w1), dev(w2), eps, x_copy=True, conv_w=dev(cw),
+        g1, g2, cp = ops.joint_residual(x, dev(a[:, t]), dev(ab), dev(w1), dev(w2), eps, x_copy=True, conv_w=dev(cw.t()),
                                         conv_state=st, row_pos=i32([t, t]), row_slot=i32([2, 0]))
         assert rel(x, want_x[:, t]) < 2e-7 and torch.equal(cp, x)
         assert rel(g1, hc[:, t]) < 2e-6 and rel(g2, h2[:, t]) < 2e-6, t
@@ -268,7 +268,7 @@ def test_residual_update_with_two_norms(W, taps, wdt):
         av = dev(torch.cat([a[0, lo:hi], a[1, lo:hi]]))
         g1, _, _ = ops.joint_residual(x, av, dev(ab), dev(w1), dev(w2), eps)
         pos, slot = list(range(lo, hi)) * 2, [1] * n + [2] * n
-        got.append(ops.conv_add_rows(g1, dev(cw), st, i32(pos), i32(slot), i32([[1, 0, n, lo], [2, n, n, lo]])).view(2, n, W))
+        got.append(ops.conv_add_rows(g1, dev(cw.t()), st, i32(pos), i32(slot), i32([[1, 0, n, lo], [2, n, n, lo]])).view(2, n, W))
     assert rel(torch.cat(got, 1), hc) < 2e-6
     # some rows only, x left as it is
     x = dev(xs[0].clone())
@@ -321,7 +321,7 @@ def test_convolved_preparation(H, Gk, dk, dv, taps, temp, shared, wdt):
     for lo, hi in ((0, 1), (1, 3), (3, 20), (20, 21), (21, 22), (22, T)):
         n = hi - lo
         act = torch.empty(2 * n, 19, device=DEV)
-        q = ops.conv_attn_prep(dev(torch.cat([proj[0, lo:hi], proj[1, lo:hi]])), dev(cw), st, H, Gk, dk, dv, dev(qw), dev(kw), eps,
+        q = ops.conv_attn_prep(dev(torch.cat([proj[0, lo:hi], proj[1, lo:hi]])), dev(cw.t()), st, H, Gk, dk, dv, dev(qw), dev(kw), eps,
                                None if shared else kc, None if shared else vc, i32(list(range(lo, hi)) * 2), i32([2] * n + [0] * n),
                                i32([[2, 0, n, lo], [0, n, n, lo]]), None if shared else bt, bias=dev(b), temp=temp,
                                act=(dev(torch.cat([z[0, lo:hi], z[1, lo:hi]])), dev(coef), dev(zb), act))
@@ -346,9 +346,9 @@ def test_convolved_preparation(H, Gk, dk, dv, taps, temp, shared, wdt):
 
 @pytest.mark.parametrize("H,dk,dv", [(2, 16, 24), (3, 21, 37), (1, 1, 1), (2, 130, 72), (4, 256, 260), (1, 5, 400), (2, 128, 128),
                                      (2, 64, 192), (3, 32, 64), (1, 96, 40)])
-@pytest.mark.parametrize("chunks", [True, False])
-def test_matrix_memory(H, dk, dv, chunks):
-    """Scan (in chunks, and token by token) and read-out in portions of two interleaved sequences (down to single tokens), from slots
+@pytest.mark.parametrize("form", ["chunks", "tokens", "step"])
+def test_matrix_memory(H, dk, dv, form):
+    """Scan (in chunks, token by token, single tokens in one launch) and read-out in portions of two interleaved sequences (down to single tokens), from slots
     an earlier request left full, against the plain recurrence; the activation that rides along."""
     from vllm_omni_draft_amd import ops
     g = torch.Generator().manual_seed(H * 1000 + dk)
@@ -361,11 +361,18 @@ def test_matrix_memory(H, dk, dv, chunks):
     z = rn(2, T, 23)
     S, N, M = (torch.full((3, H) + s, 5.0, device=DEV) for s in ((dk, dv), (dk,), ()))
     got = [[], []]
-    for lo, hi in ((0, 70), (70, 71), (71, 73), (73, 74), (74, 139), (139, 203), (203, T)):
+    for lo, hi in ((0, 1), (1, 2), (2, 70), (70, 71), (71, 73), (73, 74), (74, 139), (139, 203), (203, T)):
         n = hi - lo
         cat = lambda t: dev(torch.cat([t[0, lo:hi], t[1, lo:hi]]))
+        if form == "step" and n == 1:
+            y, a = ops.mlstm_step(cat(q), cat(k), cat(v), cat(zi), cat(zf), dev(bi), dev(bf), cap, S, N, M, i32([lo, lo]),
+                                  i32([2, 0]), cat(gate), dev(w), eps, q_scale=dk ** -0.5, act=(cat(z), dev(coef), None))
+            for s in range(2):
+                got[s].append(y[s:s + 1])
+                assert rel(a[s:s + 1], G.poly_norm(z[s, lo:hi], coef, eps)) < 2e-6
+            continue
         num, mr = ops.mlstm_scan(cat(q), cat(k), cat(v), cat(zi), cat(zf), dev(bi), dev(bf), cap, S, N, M,
-                                 i32([[2, 0, n, lo], [0, n, n, lo]]), q_scale=dk ** -0.5, chunks=chunks)
+                                 i32([[2, 0, n, lo], [0, n, n, lo]]), q_scale=dk ** -0.5, chunks=form == "chunks")
         y, a = ops.mlstm_read(num, mr, M, i32([2] * n + [0] * n), cat(gate), dev(w), eps, act=(cat(z), dev(coef), None))
         for s in range(2):
             got[s].append(y[s * n:(s + 1) * n])

@@ -221,14 +221,14 @@ def test_weights_are_stacked_per_layer():
     assert a.mix_rows == 64 and a.w_in.shape == (64 + 24, 40) and a.w_in[56:64].abs().sum() == 0    # padded to 16 rows
     assert torch.equal(a.w_in[46 - 10:46], st["l0.mix.v"][:10]) and torch.equal(a.w_in[64:], st["l0.mlp.up"])
     assert torch.equal(a.w_o, torch.cat([st["l0.mix.o"], st["l0.mlp.down"]], 1)) and torch.equal(a.w_o_bias, st["l0.mlp.down.b"])
-    assert a.conv_w.shape == (56, 4) and torch.equal(a.conv_w[24:36], st["l0.mix.k.conv"])
+    assert a.conv_w.shape == (4, 56) and torch.equal(a.conv_w[:, 24:36].t(), st["l0.mix.k.conv"])
     assert torch.equal(a.w_in_bias, torch.cat([st["l0.mix.q.b"], st["l0.mix.k.b"], st["l0.mix.v.b"]]))
     assert torch.equal(a.dist1, st["l0.mix.r1"]) and torch.equal(a.ff_coef, st["l0.mlp.act"]) and a.ff_coef.dtype == torch.float32
     assert b.mix_rows == 128 and b.w_in.shape == (128, 40) and b.w_in[126:].abs().sum() == 0
     assert torch.equal(b.w_in[120:123], st["l1.mix.i"]) and torch.equal(b.w_in[123:126], st["l1.mix.f"])
     assert torch.equal(b.gate_bias, torch.cat([st["l1.mix.i.b"], st["l1.mix.f.b"]])) and b.w_o.shape == (40, 36)
     assert b.norm2_w is None and b.w_o_bias is None and b.ff_coef is None
-    assert c.mix_rows == 32 and c.conv_w.shape == (24, 2) and c.k_norm_w is None and c.w_in_bias.shape == (24,)
+    assert c.mix_rows == 32 and c.conv_w.shape == (2, 24) and c.k_norm_w is None and c.w_in_bias.shape == (24,)
     st2 = weights.seq_random_state(mc, 0)
     assert {k: tuple(v.shape) for k, v in st2.items()} == {k: tuple(v.shape) for k, v in st.items()}
     del st["l1.mix.f.b"]

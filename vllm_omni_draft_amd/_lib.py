@@ -311,6 +311,8 @@ SIGNATURES = {
     "sd_mlstm_scratch_bytes": (C.c_size_t, [i32, i32, i32, i32, i32]),
     "sd_mlstm_scan": (i32, [vp, vp, vp, vp, vp, i64, vp, vp, C.c_float, C.c_float, vp, vp, vp, vp, i32, i32, vp, vp, i32,
                             i32, i32, vp, C.c_size_t, vp]),
+    "sd_mlstm_step": (i32, [vp, vp, vp, vp, vp, i64, vp, vp, C.c_float, C.c_float, vp, vp, vp, vp, vp, vp, vp, i32,
+                            C.c_float, vp, vp, i64, i32, i32, i32, i32, C.POINTER(PolyNorm), vp]),
     "sd_mlstm_read": (i32, [vp, vp, vp, vp, vp, i64, vp, i32, C.c_float, vp, vp, i64, i32, i32, i32,
                             C.POINTER(PolyNorm), vp]),
     "sd_seq_model_create": (vp, [C.POINTER(SeqModelDesc)]),

@@ -1631,6 +1631,13 @@ int joint_layer(const sd_seq_model& m, const sd_seq_layer& l, const sd_seq_batch
                       yb ? (void*)(yb + H * dv) : nullptr, K, l.ff};
   const sd_poly_norm* pact = l.ff > 0 ? &act : nullptr;
   if (l.kind == SD_MIX_MLSTM) {
+    if (R == b.n_entries) {
+      SQ_TRY(sd_mlstm_step(proj + c.q, proj + c.k, proj + c.v, proj + c.i, proj + c.f, ld, l.gate_bias, l.gate_bias + H,
+                           l.gate_cap, l.q_scale, l.state, l.n_state, l.m_state, b.row_pos, b.row_slot, proj + c.g,
+                           l.s_norm_w, f32, d.norm_eps, y, yb, K, R, H, dk, dv, pact, stream));
+      return seq_linear(l.w_o, l.w_o_tiled, f32, y, nullptr, K, yb, K, nullptr, (float*)(base + w.mix), W, R, W, K,
+                        wide_ws, w.wide_bytes, stream);
+    }
     float* m_rows = (float*)(base + w.step);
     SQ_TRY(sd_mlstm_scan(proj + c.q, proj + c.k, proj + c.v, proj + c.i, proj + c.f, ld, l.gate_bias, l.gate_bias + H,
                          l.gate_cap, l.q_scale, l.state, l.n_state, l.m_state, b.entries, b.n_entries, R, o, m_rows, H,

@@ -83,7 +83,7 @@ struct JointArgs {
   bf16_t* h1_b;
   float* h2;               // LN(x) w2
   bf16_t* h2_b;
-  const void* conv_w;      // [W, taps] or nullptr; rows are alone in their entries
+  const void* conv_w;      // [taps, W] or nullptr; rows are alone in their entries
   float* conv_state;
   const int32_t* row_pos;
   const int32_t* row_slot;
@@ -91,13 +91,31 @@ struct JointArgs {
 };
 
 // A workgroup per row; a thread holds up to NV pieces of V columns in registers, so the row is read
-// from memory once.
+// from memory once.  With one piece per thread and few taps everything the end of the kernel needs
+// (norm weights, convolution, state) is asked for before the row's sums are formed.
+constexpr int kEarlyTaps = 4;
 template <typename T, int V, int NV>
 __global__ __launch_bounds__(1024) void joint_residual_kernel(JointArgs g) {
   __shared__ float red[16];
-  const int i = blockIdx.x, W = g.W, np = W / V, nthr = blockDim.x;
+  const int i = blockIdx.x, W = g.W, np = W / V, nthr = blockDim.x, taps = g.taps;
   const int r = g.rows ? g.rows[i] : i;
+  const int pos = g.conv_w ? g.row_pos[r] : 0, slot = g.conv_w ? g.row_slot[r] : 0;
   float* xr = g.x + (size_t)r * W;
+  const bool early = NV == 1 && taps <= kEarlyTaps;
+  Pack<V> w1e, w2e, cwe[kEarlyTaps], ste[kEarlyTaps - 1];
+  if (early && g.w1 && (int)threadIdx.x < np) {
+    const int c = threadIdx.x * V;
+    w1e = ld_pack<V>((const T*)g.w1 + c);
+    if (g.w2) w2e = ld_pack<V>((const T*)g.w2 + c);
+    if (g.conv_w) {
+#pragma unroll
+      for (int t = 0; t < kEarlyTaps; ++t)
+        if (t < taps) cwe[t] = ld_pack<V>((const T*)g.conv_w + (size_t)t * W + c);
+#pragma unroll
+      for (int t = 0; t < kEarlyTaps - 1; ++t)
+        if (t < taps - 1) ste[t] = ld_pack<V>(g.conv_state + ((size_t)slot * (taps - 1) + t) * W + c);
+    }
+  }
   Pack<V> p[NV];
   float sum = 0.f;
 #pragma unroll
@@ -134,43 +152,53 @@ __global__ __launch_bounds__(1024) void joint_residual_kernel(JointArgs g) {
       }
     }
   const float rstd = 1.f / sqrtf(block_sum(ss, red) / (float)W + g.eps);
-  const int taps = g.taps;
-  const int pos = g.conv_w ? g.row_pos[r] : 0, slot = g.conv_w ? g.row_slot[r] : 0;
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
     if (threadIdx.x + k * nthr >= np) continue;
     const int c = (threadIdx.x + k * nthr) * V;
-    const Pack<V> w1 = ld_pack<V>((const T*)g.w1 + c);
+    const Pack<V> w1 = early ? w1e : ld_pack<V>((const T*)g.w1 + c);
     Pack<V> u;
 #pragma unroll
     for (int e = 0; e < V; ++e) u.v[e] = p[k].v[e] * rstd * w1.v[e];
-    if (g.conv_w) {
+    if (g.conv_w) {   // oldest input first; inputs move one place towards the oldest
       Pack<V> acc;
 #pragma unroll
       for (int e = 0; e < V; ++e) acc.v[e] = 0.f;
-      const T* cw = (const T*)g.conv_w + (size_t)c * taps;
       float* st = g.conv_state + (size_t)slot * (taps - 1) * W + c;
-      for (int s = 0; s < taps - 1; ++s) {     // oldest input first
-        Pack<V> in = ld_pack<V>(st + (size_t)s * W);
-        const bool there = pos - (taps - 1 - s) >= 0;
+      auto tap = [&](int t, Pack<V> in, const Pack<V>& cw) {
+        const bool there = pos - (taps - 1 - t) >= 0;
 #pragma unroll
         for (int e = 0; e < V; ++e) {
           in.v[e] = there ? in.v[e] : 0.f;
-          acc.v[e] = fmaf(ld_f(cw + e * taps + s), in.v[e], acc.v[e]);
+          acc.v[e] = fmaf(cw.v[e], in.v[e], acc.v[e]);
         }
-        if (s > 0) st_pack<V>(st + (size_t)(s - 1) * W, in);
+        if (t > 0) st_pack<V>(st + (size_t)(t - 1) * W, in);
+      };
+      Pack<V> cw;
+      if (early) {
+#pragma unroll
+        for (int t = 0; t < kEarlyTaps - 1; ++t)
+          if (t < taps - 1) tap(t, ste[t], cwe[t]);
+        cw = cwe[0];
+#pragma unroll
+        for (int t = 1; t < kEarlyTaps; ++t)
+          if (t == taps - 1) cw = cwe[t];
+      } else {
+        for (int t = 0; t < taps - 1; ++t)
+          tap(t, ld_pack<V>(st + (size_t)t * W), ld_pack<V>((const T*)g.conv_w + (size_t)t * W + c));
+        cw = ld_pack<V>((const T*)g.conv_w + (size_t)(taps - 1) * W + c);
       }
       if (taps > 1) st_pack<V>(st + (size_t)(taps - 2) * W, u);
 #pragma unroll
       for (int e = 0; e < V; ++e) {
-        acc.v[e] = fmaf(ld_f(cw + e * taps + taps - 1), u.v[e], acc.v[e]);
+        acc.v[e] = fmaf(cw.v[e], u.v[e], acc.v[e]);
         u.v[e] += acc.v[e];
       }
     }
     if (g.h1) st_pack<V>(g.h1 + (size_t)i * W + c, u);
     if (g.h1_b) st_pack<V>(g.h1_b + (size_t)i * W + c, u);
     if (g.w2) {
-      const Pack<V> w2 = ld_pack<V>((const T*)g.w2 + c);
+      const Pack<V> w2 = early ? w2e : ld_pack<V>((const T*)g.w2 + c);
       Pack<V> h;
 #pragma unroll
       for (int e = 0; e < V; ++e) h.v[e] = p[k].v[e] * rstd * w2.v[e];
@@ -188,35 +216,81 @@ __device__ __forceinline__ int rows_before(const int32_t* row_slot, int r, int t
   return t;
 }
 
+// Rows a workgroup convolves one after another, with the inputs of the last kRowTaps - 1 rows and the
+// weights in registers.
+constexpr int kRowBlock = 8;
+constexpr int kRowTaps = 8;
+
+// The input b steps before row r (of an entry with t rows before it in the batch).
+template <int V>
+__device__ __forceinline__ Pack<V> conv_input(const float* x, int64_t ldx, const float* state, int C, int taps, int r, int c,
+                                              int b, int t, int pos, int slot) {
+  if (b <= t) return ld_pack<V>(x + (size_t)(r - b) * ldx + c);
+  if (pos - b >= 0) return ld_pack<V>(state + ((size_t)slot * (taps - 1) + (taps - 1 - (b - t))) * C + c);
+  Pack<V> z;
+#pragma unroll
+  for (int e = 0; e < V; ++e) z.v[e] = 0.f;
+  return z;
+}
+
 // out = x + conv(x): x's entry rows before r, then the sequence's state, then zeros.  A workgroup
-// per (row, 256 pieces of V channels).
+// per (block of rows, 256 pieces of V channels).
 template <typename T, int V>
 __global__ __launch_bounds__(256) void conv_add_rows_kernel(
     const float* __restrict__ x, int64_t ldx, const T* __restrict__ w, const float* __restrict__ state,
     const int32_t* __restrict__ row_pos, const int32_t* __restrict__ row_slot, float* __restrict__ out,
-    bf16_t* __restrict__ out_b, int64_t ldo, int C, int taps) {
-  const int r = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * V;
+    bf16_t* __restrict__ out_b, int64_t ldo, int n_rows, int C, int taps) {
+  const int rb = blockIdx.x * kRowBlock, c = (blockIdx.y * 256 + threadIdx.x) * V;
   if (c >= C) return;
-  const int slot = row_slot[r], pos = row_pos[r], t = rows_before(row_slot, r, taps);
-  Pack<V> acc, cur;
+  const bool few = taps <= kRowTaps;
+  Pack<V> cur[kRowBlock], wt[kRowTaps], win[kRowTaps];   // wt[b], win[b]: b steps back
 #pragma unroll
-  for (int e = 0; e < V; ++e) acc.v[e] = cur.v[e] = 0.f;
-  for (int j = taps - 1; j >= 0; --j) {
-    Pack<V> in;
-    if (j <= t) in = ld_pack<V>(x + (size_t)(r - j) * ldx + c);
-    else if (pos - j >= 0) in = ld_pack<V>(state + ((size_t)slot * (taps - 1) + (taps - 1 - (j - t))) * C + c);
-    else {
+  for (int u = 0; u < kRowBlock; ++u) cur[u] = ld_pack<V>(x + (size_t)(rb + u < n_rows ? rb + u : n_rows - 1) * ldx + c);
 #pragma unroll
-      for (int e = 0; e < V; ++e) in.v[e] = 0.f;
+  for (int b = 0; b < kRowTaps; ++b)
+    if (few && b < taps) wt[b] = ld_pack<V>(w + (size_t)(taps - 1 - b) * C + c);
+  int prev = -1;
+#pragma unroll
+  for (int u = 0; u < kRowBlock; ++u) {
+    const int r = rb + u;
+    if (r >= n_rows) return;
+    const int slot = row_slot[r];
+    Pack<V> acc;
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc.v[e] = 0.f;
+    if (few) {
+      if (slot != prev) {
+        const int pos = row_pos[r], t = u == 0 ? rows_before(row_slot, r, taps) : 0;
+#pragma unroll
+        for (int b = 1; b < kRowTaps; ++b)
+          if (b < taps) win[b] = conv_input<V>(x, ldx, state, C, taps, r, c, b, t, pos, slot);
+      }
+#pragma unroll
+      for (int b = kRowTaps - 1; b >= 1; --b)
+        if (b < taps) {
+#pragma unroll
+          for (int e = 0; e < V; ++e) acc.v[e] = fmaf(wt[b].v[e], win[b].v[e], acc.v[e]);
+        }
+#pragma unroll
+      for (int e = 0; e < V; ++e) acc.v[e] = fmaf(wt[0].v[e], cur[u].v[e], acc.v[e]);
+#pragma unroll
+      for (int b = kRowTaps - 1; b >= 2; --b) win[b] = win[b - 1];
+      win[1] = cur[u];
+      prev = slot;
+    } else {
+      const int pos = row_pos[r], t = rows_before(row_slot, r, taps);
+      for (int b = taps - 1; b >= 0; --b) {
+        const Pack<V> in = conv_input<V>(x, ldx, state, C, taps, r, c, b, t, pos, slot);
+        const Pack<V> wb = ld_pack<V>(w + (size_t)(taps - 1 - b) * C + c);
+#pragma unroll
+        for (int e = 0; e < V; ++e) acc.v[e] = fmaf(wb.v[e], in.v[e], acc.v[e]);
+      }
     }
 #pragma unroll
-    for (int e = 0; e < V; ++e) acc.v[e] = fmaf(ld_f(w + (size_t)(c + e) * taps + (taps - 1 - j)), in.v[e], acc.v[e]);
-    if (j == 0) cur = in;
+    for (int e = 0; e < V; ++e) acc.v[e] += cur[u].v[e];
+    if (out) st_pack<V>(out + (size_t)r * ldo + c, acc);
+    if (out_b) st_pack<V>(out_b + (size_t)r * ldo + c, acc);
   }
-#pragma unroll
-  for (int e = 0; e < V; ++e) cur.v[e] += acc.v[e];
-  if (out) st_pack<V>(out + (size_t)r * ldo + c, cur);
-  if (out_b) st_pack<V>(out_b + (size_t)r * ldo + c, cur);
 }
 
 // An entry's last taps - 1 inputs (x + bias) become its slot's state.  A thread per channel.
@@ -239,14 +313,14 @@ __global__ void conv_tail_kernel(const float* __restrict__ x, int64_t ldx, const
 
 // ------------------------------------------------------------------ an activation of normed powers
 // out = k0 N(z) + k1 N(z^2) + k2 N(z^3) + k3, z the row + bias, N(y) = y / sqrt(mean(y^2) + eps) over
-// the row's F values.  By a whole workgroup of 256 threads; pieces of V values, the first kPolyRegs
-// of a thread held in registers between the sums and the result.
+// the row's F values.  By a whole workgroup (whole waves; red: 3 floats a wave); pieces of V values,
+// the first kPolyRegs of a thread held in registers between the sums and the result.
 constexpr int kPolyRegs = 8;
 template <typename T, int V>
 __device__ __forceinline__ void poly_norm_pieces(const float* __restrict__ z, const T* __restrict__ bias,
                                                  const float* __restrict__ coef, float eps, int F,
                                                  float* __restrict__ out, bf16_t* __restrict__ out_b, float* red) {
-  const int np = F / V;
+  const int np = F / V, nthr = blockDim.x;
   auto piece = [&](int i) {
     Pack<V> v = ld_pack<V>(z + (size_t)i * V);
     if (bias) {
@@ -268,31 +342,32 @@ __device__ __forceinline__ void poly_norm_pieces(const float* __restrict__ z, co
   };
   Pack<V> keep[kPolyRegs];
 #pragma unroll
-  for (int u = 0; u < kPolyRegs; ++u) {   // (on a piece clamped into the row: every load is issued)
-    const int i = threadIdx.x + 256 * u;
-    keep[u] = piece(i < np ? i : np - 1);
-  }
+  for (int u = 0; u < kPolyRegs; ++u)
+    if (nthr * u < np) {   // (on a piece clamped into the row)
+      const int i = threadIdx.x + nthr * u;
+      keep[u] = piece(i < np ? i : np - 1);
+    }
 #pragma unroll
   for (int u = 0; u < kPolyRegs; ++u)
-    if ((int)threadIdx.x + 256 * u < np) add(keep[u]);
-  for (int i = threadIdx.x + 256 * kPolyRegs; i < np; i += 256) add(piece(i));
+    if ((int)threadIdx.x + nthr * u < np) add(keep[u]);
+  for (int i = threadIdx.x + nthr * kPolyRegs; i < np; i += nthr) add(piece(i));
   s1 = wave_sum(s1);
   s2 = wave_sum(s2);
   s3 = wave_sum(s3);
-  const int wave = threadIdx.x >> 6;
+  const int wave = threadIdx.x >> 6, nw = nthr >> 6;
   if ((threadIdx.x & 63) == 0) {
     red[wave] = s1;
-    red[4 + wave] = s2;
-    red[8 + wave] = s3;
+    red[nw + wave] = s2;
+    red[2 * nw + wave] = s3;
   }
   __syncthreads();
   s1 = red[0];
-  s2 = red[4];
-  s3 = red[8];
-  for (int w = 1; w < 4; ++w) {
+  s2 = red[nw];
+  s3 = red[2 * nw];
+  for (int w = 1; w < nw; ++w) {
     s1 += red[w];
-    s2 += red[4 + w];
-    s3 += red[8 + w];
+    s2 += red[nw + w];
+    s3 += red[2 * nw + w];
   }
   const float n = (float)F;
   const float f1 = coef[0] / sqrtf(s1 / n + eps), f2 = coef[1] / sqrtf(s2 / n + eps),
@@ -306,8 +381,8 @@ __device__ __forceinline__ void poly_norm_pieces(const float* __restrict__ z, co
   };
 #pragma unroll
   for (int u = 0; u < kPolyRegs; ++u)
-    if ((int)threadIdx.x + 256 * u < np) write(threadIdx.x + 256 * u, keep[u]);
-  for (int i = threadIdx.x + 256 * kPolyRegs; i < np; i += 256) write(i, piece(i));
+    if ((int)threadIdx.x + nthr * u < np) write(threadIdx.x + nthr * u, keep[u]);
+  for (int i = threadIdx.x + nthr * kPolyRegs; i < np; i += nthr) write(i, piece(i));
 }
 template <typename T>
 __device__ __forceinline__ void poly_norm_row(const float* __restrict__ z, const T* __restrict__ bias,
@@ -338,7 +413,7 @@ struct ConvPrepArgs {
   const float* proj;       // [n, ld]: channels q [H*dk], k [G*dk], v [G*dv] (k, v absent: shared)
   int64_t ld;
   const void* bias;        // [C]
-  const void* conv_w;      // [C, taps]
+  const void* conv_w;      // [taps, C]
   float* conv_state;       // [slots, taps-1, C]
   const void* q_w;         // [dk]
   const void* k_w;
@@ -399,7 +474,7 @@ __global__ __launch_bounds__(256) void conv_prep_kernel(ConvPrepArgs g) {
         if (j <= t) in = pr[c - (int64_t)j * g.ld] + b;
         else if (pos - j >= 0) in = st[(size_t)(taps - 1 - (j - t)) * g.C + c];
         else in = 0.f;
-        acc = fmaf(ld_f(cw + (size_t)(ch0 + c) * taps + (taps - 1 - j)), in, acc);
+        acc = fmaf(ld_f(cw + (size_t)(taps - 1 - j) * g.C + ch0 + c), in, acc);
         // (a row alone in its entry: inputs move one place towards the oldest as they are read)
         if (g.single && j < taps - 1) st[(size_t)(taps - 2 - j) * g.C + c] = in;
       }
@@ -430,6 +505,88 @@ __global__ __launch_bounds__(256) void conv_prep_kernel(ConvPrepArgs g) {
 #pragma unroll
   for (int k = 0; k < kUnitRegs; ++k)
     if (lane + 64 * k < d) st_f(dst + lane + 64 * k, val[k]);
+}
+
+// The same for many rows: a wave takes its unit through kRowBlock rows one after another, weights and
+// the last inputs in registers (NC channels per lane).  States are left to conv_tail_kernel.
+template <typename T, int NC>
+__global__ __launch_bounds__(256) void conv_prep_block_kernel(ConvPrepArgs g, int n_rows) {
+  const int rb = blockIdx.x * kRowBlock, y = blockIdx.y;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int kind = y < g.q_wgs ? 0 : (y < g.q_wgs + g.kv_wgs ? 1 : 2);   // q, k, v
+  const int unit = (kind == 0 ? y : (kind == 1 ? y - g.q_wgs : y - g.q_wgs - g.kv_wgs)) * kUnitWaves + wave;
+  if (unit >= (kind == 0 ? g.H : g.G)) return;
+  const int d = kind == 2 ? g.dv : g.dk, taps = g.taps;
+  const int ch0 = (kind == 0 ? 0 : (kind == 1 ? g.H * g.dk : (g.H + g.G) * g.dk)) + unit * d;
+  const T* bias = (const T*)g.bias;
+  const T* nw = (const T*)(kind == 0 ? g.q_w : g.k_w);
+  float cur[kRowBlock][NC], wt[kRowTaps][NC], win[kRowTaps][NC], b[NC], norm[NC];
+  int ch[NC];
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    ch[k] = ch0 + (lane + 64 * k < d ? lane + 64 * k : d - 1);   // (clamped: results there are dropped)
+    b[k] = bias ? ld_f(bias + ch[k]) : 0.f;
+    norm[k] = kind < 2 ? ld_f(nw + ch[k] - ch0) : 1.f;
+#pragma unroll
+    for (int u = 0; u < kRowBlock; ++u) cur[u][k] = g.proj[(size_t)(rb + u < n_rows ? rb + u : n_rows - 1) * g.ld + ch[k]];
+#pragma unroll
+    for (int t = 0; t < kRowTaps; ++t)
+      if (t < taps) wt[t][k] = ld_f((const T*)g.conv_w + (size_t)(taps - 1 - t) * g.C + ch[k]);
+  }
+  int prev = -1;
+#pragma unroll
+  for (int u = 0; u < kRowBlock; ++u) {
+    const int r = rb + u;
+    if (r >= n_rows) return;
+    const int slot = g.row_slot[r], pos = g.row_pos[r];
+    if (slot != prev) {
+      const int t = u == 0 ? rows_before(g.row_slot, r, taps) : 0;
+#pragma unroll
+      for (int k = 0; k < NC; ++k)
+#pragma unroll
+        for (int s = 1; s < kRowTaps; ++s)
+          if (s < taps) {
+            if (s <= t) win[s][k] = g.proj[(size_t)(r - s) * g.ld + ch[k]] + b[k];
+            else if (pos - s >= 0) win[s][k] = g.conv_state[((size_t)slot * (taps - 1) + (taps - 1 - (s - t))) * g.C + ch[k]];
+            else win[s][k] = 0.f;
+          }
+    }
+    prev = slot;
+    float val[NC], ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < NC; ++k) {
+      const float in = cur[u][k] + b[k];
+      float acc = 0.f;
+#pragma unroll
+      for (int s = kRowTaps - 1; s >= 1; --s)
+        if (s < taps) acc = fmaf(wt[s][k], win[s][k], acc);
+      acc = fmaf(wt[0][k], in, acc);
+#pragma unroll
+      for (int s = kRowTaps - 1; s >= 2; --s) win[s][k] = win[s - 1][k];
+      win[1][k] = in;
+      val[k] = lane + 64 * k < d ? acc : 0.f;
+      ss = fmaf(val[k], val[k], ss);
+    }
+    if (kind < 2) {
+      const float f = 1.f / sqrtf(wave_sum(ss) / (float)d + g.eps);
+      const float temp = kind == 0 && g.temp_every > 0
+                             ? 1.f + g.temp_coef * logf((float)((pos + 1) / g.temp_every) + 1.f) : 1.f;
+#pragma unroll
+      for (int k = 0; k < NC; ++k) val[k] = val[k] * f * norm[k] * temp;
+    }
+    if (kind == 0) {
+      float* q = g.q_out + (size_t)r * g.H * g.dk + unit * d;
+#pragma unroll
+      for (int k = 0; k < NC; ++k)
+        if (lane + 64 * k < d) q[lane + 64 * k] = val[k];
+    } else {
+      const int pg = g.block_tables[(size_t)slot * g.max_blocks + pos / g.page];
+      T* dst = (T*)(kind == 1 ? g.k_cache : g.v_cache) + (((size_t)pg * g.G + unit) * g.page + pos % g.page) * d;
+#pragma unroll
+      for (int k = 0; k < NC; ++k)
+        if (lane + 64 * k < d) st_f(dst + lane + 64 * k, val[k]);
+    }
+  }
 }
 
 // ------------------------------------------------------------------ matrix memory with exponential gates
@@ -645,10 +802,104 @@ __global__ __launch_bounds__(256) void mlstm_post_kernel(MlstmPostArgs g) {
   if (lane == 0 && (r + 1 == (int)gridDim.x || g.row_slot[r + 1] != slot)) g.m[(size_t)slot * g.H + h] = m;
 }
 
+// Scan and read-out of rows that are alone in their entries: a workgroup per (row, head), so that the
+// head's norm needs no second launch.  A thread owns a strip of 16 key channels of one value column
+// (CT columns at a time); the same sums in the same order as mlstm_scan_kernel.
+template <typename T>
+__global__ __launch_bounds__(1024) void mlstm_step_kernel(MlstmArgs a, MlstmPostArgs g, const int32_t* __restrict__ row_pos,
+                                                          int CT, int NS) {
+  extern __shared__ float lds[];
+  __shared__ float red[48];
+  const int r = blockIdx.y, h = blockIdx.x, H = a.H, dk = a.dk, dv = a.dv, tid = threadIdx.x;
+  if (h == H) {
+    poly_norm_row<T>(g.z + (size_t)r * g.ldz, (const T*)g.z_bias, g.coef, g.eps, g.F,
+                     g.act ? g.act + (size_t)r * g.ldy : nullptr, g.act_b ? g.act_b + (size_t)r * g.ldy : nullptr, red);
+    return;
+  }
+  float* qs = lds;                 // [NS*16]
+  float* ks = qs + NS * kStrip;
+  float* part = ks + NS * kStrip;  // [NS][CT]
+  float* o = part + NS * CT;       // [dv]
+  const int slot = g.row_slot[r], pos = row_pos[r], c = tid % CT, s = tid / CT, r0 = s * kStrip;
+  const size_t at = (size_t)slot * H + h, row = (size_t)r * a.ld;
+  const bool kept = pos > 0;
+  float* st = a.S + at * dk * dv;
+  float S[kStrip];
+  auto load = [&](int col) {       // (clamped addresses; what lies outside is zeroed or dropped)
+    const int cc = col < dv ? col : dv - 1;
+#pragma unroll
+    for (int i = 0; i < kStrip; ++i) {
+      const int rr = r0 + i < dk ? r0 + i : dk - 1;
+      const float v = st[(size_t)rr * dv + cc];
+      S[i] = kept && r0 + i < dk ? v : 0.f;
+    }
+  };
+  load(c);
+  float n_old = 0.f;
+  if (tid < NS * kStrip) {
+    const int cc = tid < dk ? tid : dk - 1;
+    const float q = a.q[row + (size_t)h * dk + cc] * a.q_scale, k = a.k[row + (size_t)h * dk + cc];
+    const float n = a.nrm[at * dk + cc];
+    qs[tid] = tid < dk ? q : 0.f;
+    ks[tid] = tid < dk ? k : 0.f;
+    n_old = kept ? n : 0.f;
+  }
+  const float zi = a.zi[row + h] + a.bi[h], zf = a.zf[row + h] + a.bf[h];
+  const float li = a.cap * tanhf(zi / a.cap), lf = log_sigmoid_f(a.cap * tanhf(zf / a.cap));
+  const float m0 = kept ? a.m[at] : 0.f, m = fmaxf(lf + m0, li);
+  const float d = expf(lf + m0 - m), add = expf(li - m);
+  __syncthreads();
+  float nq = 0.f;
+  if (tid < dk) {
+    const float n = fmaf(d, n_old, ks[tid] * add);
+    a.nrm[at * dk + tid] = n;
+    nq = n * qs[tid];
+  }
+  if (tid == 0) a.m[at] = m;
+  for (int c0 = 0; c0 < dv; c0 += CT) {
+    const int col = c0 + c;
+    if (c0 > 0) load(col);
+    if (s < NS) {
+      const float av = add * a.v[row + (size_t)h * dv + (col < dv ? col : dv - 1)];
+      float acc = 0.f;
+#pragma unroll
+      for (int i = 0; i < kStrip; ++i) {
+        S[i] = fmaf(d, S[i], ks[r0 + i] * av);
+        acc = fmaf(S[i], qs[r0 + i], acc);
+      }
+      part[s * CT + c] = acc;
+      if (col < dv) {
+#pragma unroll
+        for (int i = 0; i < kStrip; ++i)
+          if (r0 + i < dk) st[(size_t)(r0 + i) * dv + col] = S[i];
+      }
+    }
+    __syncthreads();
+    if (tid < CT && c0 + tid < dv) {
+      float sum = part[tid];
+      for (int i = 1; i < NS; ++i) sum += part[i * CT + tid];
+      o[c0 + tid] = sum;
+    }
+    __syncthreads();
+  }
+  nq = block_sum(nq, red);
+  const float inv = 1.f / (fmaxf(fabsf(nq), expf(-m)) + 1e-6f);
+  float ss = 0.f;
+  for (int i = tid; i < dv; i += blockDim.x) ss = fmaf(o[i] * inv, o[i] * inv, ss);
+  const float rstd = 1.f / sqrtf(block_sum(ss, red) / (float)dv + g.eps);
+  for (int i = tid; i < dv; i += blockDim.x) {
+    const int ch = h * dv + i;
+    const float y = o[i] * inv * rstd * ld_f((const T*)g.w + ch) * sigmoid_f(g.gate[(size_t)r * g.ldg + ch]);
+    if (g.y) g.y[(size_t)r * g.ldy + ch] = y;
+    if (g.y_b) g.y_b[(size_t)r * g.ldy + ch] = (bf16_t)y;
+  }
+}
+
 // ------------------------------------------------------------------ window attention on the matrix cores
-// Many rows over bf16 caches.  A workgroup of four waves takes one kv head and a tile of query rows
-// of one portion: wh query heads of the kv head x (4 / wh) groups of 16 rows, a wave each, which
-// share the tiles of 64 keys that are staged in LDS (keys as rows, values transposed).  A wave
+// Many rows over bf16 caches.  A workgroup takes one kv head and a tile of query rows of one portion:
+// wh query heads of the kv head x (4 / wh) groups of 16 rows, a pair of waves each, which share the
+// tiles of keys that are staged in LDS (keys as rows, values transposed).  Two tiles of 64 keys are
+// staged at a time; the waves of a pair take one each and put their sums together at the end.  A wave
 // computes S^T = K Q^T, so that a query's scores sit in one column of the accumulator and are, as
 // they are, the right operand of O^T = V^T P^T (the keys of an MFMA step in the order the
 // accumulators hold them).  Queries and weights enter as the sum of two bf16 parts, keys and values
@@ -686,13 +937,21 @@ __device__ __forceinline__ bool nth_group(const int32_t* entries, int n_entries,
   return i < n_entries;
 }
 
+template <int KS, int VT>
+constexpr size_t tiled_attn_lds() {   // (the tiles' place also takes one wave group's results)
+  const size_t tiles = 2 * ((size_t)kTileKeys * (32 * KS + 8) + (size_t)16 * VT * (kTileKeys + 4)) * sizeof(bf16_t);
+  const size_t sums = (size_t)4 * SD_WAVE * (4 * VT + 2) * sizeof(float);
+  return (tiles > sums ? tiles : sums) + 8 * 80 * sizeof(float);
+}
 template <int KS, int VT>   // heads of up to 32 * KS key and 16 * VT value channels
-__global__ __launch_bounds__(256) void tiled_window_attn_kernel(TiledAttnArgs g) {
-  constexpr int KLD = 32 * KS + 8, VLD = kTileKeys + 4, NV = VT / 4;
-  __shared__ __attribute__((aligned(16))) bf16_t ks[kTileKeys * KLD];
-  __shared__ __attribute__((aligned(16))) bf16_t vs[16 * VT * VLD];
-  __shared__ float away[4][80];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, quad = lane >> 4;
+__global__ __launch_bounds__(512) void tiled_window_attn_kernel(TiledAttnArgs g) {
+  constexpr int KLD = 32 * KS + 8, VLD = kTileKeys + 4, NV = VT / 4, kStage = 2 * kTileKeys, nthr = 512;
+  extern __shared__ __attribute__((aligned(16))) char attn_lds[];
+  bf16_t* ks = reinterpret_cast<bf16_t*>(attn_lds);            // [2][64][KLD]
+  bf16_t* vs = ks + 2 * kTileKeys * KLD;                       // [2][16 * VT][VLD]
+  float* sums = reinterpret_cast<float*>(attn_lds);            // [4 * VT + 2][4][64], at the end
+  float* away = reinterpret_cast<float*>(attn_lds + tiled_attn_lds<KS, VT>() - 8 * 80 * sizeof(float)) + 80 * (threadIdx.x >> 6);
+  const int tid = threadIdx.x, group = tid >> 8, wave = (tid >> 6) & 3, lane = tid & 63, col = lane & 15, quad = lane >> 4;
   const int kvh = blockIdx.y, hgroup = blockIdx.z, qh = g.H / g.G, dk = g.dk, dv = g.dv;
   const int n_sub = 4 / g.wh, tq = 16 * n_sub;
   int e, first;
@@ -734,33 +993,33 @@ __global__ __launch_bounds__(256) void tiled_window_attn_kernel(TiledAttnArgs g)
       }
     }
   }
-  // a thread's pieces of a key tile: KS of 8 channels; of a value tile: NV of 8 channels of two keys
+  // a thread's pieces of the staged keys: KS of 8 channels; of the values: NV of 8 channels of two keys
   const u32x4 zero = {0, 0, 0, 0};
   u32x4 kr[KS], vr[NV][2];
   int kpg[KS], vpg[NV];
-  auto pages = [&](int b0) {     // the pages of the tile at b0 (clamped: rows behind `last` are zeroed)
+  auto pages = [&](int b0) {     // the pages of the keys from b0 on (clamped: rows behind `last` are zeroed)
 #pragma unroll
     for (int i = 0; i < KS; ++i) {
-      const int j = b0 + (tid + 256 * i) / (4 * KS);
+      const int j = b0 + (tid + nthr * i) / (4 * KS);
       kpg[i] = tbl[(j < last ? j : last) / kPage];
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int j = b0 + 2 * ((tid + 256 * i) / (2 * VT));
+      const int j = b0 + 2 * ((tid + nthr * i) / (2 * VT));
       vpg[i] = tbl[(j < last ? j : last) / kPage];
     }
   };
   auto fetch = [&](int b0) {
 #pragma unroll
     for (int i = 0; i < KS; ++i) {
-      const int idx = tid + 256 * i, j = b0 + idx / (4 * KS), c = 8 * (idx % (4 * KS));
+      const int idx = tid + nthr * i, j = b0 + idx / (4 * KS), c = 8 * (idx % (4 * KS));
       kr[i] = zero;
       if (j <= last && c < dk)
         kr[i] = *reinterpret_cast<const u32x4*>(g.k_cache + (((size_t)kpg[i] * g.G + kvh) * kPage + j % kPage) * dk + c);
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int idx = tid + 256 * i, j = b0 + 2 * (idx / (2 * VT)), c = 8 * (idx % (2 * VT));
+      const int idx = tid + nthr * i, j = b0 + 2 * (idx / (2 * VT)), c = 8 * (idx % (2 * VT));
       const bf16_t* v = g.v_cache + (((size_t)vpg[i] * g.G + kvh) * kPage + j % kPage) * dv + c;
       vr[i][0] = vr[i][1] = zero;
       if (j <= last && c < dv) vr[i][0] = *reinterpret_cast<const u32x4*>(v);
@@ -775,39 +1034,43 @@ __global__ __launch_bounds__(256) void tiled_window_attn_kernel(TiledAttnArgs g)
 
   pages(base);
   fetch(base);
-  pages(base + kTileKeys);
-  for (; base <= last; base += kTileKeys) {
+  pages(base + kStage);
+  for (; base <= last; base += kStage) {
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < KS; ++i) {
-      const int idx = tid + 256 * i;
+      const int idx = tid + nthr * i;
       *reinterpret_cast<u32x4*>(ks + (idx / (4 * KS)) * KLD + 8 * (idx % (4 * KS))) = kr[i];
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int idx = tid + 256 * i, c = 8 * (idx % (2 * VT)), j = 2 * (idx / (2 * VT));
+      const int idx = tid + nthr * i, c = 8 * (idx % (2 * VT)), j = 2 * (idx / (2 * VT));
       const bf16x8 a = __builtin_bit_cast(bf16x8, vr[i][0]), b = __builtin_bit_cast(bf16x8, vr[i][1]);
+      bf16_t* dst = vs + (j / kTileKeys) * 16 * VT * VLD + c * VLD + j % kTileKeys;
 #pragma unroll
-      for (int u = 0; u < 8; ++u) *reinterpret_cast<bf16x2*>(vs + (c + u) * VLD + j) = bf16x2{a[u], b[u]};
+      for (int u = 0; u < 8; ++u) *reinterpret_cast<bf16x2*>(dst + u * VLD) = bf16x2{a[u], b[u]};
     }
-    if (g.dist1) {   // entry n: distance pos0 + sub - base - 63 + n
-      const int d0 = pos0 + sub - base - (kTileKeys - 1);
-      away[wave][lane] = r1 * log1pf(r2 * (float)(d0 + lane > 0 ? d0 + lane : 0));
-      if (lane < 16) away[wave][64 + lane] = r1 * log1pf(r2 * (float)(d0 + 64 + lane > 0 ? d0 + 64 + lane : 0));
+    const int gbase = base + group * kTileKeys;              // this wave's tile
+    if (g.dist1) {   // entry n: distance pos0 + sub - gbase - 63 + n
+      const int d0 = pos0 + sub - gbase - (kTileKeys - 1);
+      away[lane] = r1 * log1pf(r2 * (float)(d0 + lane > 0 ? d0 + lane : 0));
+      if (lane < 16) away[64 + lane] = r1 * log1pf(r2 * (float)(d0 + 64 + lane > 0 ? d0 + 64 + lane : 0));
     }
     __syncthreads();
-    if (base + kTileKeys <= last) {
-      fetch(base + kTileKeys);
-      pages(base + 2 * kTileKeys);
+    if (base + kStage <= last) {
+      fetch(base + kStage);
+      pages(base + 2 * kStage);
     }
-    if (!works || base > pos0 + sub + n_rows - 1) continue;   // (keys behind this wave's last query)
+    if (!works || gbase > pos0 + sub + n_rows - 1) continue;   // (keys behind this wave's last query)
+    const bf16_t* kt = ks + group * kTileKeys * KLD;
+    const bf16_t* vt = vs + group * 16 * VT * VLD;
     f32x4 sc[4];
 #pragma unroll
     for (int t = 0; t < 4; ++t) {
       sc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int s = 0; s < KS; ++s) {
-        const bf16x8 a = *reinterpret_cast<const bf16x8*>(ks + (16 * t + col) * KLD + 32 * s + 8 * quad);
+        const bf16x8 a = *reinterpret_cast<const bf16x8*>(kt + (16 * t + col) * KLD + 32 * s + 8 * quad);
         sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qa[s], sc[t], 0, 0, 0);
         sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qb[s], sc[t], 0, 0, 0);
       }
@@ -817,11 +1080,11 @@ __global__ __launch_bounds__(256) void tiled_window_attn_kernel(TiledAttnArgs g)
     for (int t = 0; t < 4; ++t)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int kk = 16 * t + 4 * quad + i, d = p - (base + kk);
+        const int kk = 16 * t + 4 * quad + i, d = p - (gbase + kk);
         float v = sc[t][i];
         // cap tanh(v / cap) = cap - 2 cap / (e^(2 v / cap) + 1)
         if (cap > 0.f) v = fmaf(-2.f * cap, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(v * cap_in) + 1.f), cap);
-        if (g.dist1) v -= away[wave][col + kTileKeys - 1 - kk];
+        if (g.dist1) v -= away[col + kTileKeys - 1 - kk];
         v = d >= 0 && d < g.window ? v : -INFINITY;
         sc[t][i] = v;
         mx = fmaxf(mx, v);
@@ -852,7 +1115,7 @@ __global__ __launch_bounds__(256) void tiled_window_attn_kernel(TiledAttnArgs g)
     for (int t = 0; t < VT; ++t)
 #pragma unroll
       for (int u = 0; u < 2; ++u) {
-        const bf16_t* vrow = vs + (16 * t + col) * VLD + 32 * u + 4 * quad;
+        const bf16_t* vrow = vt + (16 * t + col) * VLD + 32 * u + 4 * quad;
         const bf16x4 a0 = *reinterpret_cast<const bf16x4*>(vrow), a1 = *reinterpret_cast<const bf16x4*>(vrow + 16);
         const bf16x8 a = {a0[0], a0[1], a0[2], a0[3], a1[0], a1[1], a1[2], a1[3]};
         o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pa[u], o[t], 0, 0, 0);
@@ -861,8 +1124,27 @@ __global__ __launch_bounds__(256) void tiled_window_attn_kernel(TiledAttnArgs g)
   }
   l_run += __shfl_xor(l_run, 16, SD_WAVE);
   l_run += __shfl_xor(l_run, 32, SD_WAVE);
-  if (!works || col >= n_rows) return;
-  const float inv = 1.f / l_run;
+  // the pair's sums: the second wave leaves its own, the first adds them
+  __syncthreads();
+  if (group == 1) {
+    float* mine = sums + wave * SD_WAVE + lane;
+#pragma unroll
+    for (int t = 0; t < VT; ++t)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) mine[(4 * t + i) * 4 * SD_WAVE] = o[t][i];
+    mine[4 * VT * 4 * SD_WAVE] = m_run;
+    mine[(4 * VT + 1) * 4 * SD_WAVE] = l_run;
+  }
+  __syncthreads();
+  if (group == 1 || !works || col >= n_rows) return;
+  const float* other = sums + wave * SD_WAVE + lane;
+  const float m2 = other[4 * VT * 4 * SD_WAVE], m_all = fmaxf(m_run, m2);   // (one of them saw the query's own key)
+  const float f1 = __builtin_amdgcn_exp2f((m_run - m_all) * kLog2e), f2 = __builtin_amdgcn_exp2f((m2 - m_all) * kLog2e);
+#pragma unroll
+  for (int t = 0; t < VT; ++t)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[t][i] = fmaf(o[t][i], f1, other[(4 * t + i) * 4 * SD_WAVE] * f2);
+  const float inv = 1.f / fmaf(l_run, f1, other[(4 * VT + 1) * 4 * SD_WAVE] * f2);
   const size_t at = (size_t)(row0 + sub + col) * g.ldo + (size_t)h * dv;
   const bool quads = g.ldo % 4 == 0;
 #pragma unroll
@@ -912,19 +1194,50 @@ typedef __attribute__((ext_vector_type(16))) float acc32_t;
 __device__ __forceinline__ int acc_row(int i, int half) { return 8 * (i >> 2) + 4 * half + (i & 3); }
 
 constexpr int kChunkCols = 128;   // value columns per workgroup
+// 64 rows of up to COLS columns on their way from memory to LDS, V columns a piece: all of a thread's
+// pieces are asked for at once (on addresses clamped into the valid part), then stored.
+template <int COLS, int V>
+struct ChunkRows {
+  static constexpr int N = kChunk * COLS / V / 256;
+  Pack<V> v[N];
+  __device__ __forceinline__ void load(const float* src, int64_t ld, int rows, int cols) {
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+      const int idx = threadIdx.x + 256 * u, t = idx / (COLS / V), c = idx % (COLS / V) * V;
+      v[u] = ld_pack<V>(src + (size_t)(t < rows ? t : rows - 1) * ld + (c < cols ? c : cols - V));
+    }
+  }
+  // times wt[row] (or f where wt is nullptr)
+  __device__ __forceinline__ void store(float* dst, int ldd, int rows, int cols, const float* wt, float f) {
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+      const int idx = threadIdx.x + 256 * u, t = idx / (COLS / V), c = idx % (COLS / V) * V;
+      const float w = t < rows && c < cols ? (wt ? wt[t] : f) : 0.f;
+#pragma unroll
+      for (int e = 0; e < V; ++e) dst[t * ldd + c + e] = w == 0.f ? 0.f : v[u].v[e] * w;
+    }
+  }
+};
+
+template <int DKP, int V>   // keys of up to DKP channels
 __global__ __launch_bounds__(256) void mlstm_chunk_sums_kernel(MlstmChunkArgs g) {
   extern __shared__ float lds[];
   const MlstmArgs& a = g.a;
-  const int dk = a.dk, dv = a.dv, H = a.H, nkt = (dk + 31) / 32, dkp = 32 * nkt;
-  float* ks = lds;                   // [64][dkp], times the token's weight
-  float* vs = ks + kChunk * dkp;     // [64][128]
+  const int dk = a.dk, dv = a.dv, H = a.H;
+  constexpr int nkt = DKP / 32;
+  float* ks = lds;                   // [64][DKP], times the token's weight
+  float* vs = ks + kChunk * DKP;     // [64][128]
   float* wt = vs + kChunk * kChunkCols;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l31 = lane & 31, half = lane >> 5;
-  const int h = blockIdx.y, c0 = blockIdx.z * kChunkCols;
+  const int h = blockIdx.y, c0 = blockIdx.z * kChunkCols, cols = dv - c0 < kChunkCols ? dv - c0 : kChunkCols;
   int e, first;
   if (!nth_group(a.entries, g.n_entries, kChunk, blockIdx.x, &e, &first)) return;
   const int row0 = a.entries[4 * e + 1] + first, left = a.entries[4 * e + 2] - first, nt = left < kChunk ? left : kChunk;
   const size_t at = (size_t)blockIdx.x * H + h;
+  ChunkRows<DKP, V> kr;
+  ChunkRows<kChunkCols, V> vr;
+  kr.load(a.k + (size_t)row0 * a.ld + (size_t)h * dk, a.ld, nt, dk);
+  vr.load(a.v + (size_t)row0 * a.ld + (size_t)h * dv + c0, a.ld, nt, cols);
   if (wave == 0) {
     float li, lf;
     chunk_gates(a, row0 + (lane < nt ? lane : nt - 1), h, lane < nt, &li, &lf);
@@ -942,46 +1255,22 @@ __global__ __launch_bounds__(256) void mlstm_chunk_sums_kernel(MlstmChunkArgs g)
       g.sc[at * 4 + 1] = mu;
     }
   }
-  // (four rows of k and of v in flight per thread and turn; loads on clamped addresses)
+  vr.store(vs, kChunkCols, nt, cols, nullptr, 1.f);
   __syncthreads();
-  for (int i = tid; i < kChunk * dkp; i += 256 * 8) {
-    float v[8];
-#pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = i + 256 * u, t = idx / dkp < nt ? idx / dkp : nt - 1, c = idx % dkp;
-      v[u] = a.k[(size_t)(row0 + t) * a.ld + (size_t)h * dk + (c < dk ? c : dk - 1)];
-    }
-#pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = i + 256 * u;
-      if (idx < kChunk * dkp) ks[idx] = idx / dkp < nt && idx % dkp < dk ? v[u] * wt[idx / dkp] : 0.f;
-    }
-  }
-  for (int i = tid; i < kChunk * kChunkCols; i += 256 * 8) {
-    float v[8];
-#pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = i + 256 * u, t = idx / kChunkCols < nt ? idx / kChunkCols : nt - 1, c = c0 + idx % kChunkCols;
-      v[u] = a.v[(size_t)(row0 + t) * a.ld + (size_t)h * dv + (c < dv ? c : dv - 1)];
-    }
-#pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = i + 256 * u;
-      vs[idx] = idx / kChunkCols < nt && c0 + idx % kChunkCols < dv ? v[u] : 0.f;
-    }
-  }
+  kr.store(ks, DKP, nt, dk, wt, 0.f);
   __syncthreads();
-  const int cols = dv - c0 < kChunkCols ? dv - c0 : kChunkCols, nct = (cols + 31) / 32;
+  const int nct = (cols + 31) / 32;
   float* cs = g.cs + at * dk * dv + c0;
   for (int p = wave; p < nkt * nct; p += 4) {
     const int kt = p % nkt, ct = p / nkt;
     acc32_t acc;
 #pragma unroll
     for (int i = 0; i < 16; ++i) acc[i] = 0.f;
-#pragma unroll 8
+    const float* ka = ks + half * DKP + 32 * kt + l31;
+    const float* vb = vs + half * kChunkCols + 32 * ct + l31;
+#pragma unroll
     for (int s = 0; s < kChunk; s += 2)
-      acc = __builtin_amdgcn_mfma_f32_32x32x2f32(ks[(s + half) * dkp + 32 * kt + l31],
-                                                 vs[(s + half) * kChunkCols + 32 * ct + l31], acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_32x32x2f32(ka[s * DKP], vb[s * kChunkCols], acc, 0, 0, 0);
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       const int r = 32 * kt + acc_row(i, half);
@@ -990,7 +1279,8 @@ __global__ __launch_bounds__(256) void mlstm_chunk_sums_kernel(MlstmChunkArgs g)
   }
   if (blockIdx.z == 0 && tid < dk) {
     float n = 0.f;
-    for (int s = 0; s < kChunk; ++s) n += ks[s * dkp + tid];
+#pragma unroll 16
+    for (int s = 0; s < kChunk; ++s) n += ks[s * DKP + tid];
     g.cn[at * dk + tid] = n;
   }
 }
@@ -1037,12 +1327,12 @@ __global__ __launch_bounds__(256) void mlstm_chunk_carry_kernel(MlstmChunkArgs g
   *st = val;
 }
 
-constexpr int kChunkSteps = 64;   // dk <= 128: pairs of key channels
+template <int DKP, int V>
 __global__ __launch_bounds__(256) void mlstm_chunk_reads_kernel(MlstmChunkArgs g) {
   extern __shared__ float lds[];
   const MlstmArgs& a = g.a;
-  const int dk = a.dk, dv = a.dv, H = a.H, dkp = (dk + 31) / 32 * 32, ldk = dkp + 1;
-  constexpr int kLdA = kChunk + 1;
+  const int dk = a.dk, dv = a.dv, H = a.H;
+  constexpr int ldk = DKP + 1, kLdA = kChunk + 1, kSteps = DKP / 2;
   float* qs = lds;                     // [64][ldk]
   float* ks = qs + kChunk * ldk;       // [64][ldk]
   float* vs = ks + kChunk * ldk;       // [64][128]
@@ -1051,27 +1341,29 @@ __global__ __launch_bounds__(256) void mlstm_chunk_reads_kernel(MlstmChunkArgs g
   float* lfs = lis + kChunk;
   float* ms = lfs + kChunk;
   float* carry = ms + kChunk;
-  float* ns = carry + kChunk;          // [dkp]
+  float* ns = carry + kChunk;          // [DKP]
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l31 = lane & 31, half = lane >> 5;
-  const int h = blockIdx.y, c0 = blockIdx.z * kChunkCols;
+  const int h = blockIdx.y, c0 = blockIdx.z * kChunkCols, cols = dv - c0 < kChunkCols ? dv - c0 : kChunkCols;
   int e, first;
   if (!nth_group(a.entries, g.n_entries, kChunk, blockIdx.x, &e, &first)) return;
   const int row0 = a.entries[4 * e + 1] + first, left = a.entries[4 * e + 2] - first, nt = left < kChunk ? left : kChunk;
   const size_t at = (size_t)blockIdx.x * H + h;
-  // the memory at the chunk's start: this wave's 32 columns, rows 2 j + half, asked for first
+  ChunkRows<DKP, V> qr, kr;
+  ChunkRows<kChunkCols, V> vr;
+  qr.load(a.q + (size_t)row0 * a.ld + (size_t)h * dk, a.ld, nt, dk);
+  kr.load(a.k + (size_t)row0 * a.ld + (size_t)h * dk, a.ld, nt, dk);
+  vr.load(a.v + (size_t)row0 * a.ld + (size_t)h * dv + c0, a.ld, nt, cols);
+  // the memory at the chunk's start: this wave's 32 columns, rows 2 j + half
   const int wcol = 32 * wave + l31;
-  const bool col_in = c0 + wcol < dv;
-  float S[kChunkSteps];
+  const bool col_in = wcol < cols;
+  float S[kSteps];
   {
-    const float* s0 = g.cs + at * dk * dv + (col_in ? c0 + wcol : 0);
+    const float* s0 = g.cs + at * dk * dv + c0 + (col_in ? wcol : 0);
 #pragma unroll
-    for (int j = 0; j < kChunkSteps; ++j) {
-      S[j] = 0.f;
-      if (2 * j < dkp) {
-        const int r = 2 * j + half;
-        const float v = s0[(size_t)(r < dk ? r : dk - 1) * dv];
-        S[j] = r < dk && col_in ? v : 0.f;
-      }
+    for (int j = 0; j < kSteps; ++j) {
+      const int r = 2 * j + half;
+      const float v = s0[(size_t)(r < dk ? r : dk - 1) * dv];
+      S[j] = r < dk && col_in ? v : 0.f;
     }
   }
   if (wave == 0) {
@@ -1095,39 +1387,11 @@ __global__ __launch_bounds__(256) void mlstm_chunk_reads_kernel(MlstmChunkArgs g
     carry[lane] = expf(F + m0 - m);
     if (blockIdx.z == 0 && lane < nt) a.m_rows[(size_t)(row0 + lane) * H + h] = m;
   } else {
-    for (int c = tid - 64; c < dkp; c += 192) ns[c] = c < dk ? g.cn[at * dk + c] : 0.f;
+    for (int c = tid - 64; c < DKP; c += 192) ns[c] = c < dk ? g.cn[at * dk + c] : 0.f;
   }
-  for (int i = tid; i < kChunk * dkp; i += 256 * 8) {
-    float vq[8], vk[8];
-#pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = i + 256 * u, t = idx / dkp < nt ? idx / dkp : nt - 1, c = idx % dkp;
-      const size_t from = (size_t)(row0 + t) * a.ld + (size_t)h * dk + (c < dk ? c : dk - 1);
-      vq[u] = a.q[from];
-      vk[u] = a.k[from];
-    }
-#pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = i + 256 * u, t = idx / dkp, c = idx % dkp;
-      if (idx < kChunk * dkp) {
-        qs[t * ldk + c] = t < nt && c < dk ? vq[u] * a.q_scale : 0.f;
-        ks[t * ldk + c] = t < nt && c < dk ? vk[u] : 0.f;
-      }
-    }
-  }
-  for (int i = tid; i < kChunk * kChunkCols; i += 256 * 8) {
-    float v[8];
-#pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = i + 256 * u, t = idx / kChunkCols < nt ? idx / kChunkCols : nt - 1, c = c0 + idx % kChunkCols;
-      v[u] = a.v[(size_t)(row0 + t) * a.ld + (size_t)h * dv + (c < dv ? c : dv - 1)];
-    }
-#pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = i + 256 * u;
-      vs[idx] = idx / kChunkCols < nt && c0 + idx % kChunkCols < dv ? v[u] : 0.f;
-    }
-  }
+  qr.store(qs, ldk, nt, dk, nullptr, a.q_scale);
+  kr.store(ks, ldk, nt, dk, nullptr, 1.f);
+  vr.store(vs, kChunkCols, nt, cols, nullptr, 1.f);
   __syncthreads();
   {
     // the tokens' weights: lane s, sixteen tokens t per wave; D(t, s) is summed from s on, so that a
@@ -1135,9 +1399,11 @@ __global__ __launch_bounds__(256) void mlstm_chunk_reads_kernel(MlstmChunkArgs g
     const float li = lis[lane];
     float d = 0.f;
     const int t0 = 16 * wave;
+#pragma unroll 16
     for (int t = 0; t < t0; ++t) d += t > lane ? lfs[t] : 0.f;
 #pragma unroll
-    for (int t = t0; t < t0 + 16; ++t) {
+    for (int u = 0; u < 16; ++u) {
+      const int t = t0 + u;
       d += t > lane ? lfs[t] : 0.f;
       as[t * kLdA + lane] = t >= lane ? expf(d + li - ms[t]) : 0.f;
     }
@@ -1150,8 +1416,8 @@ __global__ __launch_bounds__(256) void mlstm_chunk_reads_kernel(MlstmChunkArgs g
     const float* qa = qs + (32 * tt + l31) * ldk + half;
     const float* kb = ks + (32 * ss + l31) * ldk + half;
     if (tt >= ss) {
-#pragma unroll 8
-      for (int c = 0; c < dkp; c += 2) acc[0] = __builtin_amdgcn_mfma_f32_32x32x2f32(qa[c], kb[c], acc[0], 0, 0, 0);
+#pragma unroll
+      for (int c = 0; c < DKP; c += 2) acc[0] = __builtin_amdgcn_mfma_f32_32x32x2f32(qa[c], kb[c], acc[0], 0, 0, 0);
     }
     __syncthreads();
 #pragma unroll
@@ -1162,25 +1428,26 @@ __global__ __launch_bounds__(256) void mlstm_chunk_reads_kernel(MlstmChunkArgs g
 #pragma unroll
     for (int i = 0; i < 16; ++i) acc[u][i] = 0.f;
 #pragma unroll
-  for (int j = 0; j < kChunkSteps; ++j) {
-    if (2 * j < dkp) {
+  for (int j = 0; j < kSteps; ++j)
 #pragma unroll
-      for (int u = 0; u < 2; ++u)
-        acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(qs[(32 * u + l31) * ldk + 2 * j + half], S[j], acc[u], 0, 0, 0);
-    }
-  }
+    for (int u = 0; u < 2; ++u)
+      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(qs[(32 * u + l31) * ldk + 2 * j + half], S[j], acc[u], 0, 0, 0);
 #pragma unroll
   for (int u = 0; u < 2; ++u)
 #pragma unroll
     for (int i = 0; i < 16; ++i) acc[u][i] *= carry[32 * u + acc_row(i, half)];
   __syncthreads();
+  // (the first 32 tokens see nothing of the later ones)
 #pragma unroll
-  for (int s = 0; s < kChunk; s += 2) {
+  for (int s = 0; s < 32; s += 2) {
     const float b = vs[(s + half) * kChunkCols + wcol];
-#pragma unroll
-    for (int u = 0; u < 2; ++u)
-      if (s < 32 * (u + 1)) acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(as[(32 * u + l31) * kLdA + s + half], b, acc[u], 0, 0, 0);
+    acc[0] = __builtin_amdgcn_mfma_f32_32x32x2f32(as[l31 * kLdA + s + half], b, acc[0], 0, 0, 0);
+    acc[1] = __builtin_amdgcn_mfma_f32_32x32x2f32(as[(32 + l31) * kLdA + s + half], b, acc[1], 0, 0, 0);
   }
+#pragma unroll
+  for (int s = 32; s < 64; s += 2)
+    acc[1] = __builtin_amdgcn_mfma_f32_32x32x2f32(as[(32 + l31) * kLdA + s + half], vs[(s + half) * kChunkCols + wcol], acc[1],
+                                                  0, 0, 0);
   if (col_in) {
 #pragma unroll
     for (int u = 0; u < 2; ++u)
@@ -1193,7 +1460,7 @@ __global__ __launch_bounds__(256) void mlstm_chunk_reads_kernel(MlstmChunkArgs g
   if (blockIdx.z == 0) {   // n . q, four threads a token
     const int t = tid >> 2, part = tid & 3;
     float n = 0.f, o = 0.f;
-    for (int c = part; c < dkp; c += 4) n = fmaf(qs[t * ldk + c], ns[c], n);
+    for (int c = part; c < DKP; c += 4) n = fmaf(qs[t * ldk + c], ns[c], n);
     for (int s = part; s < kChunk; s += 4) o += as[t * kLdA + s];
     n = fmaf(n, carry[t], o);
     n += __shfl_xor(n, 1, SD_WAVE);
@@ -1202,9 +1469,27 @@ __global__ __launch_bounds__(256) void mlstm_chunk_reads_kernel(MlstmChunkArgs g
   }
 }
 
-inline size_t chunk_reads_lds(int dk) {
-  const size_t dkp = (dk + 31) / 32 * 32;
-  return sizeof(float) * (2 * kChunk * (dkp + 1) + (size_t)kChunk * kChunkCols + kChunk * (kChunk + 1) + 4 * kChunk + dkp);
+template <int DKP, int V>
+hipError_t launch_chunks(const MlstmChunkArgs& c, size_t nc, hipStream_t st) {
+  static std::once_flag once;
+  static hipError_t err = hipSuccess;
+  std::call_once(once, [] {
+    err = hipFuncSetAttribute(reinterpret_cast<const void*>(mlstm_chunk_sums_kernel<DKP, V>),
+                              hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    if (err == hipSuccess)
+      err = hipFuncSetAttribute(reinterpret_cast<const void*>(mlstm_chunk_reads_kernel<DKP, V>),
+                                hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+  });
+  if (err != hipSuccess) return err;
+  const int dk = c.a.dk, dv = c.a.dv, H = c.a.H;
+  const dim3 grid((unsigned)nc, H, (dv + kChunkCols - 1) / kChunkCols);
+  const size_t lds1 = sizeof(float) * ((size_t)kChunk * DKP + (size_t)kChunk * kChunkCols + kChunk);
+  const size_t lds2 = sizeof(float) * (2 * kChunk * (DKP + 1) + (size_t)kChunk * kChunkCols + kChunk * (kChunk + 1) +
+                                       4 * kChunk + DKP);
+  mlstm_chunk_sums_kernel<DKP, V><<<grid, 256, lds1, st>>>(c);
+  mlstm_chunk_carry_kernel<<<dim3((dk * dv + dk + 255) / 256, H, c.n_entries), 256, 0, st>>>(c);
+  mlstm_chunk_reads_kernel<DKP, V><<<grid, 256, lds2, st>>>(c);
+  return hipGetLastError();
 }
 // chunks that n_entries portions of n_rows rows in all may have
 inline size_t max_chunks(int n_rows, int n_entries) { return (size_t)n_rows / kChunk + n_entries; }
@@ -1266,8 +1551,8 @@ extern "C" int sd_conv_add_rows(const float* x, int64_t ldx, const void* w, int 
              SD_ERR_INVALID, "sd_conv_add_rows: bad argument");
   hipStream_t st = (hipStream_t)stream;
   const bool quad = C % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0;
-  dim3 grid(n_rows, ((quad ? C / 4 : C) + 255) / 256);
-#define SD_GO(T, V) conv_add_rows_kernel<T, V><<<grid, 256, 0, st>>>(x, ldx, (const T*)w, conv_state, row_pos, row_slot, out, (bf16_t*)out_bf16, ldo, C, taps)
+  dim3 grid((n_rows + kRowBlock - 1) / kRowBlock, ((quad ? C / 4 : C) + 255) / 256);
+#define SD_GO(T, V) conv_add_rows_kernel<T, V><<<grid, 256, 0, st>>>(x, ldx, (const T*)w, conv_state, row_pos, row_slot, out, (bf16_t*)out_bf16, ldo, n_rows, C, taps)
   if (w_f32) { if (quad) SD_GO(float, 4); else SD_GO(float, 1); }
   else { if (quad) SD_GO(bf16_t, 4); else SD_GO(bf16_t, 1); }
 #undef SD_GO
@@ -1316,8 +1601,29 @@ extern "C" int sd_conv_attn_prep(const float* proj, int64_t ld, const void* bias
     g.z = act->z; g.ldz = act->ldz; g.z_bias = act->bias; g.coef = act->coef; g.act = act->out;
     g.act_b = (bf16_t*)act->out_bf16; g.ldact = act->ldo; g.F = act->n;
   }
-  dim3 grid(n_rows, g.q_wgs + (shared ? 0 : 2 * g.kv_wgs) + (act ? 1 : 0));
   hipStream_t st = (hipStream_t)stream;
+  const int units = g.q_wgs + (shared ? 0 : 2 * g.kv_wgs);
+  if (!g.single && n_rows > 2 * kRowBlock && taps <= kRowTaps) {
+    if (act)
+      if (const int rc = sd_poly_norm_rows(act->z, act->ldz, act->bias, w_f32, act->coef, eps, act->out, act->out_bf16,
+                                           act->ldo, n_rows, act->n, stream))
+        return rc;
+    const dim3 gb((n_rows + kRowBlock - 1) / kRowBlock, units);
+    const int d = dk > dv ? dk : dv;
+#define SD_GO(T)                                                              \
+  do {                                                                        \
+    if (d <= 64) conv_prep_block_kernel<T, 1><<<gb, 256, 0, st>>>(g, n_rows);        \
+    else if (d <= 128) conv_prep_block_kernel<T, 2><<<gb, 256, 0, st>>>(g, n_rows);  \
+    else if (d <= 256) conv_prep_block_kernel<T, 4><<<gb, 256, 0, st>>>(g, n_rows);  \
+    else conv_prep_block_kernel<T, 8><<<gb, 256, 0, st>>>(g, n_rows);                \
+  } while (0)
+    if (w_f32) SD_GO(float);
+    else SD_GO(bf16_t);
+#undef SD_GO
+    SD_CHECK_LAUNCH("sd_conv_attn_prep");
+    return sd_conv_tail(proj, ld, bias, w_f32, conv_state, entries, n_entries, g.C, taps, stream);
+  }
+  dim3 grid(n_rows, units + (act ? 1 : 0));
   if (w_f32) conv_prep_kernel<float><<<grid, 256, 0, st>>>(g);
   else conv_prep_kernel<bf16_t><<<grid, 256, 0, st>>>(g);
   SD_CHECK_LAUNCH("sd_conv_attn_prep");
@@ -1344,28 +1650,17 @@ extern "C" int sd_mlstm_scan(const float* q, const float* k, const float* v, con
   MlstmArgs g{q, k, v, zi, zf, ld, bi, bf, cap, q_scale, S, n_state, const_cast<float*>(m_state), entries, num, m_rows, H, dk, dv};
   const size_t need = sd_mlstm_scratch_bytes(n_rows, n_entries, H, dk, dv);
   if (need > 0 && scratch && scratch_bytes >= need && sd_aligned16(scratch)) {
-    static std::once_flag once;
-    static hipError_t err = hipSuccess;
-    std::call_once(once, [] {
-      err = hipFuncSetAttribute(reinterpret_cast<const void*>(mlstm_chunk_sums_kernel),
-                                hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-      if (err == hipSuccess)
-        err = hipFuncSetAttribute(reinterpret_cast<const void*>(mlstm_chunk_reads_kernel),
-                                  hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-    });
-    SD_REQUIRE(err == hipSuccess, SD_ERR_HIP, "sd_mlstm_scan: hipFuncSetAttribute failed: %s", hipGetErrorString(err));
     const size_t nc = max_chunks(n_rows, n_entries);
     MlstmChunkArgs c{g, n_entries, (float*)scratch, nullptr, nullptr};
     c.cn = c.cs + nc * H * dk * dv;
     c.sc = c.cn + nc * H * dk;
-    const int dkp = (dk + 31) / 32 * 32, zs = (dv + kChunkCols - 1) / kChunkCols;
-    const size_t lds = sizeof(float) * ((size_t)kChunk * dkp + (size_t)kChunk * kChunkCols + kChunk);
-    mlstm_chunk_sums_kernel<<<dim3((unsigned)nc, H, zs), 256, lds, st>>>(c);
-    SD_CHECK_LAUNCH("sd_mlstm_scan (chunk sums)");
-    mlstm_chunk_carry_kernel<<<dim3((dk * dv + dk + 255) / 256, H, n_entries), 256, 0, st>>>(c);
-    SD_CHECK_LAUNCH("sd_mlstm_scan (carry)");
-    mlstm_chunk_reads_kernel<<<dim3((unsigned)nc, H, zs), 256, chunk_reads_lds(dk), st>>>(c);
-    SD_CHECK_LAUNCH("sd_mlstm_scan (reads)");
+    // (four columns a piece where every row's pieces are 16-byte aligned)
+    const bool quad = ld % 4 == 0 && dk % 4 == 0 && dv % 4 == 0 && sd_aligned16(q) && sd_aligned16(k) && sd_aligned16(v);
+    hipError_t err;
+    if (dk <= 32) err = quad ? launch_chunks<32, 4>(c, nc, st) : launch_chunks<32, 1>(c, nc, st);
+    else if (dk <= 64) err = quad ? launch_chunks<64, 4>(c, nc, st) : launch_chunks<64, 1>(c, nc, st);
+    else err = quad ? launch_chunks<128, 4>(c, nc, st) : launch_chunks<128, 1>(c, nc, st);
+    SD_REQUIRE(err == hipSuccess, SD_ERR_HIP, "sd_mlstm_scan: launch failed: %s", hipGetErrorString(err));
     return SD_OK;
   }
   const int NS = (dk + kStrip - 1) / kStrip, cols = dv + 1;
@@ -1401,11 +1696,58 @@ int sd_tiled_window_attention_(const float* q, int64_t ldq, const void* k_cache,
   const int tq = 16 * (4 / g.wh);
   dim3 grid(n_rows / tq + n_entries, G, g.n_hgroups);
   hipStream_t st = (hipStream_t)stream;
-  if (dk <= 64 && dv <= 64) tiled_window_attn_kernel<2, 4><<<grid, 256, 0, st>>>(g);
-  else if (dk <= 64) tiled_window_attn_kernel<2, 8><<<grid, 256, 0, st>>>(g);
-  else if (dv <= 64) tiled_window_attn_kernel<4, 4><<<grid, 256, 0, st>>>(g);
-  else tiled_window_attn_kernel<4, 8><<<grid, 256, 0, st>>>(g);
+#define SD_GO(KS, VT)                                                                                                    \
+  do {                                                                                                                   \
+    static std::once_flag once;                                                                                          \
+    static hipError_t err = hipSuccess;                                                                                  \
+    std::call_once(once, [] {                                                                                            \
+      err = hipFuncSetAttribute(reinterpret_cast<const void*>(tiled_window_attn_kernel<KS, VT>),                         \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);                                 \
+    });                                                                                                                  \
+    SD_REQUIRE(err == hipSuccess, SD_ERR_HIP, "sd_distance_softmax_attention: hipFuncSetAttribute failed: %s",           \
+               hipGetErrorString(err));                                                                                  \
+    tiled_window_attn_kernel<KS, VT><<<grid, 512, tiled_attn_lds<KS, VT>(), st>>>(g);                                    \
+  } while (0)
+  if (dk <= 64 && dv <= 64) SD_GO(2, 4);
+  else if (dk <= 64) SD_GO(2, 8);
+  else if (dv <= 64) SD_GO(4, 4);
+  else SD_GO(4, 8);
+#undef SD_GO
   SD_CHECK_LAUNCH("sd_distance_softmax_attention (tiled)");
+  return SD_OK;
+}
+
+extern "C" int sd_mlstm_step(const float* q, const float* k, const float* v, const float* zi, const float* zf,
+                             int64_t ld, const float* bi, const float* bf, float cap, float q_scale, float* S,
+                             float* n_state, float* m_state, const int32_t* row_pos, const int32_t* row_slot,
+                             const float* gate, const void* w, int w_f32, float eps, float* y, void* y_bf16,
+                             int64_t ldy, int n_rows, int H, int dk, int dv, const sd_poly_norm* act,
+                             sd_stream_t stream) {
+  SD_REQUIRE(q && k && v && zi && zf && bi && bf && S && n_state && m_state && row_pos && row_slot && gate && w &&
+                 (y || y_bf16) && n_rows >= 1 && H >= 1 && dv >= 1 && cap > 0.f && ldy >= (int64_t)H * dv,
+             SD_ERR_INVALID, "sd_mlstm_step: bad argument");
+  SD_REQUIRE(dk >= 1 && dk <= 256 && dv <= 4096, SD_ERR_UNSUPPORTED, "sd_mlstm_step: key size %d / value size %d", dk, dv);
+  SD_REQUIRE(!act || (act->z && act->coef && (act->out || act->out_bf16) && act->n >= 1 && act->ldz >= act->n && act->ldo == ldy),
+             SD_ERR_INVALID, "sd_mlstm_step: bad activation");
+  MlstmArgs a{q, k, v, zi, zf, ld, bi, bf, cap, q_scale, S, n_state, m_state, nullptr, nullptr, nullptr, H, dk, dv};
+  MlstmPostArgs g{};
+  g.row_slot = row_slot; g.gate = gate; g.ldg = ld; g.w = w; g.eps = eps; g.y = y; g.y_b = (bf16_t*)y_bf16; g.ldy = ldy;
+  g.H = H; g.dv = dv;
+  if (act) {
+    g.z = act->z; g.ldz = act->ldz; g.z_bias = act->bias; g.coef = act->coef; g.act = act->out;
+    g.act_b = (bf16_t*)act->out_bf16; g.F = act->n;
+  }
+  const int NS = (dk + kStrip - 1) / kStrip;
+  int CT = 1024 / NS / 64 * 64;
+  if (CT > (dv + 63) / 64 * 64) CT = (dv + 63) / 64 * 64;
+  int nthr = CT * NS;
+  if (nthr < 256) nthr = 256;
+  const size_t lds = sizeof(float) * ((size_t)2 * NS * kStrip + (size_t)NS * CT + dv);
+  hipStream_t st = (hipStream_t)stream;
+  dim3 grid(H + (act ? 1 : 0), n_rows);
+  if (w_f32) mlstm_step_kernel<float><<<grid, nthr, lds, st>>>(a, g, row_pos, CT, NS);
+  else mlstm_step_kernel<bf16_t><<<grid, nthr, lds, st>>>(a, g, row_pos, CT, NS);
+  SD_CHECK_LAUNCH("sd_mlstm_step");
   return SD_OK;
 }
 

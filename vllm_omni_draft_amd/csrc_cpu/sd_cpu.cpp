@@ -1627,6 +1627,12 @@ extern "C" int sd_mlstm_scan(const float*, const float*, const float*, const flo
                              int, int, float*, float*, int, int, int, void*, size_t, sd_stream_t) {
   UNSUPPORTED("sd_mlstm_scan");
 }
+extern "C" int sd_mlstm_step(const float*, const float*, const float*, const float*, const float*, int64_t,
+                             const float*, const float*, float, float, float*, float*, float*, const int32_t*,
+                             const int32_t*, const float*, const void*, int, float, float*, void*, int64_t, int, int,
+                             int, int, const sd_poly_norm*, sd_stream_t) {
+  UNSUPPORTED("sd_mlstm_step");
+}
 extern "C" int sd_mlstm_read(const float*, const float*, float*, const int32_t*, const float*, int64_t, const void*,
                              int, float, float*, void*, int64_t, int, int, int, const sd_poly_norm*, sd_stream_t) {
   UNSUPPORTED("sd_mlstm_read");

@@ -1483,7 +1483,7 @@ def joint_residual(x, a=None, a_bias=None, w1=None, w2=None, eps=1e-5, rows=None
                    conv_state=None, row_pos=None, row_slot=None):
     """sd_joint_residual, in place on x f32 [rows, W] (rows given: x is only read).  Returns (h1, h2,
     copy): the two layer norms (bf16: as bfloat16), h1 with its convolution added when conv_w
-    [W, taps] is given (rows alone in their entries; conv_state moves on), and the row before them."""
+    [taps, W] is given (rows alone in their entries; conv_state moves on), and the row before them."""
     _f32(x, "x")
     n, W = (rows.numel() if rows is not None else x.shape[0]), x.shape[1]
     dt = torch.bfloat16 if bf16 else torch.float32
@@ -1494,19 +1494,19 @@ def joint_residual(x, a=None, a_bias=None, w1=None, w2=None, eps=1e-5, rows=None
     f32p, b16p = (lambda t: None if bf16 else _p(t)), (lambda t: _p(t) if bf16 else None)
     _lib.check(_lib.load().sd_joint_residual(
         _p(x), _p(rows), _p(a), _p(a_bias), _p(copy), _p(w1), _p(w2), 1 if typed is None else _wkind(typed, "weights"),
-        float(eps), f32p(h1), b16p(h1), f32p(h2), b16p(h2), _p(conv_w), conv_w.shape[1] if conv_w is not None else 0,
+        float(eps), f32p(h1), b16p(h1), f32p(h2), b16p(h2), _p(conv_w), conv_w.shape[0] if conv_w is not None else 0,
         _p(conv_state), _p(row_pos), _p(row_slot), n, W, _stream()), "sd_joint_residual")
     return h1, h2, copy
 
 
 def conv_add_rows(x, w, conv_state, row_pos, row_slot, entries, bf16=False) -> torch.Tensor:
-    """x f32 [rows, C] + its causal convolution with w [C, taps] over each entry; conv_state f32
+    """x f32 [rows, C] + its causal convolution with w [taps, C] over each entry; conv_state f32
     [slots, taps-1, C] (None with one tap) moves on."""
     _f32(x, "x")
     out = torch.empty(x.shape, dtype=torch.bfloat16 if bf16 else torch.float32, device=x.device)
     _lib.check(_lib.load().sd_conv_add_rows(_p(x), x.shape[1], _p(w), _wkind(w, "w"), _p(conv_state), _p(row_pos),
                                             _p(row_slot), _p(entries), entries.shape[0], None if bf16 else _p(out),
-                                            _p(out) if bf16 else None, x.shape[1], x.shape[0], x.shape[1], w.shape[1],
+                                            _p(out) if bf16 else None, x.shape[1], x.shape[0], x.shape[1], w.shape[0],
                                             _stream()), "sd_conv_add_rows")
     return out
 
@@ -1531,14 +1531,14 @@ def _poly_norm_part(z, coef, bias, out):
 
 def conv_attn_prep(proj, conv_w, conv_state, H, G, dk, dv, q_norm_w, k_norm_w, eps, k_cache, v_cache, row_pos, row_slot,
                    entries, block_tables, bias=None, temp=(0.0, 0), act=None) -> torch.Tensor:
-    """sd_conv_attn_prep on proj f32 [rows, channels] (q | k | v; q alone when k_cache is None): returns
+    """sd_conv_attn_prep on proj f32 [rows, channels] (q | k | v; q alone when k_cache is None), conv_w [taps, channels]: returns
     the prepared q f32 [rows, H*dk]; keys and values are appended, conv_state moves on.  act (or
     None): (z, coef, bias or None, out), an activation of the same rows computed in the launch."""
     _f32(proj, "proj")
     q = torch.empty(proj.shape[0], H * dk, dtype=torch.float32, device=proj.device)
     part = _poly_norm_part(*act) if act is not None else None
     _lib.check(_lib.load().sd_conv_attn_prep(
-        _p(proj), proj.shape[1], _p(bias), _p(conv_w), conv_w.shape[1], _p(conv_state), H, G, dk, dv,
+        _p(proj), proj.shape[1], _p(bias), _p(conv_w), conv_w.shape[0], _p(conv_state), H, G, dk, dv,
         int(k_cache is None), _p(q_norm_w), _p(k_norm_w), _wkind(conv_w, "conv_w"), float(eps), float(temp[0]),
         int(temp[1]), _p(q), _p(k_cache), _p(v_cache), _p(row_pos), _p(row_slot), _p(entries), entries.shape[0],
         _p(block_tables), block_tables.shape[1] if block_tables is not None else 0, PAGE, proj.shape[0],
@@ -1595,6 +1595,26 @@ def mlstm_read(num, m_rows, m_state, row_slot, gate, w, eps, act=None) -> torch.
     if act is None:
         return buf
     return buf[:, :H * dv], buf[:, H * dv:]
+
+
+def mlstm_step(q, k, v, zi, zf, bi, bf, cap, state, n_state, m_state, row_pos, row_slot, gate, w, eps, q_scale=1.0,
+               act=None):
+    """mlstm_scan and mlstm_read in one launch for rows alone in their entries: f32 [rows, H*dv] (and the
+    activation's result, when act is given as mlstm_read takes it); all states move on."""
+    buf = torch.cat([q, k, v, gate, zi, zf], dim=1).contiguous()
+    n, H, dk, dv = q.shape[0], *state.shape[1:]
+    at, ptr = 0, []
+    for t in (q, k, v, gate, zi, zf):
+        ptr.append(buf.data_ptr() + 4 * at)
+        at += t.shape[1]
+    F = act[0].shape[1] if act is not None else 0
+    y = torch.empty(n, H * dv + F, dtype=torch.float32, device=q.device)
+    part = _poly_norm_part(act[0], act[1], act[2], y[:, H * dv:]) if act is not None else None
+    _lib.check(_lib.load().sd_mlstm_step(ptr[0], ptr[1], ptr[2], ptr[4], ptr[5], buf.shape[1], _p(bi), _p(bf), float(cap),
+                                         float(q_scale), _p(state), _p(n_state), _p(m_state), _p(row_pos), _p(row_slot),
+                                         ptr[3], _p(w), _wkind(w, "w"), float(eps), _p(y), None, H * dv + F, n, H, dk, dv,
+                                         C.byref(part) if part is not None else None, _stream()), "sd_mlstm_step")
+    return y if act is None else (y[:, :H * dv], y[:, H * dv:])
 
 
 def matmul_rows_batched(x, w) -> torch.Tensor:

@@ -369,7 +369,7 @@ class SeqLayerTensors:
     # layers whose sublayers read the same residual: w_in [mixer rows, padded to mix_rows | ff up rows],
     # w_o [width, mixer output | ff] (the mixer's output matrix and the feed-forward's down matrix)
     mix_rows: int = 0
-    in_conv_w: Optional[torch.Tensor] = None   # [width, taps]: the mixer's input convolution
+    in_conv_w: Optional[torch.Tensor] = None   # [taps, width]: the mixer's input convolution (conv_w too: taps first)
     dist1: Optional[torch.Tensor] = None       # f32 [heads]
     dist2: Optional[torch.Tensor] = None
     gate_bias: Optional[torch.Tensor] = None   # f32 [2*heads]: input gates', then forget gates'
@@ -610,7 +610,7 @@ def _joint_layer(cfg, i: int, get, dev, mat) -> SeqLayerTensors:
     """Layer i of a model whose sublayers read the same residual: the matrices that read the mixer's
     input stacked, padded with zero rows to a multiple of 16 and followed by the feed-forward's up
     matrix; the mixer's output matrix and the down matrix side by side, so that one product adds
-    both sublayers; the convolutions of q, k and v as one over the stacked channels."""
+    both sublayers; the convolutions of q, k and v as one over the stacked channels, taps first."""
     l, p, W = cfg.layers[i], f"l{i}.", cfg.width
     m = l.mixer
     H, G, dk, dv, F = m.heads, m.kv_heads, m.dim, m.vdim, l.ff
@@ -629,12 +629,12 @@ def _joint_layer(cfg, i: int, get, dev, mat) -> SeqLayerTensors:
     lt = SeqLayerTensors(norm_w=dev(get(p + "norm1", (W,))), w_in=mat(torch.cat(parts)), w_o=mat(torch.cat(out, dim=1)),
                          r1_bias=None, mix_rows=mix_rows)
     if l.in_taps:
-        lt.in_conv_w = dev(get(p + "canon1", (W, l.in_taps)))
+        lt.in_conv_w = dev(get(p + "canon1", (W, l.in_taps)).t())
     if m.kind == "mlstm":
         lt.gate_bias = dev(torch.cat([get(p + "mix.i.b", (H,)).float(), get(p + "mix.f.b", (H,)).float()]), torch.float32)
         lt.s_norm_w = dev(get(p + "mix.norm", (H * dv,)))
     else:
-        lt.conv_w = dev(torch.cat([get(p + f"mix.{n}.conv", (rows, m.conv_taps)) for n, rows in names]))
+        lt.conv_w = dev(torch.cat([get(p + f"mix.{n}.conv", (rows, m.conv_taps)) for n, rows in names]).t())
         if m.qkv_bias:
             lt.w_in_bias = dev(torch.cat([get(p + f"mix.{n}.b", (rows,)) for n, rows in names]))
         lt.q_norm_w = dev(get(p + "mix.q.norm", (dk,)))
