@@ -1314,6 +1314,27 @@ def guf_kernel_rooflines(cfg, device, ctx, rows):
         out.append(("joint_residual", "gated_residual_norm", us, rows * W * 20, 0.0, F32_VALU_PEAK_TFLOPS))
         us = _events(lambda: ops.conv_add_rows(x, icw, ics, pos, slot, ent, bf16=True), 5)
         out.append(("conv_add_rows", "causal_conv_rows", us, rows * W * 6, 0.0, F32_VALU_PEAK_TFLOPS))
+        us = _events(lambda: ops.causal_conv_rows(x, icw.t().contiguous(), None, ics, pos, slot, ent), 5)
+        out.append(("causal_conv_rows (as conv_add_rows; like kernel)", "", us, rows * W * 8, 0.0, F32_VALU_PEAK_TFLOPS))
+    if rows == 1:
+        us = _events(lambda: ops.mlstm_step(qm, km, vm, zi, zf, bi, bff, mem.gate_cap, S, N_, M_, pos, slot, gate, w, 1e-5,
+                                            q_scale=dk ** -0.5), 5)
+        out.append(("mlstm_step (wrapper copy included)", "decay_scan_rows", us,
+                    4 * (2 * Hm * dk + 3 * Hm * dv + 2 * Hm + 2 * Hm * dk * (dv + 1)), Hm * dk * (dv + 1) * 5.0,
+                    F32_VALU_PEAK_TFLOPS))
+    # the like kernels of other families at the same sizes
+    k2, v2, q2 = rn(rows, G * D), rn(rows, G * D), rn(rows, H * D)
+    us = _events(lambda: ops.qk_head_norm_append(q2, qw, k2, kw, v2, H, G, D, D, 1e-5, kc, vc, pos, slot, tables), 5)
+    out.append(("qk_head_norm_append (like kernel, wrapper copies included)", "", us,
+                rows * (8 * (H + G) * D + 4 * G * D + 4 * G * D), 0.0, F32_VALU_PEAK_TFLOPS))
+    us = _events(lambda: ops.head_post(vm, gate, Hm, dv, norm_w=w[:dv], unit_norm=True), 5)
+    out.append(("head_post (like kernel)", "", us, rows * Hm * dv * 12, 0.0, F32_VALU_PEAK_TFLOPS))
+    z2 = rn(rows, F)
+    us = _events(lambda: ops.relu_mul_rows(z, z2), 5)
+    out.append(("relu_mul_rows (like kernel)", "", us, rows * F * 10, 0.0, F32_VALU_PEAK_TFLOPS))
+    z1 = rn(rows, W)
+    us = _events(lambda: ops.gated_residual_norm(x, z1, a, w1, 1e-5), 5)
+    out.append(("gated_residual_norm (like kernel)", "", us, rows * W * 22, 0.0, F32_VALU_PEAK_TFLOPS))
     res = []
     for name, like, us, nbytes, flops, peak in out:
         floor_us = max(nbytes / (HBM_PEAK_GBS * 1e3), flops / (peak * 1e6))

@@ -1102,7 +1102,8 @@ SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
       if (l.kind == SD_MIX_MLSTM) {
         up(hv, (size_t)l.heads * (l.vdim + 1));
         up(sh, (size_t)l.heads);
-        up(mem, sd_mlstm_scratch_bytes(rows, rows < kPlanEntries ? rows : kPlanEntries, l.heads, l.dim, l.vdim));
+        const int ents = rows < kPlanEntries ? rows : kPlanEntries;   // (enough for any number of portions up to it)
+        up(mem, sd_mlstm_scratch_bytes(rows + ents, ents, l.heads, l.dim, l.vdim));
       } else {
         up(pq, (size_t)l.heads * l.dim);
         up(attn, sd_multimap_softmax_attention_scratch_bytes(rows, l.heads, 1, l.vdim, l.window, 0, 0, max_ctx));

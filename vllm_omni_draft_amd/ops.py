@@ -1465,7 +1465,7 @@ def distance_softmax_attention(q, k_cache, v_cache, row_pos, row_slot, block_tab
     _f32(q, "q")
     window, ldo = int(window) or 0x7fffffff, int(ldo) or H * dv
     dt = torch.bfloat16 if bf16_only else torch.float32
-    out = torch.zeros(q.shape[0], ldo, dtype=dt, device=q.device)
+    out = torch.empty(q.shape[0], ldo, dtype=dt, device=q.device)
     lib = _lib.load()
     n = int(lib.sd_multimap_softmax_attention_scratch_bytes(q.shape[0], H, 1, dv, window, 0, 0,
                                                             block_tables.shape[1] * PAGE)) if split else 0
