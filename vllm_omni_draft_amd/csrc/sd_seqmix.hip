@@ -1802,8 +1802,8 @@ extern "C" int sd_seq_model_forward(sd_seq_model* m, const sd_seq_batch* b, void
                                nullptr, d.final_norm_w, nullptr, f32, d.norm_eps, hout, d.head_tiled ? houtb : nullptr,
                                nullptr, nullptr, nullptr, 0, nullptr, nullptr, nullptr, b->n_out, W, stream));
     else
-    SQ_TRY(sd_rmsnorm_rows(x, b->out_rows, d.final_norm_w, f32, d.plain_norm ? 0.f : 1.f, d.norm_eps, hout,
-                           d.head_tiled ? houtb : nullptr, b->n_out, W, stream));
+      SQ_TRY(sd_rmsnorm_rows(x, b->out_rows, d.final_norm_w, f32, d.plain_norm ? 0.f : 1.f, d.norm_eps, hout,
+                             d.head_tiled ? houtb : nullptr, b->n_out, W, stream));
     SQ_TRY(seq_linear(d.head ? d.head : d.embed, d.head_tiled, f32, hout, nullptr, W, houtb, W, nullptr, b->logits,
                       d.vocab, b->n_out, d.vocab, W, wide_ws, w.wide_bytes, stream));
     if (d.logit_scale != 0.f && d.logit_scale != 1.f)

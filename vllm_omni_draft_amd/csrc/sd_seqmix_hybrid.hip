@@ -1990,7 +1990,7 @@ extern "C" int sd_distance_softmax_attention(const float* q, int64_t ldq, const 
              "sd_masked_softmax_attention: value size %d outside 1..512 (or above the key row it is part of)", dv);
   hipStream_t st = (hipStream_t)stream;
   if (entries && !cache_f32 && n_rows > kSplitRows && maps == 1 && !sinks && keep_first == 0 && chunk == 0 && v_cache) {
-    const int rc = sd_tiled_window_attention_(q, ldq, k_cache, v_cache, row_pos, block_tables, max_blocks, page, n_rows,
+    const int rc = sd_tiled_window_attention_(q, ldq, k_cache, v_cache, block_tables, max_blocks, page, n_rows,
                                               H, G, dk, dv, window, scale, softcap, dist1, dist2, entries, n_entries, out,
                                               out_bf16, ldo, stream);
     if (rc != SD_ERR_UNSUPPORTED) return rc;

@@ -1680,11 +1680,10 @@ extern "C" int sd_mlstm_scan(const float* q, const float* k, const float* v, con
 }
 
 int sd_tiled_window_attention_(const float* q, int64_t ldq, const void* k_cache, const void* v_cache,
-                               const int32_t* row_pos, const int32_t* block_tables, int max_blocks, int page, int n_rows,
-                               int H, int G, int dk, int dv, int window, float scale, float softcap, const float* dist1,
+                               const int32_t* block_tables, int max_blocks, int page, int n_rows, int H,
+                               int G, int dk, int dv, int window, float scale, float softcap, const float* dist1,
                                const float* dist2, const int32_t* entries, int n_entries, float* out, void* out_bf16,
                                int64_t ldo, sd_stream_t stream) {
-  (void)row_pos;
   if (page != kPage || dk % 8 || dv % 8 || dk > 128 || dv > 128 || ldq % 4 || !sd_aligned16(q) || !sd_aligned16(k_cache) ||
       !sd_aligned16(v_cache) || !(ldo % 4 || (sd_aligned16(out) && sd_aligned16(out_bf16))))
     return SD_ERR_UNSUPPORTED;
