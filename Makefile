@@ -2,7 +2,7 @@
 HIPCC ?= /opt/rocm/bin/hipcc
 ARCH  ?= gfx950
 CSRC  := vllm_omni_draft_amd/csrc
-SRCS  := $(CSRC)/sd_base.hip $(CSRC)/sd_runtime.hip $(CSRC)/sd_sampling.hip $(CSRC)/sd_linear.hip $(CSRC)/sd_linear_wide.hip $(CSRC)/sd_attention.hip $(CSRC)/sd_ipc.hip $(CSRC)/sd_chain.hip $(CSRC)/sd_draft_layer.hip $(CSRC)/sd_seqmix.hip $(CSRC)/sd_seqmix_hybrid.hip $(CSRC)/sd_seqmix_joint.hip
+SRCS  := $(CSRC)/sd_base.hip $(CSRC)/sd_runtime.hip $(CSRC)/sd_sampling.hip $(CSRC)/sd_linear.hip $(CSRC)/sd_linear_wide.hip $(CSRC)/sd_attention.hip $(CSRC)/sd_ipc.hip $(CSRC)/sd_chain.hip $(CSRC)/sd_draft_layer.hip $(CSRC)/sd_seqmix.hip $(CSRC)/sd_seqmix_hybrid.hip $(CSRC)/sd_seqmix_joint.hip $(CSRC)/sd_seqmix_streams.hip
 OBJS  := $(SRCS:.hip=.o)
 LIB   := vllm_omni_draft_amd/libsd_amd.so
 EXTRA ?=
@@ -38,7 +38,7 @@ SEQ_LIB  := vllm_omni_draft_amd/libsd_seq.so
 # (these models call the many-row linear family with bf16 weights and its f32 epilogue only: that file is
 # compiled for them without its other instantiations, which take most of the whole library's build time)
 # (... and in two parts side by side, the kernels of few and of many token tiles)
-SEQ_OBJS := $(CSRC)/sd_base.o $(CSRC)/sd_seqmix.o $(CSRC)/sd_seqmix_hybrid.o $(CSRC)/sd_seqmix_joint.o $(CSRC)/sd_sampling.o $(CSRC)/sd_linear.o \
+SEQ_OBJS := $(CSRC)/sd_base.o $(CSRC)/sd_seqmix.o $(CSRC)/sd_seqmix_hybrid.o $(CSRC)/sd_seqmix_joint.o $(CSRC)/sd_seqmix_streams.o $(CSRC)/sd_sampling.o $(CSRC)/sd_linear.o \
 	$(CSRC)/sd_linear_wide_seq1.o $(CSRC)/sd_linear_wide_seq2.o
 $(CSRC)/sd_linear_wide_seq%.o: $(CSRC)/sd_linear_wide.hip $(CSRC)/sd_common.h include/sd_amd.h
 	$(HIPCC) $(FLAGS) -DSD_WIDE_F32_ONLY -DSD_WIDE_PART=$* -c $< -o $@

@@ -1456,6 +1456,119 @@ int sd_mlstm_step(const float* q, const float* k, const float* v, const float* z
                   const float* gate, const void* w, int w_f32, float eps, float* y, void* y_bf16,
                   int64_t ldy, int n_rows, int H, int dk, int dv, const sd_poly_norm* act,
                   sd_stream_t stream);
+/* sd_distance_softmax_attention whose output rows are gated: unit u of row r is multiplied by
+ * sigmoid(gates[r*ldg + u]) (gates f32, or NULL: not).  Its tiled form takes sinks, kept first tokens
+ * and gates too; the cut and the sweeping form take everything.                             */
+int sd_gated_softmax_attention(const float* q, int64_t ldq, const void* k_cache, const void* v_cache,
+                               int cache_f32, const int32_t* row_pos, const int32_t* row_slot,
+                               const int32_t* block_tables, int max_blocks, int page, int n_rows, int H, int G,
+                               int maps, int dk, int dv, int window, int keep_first, int chunk, float scale,
+                               float softcap, const float* sinks, const float* dist1, const float* dist2,
+                               const float* gates, int64_t ldg, const int32_t* entries, int n_entries, float* out,
+                               void* out_bf16, int64_t ldo, void* scratch, size_t scratch_bytes, sd_stream_t stream);
+/* sd_moe_route_rows_biased with a correction (f32 [E], or NULL): the experts with the largest score +
+ * correction are chosen, their weights are the scores without it.                           */
+int sd_moe_route_rows_corrected(const float* x, int64_t ldx, const void* w_router, const float* router_bias,
+                                const float* correction, int w_f32, float* logits, int32_t* sel_expert,
+                                float* sel_weight, int n_rows, int E, int K, int top, int score_kind, int renorm,
+                                float renorm_eps, float weight_scale, const void* w_gate, int n_gate, float* gate_out,
+                                sd_stream_t stream);
+/* sd_moe_experts with one more activation, act_kind 2 (gated experts): g = min(gate, limit), c = up
+ * clamped to +-limit, g sigmoid(1.702 g) (c + 1).  A chosen index outside 0 .. E-1 is none of these
+ * experts: its row of out is not written (in every form of sd_moe_experts).                 */
+int sd_moe_experts_clamped(const float* x, const void* x_bf16, int64_t ldx, const int32_t* sel_expert,
+                           const float* sel_weight, const void* w_gate_up, const void* w_down, int w_f32, float* out,
+                           int n_rows, int top, int E, int F, int W, int scale_input, int act_kind, float limit,
+                           void* scratch, size_t scratch_bytes, sd_stream_t stream);
+/* x[r, c] = cap tanh(x[r, c] / cap)                                                        */
+int sd_cap_rows(float* x, int64_t ld, float cap, int n_rows, int n_cols, sd_stream_t stream);
+
+/* ---- mechanisms of decoders that keep several copies of the residual (streams).  Same conventions.  */
+
+/* Streams x [rows, streams, W] f32.  Per row, in one launch:
+ *   tokens != NULL:  x_s = embed[token] for every stream
+ *   a != NULL:  y = the sublayer's result (below);  x_t <- sum_s mix[s*streams + t] x_s + out[t] y, all
+ *               streams at once from the old ones
+ *   x_copy[r] = sum_s x_s                                  (x_copy != NULL)
+ *   w_next != NULL:  u = sum_s in[s] x_s (in NULL: every factor 1), h = rms_norm(u) * (1 + w_next), h_bf16
+ *               the same (either may be NULL)
+ * y: b == NULL: the sum of the row's n_a rows of a ([rows*n_a, lda]); with sel_expert / sel_weight
+ * [rows, n_a] only rows whose chosen expert is below n_experts count, and the weights of the others are
+ * added up and multiply the sublayer's own input ([rows, W]; may be h).  b != NULL (row stride lda):
+ * half the sum of rms_norm(a) * w_a and rms_norm(b) * w_b.  rows (int32 [n_rows], or NULL): output row i
+ * comes from row rows[i], and x is left as it is.  mix, out, in f32; norm weights and the table in the
+ * model's element type.                                                                    */
+typedef struct {
+  float* x;
+  int streams;
+  const int32_t* rows;
+  const int32_t* tokens;
+  const void* embed;        /* [vocab, W] */
+  int vocab;
+  const float* a;
+  int64_t lda;
+  int n_a;
+  const int32_t* sel_expert;
+  const float* sel_weight;
+  int n_experts;
+  const float* input;
+  const float* b;
+  const void* w_a;
+  const void* w_b;
+  const float* mix;
+  const float* out;
+  float* x_copy;
+  const float* in;
+  const void* w_next;
+  float* h;
+  void* h_bf16;
+} sd_streams_update;
+int sd_streams_residual(const sd_streams_update* u, int w_f32, float eps, int n_rows, int W, int round_bf16_out,
+                        sd_stream_t stream);
+/* Linear attention with a decay per key channel, one token per row: with d = sigmoid(a2 a1 + a2_bias)^(1/tau)
+ * (a1 [rank], a2 [heads*dim, rank]), per head  S <- diag(d) S + k v^T,  o = S^T (q_scale q), then o / sqrt(mean(o^2)
+ * + eps) * norm_w * silu(gate) to y / y_bf16 [rows, heads*vdim] (row stride ldy, either may be NULL).  q, k, v,
+ * a1, gate have row stride ld; state f32 [slots, heads, dim, vdim].  dim <= 256.              */
+typedef struct {
+  const float* q;
+  const float* k;
+  const float* v;
+  const float* a1;
+  const float* gate;
+  int64_t ld;
+  const void* a2;
+  const float* a2_bias;
+  int rank;
+  float tau, q_scale;
+  float* state;
+  const void* norm_w;       /* [vdim] */
+  float* y;
+  void* y_bf16;
+  int64_t ldy;
+  int heads, dim, vdim;
+} sd_decay_step;
+/* Every row must be alone in its entry (a decoding step); a row at position 0 starts from zero. */
+int sd_decay_step_rows(const sd_decay_step* step, int w_f32, float eps, const int32_t* row_pos,
+                       const int32_t* row_slot, int n_rows, sd_stream_t stream);
+/* Attention inputs with biases (each may be NULL, model element type): q [rows, H*dk] + q_bias RMS-normed per
+ * head (weight [dk]) in place; k [rows, G*dk] + k_bias normed per head and v [rows, G*dv] + v_bias appended as
+ * sd_cache_append does.  Row stride ld.  dk, dv <= 512.  step (or NULL): sd_decay_step_rows in the same launch. */
+int sd_biased_qkv_prep(float* q, const float* k, const float* v, int64_t ld, const void* q_bias, const void* k_bias,
+                       const void* v_bias, int H, int G, int dk, int dv, const void* q_norm_w, const void* k_norm_w,
+                       int w_f32, float eps, void* k_cache, void* v_cache, const int32_t* row_pos,
+                       const int32_t* row_slot, const int32_t* block_tables, int max_blocks, int page, int n_rows,
+                       const sd_decay_step* step, sd_stream_t stream);
+/* out[r, c] = sigmoid(a2[c] . a1[r] + a2_bias[c])^(1/tau); a1 [rows, rank] (row stride ld), a2 [n_cols, rank]. */
+int sd_low_rank_decay(const float* a1, int64_t ld, const void* a2, const float* a2_bias, int w_f32, int rank, float tau,
+                      float* out, int n_rows, int n_cols, sd_stream_t stream);
+/* The recurrence of sd_decay_scan with decays per key channel ([rows, H*dk]) and q multiplied by q_scale, in
+ * blocks of 16 tokens on the f32 matrix instruction.  With scratch of sd_decay_chunks_scratch_bytes bytes (0: few
+ * rows) long portions run in chunks side by side: the chunks' own sums, a pass over the chunks, then the tokens'
+ * results; otherwise a portion runs in one go.                                              */
+size_t sd_decay_chunks_scratch_bytes(int n_rows, int n_entries, int H, int dk, int dv);
+int sd_decay_chunks(const float* q, const float* k, const float* v, int64_t ld, const float* decay, float q_scale,
+                    float* state, const int32_t* entries, int n_entries, int n_rows, float* out, int H, int dk, int dv,
+                    void* scratch, size_t scratch_bytes, sd_stream_t stream);
 /* x[r, c] *= s                                                                             */
 int sd_scale_rows(float* x, int64_t ld, float s, int n_rows, int n_cols, sd_stream_t stream);
 
@@ -1466,14 +1579,16 @@ typedef enum {
   SD_MIX_LATENT = 3,        /* softmax window attention over latent keys / values */
   SD_MIX_SOFTMAX_SSD = 4,   /* softmax window attention and a state-space recurrence side by side */
   SD_MIX_SOFTMAX = 5,       /* grouped-query softmax attention (sd_masked_softmax_attention), no rotation */
-  SD_MIX_MLSTM = 6          /* matrix memory with exponential gates (sd_mlstm_scan) */
+  SD_MIX_MLSTM = 6,         /* matrix memory with exponential gates (sd_mlstm_scan) */
+  SD_MIX_SOFTMAX_DECAY = 7  /* softmax window attention and linear attention with a decay per key channel side by side */
 } sd_mixer_kind;
 
 typedef enum {
   SD_BLOCK_GATED = 0,       /* h = norm(x); x += sigmoid(r1) mixer(h) + sigmoid(r2) ff(h) */
   SD_BLOCK_POSTNORM = 1,    /* x += norm1(mixer(x)); x += norm2(ff(x)) */
   SD_BLOCK_SANDWICH = 2,    /* x += post_norm(mixer(norm(x))); x += post_norm2(ff(norm2(x))) */
-  SD_BLOCK_JOINT = 3        /* x += mixer(u + conv(u)) + ff(LN2(x)), u = LN1(x): layer norms */
+  SD_BLOCK_JOINT = 3,       /* x += mixer(u + conv(u)) + ff(LN2(x)), u = LN1(x): layer norms */
+  SD_BLOCK_STREAMS = 4      /* several copies of the residual, mixed around each sublayer (sd_streams_residual) */
 } sd_block_kind;
 
 /* One layer: h = norm(x); x += sigmoid(r1) * mixer(h) + sigmoid(r2) * ff(h).  w_in stacks every
@@ -1615,6 +1730,27 @@ typedef struct {
   /* feed-forward (ff > 0): an activation of normed powers */
   const void* ff_bias;      /* [ff] the up matrix's bias, or NULL */
   const float* ff_coef;     /* [4] */
+  /* ---- SD_BLOCK_STREAMS layers (all zero otherwise).  norm_w / norm2_w are stored around zero.
+   * SD_MIX_SOFTMAX_DECAY: w_in stacks q [heads*dim], k [kv_heads*dim], v [kv_heads*vdim], then the linear
+   * attention's q [s_heads*s_state], k [s_heads*s_state], v [s_heads*s_vdim], g [s_heads*s_vdim], a1 [rank],
+   * then the head gates [heads]; w_in_bias has one element per row of the first three (or NULL); q_norm_w
+   * / k_norm_w [dim]; s_norm_w [s_vdim], w_a2, b_a2, tau, state [slots, s_heads, s_state, s_vdim].  The two
+   * output matrices are w_o [width, heads*vdim] and w_o2 [width, s_heads*s_vdim], or, out_stacked (equal
+   * input widths; tiled: a width that is a multiple of 16), w_o holds the rows of both.  out_norm_w / out_norm2_w
+   * norm their results.  The feed-forward is absent, dense (w_ff_in, w_down, ff_act) or routed experts:
+   * n_experts with matrices and n_identity more that return their input. */
+  const float* hc_in;       /* [streams] factors around the mixer */
+  const float* hc_out;      /* [streams] */
+  const float* hc_mix;      /* [streams, streams], from, to */
+  const float* hc2_in;      /* around the feed-forward */
+  const float* hc2_out;
+  const float* hc2_mix;
+  int out_stacked;
+  const void* out_norm_w;   /* [width] */
+  const void* out_norm2_w;
+  int n_identity;           /* w_router has n_experts + n_identity rows */
+  const float* route_correction; /* f32 [n_experts + n_identity] or NULL: sd_moe_route_rows_corrected */
+  float expert_limit;       /* sd_moe_experts_clamped */
 } sd_seq_layer;
 
 typedef struct {
@@ -1632,6 +1768,8 @@ typedef struct {
   int buckets, mul_prev, mul_cur;
   const void* head;        /* [vocab, width] row-major, or NULL: the embedding table is the head */
   float logit_scale;       /* 0: 1 */
+  int streams;             /* SD_BLOCK_STREAMS models: copies of the residual */
+  float logit_softcap;     /* logits become cap tanh(z / cap); 0: they stay */
 } sd_seq_model_desc;
 
 typedef struct {

@@ -106,7 +106,10 @@ class SeqLayer(C.Structure):
                 ("mix_rows", i32), ("in_conv_w", vp), ("in_taps", i32), ("in_conv_state", vp),
                 ("q_temp_coef", C.c_float), ("q_temp_every", i32), ("dist1", vp), ("dist2", vp),
                 ("n_state", vp), ("m_state", vp), ("gate_bias", vp), ("gate_cap", C.c_float),
-                ("ff_bias", vp), ("ff_coef", vp)]
+                ("ff_bias", vp), ("ff_coef", vp),
+                ("hc_in", vp), ("hc_out", vp), ("hc_mix", vp), ("hc2_in", vp), ("hc2_out", vp), ("hc2_mix", vp),
+                ("out_stacked", i32), ("out_norm_w", vp), ("out_norm2_w", vp), ("n_identity", i32),
+                ("route_correction", vp), ("expert_limit", C.c_float)]
 
 
 class PolyNorm(C.Structure):
@@ -115,12 +118,28 @@ class PolyNorm(C.Structure):
                 ("n", i32)]
 
 
+class StreamsUpdate(C.Structure):
+    """sd_streams_update"""
+    _fields_ = [("x", vp), ("streams", i32), ("rows", vp), ("tokens", vp), ("embed", vp), ("vocab", i32),
+                ("a", vp), ("lda", i64), ("n_a", i32), ("sel_expert", vp), ("sel_weight", vp), ("n_experts", i32),
+                ("input", vp), ("b", vp), ("w_a", vp), ("w_b", vp), ("mix", vp), ("out", vp), ("x_copy", vp),
+                ("in_", vp), ("w_next", vp), ("h", vp), ("h_bf16", vp)]
+
+
+class DecayStep(C.Structure):
+    """sd_decay_step"""
+    _fields_ = [("q", vp), ("k", vp), ("v", vp), ("a1", vp), ("gate", vp), ("ld", i64), ("a2", vp), ("a2_bias", vp),
+                ("rank", i32), ("tau", C.c_float), ("q_scale", C.c_float), ("state", vp), ("norm_w", vp), ("y", vp),
+                ("y_bf16", vp), ("ldy", i64), ("heads", i32), ("dim", i32), ("vdim", i32)]
+
+
 class SeqModelDesc(C.Structure):
     _fields_ = [("n_layers", i32), ("width", i32), ("vocab", i32), ("weights_f32", i32),
                 ("norm_eps", C.c_float), ("embed", vp), ("head_tiled", vp), ("final_norm_w", vp),
                 ("layers", C.POINTER(SeqLayer)),
                 ("plain_norm", i32), ("embed_scale", C.c_float), ("bigram", vp), ("buckets", i32),
-                ("mul_prev", i32), ("mul_cur", i32), ("head", vp), ("logit_scale", C.c_float)]
+                ("mul_prev", i32), ("mul_cur", i32), ("head", vp), ("logit_scale", C.c_float), ("streams", i32),
+                ("logit_softcap", C.c_float)]
 
 
 class SeqBatch(C.Structure):
@@ -276,6 +295,21 @@ SIGNATURES = {
     "sd_moe_experts_scratch_bytes": (C.c_size_t, [i32, i32, i32, i32, i32]),
     "sd_moe_experts": (i32, [vp, vp, i64, vp, vp, vp, vp, i32, vp, i32, i32, i32, i32, i32, i32, i32, vp, C.c_size_t, vp]),
     "sd_postnorm_residual": (i32, [vp, vp, i32, C.c_float, vp, C.c_float, vp, i32, C.c_float, vp, i32, i32, vp]),
+    "sd_gated_softmax_attention": (i32, [vp, i64, vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, i32,
+                                         i32, i32, C.c_float, C.c_float, vp, vp, vp, vp, i64, vp, i32, vp, vp, i64, vp,
+                                         C.c_size_t, vp]),
+    "sd_moe_route_rows_corrected": (i32, [vp, i64, vp, vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, i32, C.c_float,
+                                          C.c_float, vp, i32, vp, vp]),
+    "sd_moe_experts_clamped": (i32, [vp, vp, i64, vp, vp, vp, vp, i32, vp, i32, i32, i32, i32, i32, i32, i32, C.c_float,
+                                     vp, C.c_size_t, vp]),
+    "sd_cap_rows": (i32, [vp, i64, C.c_float, i32, i32, vp]),
+    "sd_streams_residual": (i32, [C.POINTER(StreamsUpdate), i32, C.c_float, i32, i32, i32, vp]),
+    "sd_decay_step_rows": (i32, [C.POINTER(DecayStep), i32, C.c_float, vp, vp, i32, vp]),
+    "sd_biased_qkv_prep": (i32, [vp, vp, vp, i64, vp, vp, vp, i32, i32, i32, i32, vp, vp, i32, C.c_float, vp, vp, vp, vp,
+                                 vp, i32, i32, i32, C.POINTER(DecayStep), vp]),
+    "sd_low_rank_decay": (i32, [vp, i64, vp, vp, i32, i32, C.c_float, vp, i32, i32, vp]),
+    "sd_decay_chunks_scratch_bytes": (C.c_size_t, [i32, i32, i32, i32, i32]),
+    "sd_decay_chunks": (i32, [vp, vp, vp, i64, vp, C.c_float, vp, vp, i32, i32, vp, i32, i32, i32, vp, C.c_size_t, vp]),
     "sd_scale_rows": (i32, [vp, i64, C.c_float, i32, i32, vp]),
     "sd_masked_softmax_attention_scratch_bytes": (C.c_size_t, [i32, i32, i32, i32, i32, i32, i32]),
     "sd_masked_softmax_attention": (i32, [vp, i64, vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32,

@@ -251,7 +251,10 @@ class ExpertsSpec:
     two matrices, down(relu(up h)^2).  The chosen weights are divided by (their sum + renorm_eps)
     when renorm, then multiplied by scale.  shared_ff > 0: one more expert of that width and the
     same form runs for every token and is added, times sigmoid(g . h) when shared_gate.  A softmax
-    score that is renormed over the chosen experts is the softmax over the chosen logits alone."""
+    score that is renormed over the chosen experts is the softmax over the chosen logits alone.  act
+    "clamped_gate": g = min(gate h, limit), c = up h clamped to +-limit, down(g sigmoid(1.702 g) (c + 1)).
+    correction: a learned number per expert is added to the scores for the choice alone.  identity:
+    that many experts more, the last ones, whose output is their input."""
     experts: int
     top: int
     ff: int
@@ -264,14 +267,44 @@ class ExpertsSpec:
     shared_ff: int = 0
     shared_gate: bool = True
     router_bias: bool = False      # a bias on the router's logits
+    limit: float = 0.0             # "clamped_gate"
+    correction: bool = False
+    identity: int = 0
+
+    @property
+    def outputs(self) -> int:
+        """Rows of the router: the experts with matrices, then the identity experts."""
+        return self.experts + self.identity
 
     def validate(self) -> None:
-        if self.experts < 1 or not 1 <= self.top <= self.experts or self.ff < 1 or self.shared_ff < 0:
-            raise ValueError(f"experts {self.experts}, top {self.top}, ff {self.ff}, shared ff {self.shared_ff}")
+        if self.experts < 1 or self.identity < 0 or not 1 <= self.top <= self.outputs or self.ff < 1 or self.shared_ff < 0:
+            raise ValueError(f"experts {self.experts} (and {self.identity} identity experts), top {self.top}, ff {self.ff}, "
+                             f"shared ff {self.shared_ff}")
         if self.score not in ("sigmoid", "softmax"):
             raise ValueError(f"unknown router score {self.score!r}")
-        if self.act not in ("silu", "relu2"):
+        if self.act not in ("silu", "relu2", "clamped_gate"):
             raise ValueError(f"unknown expert activation {self.act!r}")
+        if self.act == "clamped_gate" and not self.limit > 0:
+            raise ValueError("a clamped activation needs limit > 0")
+
+
+@dataclass
+class LinearSpec:
+    """Linear attention with a decay per key channel, sigmoid(z)^(1/tau) with z from the input through a
+    low-rank pair of matrices (the "gla" mixer as one side of a "parallel" mixer): each head's result is
+    normed over vdim with one weight for all heads and gated by silu."""
+    heads: int
+    dim: int
+    vdim: int
+    rank: int                      # inner size of the low-rank pair (a tensor's shape gives it)
+    tau: float = 1.0
+
+    def validate(self) -> None:
+        if min(self.heads, self.dim, self.vdim, self.rank) < 1 or not self.tau > 0:
+            raise ValueError(f"linear attention: heads {self.heads}, dim {self.dim}, vdim {self.vdim}, rank {self.rank}, "
+                             f"tau {self.tau}")
+        if self.dim > 256 or self.rank > 1536:
+            raise ValueError("linear attention: dim above 256 or rank above 1536 is not supported")
 
 
 @dataclass
@@ -286,7 +319,9 @@ class MixerSpec:
     shared by the heads (queries through a latent of q_rank channels; dim counts the unrotated
     channels of a head); "parallel": grouped-query softmax attention without rotation, q and k
     normed over the whole projection, over a window that also keeps the first keep_first tokens,
-    beside a state-space recurrence (ssd) on the same input, summed with two scales;
+    beside a state-space recurrence (ssd) on the same input, summed with two scales, or beside linear
+    attention (linear), half the sum of both results, each normed over the width (then with q and k
+    normed per head, and biases, a cap, a sink and head gates as a softmax attention may have them);
     "softmax_attention": grouped-query softmax attention without rotation, q and k normed per
     head with one weight of `dim` channels each (qk_head_norm), scores capped by softcap *
     tanh(s / softcap), keys of the query's own chunk of `chunk` positions only.  A latent
@@ -327,7 +362,8 @@ class MixerSpec:
     kv_rank: int = 0
     rot_dim: int = 0               # latent_attention: rotated channels per head (behind the `dim` unrotated)
     rot_scaling: Optional[dict] = None  # frequency blending {factor, original, fast, slow}
-    ssd: Optional[SsdSpec] = None  # parallel
+    ssd: Optional[SsdSpec] = None  # parallel: the recurrence beside the attention,
+    linear: Optional[LinearSpec] = None  # ... or linear attention beside it
     left_scale: float = 1.0        # parallel: factor of the attention
     right_scale: float = 1.0       # parallel: factor of the recurrence
     chunk: int = 0                 # softmax attention: keys of the query's own chunk only (0: no chunks)
@@ -387,6 +423,14 @@ class MixerSpec:
                 raise ValueError("softmax attention: one or two score maps, one kind of q/k norm, one kind of sink")
             if self.value_is_key and (self.maps != 1 or self.vdim != self.dim or self.kv_from >= 0):
                 raise ValueError("values taken from the keys need one score map, vdim == dim and keys of the layer's own")
+            return
+        if self.kind == "parallel" and self.linear is not None:
+            if self.window < 0 or self.keep_first < 0 or self.softcap < 0 or self.rot_dims or self.ssd is not None:
+                raise ValueError("attention beside linear attention needs window >= 0, keep_first >= 0, softcap >= 0, no "
+                                 "rotation and no state-space part")
+            if self.dim > 512 or self.vdim > 512 or not self.qk_head_norm:
+                raise ValueError("attention beside linear attention norms q and k per head, of at most 512 channels")
+            self.linear.validate()
             return
         if self.kind == "parallel":
             if self.window < 1 or self.keep_first < 0 or self.rot_dims or self.ssd is None or self.vdim > 512:
@@ -465,6 +509,9 @@ class SeqModelConfig:
     # feed-forward is gated, a set of routed experts (with or without a shared one), or absent.
     # "joint": x += mixer(u + conv(u)) + ff(norm2(x)), u = norm1(x): both sublayers read the same x;
     # layer norms with a weight and no bias, a causal convolution of the mixer's input.
+    # "streams": several copies x_s of the residual; a sublayer reads norm(sum_s a_s x_s), norm weights
+    # stored around zero, and with its result y every copy becomes sum_s M[s, t] x_s + b_t y (a, M, b
+    # learned per sublayer); the feed-forward is gated, a set of routed experts, or absent.
     block: str = "gated"
     embed_scale: float = 1.0
     bigram: Optional[dict] = None  # {buckets, mul_prev, mul_cur}: a hashed table of token pairs added to the embedding
@@ -475,6 +522,8 @@ class SeqModelConfig:
     # stream before pass t.
     loop: Optional[dict] = None
     residual_mult: float = 1.0     # "sandwich": both residual updates are multiplied by it
+    streams: int = 1               # "streams": copies of the residual
+    logit_softcap: float = 0.0     # logits become cap tanh(z / cap) (0: they stay)
 
     @property
     def runs(self) -> List[tuple]:
@@ -543,11 +592,35 @@ class SeqModelConfig:
                     raise ValueError(f"layer {i}: layer {m.kv_from} must be an earlier attention layer that projects "
                                      "keys and values of its own, with this layer's head counts and sizes")
 
+    def _validate_streams(self) -> None:
+        if self.loop is not None or self.bigram is not None or self.tied_head:
+            raise ValueError("a 'streams' model has no repeated span, no bigram table and a head of its own")
+        if not 1 <= self.streams <= 16 or self.width > 15360 or self.logit_softcap < 0:
+            raise ValueError(f"streams {self.streams} (1..16), width {self.width} (up to 15360), logit cap {self.logit_softcap}")
+        for l in self.layers:
+            l.mixer.validate()
+            if l.mixer.kind != "parallel" or l.mixer.linear is None:
+                raise ValueError("a 'streams' model's mixers are attention beside linear attention")
+            if l.ff < 0 or (l.ff and (l.ff_act not in ("relu", "silu") or l.experts is not None)):
+                raise ValueError("a layer's feed-forward is gated (ff > 0, relu or silu) or routed experts, not both")
+            if l.experts is not None:
+                l.experts.validate()
+                if l.experts.scale_input or l.experts.shared_ff:
+                    raise ValueError("a 'streams' model's experts are weighted on their outputs and have no shared one")
+
     def validate(self) -> None:
         if self.width < 1 or self.vocab < 1 or not self.layers:
             raise ValueError("a model needs width, vocab and at least one layer")
-        if self.block not in ("gated", "postnorm", "sandwich", "joint"):
+        if self.block not in ("gated", "postnorm", "sandwich", "joint", "streams"):
             raise ValueError(f"unknown block {self.block!r}")
+        if self.block == "streams":
+            return self._validate_streams()
+        if any(l.mixer.linear is not None or (l.experts is not None and (
+                l.experts.identity or l.experts.correction or l.experts.act == "clamped_gate")) for l in self.layers):
+            raise ValueError("linear attention beside attention, identity experts, a corrected choice and clamped "
+                             "activations belong to 'streams' models")
+        if self.streams != 1 or self.logit_softcap:
+            raise ValueError("several residual streams and capped logits belong to 'streams' models")
         if self.block == "joint":
             return self._validate_joint()
         if self.block == "sandwich":
@@ -586,6 +659,17 @@ class SeqModelConfig:
             n += int(self.loop["times"]) * W
         for l in self.layers:
             m = l.mixer
+            if self.block == "streams":
+                r, ex, S = m.linear, l.experts, self.streams
+                nq, nk, nv = m.heads * m.dim, m.kv_heads * m.dim, m.kv_heads * m.vdim
+                n += 3 * W + S * (S + 2) + W * (nq + nk + nv + m.heads * m.vdim) + 2 * m.dim
+                n += (nq + nk + nv if m.qkv_bias else 0) + (m.heads if m.sink else 0) + (W * m.heads if m.head_gate else 0)
+                n += W * (2 * r.heads * r.dim + 3 * r.heads * r.vdim + r.rank) + r.heads * r.dim * (r.rank + 1) + r.vdim
+                n += W + S * (S + 2) if l.ff or ex else 0
+                n += 3 * l.ff * W
+                if ex is not None:
+                    n += ex.outputs * (W + (1 if ex.correction else 0)) + 3 * ex.experts * ex.ff * W
+                continue
             if self.block == "joint":
                 n += W + l.in_taps * W + m.heads * m.vdim * W
                 if m.kind == "mlstm":
@@ -636,7 +720,9 @@ class SeqModelConfig:
         n = 0
         for l in self.layers:
             m = l.mixer
-            if m.kind == "parallel":
+            if m.linear is not None:
+                n += 4 * m.linear.heads * m.linear.dim * m.linear.vdim
+            elif m.kind == "parallel":
                 n += 4 * (m.ssd.heads * m.ssd.state * m.ssd.vdim + (m.ssd.taps - 1) * m.ssd.conv_channels)
             elif m.kind in ("retention", "gla"):
                 n += 4 * m.heads * m.dim * m.vdim
@@ -870,9 +956,55 @@ def gufasun_config(cfg: dict, tensor_shapes: Optional[dict] = None, **overrides)
     return out
 
 
+def tovapel_config(cfg: dict, tensor_shapes: Optional[dict] = None, **overrides) -> SeqModelConfig:
+    """A Tovapel config.json: several residual streams, mixed around each sublayer; every mixer is softmax
+    attention (left: biases, q and k normed per head, no rotation, capped scores, a window that keeps the
+    first tokens, a learned sink and a gate per head) beside linear attention with a decay per key channel
+    (right), half the sum of both results normed over the width; a gated feed-forward, routed experts
+    with clamped activations among which some are the identity (the choice by corrected scores), or
+    none; capped logits and an untied head.  tensor_shapes (name -> shape) supplies the inner size of the
+    low-rank pairs."""
+    layers = []
+    for i, l in enumerate(cfg["layers"]):
+        if l["type"] != "parallel":
+            raise ValueError(f"layer {i}: unknown mixer type {l['type']!r}")
+        a, b = l["mixer"]["left"], l["mixer"]["right"]
+        mask, shape = a.get("mask") or {}, (tensor_shapes or {}).get(f"l{i}.mix.right.a1")
+        spec = MixerSpec(kind="parallel", heads=int(a["heads"]), kv_heads=int(a.get("kv_heads") or 0), dim=int(a["dim"]),
+                         vdim=int(a["vdim"]), scale=float(a["scale"]), softcap=float(a.get("softcap") or 0.0),
+                         window=int(mask.get("size") or 0), keep_first=int(mask.get("keep_first") or 0), qkv_bias=True,
+                         qk_head_norm=True, sink=True, head_gate=True,
+                         linear=LinearSpec(heads=int(b["heads"]), dim=int(b["dim"]), vdim=int(b["vdim"]),
+                                           rank=int(shape[0]) if shape is not None else int(b["rank"]), tau=float(b["tau"])))
+        mlp = l.get("mlp")
+        ff, experts = 0, None
+        if mlp:
+            mk = mlp.get("kind", "dense")
+            if mk == "dense":
+                ff = int(mlp["ff"])
+            elif mk == "moe":
+                r, ex = mlp["router"], mlp["expert"]
+                experts = ExpertsSpec(experts=int(r["experts"]), top=int(r["top"]), ff=int(ex["ff"]), score="softmax",
+                                      scale_input=False, act="clamped_gate", limit=float(ex["limit"]), correction=True,
+                                      identity=int(r.get("identity") or 0))
+            else:
+                raise ValueError(f"layer {i}: feed-forward kind {mk!r} is not supported")
+        layers.append(SeqLayerSpec(spec, ff, experts, ff_act="silu"))
+    out = SeqModelConfig(arch="tovapel", width=int(cfg["width"]), vocab=int(cfg["vocab"]), layers=layers,
+                         norm_eps=float(cfg["norm"]["eps"]), name=cfg.get("architecture", "Tovapel"), block="streams",
+                         tied_head=False, streams=int(cfg.get("streams") or 1),
+                         logit_softcap=float(cfg.get("logit_softcap") or 0.0))
+    for k, v in overrides.items():
+        if not hasattr(out, k):
+            raise ValueError(f"Unknown config parameter: {k}")
+        setattr(out, k, v)
+    out.validate()
+    return out
+
+
 # config.json "architecture" -> builder of a layer-list config
 SEQ_ARCHITECTURES = {"Puguzen": puguzen_config, "Naburax": naburax_config, "Fepopel": fepopel_config,
-                     "Zopupel": zopupel_config, "Gufasun": gufasun_config}
+                     "Zopupel": zopupel_config, "Gufasun": gufasun_config, "Tovapel": tovapel_config}
 
 
 def safetensors_shapes(path: str) -> dict:

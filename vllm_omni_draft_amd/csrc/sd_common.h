@@ -34,12 +34,13 @@ sd_pf_range sd_linear_pf_range(const void* W, int N, int K, int epi, int fp8, in
 // Applies to the next attention launch of this host thread (then forgotten); n <= 2.
 void sd_attn_prefetch_next(const sd_pf_range* r, int n);
 
-// sd_distance_softmax_attention's tiled form (sd_seqmix_joint.hip); SD_ERR_UNSUPPORTED: sizes it does
+// sd_gated_softmax_attention's tiled form (sd_seqmix_joint.hip); SD_ERR_UNSUPPORTED: sizes it does
 // not take.
 int sd_tiled_window_attention_(const float* q, int64_t ldq, const void* k_cache, const void* v_cache,
                                const int32_t* block_tables, int max_blocks, int page, int n_rows, int H,
-                               int G, int dk, int dv, int window, float scale, float softcap, const float* dist1,
-                               const float* dist2, const int32_t* entries, int n_entries, float* out, void* out_bf16,
+                               int G, int dk, int dv, int window, int keep_first, float scale, float softcap,
+                               const float* sinks, const float* dist1, const float* dist2, const float* gates,
+                               int64_t ldg, const int32_t* entries, int n_entries, float* out, void* out_bf16,
                                int64_t ldo, sd_stream_t stream);
 
 #define SD_REQUIRE(cond, code, ...)            \

@@ -1002,6 +1002,7 @@ struct SeqWs {
   // layers normed on their output
   size_t pq, qe, cqb, conv, step, decay, rlog, sel_e, sel_w, dn, moe, moe_bytes;
   size_t hc, h2b, mem, mem_bytes;   // layers whose sublayers read norms of their own
+  size_t o2, y2, y2b;               // two mixers side by side on several streams
 };
 // column offsets inside the fused input projection of a layer normed on its output
 struct PnCols {
@@ -1052,6 +1053,26 @@ JtCols jt_cols(const sd_seq_layer& l) {
   c.total = c.mix + l.ff;
   return c;
 }
+// column offsets inside the fused input projection of two mixers side by side on several streams
+struct StCols {
+  int q, k, v, rq, rk, rv, rg, a1, g, total, ld;
+};
+StCols st_cols(const sd_seq_layer& l) {
+  StCols c = {};
+  int at = 0;
+  c.q = at;  at += l.heads * l.dim;
+  c.k = at;  at += l.kv_heads * l.dim;
+  c.v = at;  at += l.kv_heads * l.vdim;
+  c.rq = at; at += l.s_heads * l.s_state;
+  c.rk = at; at += l.s_heads * l.s_state;
+  c.rv = at; at += l.s_heads * l.s_vdim;
+  c.rg = at; at += l.s_heads * l.s_vdim;
+  c.a1 = at; at += l.rank;
+  c.g = at;  at += l.heads;
+  c.total = at;
+  c.ld = (at + 15) / 16 * 16;
+  return c;
+}
 // whether a grouped-query softmax layer needs the general preparation (sd_attn_prep) rather than
 // norms per head alone (sd_qk_head_norm_append)
 inline bool general_prep(const sd_seq_layer& l) {
@@ -1081,7 +1102,8 @@ PnCols pn_cols(const sd_seq_layer& l) {
 SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
   const int W = m.d.width;
   size_t proj = 0, hk = 0, hv = 0, ff = 0, wide = 0, attn = 0;
-  size_t pq = 0, qe = 0, cq = 0, conv = 0, sh = 0, ne = 0, top = 0, moe = 0, joint = 0, mem = 0;
+  size_t pq = 0, qe = 0, cq = 0, conv = 0, sh = 0, ne = 0, top = 0, moe = 0, joint = 0, mem = 0, hv2 = 0;
+  const size_t copies = m.d.streams > 1 ? m.d.streams : 1;
   const int wr = rows < kWideRows ? rows : kWideRows;
   auto up = [](size_t& a, size_t b) { a = b > a ? b : a; };
   auto need = [&](const void* tiled, int M, int N, int K) {
@@ -1090,6 +1112,32 @@ SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
     wide = n > wide ? n : wide;
   };
   for (const sd_seq_layer& l : m.layers) {
+    if (l.block == SD_BLOCK_STREAMS) {
+      const StCols c = st_cols(l);
+      const int K1 = l.heads * l.vdim, K2 = l.s_heads * l.s_vdim;
+      up(proj, (size_t)c.ld);
+      up(hk, (size_t)l.s_heads * l.s_state);
+      up(hv, (size_t)K1);
+      up(hv2, (size_t)K2);
+      need(l.w_in_tiled, wr, c.total, W);
+      need(l.w_o_tiled, wr, W, K1);
+      need(l.out_stacked ? l.w_o_tiled : l.w_o2_tiled, wr, W, K2);
+      up(attn, sd_multimap_softmax_attention_scratch_bytes(rows, l.heads, 1, l.vdim, l.window, l.keep_first, 0, max_ctx));
+      const int ents = rows < kPlanEntries ? rows : kPlanEntries;   // (enough for any number of portions up to it)
+      up(mem, sd_decay_chunks_scratch_bytes(rows + ents, ents, l.s_heads, l.s_state, l.s_vdim));
+      if (l.ff > 0) {
+        up(proj, (size_t)2 * l.ff);
+        up(ff, (size_t)l.ff);
+        need(l.w_ff_in_tiled, wr, 2 * l.ff, W);
+        need(l.w_down_tiled, wr, W, l.ff);
+      }
+      if (l.n_experts > 0) {
+        up(ne, (size_t)l.n_experts + l.n_identity);
+        up(top, (size_t)l.top);
+        up(moe, sd_moe_experts_scratch_bytes(rows, l.top, l.n_experts, l.expert_ff, W));
+      }
+      continue;
+    }
     if (l.block == SD_BLOCK_JOINT) {
       const JtCols c = jt_cols(l);
       const int K = l.heads * l.vdim + l.ff;
@@ -1188,13 +1236,13 @@ SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
   SeqWs w;
   size_t off = 0;
   const size_t R = (size_t)rows, f = sizeof(float);
-  w.x = off;    off += al(R * W * f);
+  w.x = off;    off += al(R * copies * W * f);
   w.h = off;    off += al(R * W * f);
   w.proj = off; off += al(R * proj * f);
   w.dec = off;  off += al(R * hk * f);   // low-rank decay logits, then decays
   w.o = off;    off += al(R * hv * f);
   w.y = off;    off += al(R * hv * f);
-  w.mix = off;  off += al(R * W * f);
+  w.mix = off;  off += al(R * W * f * (hv2 > 0 ? 2 : 1));   // (two mixers' results side by side)
   w.ffo = off;  off += al(R * W * f);
   w.hout = off; off += al((size_t)no * W * f);
   // bf16 copies of the matrix products' operands, for the tiled linear kernels
@@ -1223,6 +1271,9 @@ SeqWs plan_seq(const sd_seq_model& m, int rows, int n_out, int max_ctx) {
   w.h2b = off;   off += al(R * joint * 2);
   w.mem_bytes = mem;
   w.mem = off;   off += al(mem ? mem : 16);
+  w.o2 = off;    off += al(R * hv2 * f);
+  w.y2 = off;    off += al(R * hv2 * f);
+  w.y2b = off;   off += al(R * hv2 * 2);
   w.total = off;
   return w;
 }
@@ -1258,6 +1309,25 @@ extern "C" sd_seq_model* sd_seq_model_create(const sd_seq_model_desc* desc) {
   for (int i = 0; i < desc->n_layers; ++i) {
     const sd_seq_layer& l = m->layers[i];
     const char* bad = nullptr;
+    if (l.block == SD_BLOCK_STREAMS) {
+      const bool f32 = desc->weights_f32;
+      const int K1 = l.heads * l.vdim, K2 = l.s_heads * l.s_vdim;
+      if (desc->streams < 1 || desc->streams > 16) bad = "streams outside 1..16";
+      else if (l.kind != SD_MIX_SOFTMAX_DECAY) bad = "a layer on several streams takes softmax attention beside linear attention with decays";
+      else if (i > 0 && m->layers[i - 1].block != SD_BLOCK_STREAMS) bad = "it follows a layer of another kind";
+      else if (l.heads < 1 || l.kv_heads < 1 || l.heads % l.kv_heads || l.dim < 1 || l.vdim < 1 || l.dim > 512 || l.vdim > 512 || l.window < 1 || l.keep_first < 0 || l.softcap < 0.f) bad = "attention's head counts / sizes / window / cap";
+      else if (l.s_heads < 1 || l.s_state < 1 || l.s_state > 256 || l.s_vdim < 1 || l.rank < 1 || l.rank > 1536 || !(l.tau > 0.f)) bad = "linear attention's head count / sizes / rank / tau";
+      else if (!l.norm_w || !(l.w_in || l.w_in_tiled) || !(l.w_o || l.w_o_tiled) || !l.q_norm_w || !l.k_norm_w || !l.out_norm_w || !l.out_norm2_w) bad = "a null weight";
+      else if (l.out_stacked ? K1 != K2 || (l.w_o_tiled && desc->width % 16) : !(l.w_o2 || l.w_o2_tiled) || !l.w_o_tiled != !l.w_o2_tiled) bad = "two output matrices, stacked only with equal input widths, are both tiled or neither";
+      else if (!l.k_cache || !l.v_cache || !l.state || !l.w_a2 || !l.b_a2 || !l.s_norm_w) bad = "a null cache, state or decay weight";
+      else if ((l.w_in_tiled || l.w_o_tiled || l.w_ff_in_tiled || l.w_down_tiled) && f32) bad = "tiled matrices are bf16";
+      else if ((l.w_in_tiled && desc->width % 32) || (l.w_o_tiled && (K1 % 32 || K2 % 32)) || (l.w_ff_in_tiled && desc->width % 32) || (l.w_down_tiled && l.ff % 32)) bad = "a tiled matrix needs an input width that is a multiple of 32";
+      else if (!l.hc_in || !l.hc_out || !l.hc_mix) bad = "the mixer's stream factors";
+      else if (l.ff < 0 || (l.ff > 0 && (l.n_experts > 0 || l.ff_act < 0 || l.ff_act > 1 || !(l.w_ff_in || l.w_ff_in_tiled) || !(l.w_down || l.w_down_tiled)))) bad = "a dense feed-forward needs its two matrices and a gated activation, and excludes experts";
+      else if (l.n_experts > 0 && (l.n_identity < 0 || l.top < 1 || l.top > l.n_experts + l.n_identity || l.expert_ff < 1 || !l.w_router || !l.w_gate_up || !l.w_down_e || l.expert_act < 0 || l.expert_act > 2 || l.expert_scale_input)) bad = "routed experts need top <= experts, their matrices, a known activation and weighted outputs";
+      else if ((l.ff > 0 || l.n_experts > 0) && (!l.norm2_w || !l.hc2_in || !l.hc2_out || !l.hc2_mix)) bad = "a feed-forward needs its norm and stream factors";
+      else if (desc->width > 15360) bad = "a width above 15360";
+    } else
     if (l.block == SD_BLOCK_JOINT) {
       const bool f32 = desc->weights_f32;
       if (l.kind != SD_MIX_SOFTMAX && l.kind != SD_MIX_MLSTM) bad = "a layer whose sublayers read the same residual takes grouped-query softmax attention or a matrix memory";
@@ -1660,6 +1730,146 @@ int joint_layer(const sd_seq_model& m, const sd_seq_layer& l, const sd_seq_batch
   return seq_linear(l.w_o, l.w_o_tiled, f32, y, nullptr, K, yb, K, nullptr, (float*)(base + w.mix), W, R, W, K, wide_ws,
                     w.wide_bytes, stream);
 }
+
+// The wanted rows' logits from their final norm (hout / houtb).
+int head_logits(const sd_seq_model& m, const sd_seq_batch& b, char* base, const SeqWs& w, sd_stream_t stream) {
+  const sd_seq_model_desc& d = m.d;
+  const int W = d.width;
+  SQ_TRY(seq_linear(d.head ? d.head : d.embed, d.head_tiled, d.weights_f32, (float*)(base + w.hout), nullptr, W,
+                    base + w.houtb, W, nullptr, b.logits, d.vocab, b.n_out, d.vocab, W, base + w.wide, w.wide_bytes,
+                    stream));
+  if (d.logit_scale != 0.f && d.logit_scale != 1.f)
+    SQ_TRY(sd_scale_rows(b.logits, d.vocab, d.logit_scale, b.n_out, d.vocab, stream));
+  if (d.logit_softcap > 0.f) SQ_TRY(sd_cap_rows(b.logits, d.vocab, d.logit_softcap, b.n_out, d.vocab, stream));
+  return SD_OK;
+}
+
+// Where a layer on several streams leaves the next sublayer's input: the next layer's mixer, or nothing
+// behind the last layer (the final norm reads the streams themselves).
+void next_input(const sd_seq_layer* next, sd_streams_update* u) {
+  u->in = next ? next->hc_in : nullptr;
+  u->w_next = next ? next->norm_w : nullptr;
+}
+
+// One layer on several streams.  On entry h / hb hold the mixer's input.  On return the streams hold
+// the layer's result and h / hb the next layer's input, unless *last is set: then what the layer's last
+// sublayer left waits in *last, and the final norm applies it to the rows it reads.
+int streams_layer(const sd_seq_model& m, const sd_seq_layer& l, const sd_seq_layer* next, const sd_seq_batch& b,
+                  char* base, const SeqWs& w, float* x_copy, sd_streams_update* last, sd_stream_t stream) {
+  const sd_seq_model_desc& d = m.d;
+  const int W = d.width, R = b.n_rows, f32 = d.weights_f32, rnd = !f32;
+  const float eps = d.norm_eps;
+  float* h = (float*)(base + w.h);
+  float* proj = (float*)(base + w.proj);
+  float* mix = (float*)(base + w.mix);
+  bf16_t* hb = (bf16_t*)(base + w.hb);
+  bf16_t* yb = (bf16_t*)(base + w.yb);
+  bf16_t* y2b = (bf16_t*)(base + w.y2b);
+  float* y2 = (float*)(base + w.y2);
+  void* wide_ws = base + w.wide;
+  const StCols c = st_cols(l);
+  const int64_t ld = c.ld;
+  const int H = l.heads, G = l.kv_heads, dk = l.dim, dv = l.vdim, Hs = l.s_heads, N = l.s_state, P = l.s_vdim;
+  const int K1 = H * dv, K2 = Hs * P;
+  const bool tiled = l.w_o_tiled != nullptr, single = R == b.n_entries;
+  float* o = tiled ? nullptr : (float*)(base + w.o);
+  const size_t es = f32 ? sizeof(float) : sizeof(bf16_t);
+  SQ_TRY(seq_linear(l.w_in, l.w_in_tiled, f32, h, nullptr, W, hb, W, nullptr, proj, ld, R, c.total, W, wide_ws,
+                    w.wide_bytes, stream));
+  // attention's inputs; a decoding step moves the linear attention's states on, and reads them, in the same launch
+  const char* bias = (const char*)l.w_in_bias;
+  sd_decay_step step = {proj + c.rq, proj + c.rk, proj + c.rv, proj + c.a1, proj + c.rg, ld, l.w_a2, l.b_a2, l.rank, l.tau,
+                        l.q_scale, l.state, l.s_norm_w, tiled ? nullptr : y2, tiled ? (void*)y2b : nullptr, K2, Hs, N, P};
+  SQ_TRY(sd_biased_qkv_prep(proj + c.q, proj + c.k, proj + c.v, ld, bias ? bias + (size_t)c.q * es : nullptr,
+                            bias ? bias + (size_t)c.k * es : nullptr, bias ? bias + (size_t)c.v * es : nullptr, H, G, dk,
+                            dv, l.q_norm_w, l.k_norm_w, f32, eps, l.k_cache, l.v_cache, b.row_pos, b.row_slot,
+                            b.block_tables, b.max_blocks, b.page, R, single ? &step : nullptr, stream));
+  SQ_TRY(sd_gated_softmax_attention(proj + c.q, ld, l.k_cache, l.v_cache, f32, b.row_pos, b.row_slot, b.block_tables,
+                                    b.max_blocks, b.page, R, H, G, 1, dk, dv, l.window, l.keep_first, 0, l.score_scale,
+                                    l.softcap, l.sinks, nullptr, nullptr, l.head_gate ? proj + c.g : nullptr, ld,
+                                    b.entries, b.n_entries, o, tiled ? yb : nullptr, K1, base + w.attn, w.attn_bytes,
+                                    stream));
+  if (!single) {
+    float* dec = (float*)(base + w.dec);
+    float* o2 = (float*)(base + w.o2);
+    SQ_TRY(sd_low_rank_decay(proj + c.a1, ld, l.w_a2, l.b_a2, f32, l.rank, l.tau, dec, R, Hs * N, stream));
+    SQ_TRY(sd_decay_chunks(proj + c.rq, proj + c.rk, proj + c.rv, ld, dec, l.q_scale, l.state, b.entries, b.n_entries, R,
+                           o2, Hs, N, P, base + w.mem, w.mem_bytes, stream));
+    SQ_TRY(sd_head_post(o2, proj + c.rg, ld, l.s_norm_w, f32, 1, eps, 0, y2, tiled ? y2b : nullptr, R, Hs, P, rnd, stream));
+  }
+  // both output matrices: one launch for a few rows where they are stacked
+  if (l.out_stacked && tiled && R <= 16) {
+    SQ_TRY(sd_linear_two_inputs(l.w_o_tiled, yb, y2b, K1, W, mix, 2 * (int64_t)W, R, 2 * W, K1, stream));
+  } else {
+    const void* w2 = l.w_o2;
+    const void* w2_t = l.w_o2_tiled;
+    if (l.out_stacked) {
+      w2 = l.w_o ? (const char*)l.w_o + (size_t)W * K1 * es : nullptr;
+      w2_t = tiled ? (const char*)l.w_o_tiled + (size_t)W * K1 * sizeof(bf16_t) : nullptr;
+    }
+    SQ_TRY(seq_linear(l.w_o, l.w_o_tiled, f32, o, nullptr, K1, yb, K1, nullptr, mix, 2 * (int64_t)W, R, W, K1, wide_ws,
+                      w.wide_bytes, stream));
+    SQ_TRY(seq_linear(w2, w2_t, f32, y2, nullptr, K2, y2b, K2, nullptr, mix + W, 2 * (int64_t)W, R, W, K2, wide_ws,
+                      w.wide_bytes, stream));
+  }
+  sd_streams_update u = {};
+  u.x = (float*)(base + w.x);
+  u.streams = d.streams;
+  u.h = h;
+  u.h_bf16 = hb;
+  u.a = mix;
+  u.b = mix + W;
+  u.lda = 2 * (int64_t)W;
+  u.n_a = 1;
+  u.w_a = l.out_norm_w;
+  u.w_b = l.out_norm2_w;
+  u.mix = l.hc_mix;
+  u.out = l.hc_out;
+  if (l.ff > 0 || l.n_experts > 0) {
+    u.in = l.hc2_in;
+    u.w_next = l.norm2_w;
+    SQ_TRY(sd_streams_residual(&u, f32, eps, R, W, rnd, stream));
+    u.b = nullptr;
+    u.lda = W;
+    u.mix = l.hc2_mix;
+    u.out = l.hc2_out;
+  }
+  if (l.ff > 0) {
+    const int F = l.ff;
+    float* ffo = (float*)(base + w.ffo);
+    bf16_t* actb = (bf16_t*)(base + w.actb);
+    SQ_TRY(seq_linear(l.w_ff_in, l.w_ff_in_tiled, f32, h, nullptr, W, hb, W, nullptr, proj, 2 * (int64_t)F, R, 2 * F, W,
+                      wide_ws, w.wide_bytes, stream));
+    SQ_TRY(sd_act_rows(proj, proj + F, 2 * (int64_t)F, l.w_down_tiled ? nullptr : proj, 2 * (int64_t)F,
+                       l.w_down_tiled ? actb : nullptr, F, R, F, l.ff_act, rnd, stream));
+    SQ_TRY(seq_linear(l.w_down, l.w_down_tiled, f32, proj, nullptr, 2 * (int64_t)F, actb, F, nullptr, ffo, W, R, W, F,
+                      wide_ws, w.wide_bytes, stream));
+    u.a = ffo;
+  } else if (l.n_experts > 0) {
+    int32_t* sel_e = (int32_t*)(base + w.sel_e);
+    float* sel_w = (float*)(base + w.sel_w);
+    float* dn = (float*)(base + w.dn);
+    SQ_TRY(sd_moe_route_rows_corrected(h, W, l.w_router, l.router_bias, l.route_correction, f32, (float*)(base + w.rlog),
+                                       sel_e, sel_w, R, l.n_experts + l.n_identity, W, l.top, l.route_score,
+                                       l.route_renorm, l.route_renorm_eps, l.route_scale != 0.f ? l.route_scale : 1.f,
+                                       nullptr, 0, nullptr, stream));
+    SQ_TRY(sd_moe_experts_clamped(h, hb, W, sel_e, sel_w, l.w_gate_up, l.w_down_e, f32, dn, R, l.top, l.n_experts,
+                                  l.expert_ff, W, 0, l.expert_act, l.expert_limit, base + w.moe, w.moe_bytes, stream));
+    u.a = dn;
+    u.n_a = l.top;
+    u.sel_expert = sel_e;
+    u.sel_weight = sel_w;
+    u.n_experts = l.n_experts;
+    u.input = h;
+  }
+  u.x_copy = x_copy;
+  next_input(next, &u);
+  if (!next && !x_copy) {
+    *last = u;
+    return SD_OK;
+  }
+  return sd_streams_residual(&u, f32, eps, R, W, rnd, stream);
+}
 }  // namespace
 
 extern "C" int sd_seq_model_forward(sd_seq_model* m, const sd_seq_batch* b, void* workspace,
@@ -1693,6 +1903,31 @@ extern "C" int sd_seq_model_forward(sd_seq_model* m, const sd_seq_batch* b, void
   bf16_t* houtb = (bf16_t*)(base + w.houtb);
   void* wide_ws = base + w.wide;
 
+  sd_streams_update last = {};   // (models on several streams: what the last layer leaves to the final norm)
+  if (m->layers[0].block == SD_BLOCK_STREAMS) {
+    last.x = x;
+    last.streams = d.streams;
+    sd_streams_update u = last;
+    u.tokens = b->tokens;
+    u.embed = d.embed;
+    u.vocab = d.vocab;
+    u.h = h;
+    u.h_bf16 = hb;
+    next_input(&m->layers[0], &u);
+    SQ_TRY(sd_streams_residual(&u, f32, d.norm_eps, R, W, rnd, stream));
+    for (int li = 0; li < d.n_layers; ++li)
+      SQ_TRY(streams_layer(*m, m->layers[li], li + 1 < d.n_layers ? &m->layers[li + 1] : nullptr, *b, base, w,
+                           b->layer_out ? b->layer_out + (size_t)li * R * W : nullptr, &last, stream));
+    if (b->n_out > 0) {
+      last.rows = b->out_rows;
+      last.w_next = d.final_norm_w;
+      last.h = hout;
+      last.h_bf16 = houtb;
+      SQ_TRY(sd_streams_residual(&last, f32, d.norm_eps, b->n_out, W, rnd, stream));
+      return head_logits(*m, *b, base, w, stream);
+    }
+    return SD_OK;
+  }
   const bool hashed = d.bigram || (d.embed_scale != 0.f && d.embed_scale != 1.f) || m->layers[0].block != SD_BLOCK_GATED;
   if (hashed) {
     SD_REQUIRE(!d.bigram || b->prev_tokens, SD_ERR_INVALID, "sd_seq_model_forward: a bigram table needs prev_tokens");
@@ -1804,10 +2039,7 @@ extern "C" int sd_seq_model_forward(sd_seq_model* m, const sd_seq_batch* b, void
     else
       SQ_TRY(sd_rmsnorm_rows(x, b->out_rows, d.final_norm_w, f32, d.plain_norm ? 0.f : 1.f, d.norm_eps, hout,
                              d.head_tiled ? houtb : nullptr, b->n_out, W, stream));
-    SQ_TRY(seq_linear(d.head ? d.head : d.embed, d.head_tiled, f32, hout, nullptr, W, houtb, W, nullptr, b->logits,
-                      d.vocab, b->n_out, d.vocab, W, wide_ws, w.wide_bytes, stream));
-    if (d.logit_scale != 0.f && d.logit_scale != 1.f)
-      SQ_TRY(sd_scale_rows(b->logits, d.vocab, d.logit_scale, b->n_out, d.vocab, stream));
+    SQ_TRY(head_logits(*m, *b, base, w, stream));
   }
   return SD_OK;
 }

@@ -198,6 +198,7 @@ __device__ __forceinline__ void score_key(const KT_* __restrict__ kr, const floa
 // n_splits > 1 (few rows): workgroup (.., .., z) takes tile z / n_hgroups of the row's keys only
 // and leaves its maximum, its sum of weights and its unnormalised weighted values in part_ml /
 // part_acc; softmax_merge_kernel puts a row's tiles together in tile order.
+// gates [rows, units] (or nullptr): a unit's output is multiplied by sigmoid of its gate.
 // dist1 / dist2 (per unit, or nullptr): a score, capped already, loses dist1 ln(1 + dist2 (i - j)).
 // maps > 1: a head holds `maps` queries of dk channels (unit h * maps + m of a row of q), the key
 // cache `maps` key rows per kv head (cache head g * maps + m), and every map reads the kv head's
@@ -210,7 +211,7 @@ __global__ __launch_bounds__(256) void window_softmax_attn_kernel(
     int keep_first, float scale, float* __restrict__ out, bf16_t* __restrict__ out_b, int n_hgroups, int n_splits,
     float* __restrict__ part_acc, float* __restrict__ part_ml, int chunk, float softcap,
     const float* __restrict__ sinks, int maps, const float* __restrict__ dist1, const float* __restrict__ dist2,
-    int64_t ldo) {
+    int64_t ldo, const float* __restrict__ gates, int64_t ldg) {
   extern __shared__ float lds[];
   constexpr int nthr = 256, nw = 4, PARTS = nthr / KT, KW = KT / 64;
   unsigned long long* vat = reinterpret_cast<unsigned long long*>(lds);  // [KT] cache row of the key
@@ -371,7 +372,8 @@ __global__ __launch_bounds__(256) void window_softmax_attn_kernel(
         if (lane + 64 * m < dv) red[wave * dv + lane + 64 * m] = acc[hq][m];
       __syncthreads();
       // (no key and no sink: a row past its own keys, which a cut launch's merge skips)
-      const float inv = n_splits > 1 ? 1.f : 1.f / l_run[hq];
+      float inv = n_splits > 1 ? 1.f : 1.f / l_run[hq];
+      if (gates && n_splits == 1) inv *= sigmoid_f(gates[(size_t)r * ldg + h0 + hq * maps]);
       for (int c = tid; c < dv; c += nthr) {
         float o = red[c];
 #pragma unroll
@@ -395,13 +397,14 @@ __global__ __launch_bounds__(256) void window_softmax_attn_kernel(
   }
 }
 
-// out[r, h] = sum_s acc_s exp(m_s - M) / sum_s l_s exp(m_s - M), M = max m_s.  The first wave takes
+// out[r, h] = sum_s acc_s exp(m_s - M) / sum_s l_s exp(m_s - M), M = max m_s (times the head's gate,
+// sigmoid(gates[r, h]), where there is one).  The first wave takes
 // the tiles' maxima and sums a lane per tile (butterfly sums: a fixed order) and leaves every
 // tile's factor in LDS; then a thread per column adds the tiles' rows in tile order, eight loads
 // in flight.
 __global__ void softmax_merge_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
                                      int n_splits, float* __restrict__ out, bf16_t* __restrict__ out_b, int H, int dv,
-                                     int64_t ldo) {
+                                     int64_t ldo, const float* __restrict__ gates, int64_t ldg) {
   extern __shared__ float fac[];   // [n_splits]
   __shared__ float inv_l;
   const int r = blockIdx.x, h = blockIdx.y, R = gridDim.x, tid = threadIdx.x;
@@ -419,7 +422,7 @@ __global__ void softmax_merge_kernel(const float* __restrict__ part_acc, const f
       L += ml[1] * f;
     }
     L = wave_sum(L);
-    if (tid == 0) inv_l = 1.f / L;
+    if (tid == 0) inv_l = (gates ? sigmoid_f(gates[(size_t)r * ldg + h]) : 1.f) / L;
   }
   __syncthreads();
   constexpr int kU = 8;
@@ -452,13 +455,13 @@ void launch_softmax_nc(dim3 grid, int kt, size_t lds, hipStream_t st, int nc, co
                        const int32_t* bt, int max_blocks, int page, int H, int G, int dk, int dv, int window,
                        int keep_first, float scale, float* out, bf16_t* out_b, int n_hgroups, int n_splits,
                        float* part_acc, float* part_ml, int chunk, float softcap, const float* sinks, int maps,
-                       const float* dist1, const float* dist2, int64_t ldo) {
+                       const float* dist1, const float* dist2, int64_t ldo, const float* gates, int64_t ldg) {
 #define SD_GO2(NC, KT)                                                                                               \
   window_softmax_attn_kernel<T, NH, NC, KT><<<grid, 256, lds, st>>>(q, ldq, (const T*)kc, (const T*)vc, v_row, row_pos, \
                                                                     row_slot, bt, max_blocks, page, H, G, dk, dv,       \
                                                                     window, keep_first, scale, out, out_b, n_hgroups,   \
                                                                     n_splits, part_acc, part_ml, chunk, softcap, sinks, \
-                                                                    maps, dist1, dist2, ldo)
+                                                                    maps, dist1, dist2, ldo, gates, ldg)
 #define SD_GO(NC)                                          \
   do {                                                     \
     if constexpr (NH <= 4) {                               \
@@ -974,7 +977,8 @@ __global__ void moe_route_kernel(const float* __restrict__ logits, int64_t ld, i
 
 // The router's product and the choice in one launch: a workgroup per row, a wave per expert
 // (lanes stride over the row's channels, then a butterfly sum: an order that no other row
-// changes), then the first wave chooses as moe_route_kernel does.
+// changes), then the first wave chooses as moe_route_kernel does; with a correction [E] the choice is
+// made by score + correction, the weight is the score.
 template <typename T>
 __global__ __launch_bounds__(1024) void moe_route_rows_kernel(const float* __restrict__ x, int64_t ldx,
                                                              const T* __restrict__ w, float* __restrict__ logits,
@@ -983,7 +987,8 @@ __global__ __launch_bounds__(1024) void moe_route_rows_kernel(const float* __res
                                                              int round, float renorm_eps, float weight_scale,
                                                              const T* __restrict__ w_gate, int n_gate,
                                                              float* __restrict__ gate_out,
-                                                             const float* __restrict__ bias) {
+                                                             const float* __restrict__ bias,
+                                                             const float* __restrict__ correction) {
   extern __shared__ float sc[];   // [E]
   const int r = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
   const float* xr = x + (size_t)r * ldx;
@@ -1037,7 +1042,7 @@ __global__ __launch_bounds__(1024) void moe_route_rows_kernel(const float* __res
     float best = -INFINITY;
     int bi = 0x7fffffff;
     for (int e = lane; e < E; e += 64) {
-      const float v = sc[e];
+      const float v = correction ? sc[e] + correction[e] : sc[e];   // (the choice alone sees the correction)
       if (v > best) {
         best = v;
         bi = e;
@@ -1052,10 +1057,11 @@ __global__ __launch_bounds__(1024) void moe_route_rows_kernel(const float* __res
         bi = oi;
       }
     }
+    if (correction) best = sc[bi < E ? bi : 0];
     if (lane == 0) {
       sel_e[(size_t)r * top + j] = bi;
       sel_w[(size_t)r * top + j] = best;
-      sc[bi] = -INFINITY;
+      sc[bi < E ? bi : 0] = -INFINITY;
     }
     total += best;
   }
@@ -1067,8 +1073,13 @@ __global__ __launch_bounds__(1024) void moe_route_rows_kernel(const float* __res
 }
 
 // An expert's activation from its (scaled) first product a and, when gated, its second product u:
-// kind 0 silu(a) u; kind 1 relu(a)^2, an expert of two matrices only.
-__device__ __forceinline__ float expert_act(float a, float u, int kind) {
+// kind 0 silu(a) u; kind 1 relu(a)^2, an expert of two matrices only; kind 2 g sigmoid(1.702 g) (c + 1)
+// of g = min(a, limit) and c = u clamped to +-limit.
+__device__ __forceinline__ float expert_act(float a, float u, int kind, float limit) {
+  if (kind == 2) {
+    const float g = fminf(a, limit), c = fminf(fmaxf(u, -limit), limit);
+    return g * sigmoid_f(1.702f * g) * (c + 1.f);
+  }
   if (kind == 1) {
     const float p = fmaxf(a, 0.f);
     return p * p;
@@ -1132,9 +1143,9 @@ template <typename T>
 __global__ __launch_bounds__(256) void moe_gate_up_kernel(
     const float* __restrict__ X, int64_t ldx, const int32_t* __restrict__ perm, const int32_t* __restrict__ tiles,
     const int32_t* __restrict__ n_tiles, const float* __restrict__ sel_w, const T* __restrict__ Wgu,
-    float* __restrict__ act, int top, int F, int K, int scale_input, int round, int act_kind) {
+    float* __restrict__ act, int top, int E, int F, int K, int scale_input, int round, int act_kind, float limit) {
   constexpr int BM = kMoeBM, BN = 64, BK = 16, TM = 2, TN = 4;
-  const bool gated = act_kind == 0;   // (else Wgu holds one matrix [F, K] per expert)
+  const bool gated = act_kind != 1;   // (else Wgu holds one matrix [F, K] per expert)
   if (tiles && (int)blockIdx.y >= n_tiles[0]) return;
   __shared__ float xs[BK][BM + 1];
   __shared__ float wg[BK][BN + 1];
@@ -1142,6 +1153,7 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(
   __shared__ int arow[BM];
   // (tiles == nullptr: assignment blockIdx.y alone, perm is then the chosen experts themselves)
   const int e = tiles ? tiles[3 * blockIdx.y] : perm[blockIdx.y];
+  if ((unsigned)e >= (unsigned)E) return;   // (not one of these experts: its row is not written)
   const int p0 = tiles ? tiles[3 * blockIdx.y + 1] : blockIdx.y, rows = tiles ? tiles[3 * blockIdx.y + 2] : 1;
   const int tid = threadIdx.x, tx = tid % (BN / TN), ty = tid / (BN / TN);
   const int n0 = blockIdx.x * BN;
@@ -1195,7 +1207,7 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(
 #pragma unroll
     for (int j = 0; j < TN; ++j) {
       const int n = n0 + tx * TN + j;
-      if (n < F) act[(size_t)a * F + n] = maybe_round(expert_act(s * ag[i][j], s * au[i][j], act_kind), round);
+      if (n < F) act[(size_t)a * F + n] = maybe_round(expert_act(s * ag[i][j], s * au[i][j], act_kind, limit), round);
     }
   }
 }
@@ -1205,7 +1217,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void moe_down_kernel(
     const float* __restrict__ act, const int32_t* __restrict__ perm, const int32_t* __restrict__ tiles,
     const int32_t* __restrict__ n_tiles, const float* __restrict__ sel_w, const T* __restrict__ Wd,
-    float* __restrict__ out, int N, int K, int scale_input) {
+    float* __restrict__ out, int E, int N, int K, int scale_input) {
   constexpr int BM = kMoeBM, BN = 64, BK = 16, TM = 2, TN = 4;
   if (tiles && (int)blockIdx.y >= n_tiles[0]) return;
   __shared__ float xs[BK][BM + 1];
@@ -1213,6 +1225,7 @@ __global__ __launch_bounds__(256) void moe_down_kernel(
   __shared__ int arow[BM];
   // (tiles == nullptr: assignment blockIdx.y alone, perm is then the chosen experts themselves)
   const int e = tiles ? tiles[3 * blockIdx.y] : perm[blockIdx.y];
+  if ((unsigned)e >= (unsigned)E) return;   // (not one of these experts: its row is not written)
   const int p0 = tiles ? tiles[3 * blockIdx.y + 1] : blockIdx.y, rows = tiles ? tiles[3 * blockIdx.y + 2] : 1;
   const int tid = threadIdx.x, tx = tid % (BN / TN), ty = tid / (BN / TN);
   const int n0 = blockIdx.x * BN;
@@ -1277,13 +1290,15 @@ template <int MT, int KC, bool GATED>
 __global__ __launch_bounds__(256) void moe_gate_up_mfma_kernel(
     const float* __restrict__ X, const bf16_t* __restrict__ Xb, int64_t ldx, const int32_t* __restrict__ perm,
     const int32_t* __restrict__ tiles, const int32_t* __restrict__ n_tiles, const float* __restrict__ sel_w,
-    const bf16_t* __restrict__ Wgu, bf16_t* __restrict__ act, int top, int F, int K, int scale_input) {
+    const bf16_t* __restrict__ Wgu, bf16_t* __restrict__ act, int top, int E, int F, int K, int scale_input, int act_kind,
+    float limit) {
   if (tiles && (int)blockIdx.y >= n_tiles[0]) return;
   constexpr int BM = 16 * MT, LD = KC + 8;   // LDS row stride: 16 rows at one k fall into distinct banks
   __shared__ __attribute__((aligned(16))) bf16_t xs[BM * LD];
   __shared__ int arow[BM];
   // (tiles == nullptr: assignment blockIdx.y alone, perm is then the chosen experts themselves)
   const int e = tiles ? tiles[3 * blockIdx.y] : perm[blockIdx.y];
+  if ((unsigned)e >= (unsigned)E) return;   // (not one of these experts: its row is not written)
   const int p0 = tiles ? tiles[3 * blockIdx.y + 1] : blockIdx.y, rows = tiles ? tiles[3 * blockIdx.y + 2] : 1;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, lr = lane & 15, kq = lane >> 4;
   const int n0 = blockIdx.x * 128 + wave * 32 + lr, n1 = n0 + 16;
@@ -1351,8 +1366,8 @@ __global__ __launch_bounds__(256) void moe_gate_up_mfma_kernel(
       const int a = arow[mt * 16 + 4 * kq + i];
       if (a < 0) continue;
       const float sc = scale_input ? sel_w[a] : 1.f;
-      if (n0 < F) act[(size_t)a * F + n0] = (bf16_t)expert_act(sc * ag[mt][0][i], sc * au[mt][0][i], GATED ? 0 : 1);
-      if (n1 < F) act[(size_t)a * F + n1] = (bf16_t)expert_act(sc * ag[mt][1][i], sc * au[mt][1][i], GATED ? 0 : 1);
+      if (n0 < F) act[(size_t)a * F + n0] = (bf16_t)expert_act(sc * ag[mt][0][i], sc * au[mt][0][i], act_kind, limit);
+      if (n1 < F) act[(size_t)a * F + n1] = (bf16_t)expert_act(sc * ag[mt][1][i], sc * au[mt][1][i], act_kind, limit);
     }
 }
 
@@ -1361,12 +1376,13 @@ template <int MT, int KC>
 __global__ __launch_bounds__(256) void moe_down_mfma_kernel(
     const bf16_t* __restrict__ act, const int32_t* __restrict__ perm, const int32_t* __restrict__ tiles,
     const int32_t* __restrict__ n_tiles, const float* __restrict__ sel_w, const bf16_t* __restrict__ Wd,
-    float* __restrict__ out, int N, int K, int scale_input) {
+    float* __restrict__ out, int E, int N, int K, int scale_input) {
   if (tiles && (int)blockIdx.y >= n_tiles[0]) return;
   constexpr int BM = 16 * MT, LD = KC + 8;
   __shared__ __attribute__((aligned(16))) bf16_t xs[BM * LD];
   __shared__ int arow[BM];
   const int e = tiles ? tiles[3 * blockIdx.y] : perm[blockIdx.y];
+  if ((unsigned)e >= (unsigned)E) return;   // (not one of these experts: its row is not written)
   const int p0 = tiles ? tiles[3 * blockIdx.y + 1] : blockIdx.y, rows = tiles ? tiles[3 * blockIdx.y + 2] : 1;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, lr = lane & 15, kq = lane >> 4;
   const int n0 = blockIdx.x * 128 + wave * 32 + lr, n1 = n0 + 16;
@@ -1424,9 +1440,11 @@ constexpr int kGemvMaxK = 8192;
 template <bool GATED>
 __global__ __launch_bounds__(256) void moe_gemv_gate_up_kernel(
     const float* __restrict__ X, int64_t ldx, const int32_t* __restrict__ sel_e, const float* __restrict__ sel_w,
-    const bf16_t* __restrict__ Wgu, bf16_t* __restrict__ act, int top, int F, int K, int scale_input) {
+    const bf16_t* __restrict__ Wgu, bf16_t* __restrict__ act, int top, int E, int F, int K, int scale_input, int act_kind,
+    float limit) {
   extern __shared__ float xs[];   // [K]
   const int a = blockIdx.y, e = sel_e[a], tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  if ((unsigned)e >= (unsigned)E) return;   // (not one of these experts)
   const float* xr = X + (size_t)(a / top) * ldx;
   for (int k = tid; k < K; k += 256) xs[k] = round_bf16(xr[k]);
   __syncthreads();
@@ -1473,12 +1491,12 @@ __global__ __launch_bounds__(256) void moe_gemv_gate_up_kernel(
   if (lane == 0) {
     const float sc = scale_input ? sel_w[a] : 1.f;
     if constexpr (GATED) {
-      act[(size_t)a * F + n0] = (bf16_t)expert_act(sc * acc[0], sc * acc[1], 0);
-      if (n0 + 1 < F) act[(size_t)a * F + n0 + 1] = (bf16_t)expert_act(sc * acc[2], sc * acc[3], 0);
+      act[(size_t)a * F + n0] = (bf16_t)expert_act(sc * acc[0], sc * acc[1], act_kind, limit);
+      if (n0 + 1 < F) act[(size_t)a * F + n0 + 1] = (bf16_t)expert_act(sc * acc[2], sc * acc[3], act_kind, limit);
     } else {
 #pragma unroll
       for (int j = 0; j < 4; ++j)
-        if (n0 + j < F) act[(size_t)a * F + n0 + j] = (bf16_t)expert_act(sc * acc[j], 0.f, 1);
+        if (n0 + j < F) act[(size_t)a * F + n0 + j] = (bf16_t)expert_act(sc * acc[j], 0.f, 1, limit);
     }
   }
 }
@@ -1486,9 +1504,10 @@ __global__ __launch_bounds__(256) void moe_gemv_gate_up_kernel(
 // out[a, n] = down_e[n] . act[a]; wave: four columns.
 __global__ __launch_bounds__(256) void moe_gemv_down_kernel(
     const bf16_t* __restrict__ act, const int32_t* __restrict__ sel_e, const float* __restrict__ sel_w,
-    const bf16_t* __restrict__ Wd, float* __restrict__ out, int N, int K, int scale_input) {
+    const bf16_t* __restrict__ Wd, float* __restrict__ out, int E, int N, int K, int scale_input) {
   extern __shared__ float xs[];   // [K]
   const int a = blockIdx.y, e = sel_e[a], tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  if ((unsigned)e >= (unsigned)E) return;   // (not one of these experts)
   for (int k = tid; k < K; k += 256) xs[k] = (float)act[(size_t)a * K + k];
   __syncthreads();
   const int n0 = blockIdx.x * 16 + wave * 4;
@@ -1979,9 +1998,24 @@ extern "C" int sd_distance_softmax_attention(const float* q, int64_t ldq, const 
                                              const float* dist2, const int32_t* entries, int n_entries, float* out,
                                              void* out_bf16, int64_t ldo, void* scratch, size_t scratch_bytes,
                                              sd_stream_t stream) {
+  return sd_gated_softmax_attention(q, ldq, k_cache, v_cache, cache_f32, row_pos, row_slot, block_tables, max_blocks,
+                                    page, n_rows, H, G, maps, dk, dv, window, keep_first, chunk, scale, softcap, sinks,
+                                    dist1, dist2, nullptr, 0, entries, n_entries, out, out_bf16, ldo, scratch,
+                                    scratch_bytes, stream);
+}
+
+extern "C" int sd_gated_softmax_attention(const float* q, int64_t ldq, const void* k_cache, const void* v_cache,
+                                          int cache_f32, const int32_t* row_pos, const int32_t* row_slot,
+                                          const int32_t* block_tables, int max_blocks, int page, int n_rows, int H,
+                                          int G, int maps, int dk, int dv, int window, int keep_first, int chunk,
+                                          float scale, float softcap, const float* sinks, const float* dist1,
+                                          const float* dist2, const float* gates, int64_t ldg, const int32_t* entries,
+                                          int n_entries, float* out, void* out_bf16, int64_t ldo, void* scratch,
+                                          size_t scratch_bytes, sd_stream_t stream) {
   SD_REQUIRE(q && k_cache && row_pos && row_slot && block_tables && (out || out_bf16) && !dist1 == !dist2, SD_ERR_INVALID,
              "sd_masked_softmax_attention: null argument");
   SD_REQUIRE(ldo >= (int64_t)H * maps * dv, SD_ERR_INVALID, "sd_masked_softmax_attention: output rows too short");
+  SD_REQUIRE(!gates || ldg >= (int64_t)H * maps, SD_ERR_INVALID, "sd_gated_softmax_attention: gate rows too short");
   SD_REQUIRE(n_rows >= 1 && H >= 1 && G >= 1 && H % G == 0 && dk >= 1 && window >= 1 && keep_first >= 0 && page >= 1 &&
                  chunk >= 0 && softcap >= 0.f && maps >= 1 && (maps == 1 || v_cache) &&
                  ldq >= (int64_t)H * maps * dk,
@@ -1989,10 +2023,10 @@ extern "C" int sd_distance_softmax_attention(const float* q, int64_t ldq, const 
   SD_REQUIRE(dv >= 1 && dv <= 512 && (v_cache || dv <= dk), SD_ERR_UNSUPPORTED,
              "sd_masked_softmax_attention: value size %d outside 1..512 (or above the key row it is part of)", dv);
   hipStream_t st = (hipStream_t)stream;
-  if (entries && !cache_f32 && n_rows > kSplitRows && maps == 1 && !sinks && keep_first == 0 && chunk == 0 && v_cache) {
+  if (entries && !cache_f32 && n_rows > kSplitRows && maps == 1 && chunk == 0 && v_cache) {
     const int rc = sd_tiled_window_attention_(q, ldq, k_cache, v_cache, block_tables, max_blocks, page, n_rows,
-                                              H, G, dk, dv, window, scale, softcap, dist1, dist2, entries, n_entries, out,
-                                              out_bf16, ldo, stream);
+                                              H, G, dk, dv, window, keep_first, scale, softcap, sinks, dist1, dist2, gates,
+                                              ldg, entries, n_entries, out, out_bf16, ldo, stream);
     if (rc != SD_ERR_UNSUPPORTED) return rc;
   }
   const int qh = H / G;
@@ -2020,7 +2054,7 @@ extern "C" int sd_distance_softmax_attention(const float* q, int64_t ldq, const 
 #define SD_NH(T, N)                                                                                                  \
   launch_softmax_nc<T, N>(grid, kt, lds, st, nc, q, ldq, k_cache, vc, v_row, row_pos, row_slot, block_tables,      \
                           max_blocks, page, H, G, dk, dv, window, keep_first, scale, out, (bf16_t*)out_bf16, n_hgroups, \
-                          n_splits, part_acc, part_ml, chunk, softcap, sinks, maps, dist1, dist2, ldo)
+                          n_splits, part_acc, part_ml, chunk, softcap, sinks, maps, dist1, dist2, ldo, gates, ldg)
 #define SD_T(T)                      \
   do {                               \
     if (NH == 1) SD_NH(T, 1);        \
@@ -2035,7 +2069,7 @@ extern "C" int sd_distance_softmax_attention(const float* q, int64_t ldq, const 
   SD_CHECK_LAUNCH("sd_masked_softmax_attention");
   if (split) {
     softmax_merge_kernel<<<dim3(n_rows, HM), dv <= 64 ? 64 : (dv <= 128 ? 128 : 256), sizeof(float) * n_splits, st>>>(
-        part_acc, part_ml, n_splits, out, (bf16_t*)out_bf16, HM, dv, ldo);
+        part_acc, part_ml, n_splits, out, (bf16_t*)out_bf16, HM, dv, ldo, gates, ldg);
     SD_CHECK_LAUNCH("sd_masked_softmax_attention (merge)");
   }
   return SD_OK;
@@ -2151,6 +2185,16 @@ extern "C" int sd_moe_route_rows_biased(const float* x, int64_t ldx, const void*
                                         int E, int K, int top, int score_kind, int renorm, float renorm_eps,
                                         float weight_scale, const void* w_gate, int n_gate, float* gate_out,
                                         sd_stream_t stream) {
+  return sd_moe_route_rows_corrected(x, ldx, w_router, router_bias, nullptr, w_f32, logits, sel_expert, sel_weight,
+                                     n_rows, E, K, top, score_kind, renorm, renorm_eps, weight_scale, w_gate, n_gate,
+                                     gate_out, stream);
+}
+
+extern "C" int sd_moe_route_rows_corrected(const float* x, int64_t ldx, const void* w_router, const float* router_bias,
+                                           const float* correction, int w_f32, float* logits, int32_t* sel_expert,
+                                           float* sel_weight, int n_rows, int E, int K, int top, int score_kind,
+                                           int renorm, float renorm_eps, float weight_scale, const void* w_gate,
+                                           int n_gate, float* gate_out, sd_stream_t stream) {
   SD_REQUIRE(x && w_router && sel_expert && sel_weight && n_rows >= 1 && E >= 1 && K >= 1 && top >= 1 && top <= E &&
                  ldx >= K,
              SD_ERR_INVALID, "sd_moe_route_rows: bad argument (E=%d top=%d)", E, top);
@@ -2162,11 +2206,11 @@ extern "C" int sd_moe_route_rows_biased(const float* x, int64_t ldx, const void*
   if (w_f32)
     moe_route_rows_kernel<float><<<n_rows, nthr, sizeof(float) * E, st>>>(
         x, ldx, (const float*)w_router, logits, sel_expert, sel_weight, E, K, top, score_kind, renorm, 0, renorm_eps,
-        weight_scale, (const float*)w_gate, n_gate, gate_out, router_bias);
+        weight_scale, (const float*)w_gate, n_gate, gate_out, router_bias, correction);
   else
     moe_route_rows_kernel<bf16_t><<<n_rows, nthr, sizeof(float) * E, st>>>(
         x, ldx, (const bf16_t*)w_router, logits, sel_expert, sel_weight, E, K, top, score_kind, renorm, 1, renorm_eps,
-        weight_scale, (const bf16_t*)w_gate, n_gate, gate_out, router_bias);
+        weight_scale, (const bf16_t*)w_gate, n_gate, gate_out, router_bias, correction);
   SD_CHECK_LAUNCH("sd_moe_route_rows");
   return SD_OK;
 }
@@ -2189,10 +2233,19 @@ extern "C" int sd_moe_experts(const float* x, const void* x_bf16, int64_t ldx, c
                               const void* w_gate_up, const void* w_down, int w_f32, float* out, int n_rows, int top,
                               int E, int F, int W, int scale_input, int act_kind, void* scratch, size_t scratch_bytes,
                               sd_stream_t stream) {
+  SD_REQUIRE(act_kind == 0 || act_kind == 1, SD_ERR_UNSUPPORTED, "sd_moe_experts: activation %d is not provided", act_kind);
+  return sd_moe_experts_clamped(x, x_bf16, ldx, sel_expert, sel_weight, w_gate_up, w_down, w_f32, out, n_rows, top, E, F,
+                                W, scale_input, act_kind, 0.f, scratch, scratch_bytes, stream);
+}
+
+extern "C" int sd_moe_experts_clamped(const float* x, const void* x_bf16, int64_t ldx, const int32_t* sel_expert,
+                                      const float* sel_weight, const void* w_gate_up, const void* w_down, int w_f32,
+                                      float* out, int n_rows, int top, int E, int F, int W, int scale_input, int act_kind,
+                                      float limit, void* scratch, size_t scratch_bytes, sd_stream_t stream) {
   SD_REQUIRE(x && sel_expert && sel_weight && w_gate_up && w_down && out && scratch, SD_ERR_INVALID,
              "sd_moe_experts: null argument");
   SD_REQUIRE(n_rows >= 1 && top >= 1 && E >= 1 && F >= 1 && W >= 1 && ldx >= W, SD_ERR_INVALID, "sd_moe_experts: bad shape");
-  SD_REQUIRE(act_kind == 0 || act_kind == 1, SD_ERR_UNSUPPORTED, "sd_moe_experts: activation %d is not provided", act_kind);
+  SD_REQUIRE(act_kind >= 0 && act_kind <= 2, SD_ERR_UNSUPPORTED, "sd_moe_experts: activation %d is not provided", act_kind);
   const MoeScratch p = moe_plan(n_rows, top, E, F);
   SD_REQUIRE(scratch_bytes >= p.total, SD_ERR_WORKSPACE, "sd_moe_experts: scratch %zu < %zu bytes", scratch_bytes, p.total);
   SD_REQUIRE(sd_aligned16(scratch), SD_ERR_INVALID, "sd_moe_experts: scratch unaligned");
@@ -2223,42 +2276,42 @@ extern "C" int sd_moe_experts(const float* x, const void* x_bf16, int64_t ldx, c
   }
   if (w_f32) {
     moe_gate_up_kernel<float><<<dim3((F + 63) / 64, tiles_y), 256, 0, st>>>(x, ldx, perm, tiles, n_tiles, sel_weight,
-                                                                            (const float*)w_gate_up, act, top, F, W, scale_input, 0, act_kind);
+                                                                            (const float*)w_gate_up, act, top, E, F, W, scale_input, 0, act_kind, limit);
     SD_CHECK_LAUNCH("sd_moe_experts (gate, up)");
     moe_down_kernel<float><<<dim3((W + 63) / 64, tiles_y), 256, 0, st>>>(act, perm, tiles, n_tiles, sel_weight,
-                                                                         (const float*)w_down, out, W, F, scale_input);
+                                                                         (const float*)w_down, out, E, W, F, scale_input);
   } else if (!tiles && W % 8 == 0 && F % 8 == 0 && W <= kGemvMaxK && F <= kGemvMaxK && sd_aligned16(w_gate_up) &&
              sd_aligned16(w_down)) {
     bf16_t* act_b = (bf16_t*)act;
-    if (act_kind == 0)
+    if (act_kind != 1)
       moe_gemv_gate_up_kernel<true><<<dim3((F + 7) / 8, n), 256, sizeof(float) * W, st>>>(
-          x, ldx, sel_expert, sel_weight, (const bf16_t*)w_gate_up, act_b, top, F, W, scale_input);
+          x, ldx, sel_expert, sel_weight, (const bf16_t*)w_gate_up, act_b, top, E, F, W, scale_input, act_kind, limit);
     else
       moe_gemv_gate_up_kernel<false><<<dim3((F + 15) / 16, n), 256, sizeof(float) * W, st>>>(
-          x, ldx, sel_expert, sel_weight, (const bf16_t*)w_gate_up, act_b, top, F, W, scale_input);
+          x, ldx, sel_expert, sel_weight, (const bf16_t*)w_gate_up, act_b, top, E, F, W, scale_input, act_kind, limit);
     SD_CHECK_LAUNCH("sd_moe_experts (gate, up)");
     moe_gemv_down_kernel<<<dim3((W + 15) / 16, n), 256, sizeof(float) * F, st>>>(
-        act_b, sel_expert, sel_weight, (const bf16_t*)w_down, out, W, F, scale_input);
+        act_b, sel_expert, sel_weight, (const bf16_t*)w_down, out, E, W, F, scale_input);
   } else if (mfma) {
     // (act holds n * F floats: its first half serves as the bf16 activations)
     bf16_t* act_b = (bf16_t*)act;
     const dim3 g1((F + 127) / 128, tiles_y), g2((W + 127) / 128, tiles_y);
     const bf16_t* xb = (const bf16_t*)x_bf16;
-    if (act_kind == 0)
+    if (act_kind != 1)
       moe_gate_up_mfma_kernel<2, 512, true><<<g1, 256, 0, st>>>(x, xb, ldx, perm, tiles, n_tiles, sel_weight,
-                                                                (const bf16_t*)w_gate_up, act_b, top, F, W, scale_input);
+                                                                (const bf16_t*)w_gate_up, act_b, top, E, F, W, scale_input, act_kind, limit);
     else
       moe_gate_up_mfma_kernel<2, 512, false><<<g1, 256, 0, st>>>(x, xb, ldx, perm, tiles, n_tiles, sel_weight,
-                                                                 (const bf16_t*)w_gate_up, act_b, top, F, W, scale_input);
+                                                                 (const bf16_t*)w_gate_up, act_b, top, E, F, W, scale_input, act_kind, limit);
     SD_CHECK_LAUNCH("sd_moe_experts (gate, up)");
     moe_down_mfma_kernel<2, 512><<<g2, 256, 0, st>>>(act_b, perm, tiles, n_tiles, sel_weight, (const bf16_t*)w_down,
-                                                     out, W, F, scale_input);
+                                                     out, E, W, F, scale_input);
   } else {
     moe_gate_up_kernel<bf16_t><<<dim3((F + 63) / 64, tiles_y), 256, 0, st>>>(x, ldx, perm, tiles, n_tiles, sel_weight,
-                                                                             (const bf16_t*)w_gate_up, act, top, F, W, scale_input, 1, act_kind);
+                                                                             (const bf16_t*)w_gate_up, act, top, E, F, W, scale_input, 1, act_kind, limit);
     SD_CHECK_LAUNCH("sd_moe_experts (gate, up)");
     moe_down_kernel<bf16_t><<<dim3((W + 63) / 64, tiles_y), 256, 0, st>>>(act, perm, tiles, n_tiles, sel_weight,
-                                                                          (const bf16_t*)w_down, out, W, F, scale_input);
+                                                                          (const bf16_t*)w_down, out, E, W, F, scale_input);
   }
   SD_CHECK_LAUNCH("sd_moe_experts (down)");
   return SD_OK;

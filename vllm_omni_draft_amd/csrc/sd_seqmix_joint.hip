@@ -904,7 +904,8 @@ __global__ __launch_bounds__(1024) void mlstm_step_kernel(MlstmArgs a, MlstmPost
 // they are, the right operand of O^T = V^T P^T (the keys of an MFMA step in the order the
 // accumulators hold them).  Queries and weights enter as the sum of two bf16 parts, keys and values
 // are the cache's bf16 values: products carry 2^-17 of their operands, sums, softmax, cap and
-// distance are f32.  The distance's logarithm is formed once per distinct distance of a tile.
+// distance are f32.  The distance's logarithm is formed once per distinct distance of a tile.  Kept
+// first tokens that lie before the window's first page come first, in stages of their own.
 struct TiledAttnArgs {
   const float* q;
   int64_t ldq;
@@ -912,13 +913,16 @@ struct TiledAttnArgs {
   const bf16_t* v_cache;
   const int32_t* block_tables;
   const int32_t* entries;
+  const float* sinks;      // [H] or nullptr: one more term exp(sink) of the denominator
   const float* dist1;      // or nullptr
   const float* dist2;
+  const float* gates;      // [rows, ldg] or nullptr: heads' outputs times sigmoid of it
+  int64_t ldg;
   float* out;
   bf16_t* out_b;
   int64_t ldo;
   float scale, softcap;
-  int n_entries, max_blocks, H, G, dk, dv, window, wh, n_hgroups;
+  int n_entries, max_blocks, H, G, dk, dv, window, keep_first, wh, n_hgroups;
 };
 constexpr int kTileKeys = 64;
 constexpr int kPage = 16;
@@ -964,8 +968,11 @@ __global__ __launch_bounds__(512) void tiled_window_attn_kernel(TiledAttnArgs g)
   const int p = pos0 + sub + col;                            // this lane's query
   const int32_t* tbl = g.block_tables + (size_t)slot * g.max_blocks;
   const int last = pos0 + (len < first + tq ? len : first + tq) - 1;   // the workgroup's last position
-  int base = pos0 + first - g.window + 1;
-  base = base > 0 ? base & ~(kPage - 1) : 0;
+  int base0 = pos0 + first - g.window + 1;                   // the window's first page
+  base0 = base0 > 0 ? base0 & ~(kPage - 1) : 0;
+  const int n_kept = g.keep_first < base0 ? g.keep_first : base0;   // kept tokens before it
+  const int kept_stages = (n_kept + kStage - 1) / kStage, stages = kept_stages + (last - base0) / kStage + 1;
+  auto stage_base = [&](int s) { return s < kept_stages ? s * kStage : base0 + (s - kept_stages) * kStage; };
   const float r1 = g.dist1 ? g.dist1[h] : 0.f, r2 = g.dist1 ? g.dist2[h] : 0.f;
 
   bf16x8 qa[KS], qb[KS];                                     // the query's two parts
@@ -1029,13 +1036,18 @@ __global__ __launch_bounds__(512) void tiled_window_attn_kernel(TiledAttnArgs g)
   f32x4 o[VT];
 #pragma unroll
   for (int t = 0; t < VT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m_run = -INFINITY, l_run = 0.f;
+  // (a sink opens the first wave group's running maximum and sum; a query's sum is spread over its four lanes)
+  const bool sunk = g.sinks && group == 0;
+  float m_run = sunk ? g.sinks[h] : -INFINITY, l_run = sunk && quad == 0 ? 1.f : 0.f;
   const float cap = g.softcap, cap_in = cap > 0.f ? 2.f * kLog2e / cap : 0.f;
 
-  pages(base);
-  fetch(base);
-  pages(base + kStage);
-  for (; base <= last; base += kStage) {
+  pages(stage_base(0));
+  fetch(stage_base(0));
+  pages(stage_base(1));
+  for (int stage = 0; stage < stages; ++stage) {
+    const int base = stage_base(stage);
+    // (a stage of kept tokens holds no key of the window; in the window's stages kept tokens are seen too)
+    const int key_end = stage < kept_stages ? n_kept : 0x7fffffff;
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < KS; ++i) {
@@ -1057,11 +1069,11 @@ __global__ __launch_bounds__(512) void tiled_window_attn_kernel(TiledAttnArgs g)
       if (lane < 16) away[64 + lane] = r1 * log1pf(r2 * (float)(d0 + 64 + lane > 0 ? d0 + 64 + lane : 0));
     }
     __syncthreads();
-    if (base + kStage <= last) {
-      fetch(base + kStage);
-      pages(base + 2 * kStage);
+    if (stage + 1 < stages) {
+      fetch(stage_base(stage + 1));
+      pages(stage_base(stage + 2));
     }
-    if (!works || gbase > pos0 + sub + n_rows - 1) continue;   // (keys behind this wave's last query)
+    if (!works || gbase > pos0 + sub + n_rows - 1 || gbase >= key_end) continue;   // (keys behind this wave's last query)
     const bf16_t* kt = ks + group * kTileKeys * KLD;
     const bf16_t* vt = vs + group * 16 * VT * VLD;
     f32x4 sc[4];
@@ -1085,7 +1097,8 @@ __global__ __launch_bounds__(512) void tiled_window_attn_kernel(TiledAttnArgs g)
         // cap tanh(v / cap) = cap - 2 cap / (e^(2 v / cap) + 1)
         if (cap > 0.f) v = fmaf(-2.f * cap, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(v * cap_in) + 1.f), cap);
         if (g.dist1) v -= away[col + kTileKeys - 1 - kk];
-        v = d >= 0 && d < g.window ? v : -INFINITY;
+        const int j = gbase + kk;
+        v = d >= 0 && (d < g.window || j < g.keep_first) && j < key_end ? v : -INFINITY;
         sc[t][i] = v;
         mx = fmaxf(mx, v);
       }
@@ -1144,7 +1157,8 @@ __global__ __launch_bounds__(512) void tiled_window_attn_kernel(TiledAttnArgs g)
   for (int t = 0; t < VT; ++t)
 #pragma unroll
     for (int i = 0; i < 4; ++i) o[t][i] = fmaf(o[t][i], f1, other[(4 * t + i) * 4 * SD_WAVE] * f2);
-  const float inv = 1.f / fmaf(l_run, f1, other[(4 * VT + 1) * 4 * SD_WAVE] * f2);
+  float inv = 1.f / fmaf(l_run, f1, other[(4 * VT + 1) * 4 * SD_WAVE] * f2);
+  if (g.gates) inv *= sigmoid_f(g.gates[(size_t)(row0 + sub + col) * g.ldg + h]);
   const size_t at = (size_t)(row0 + sub + col) * g.ldo + (size_t)h * dv;
   const bool quads = g.ldo % 4 == 0;
 #pragma unroll
@@ -1681,15 +1695,17 @@ extern "C" int sd_mlstm_scan(const float* q, const float* k, const float* v, con
 
 int sd_tiled_window_attention_(const float* q, int64_t ldq, const void* k_cache, const void* v_cache,
                                const int32_t* block_tables, int max_blocks, int page, int n_rows, int H,
-                               int G, int dk, int dv, int window, float scale, float softcap, const float* dist1,
-                               const float* dist2, const int32_t* entries, int n_entries, float* out, void* out_bf16,
+                               int G, int dk, int dv, int window, int keep_first, float scale, float softcap,
+                               const float* sinks, const float* dist1, const float* dist2, const float* gates,
+                               int64_t ldg, const int32_t* entries, int n_entries, float* out, void* out_bf16,
                                int64_t ldo, sd_stream_t stream) {
   if (page != kPage || dk % 8 || dv % 8 || dk > 128 || dv > 128 || ldq % 4 || !sd_aligned16(q) || !sd_aligned16(k_cache) ||
       !sd_aligned16(v_cache) || !(ldo % 4 || (sd_aligned16(out) && sd_aligned16(out_bf16))))
     return SD_ERR_UNSUPPORTED;
   const int qh = H / G;
-  TiledAttnArgs g{q, ldq, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, entries, dist1, dist2, out,
-                  (bf16_t*)out_bf16, ldo, scale, softcap, n_entries, max_blocks, H, G, dk, dv, window, 0, 0};
+  TiledAttnArgs g{q, ldq, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, entries, sinks, dist1, dist2,
+                  gates, ldg, out, (bf16_t*)out_bf16, ldo, scale, softcap, n_entries, max_blocks, H, G, dk, dv, window,
+                  keep_first, 0, 0};
   g.wh = qh >= 4 ? 4 : (qh >= 2 ? 2 : 1);
   g.n_hgroups = (qh + g.wh - 1) / g.wh;
   const int tq = 16 * (4 / g.wh);

@@ -1637,6 +1637,44 @@ extern "C" int sd_mlstm_read(const float*, const float*, float*, const int32_t*,
                              int, float, float*, void*, int64_t, int, int, int, const sd_poly_norm*, sd_stream_t) {
   UNSUPPORTED("sd_mlstm_read");
 }
+extern "C" int sd_gated_softmax_attention(const float*, int64_t, const void*, const void*, int, const int32_t*,
+                                          const int32_t*, const int32_t*, int, int, int, int, int, int, int, int, int,
+                                          int, int, float, float, const float*, const float*, const float*,
+                                          const float*, int64_t, const int32_t*, int, float*, void*, int64_t, void*,
+                                          size_t, sd_stream_t) {
+  UNSUPPORTED("sd_gated_softmax_attention");
+}
+extern "C" int sd_moe_route_rows_corrected(const float*, int64_t, const void*, const float*, const float*, int, float*,
+                                           int32_t*, float*, int, int, int, int, int, int, float, float, const void*,
+                                           int, float*, sd_stream_t) {
+  UNSUPPORTED("sd_moe_route_rows_corrected");
+}
+extern "C" int sd_moe_experts_clamped(const float*, const void*, int64_t, const int32_t*, const float*, const void*,
+                                      const void*, int, float*, int, int, int, int, int, int, int, float, void*, size_t,
+                                      sd_stream_t) {
+  UNSUPPORTED("sd_moe_experts_clamped");
+}
+extern "C" int sd_cap_rows(float*, int64_t, float, int, int, sd_stream_t) { UNSUPPORTED("sd_cap_rows"); }
+extern "C" int sd_streams_residual(const sd_streams_update*, int, float, int, int, int, sd_stream_t) {
+  UNSUPPORTED("sd_streams_residual");
+}
+extern "C" int sd_decay_step_rows(const sd_decay_step*, int, float, const int32_t*, const int32_t*, int, sd_stream_t) {
+  UNSUPPORTED("sd_decay_step_rows");
+}
+extern "C" int sd_biased_qkv_prep(float*, const float*, const float*, int64_t, const void*, const void*, const void*, int,
+                                  int, int, int, const void*, const void*, int, float, void*, void*, const int32_t*,
+                                  const int32_t*, const int32_t*, int, int, int, const sd_decay_step*, sd_stream_t) {
+  UNSUPPORTED("sd_biased_qkv_prep");
+}
+extern "C" int sd_low_rank_decay(const float*, int64_t, const void*, const float*, int, int, float, float*, int, int,
+                                 sd_stream_t) {
+  UNSUPPORTED("sd_low_rank_decay");
+}
+extern "C" size_t sd_decay_chunks_scratch_bytes(int, int, int, int, int) { return 0; }
+extern "C" int sd_decay_chunks(const float*, const float*, const float*, int64_t, const float*, float, float*,
+                               const int32_t*, int, int, float*, int, int, int, void*, size_t, sd_stream_t) {
+  UNSUPPORTED("sd_decay_chunks");
+}
 extern "C" int sd_scale_rows(float*, int64_t, float, int, int, sd_stream_t) { UNSUPPORTED("sd_scale_rows"); }
 extern "C" sd_seq_model* sd_seq_model_create(const sd_seq_model_desc*) {
   set_error("sd_seq_model_create: not provided by the CPU build of the library");

@@ -148,7 +148,8 @@ class SeqCache:
     means pk / pv f32 [pages, kv_heads, pooled slots per page, dim | vdim]; one page table per
     slot serves all window layers.  Latent attention keeps one row [kv_rank + rot_dim] per token
     in k only; a state-space recurrence keeps state[layer] [slots, heads, state, vdim] and the
-    tail of its convolution's inputs conv[layer] f32 [slots, taps - 1, channels].  The tensors are
+    tail of its convolution's inputs conv[layer] f32 [slots, taps - 1, channels]; linear attention beside
+    softmax attention keeps state[layer] [slots, heads, dim, vdim] of its own sizes.  The tensors are
     keyed by the layer's place in the order of running (cfg.runs): a layer that runs several
     times over keeps a cache for every pass.  A softmax attention with several score maps per head
     keeps that many key rows per kv head and token (cache head = kv head * maps + map) and one value
@@ -197,6 +198,11 @@ class SeqCache:
                 # one row per token serves as key and value: the latent, then the shared rotated part
                 self.has_pages = True
                 self.k[i] = torch.zeros(num_pages, 1, PAGE, m.kv_rank + m.rot_dim, dtype=dtype, device=device)
+            elif m.linear is not None:
+                self.has_pages = True
+                self.k[i] = torch.zeros(num_pages, m.kv_heads, PAGE, m.dim, dtype=dtype, device=device)
+                self.v[i] = torch.zeros(num_pages, m.kv_heads, PAGE, m.vdim, dtype=dtype, device=device)
+                self.state[i] = f32(max_seqs, m.linear.heads, m.linear.dim, m.linear.vdim)
             elif m.kind == "parallel":
                 self.has_pages = True
                 sd = m.ssd

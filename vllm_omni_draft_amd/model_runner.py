@@ -203,6 +203,7 @@ class DecoderModel:
 # ---------------------------------------------------------------------------------------------
 _MIX_KIND = {"retention": 0, "gla": 1, "attention": 2, "latent_attention": 3, "parallel": 4, "softmax_attention": 5,
              "mlstm": 6}
+_EXPERT_ACT = {"silu": 0, "relu2": 1, "clamped_gate": 2}
 
 
 class SeqModel:
@@ -268,6 +269,31 @@ class SeqModel:
                     w_shared_down=rm(t.w_shared_down), w_shared_down_tiled=tl(t.w_shared_down),
                     w_shared_gate=_ptr(t.w_shared_gate))
                 continue
+            if cfg.block == "streams":
+                r, ex = m.linear, spec.experts
+                layers[i] = _lib.SeqLayer(
+                    kind=7, block=4, heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, ff=spec.ff,
+                    ff_act={"relu": 0, "silu": 1}[spec.ff_act], q_scale=r.dim ** -0.5, score_scale=m.scale,
+                    window=m.window or 0x7fffffff, keep_first=m.keep_first, softcap=m.softcap, sinks=_ptr(t.sinks),
+                    head_gate=int(m.head_gate), norm_w=_ptr(t.norm_w), norm2_w=_ptr(t.norm2_w),
+                    w_in=rm(t.w_in), w_in_tiled=tl(t.w_in), w_in_bias=_ptr(t.w_in_bias), w_o=rm(t.w_o),
+                    w_o_tiled=tl(t.w_o), w_o2=rm(t.w_o2), w_o2_tiled=tl(t.w_o2), out_stacked=int(t.out_stacked),
+                    q_norm_w=_ptr(t.q_norm_w), k_norm_w=_ptr(t.k_norm_w),
+                    s_heads=r.heads, s_state=r.dim, s_vdim=r.vdim, rank=r.rank, tau=r.tau, w_a2=_ptr(t.w_a2),
+                    b_a2=_ptr(t.b_a2), s_norm_w=_ptr(t.s_norm_w), out_norm_w=_ptr(t.out_norm_w),
+                    out_norm2_w=_ptr(t.out_norm2_w), state=_ptr(cache.state.get(i)),
+                    k_cache=_ptr(cache.keys_of(i)), v_cache=_ptr(cache.values_of(i)),
+                    hc_in=_ptr(t.hc_in), hc_out=_ptr(t.hc_out), hc_mix=_ptr(t.hc_mix), hc2_in=_ptr(t.hc2_in),
+                    hc2_out=_ptr(t.hc2_out), hc2_mix=_ptr(t.hc2_mix),
+                    w_ff_in=rm(t.w_ff_in), w_ff_in_tiled=tl(t.w_ff_in), w_down=rm(t.w_down), w_down_tiled=tl(t.w_down),
+                    n_experts=ex.experts if ex else 0, n_identity=ex.identity if ex else 0, top=ex.top if ex else 0,
+                    expert_ff=ex.ff if ex else 0, w_router=_ptr(t.w_router), w_gate_up=_ptr(t.w_gate_up),
+                    w_down_e=_ptr(t.w_down_e), expert_act=_EXPERT_ACT[ex.act] if ex else 0,
+                    expert_limit=ex.limit if ex else 0.0, route_score=int(ex.score == "softmax") if ex else 0,
+                    route_renorm=int(ex.renorm) if ex else 0, route_renorm_eps=ex.renorm_eps if ex else 0.0,
+                    route_scale=ex.scale if ex else 1.0, router_bias=_ptr(t.router_bias),
+                    route_correction=_ptr(t.route_correction))
+                continue
             if cfg.block == "joint":
                 layers[i] = _lib.SeqLayer(
                     kind=_MIX_KIND[m.kind], block=3, heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim,
@@ -328,7 +354,8 @@ class SeqModel:
                                  bigram=_ptr(weights.bigram), buckets=(cfg.bigram or {}).get("buckets", 0),
                                  mul_prev=(cfg.bigram or {}).get("mul_prev", 0),
                                  mul_cur=(cfg.bigram or {}).get("mul_cur", 0), head=_ptr(weights.head),
-                                 logit_scale=cfg.logit_scale)
+                                 logit_scale=cfg.logit_scale, streams=cfg.streams,
+                                 logit_softcap=cfg.logit_softcap)
         self._handle = _lib.load().sd_seq_model_create(C.byref(desc))
         if not self._handle:
             raise _lib.SdError(f"sd_seq_model_create failed: {_lib.last_error()}")

@@ -375,6 +375,19 @@ class SeqLayerTensors:
     gate_bias: Optional[torch.Tensor] = None   # f32 [2*heads]: input gates', then forget gates'
     ff_bias: Optional[torch.Tensor] = None     # [ff]
     ff_coef: Optional[torch.Tensor] = None     # f32 [4]
+    # layers on several residual streams (norm_w / norm2_w stored around zero); hc: in, out [streams], mix
+    # [streams, streams], f32, around the mixer; hc2: around the feed-forward.  w_o holds the rows of both
+    # output matrices when out_stacked, else w_o2 is the second one
+    hc_in: Optional[torch.Tensor] = None
+    hc_out: Optional[torch.Tensor] = None
+    hc_mix: Optional[torch.Tensor] = None
+    hc2_in: Optional[torch.Tensor] = None
+    hc2_out: Optional[torch.Tensor] = None
+    hc2_mix: Optional[torch.Tensor] = None
+    out_stacked: bool = False
+    out_norm_w: Optional[torch.Tensor] = None  # [width]: norms of the two mixers' results
+    out_norm2_w: Optional[torch.Tensor] = None
+    route_correction: Optional[torch.Tensor] = None   # f32 [router rows]
 
 
 @dataclass
@@ -435,8 +448,8 @@ def seq_from_state_dict(cfg, state: Dict[str, torch.Tensor], device="cuda",
             return ops.tile_weights(d, ops.TILE_PLAIN)
         return d
 
-    if cfg.block in ("sandwich", "joint"):
-        one = _sandwich_layer if cfg.block == "sandwich" else _joint_layer
+    if cfg.block in ("sandwich", "joint", "streams"):
+        one = {"sandwich": _sandwich_layer, "joint": _joint_layer, "streams": _streams_layer}[cfg.block]
         layers = [one(cfg, i, get, dev, mat) for i in range(cfg.n_layers)]
         head = mat(get("head", (cfg.vocab, W)))
         return SeqModelWeights(cfg, dtype, dev(get("embed", (cfg.vocab, W))), dev(get("final.norm", (W,))), layers,
@@ -647,6 +660,60 @@ def _joint_layer(cfg, i: int, get, dev, mat) -> SeqLayerTensors:
     return lt
 
 
+def _streams_layer(cfg, i: int, get, dev, mat) -> SeqLayerTensors:
+    """Layer i of a model on several residual streams: the matrices that read the mixer's input stacked
+    into w_in (attention's q, k, v, linear attention's q, k, v, g and the first of its low-rank pair, the
+    head gates last), both output matrices stacked where their input widths are equal."""
+    l, p, W, S = cfg.layers[i], f"l{i}.", cfg.width, cfg.streams
+    m, r = l.mixer, l.mixer.linear
+    H, G, dk, dv = m.heads, m.kv_heads, m.dim, m.vdim
+    left, right, f32 = p + "mix.left.", p + "mix.right.", torch.float32
+    qkv = [("q", H * dk), ("k", G * dk), ("v", G * dv)]
+    parts = [get(left + n, (rows, W)) for n, rows in qkv]
+    parts += [get(right + n, (rows, W)) for n, rows in (("q", r.heads * r.dim), ("k", r.heads * r.dim), ("v", r.heads * r.vdim),
+                                                        ("g", r.heads * r.vdim), ("a1", r.rank))]
+    if m.head_gate:
+        parts.append(get(left + "g", (H, W)))
+    else:
+        parts.append(torch.zeros(H, W))
+    o1, o2 = get(left + "o", (W, H * dv)).float(), get(right + "o", (W, r.heads * r.vdim)).float()
+    lt = SeqLayerTensors(norm_w=dev(get(p + "norm1", (W,))), w_in=mat(torch.cat([t.float() for t in parts])), w_o=None,
+                         r1_bias=None)
+    lt.out_stacked = o1.shape[1] == o2.shape[1] and W % 16 == 0
+    if lt.out_stacked:
+        lt.w_o = mat(torch.cat([o1, o2]))
+    else:
+        lt.w_o, lt.w_o2 = mat(o1), mat(o2)
+        if isinstance(lt.w_o, ops.TiledWeight) != isinstance(lt.w_o2, ops.TiledWeight):
+            lt.w_o, lt.w_o2 = dev(o1), dev(o2)
+    if m.qkv_bias:
+        lt.w_in_bias = dev(torch.cat([get(left + n + ".b", (rows,)).float() for n, rows in qkv]))
+    lt.q_norm_w, lt.k_norm_w = dev(get(left + "q.norm", (dk,))), dev(get(left + "k.norm", (dk,)))
+    if m.sink:
+        lt.sinks = dev(get(left + "sink", (H,)), f32)
+    lt.w_a2, lt.b_a2 = dev(get(right + "a2", (r.heads * r.dim, r.rank))), dev(get(right + "a2.b", (r.heads * r.dim,)), f32)
+    lt.s_norm_w = dev(get(right + "norm", (r.vdim,)))
+    lt.out_norm_w, lt.out_norm2_w = dev(get(left + "out", (W,))), dev(get(right + "out", (W,)))
+    lt.hc_in, lt.hc_out = dev(get(p + "hc1.in", (S,)), f32), dev(get(p + "hc1.out", (S,)), f32)
+    lt.hc_mix = dev(get(p + "hc1.mix", (S, S)), f32)
+    ex = l.experts
+    if l.ff or ex is not None:
+        lt.norm2_w = dev(get(p + "norm2", (W,)))
+        lt.hc2_in, lt.hc2_out = dev(get(p + "hc2.in", (S,)), f32), dev(get(p + "hc2.out", (S,)), f32)
+        lt.hc2_mix = dev(get(p + "hc2.mix", (S, S)), f32)
+    if l.ff:
+        lt.w_ff_in = mat(torch.cat([get(p + "mlp.gate", (l.ff, W)).float(), get(p + "mlp.up", (l.ff, W)).float()]))
+        lt.w_down = mat(get(p + "mlp.down", (W, l.ff)))
+    if ex is not None:
+        lt.w_router = dev(get(p + "mlp.router", (ex.outputs, W)))
+        if ex.correction:
+            lt.route_correction = dev(get(p + "mlp.correction", (ex.outputs,)), f32)
+        lt.w_gate_up = dev(torch.stack([torch.cat([get(p + f"mlp.e{e}.gate", (ex.ff, W)), get(p + f"mlp.e{e}.up", (ex.ff, W))])
+                                        for e in range(ex.experts)]))
+        lt.w_down_e = dev(torch.stack([get(p + f"mlp.e{e}.down", (W, ex.ff)) for e in range(ex.experts)]))
+    return lt
+
+
 def seq_from_safetensors_dir(cfg, model_dir: str, device="cuda",
                              dtype: torch.dtype = torch.bfloat16) -> SeqModelWeights:
     from safetensors import safe_open
@@ -677,6 +744,8 @@ def seq_random_state(cfg, seed: int = 0) -> Dict[str, torch.Tensor]:
         return _sandwich_random_state(cfg, rn)
     if cfg.block == "joint":
         return _joint_random_state(cfg, rn)
+    if cfg.block == "streams":
+        return _streams_random_state(cfg, rn)
     st = {"embed": rn(cfg.vocab, W, s=1.0), "final.norm": rn(W, s=0.1)}
     for i, l in enumerate(cfg.layers):
         m, p = l.mixer, f"l{i}."
@@ -822,6 +891,45 @@ def _joint_random_state(cfg, rn) -> Dict[str, torch.Tensor]:
             st[p + "norm2"], st[p + "mlp.act"] = 1 + rn(W, s=0.1), rn(4, s=0.5)
             st[p + "mlp.up"], st[p + "mlp.up.b"] = rn(l.ff, W, s=W ** -0.5), rn(l.ff, s=0.2)
             st[p + "mlp.down"], st[p + "mlp.down.b"] = rn(W, l.ff, s=l.ff ** -0.5), rn(W, s=0.2)
+    return st
+
+
+def _streams_random_state(cfg, rn) -> Dict[str, torch.Tensor]:
+    W, S = cfg.width, cfg.streams
+    st = {"embed": rn(cfg.vocab, W, s=1.0), "final.norm": rn(W, s=0.1), "head": rn(cfg.vocab, W, s=W ** -0.5)}
+    for i, l in enumerate(cfg.layers):
+        m, r, ex, p = l.mixer, l.mixer.linear, l.experts, f"l{i}."
+        for n in (1, 2) if l.ff or ex else (1,):
+            st[p + f"norm{n}"] = rn(W, s=0.1)
+            st[p + f"hc{n}.in"], st[p + f"hc{n}.out"] = rn(S, s=0.1) + 1.0 / S, rn(S, s=0.1) + 0.5
+            st[p + f"hc{n}.mix"] = (torch.eye(S) + rn(S, S, s=0.05)).to(torch.bfloat16)
+        left, right = p + "mix.left.", p + "mix.right."
+        for n, rows in (("q", m.heads * m.dim), ("k", m.kv_heads * m.dim), ("v", m.kv_heads * m.vdim)):
+            st[left + n] = rn(rows, W, s=W ** -0.5)
+            if m.qkv_bias:
+                st[left + n + ".b"] = rn(rows, s=0.2)
+        st[left + "q.norm"], st[left + "k.norm"], st[left + "out"] = 1 + rn(m.dim, s=0.1), 1 + rn(m.dim, s=0.1), 1 + rn(W, s=0.1)
+        st[left + "o"] = rn(W, m.heads * m.vdim, s=(m.heads * m.vdim) ** -0.5)
+        if m.sink:
+            st[left + "sink"] = rn(m.heads, s=1.0)
+        if m.head_gate:
+            st[left + "g"] = rn(m.heads, W, s=W ** -0.5)
+        for n, rows in (("q", r.heads * r.dim), ("k", r.heads * r.dim), ("v", r.heads * r.vdim), ("g", r.heads * r.vdim),
+                        ("a1", r.rank)):
+            st[right + n] = rn(rows, W, s=W ** -0.5)
+        st[right + "a2"], st[right + "a2.b"] = rn(r.heads * r.dim, r.rank, s=r.rank ** -0.5), rn(r.heads * r.dim, s=1.0) + 3.0
+        st[right + "norm"], st[right + "out"] = 1 + rn(r.vdim, s=0.1), 1 + rn(W, s=0.1)
+        st[right + "o"] = rn(W, r.heads * r.vdim, s=(r.heads * r.vdim) ** -0.5)
+        if l.ff:
+            st[p + "mlp.gate"], st[p + "mlp.up"] = rn(l.ff, W, s=W ** -0.5), rn(l.ff, W, s=W ** -0.5)
+            st[p + "mlp.down"] = rn(W, l.ff, s=l.ff ** -0.5)
+        if ex is not None:
+            st[p + "mlp.router"] = rn(ex.outputs, W, s=W ** -0.5)
+            if ex.correction:
+                st[p + "mlp.correction"] = rn(ex.outputs, s=0.02)
+            for e in range(ex.experts):
+                st[p + f"mlp.e{e}.gate"], st[p + f"mlp.e{e}.up"] = rn(ex.ff, W, s=W ** -0.5), rn(ex.ff, W, s=W ** -0.5)
+                st[p + f"mlp.e{e}.down"] = rn(W, ex.ff, s=ex.ff ** -0.5)
     return st
 
 
