@@ -227,4 +227,4 @@ def random_tensors(cfg, ranks, seed=0):
         for e in range(E):
             st[q + f"e{e}.gate"], st[q + f"e{e}.up"] = rn(F, W, s=1.5 * W ** -0.5), rn(F, W, s=1.5 * W ** -0.5)
             st[q + f"e{e}.down"] = rn(W, F, s=F ** -0.5)
-    return st
+    return {k: v.to(torch.bfloat16).float() for k, v in st.items()}

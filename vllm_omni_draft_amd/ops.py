@@ -1617,6 +1617,174 @@ def mlstm_step(q, k, v, zi, zf, bi, bf, cap, state, n_state, m_state, row_pos, r
     return y if act is None else (y[:, :H * dv], y[:, H * dv:])
 
 
+# ------------------------------------------------------- several residual streams, linear attention with decays
+def gated_softmax_attention(q, k_cache, v_cache, row_pos, row_slot, block_tables, H, G, dk, dv, scale, window=0,
+                            keep_first=0, softcap=0.0, sinks=None, gates=None, entries=None, split=True, ldo=0,
+                            bf16_only=False) -> torch.Tensor:
+    """masked_softmax_attention whose heads' outputs are multiplied by sigmoid(gates f32 [rows, H]).  entries
+    int32 [n, 4]: the rows' portions; many rows over bfloat16 caches then run on the matrix cores.
+    ldo: elements between output rows; bf16_only: the result in bfloat16 alone."""
+    _f32(q, "q")
+    for t, nm in ((sinks, "sinks"), (gates, "gates")):
+        if t is not None:
+            _f32(t, nm)
+    n, window = q.shape[0], int(window) or 0x7fffffff
+    ldo = ldo or H * dv
+    out = torch.empty(n, ldo, dtype=torch.bfloat16 if bf16_only else torch.float32, device=q.device)
+    lib = _lib.load()
+    nb = int(lib.sd_multimap_softmax_attention_scratch_bytes(n, H, 1, dv, window, int(keep_first), 0,
+                                                             block_tables.shape[1] * PAGE)) if split else 0
+    scratch = torch.empty(nb, dtype=torch.uint8, device=q.device) if nb else None
+    _lib.check(lib.sd_gated_softmax_attention(
+        _p(q), q.shape[1], _p(k_cache), _p(v_cache), int(k_cache.dtype == torch.float32), _p(row_pos), _p(row_slot),
+        _p(block_tables), block_tables.shape[1], PAGE, n, H, G, 1, dk, dv, window, int(keep_first), 0, float(scale),
+        float(softcap), _p(sinks), None, None, _p(gates), gates.shape[1] if gates is not None else 0, _p(entries),
+        entries.shape[0] if entries is not None else 0, None if bf16_only else _p(out), _p(out) if bf16_only else None,
+        ldo, _p(scratch), nb, _stream()), "sd_gated_softmax_attention")
+    return out[:, :H * dv]
+
+
+def moe_route_rows_corrected(x, w_router, correction, top, score="softmax"):
+    """moe_route_rows whose choice is made by score + correction f32 [E]: (experts, weights, logits)."""
+    _f32(x, "x")
+    _f32(correction, "correction")
+    n, K = x.shape
+    E = w_router.shape[0]
+    sel_e = torch.empty(n, top, dtype=torch.int32, device=x.device)
+    sel_w = torch.empty(n, top, dtype=torch.float32, device=x.device)
+    logits = torch.empty(n, E, dtype=torch.float32, device=x.device)
+    _lib.check(_lib.load().sd_moe_route_rows_corrected(
+        _p(x), K, _p(w_router), None, _p(correction), _wkind(w_router, "w_router"), _p(logits), _p(sel_e), _p(sel_w), n, E,
+        K, top, {"sigmoid": 0, "softmax": 1}[score], 0, 0.0, 1.0, None, 0, None, _stream()), "sd_moe_route_rows_corrected")
+    return sel_e, sel_w, logits
+
+
+def moe_experts_clamped(x, sel_e, sel_w, w_gate_up, w_down, limit, bf16_copy=False) -> torch.Tensor:
+    """moe_experts with weighted outputs and the clamped activation: f32 [rows, top, W].  Rows of a chosen index
+    outside the experts with matrices hold what the buffer held (here: NaN)."""
+    _f32(x, "x")
+    n, W = x.shape
+    top, E, F = sel_e.shape[1], w_gate_up.shape[0], w_down.shape[2]
+    lib = _lib.load()
+    nb = int(lib.sd_moe_experts_scratch_bytes(n, top, E, F, W))
+    scratch = torch.empty(nb, dtype=torch.uint8, device=x.device)
+    out = torch.full((n, top, W), float("nan"), dtype=torch.float32, device=x.device)
+    xb = x.to(torch.bfloat16) if bf16_copy else None
+    _lib.check(lib.sd_moe_experts_clamped(_p(x), _p(xb), W, _p(sel_e), _p(sel_w), _p(w_gate_up), _p(w_down),
+                                          _wkind(w_down, "w_down"), _p(out), n, top, E, F, W, 0, 2, float(limit), _p(scratch),
+                                          nb, _stream()), "sd_moe_experts_clamped")
+    return out
+
+
+def cap_rows(x, cap) -> None:
+    """x = cap tanh(x / cap), in place on f32 [rows, n]."""
+    _f32(x, "x")
+    _lib.check(_lib.load().sd_cap_rows(_p(x), x.shape[1], float(cap), x.shape[0], x.shape[1], _stream()), "sd_cap_rows")
+
+
+def streams_residual(x, *, tokens=None, embed=None, a=None, n_a=1, sel=None, input=None, b=None, w_a=None, w_b=None,
+                     mix=None, out=None, in_=None, w_next=None, rows=None, eps=1e-5, want_copy=False, bf16=False,
+                     h=None):
+    """sd_streams_residual on x f32 [rows, streams, W].  sel: (chosen int32 [rows, n_a], weights f32
+    [rows, n_a], number of experts with matrices).  Returns (h or None, the streams' sums or None); h
+    may be given (a sublayer's input that is read and replaced)."""
+    _f32(x, "x")
+    for t, nm in ((a, "a"), (b, "b"), (mix, "mix"), (out, "out"), (in_, "in"), (input, "input")):
+        if t is not None:
+            _f32(t, nm)
+    S, W = x.shape[1], x.shape[2]
+    n = rows.numel() if rows is not None else x.shape[0]
+    typed = next((t for t in (w_next, w_a, embed) if t is not None), None)
+    copy = torch.empty(x.shape[0], W, dtype=torch.float32, device=x.device) if want_copy else None
+    if w_next is not None and h is None:
+        h = torch.empty(n, W, dtype=torch.float32, device=x.device)
+    hb = torch.empty(n, W, dtype=torch.bfloat16, device=x.device) if bf16 else None
+    u = _lib.StreamsUpdate(x=_p(x), streams=S, rows=_p(rows), tokens=_p(tokens), embed=_p(embed),
+                           vocab=embed.shape[0] if embed is not None else 0, a=_p(a), lda=W, n_a=n_a,
+                           sel_expert=_p(sel[0]) if sel else None, sel_weight=_p(sel[1]) if sel else None,
+                           n_experts=sel[2] if sel else 0, input=_p(input), b=_p(b), w_a=_p(w_a), w_b=_p(w_b), mix=_p(mix),
+                           out=_p(out), x_copy=_p(copy), in_=_p(in_), w_next=_p(w_next),
+                           h=None if bf16 or w_next is None else _p(h), h_bf16=_p(hb))
+    _lib.check(_lib.load().sd_streams_residual(C.byref(u), int(typed is None or typed.dtype == torch.float32), float(eps), n,
+                                               W, 0, _stream()), "sd_streams_residual")
+    return (hb if bf16 else h), copy
+
+
+def _decay_step(buf, sizes, a2, a2_bias, tau, q_scale, state, norm_w, y):
+    """The sd_decay_step over buf [rows, ld], which stacks q, k, v, gate, a1 at column `sizes` starts."""
+    H, dk, dv = state.shape[1:]
+    p = [buf.data_ptr() + 4 * s for s in sizes]
+    return _lib.DecayStep(q=p[0], k=p[1], v=p[2], a1=p[4], gate=p[3], ld=buf.shape[1], a2=_p(a2), a2_bias=_p(a2_bias),
+                          rank=a2.shape[1], tau=float(tau), q_scale=float(q_scale), state=_p(state), norm_w=_p(norm_w),
+                          y=_p(y), y_bf16=None, ldy=H * dv, heads=H, dim=dk, vdim=dv)
+
+
+def decay_step_rows(q, k, v, gate, a1, a2, a2_bias, tau, state, norm_w, eps, row_pos, row_slot, q_scale=1.0):
+    """Linear attention with decays, rows alone in their entries: f32 [rows, H*dv]; state f32 [slots, H, dk, dv]
+    moves on.  q, k [rows, H*dk], v, gate [rows, H*dv], a1 [rows, rank], a2 [H*dk, rank]."""
+    buf = torch.cat([q, k, v, gate, a1], dim=1).contiguous()
+    at = [0]
+    for t in (q, k, v, gate):
+        at.append(at[-1] + t.shape[1])
+    y = torch.empty(q.shape[0], v.shape[1], dtype=torch.float32, device=q.device)
+    s = _decay_step(buf, at, a2, a2_bias, tau, q_scale, state, norm_w, y)
+    _lib.check(_lib.load().sd_decay_step_rows(C.byref(s), _wkind(a2, "a2"), float(eps), _p(row_pos), _p(row_slot), q.shape[0],
+                                              _stream()), "sd_decay_step_rows")
+    return y
+
+
+def biased_qkv_prep(q, k, v, biases, G, dk, dv, q_norm_w, k_norm_w, eps, k_cache, v_cache, row_pos, row_slot,
+                    block_tables, step=None):
+    """sd_biased_qkv_prep on q f32 [rows, H*dk], k [rows, G*dk], v [rows, G*dv]; biases: (q, k, v), each may be
+    None.  Returns the prepared q; keys and values go to the caches.  step: the arguments of
+    decay_step_rows up to norm_w (and q_scale), whose result is then returned too."""
+    buf = torch.cat([q, k, v], dim=1).contiguous()
+    nq, nk, ld = q.shape[1], k.shape[1], buf.shape[1]
+    y, s = None, None
+    if step is not None:
+        sq, sk, sv, gate, a1, a2, a2_bias, tau, state, norm_w, q_scale = step
+        buf2 = torch.cat([sq, sk, sv, gate, a1], dim=1).contiguous()
+        at = [0]
+        for t in (sq, sk, sv, gate):
+            at.append(at[-1] + t.shape[1])
+        y = torch.empty(q.shape[0], sv.shape[1], dtype=torch.float32, device=q.device)
+        s = _decay_step(buf2, at, a2, a2_bias, tau, q_scale, state, norm_w, y)
+    _lib.check(_lib.load().sd_biased_qkv_prep(
+        buf.data_ptr(), buf.data_ptr() + 4 * nq, buf.data_ptr() + 4 * (nq + nk), ld, _p(biases[0]), _p(biases[1]),
+        _p(biases[2]), nq // dk, G, dk, dv, _p(q_norm_w), _p(k_norm_w), _wkind(q_norm_w, "q_norm_w"), float(eps), _p(k_cache),
+        _p(v_cache), _p(row_pos), _p(row_slot), _p(block_tables), block_tables.shape[1], PAGE, q.shape[0],
+        C.byref(s) if s is not None else None, _stream()), "sd_biased_qkv_prep")
+    out = buf[:, :nq].contiguous()
+    return out if step is None else (out, y)
+
+
+def low_rank_decay(a1, a2, a2_bias, tau) -> torch.Tensor:
+    """sigmoid(a1 a2^T + a2_bias)^(1/tau): f32 [rows, n] for a1 f32 [rows, rank], a2 [n, rank]."""
+    _f32(a1, "a1")
+    _f32(a2_bias, "a2_bias")
+    out = torch.empty(a1.shape[0], a2.shape[0], dtype=torch.float32, device=a1.device)
+    _lib.check(_lib.load().sd_low_rank_decay(_p(a1), a1.shape[1], _p(a2), _p(a2_bias), _wkind(a2, "a2"), a2.shape[1],
+                                             float(tau), _p(out), a1.shape[0], a2.shape[0], _stream()), "sd_low_rank_decay")
+    return out
+
+
+def decay_chunks(q, k, v, decay, state, entries, q_scale=1.0, cut=True) -> torch.Tensor:
+    """The recurrence with decays per key channel over portions: q, k, decay f32 [rows, H*dk], v [rows, H*dv], state
+    f32 [slots, H, dk, dv] (moves on) -> f32 [rows, H*dv].  cut=False: every portion in one go."""
+    for t, nm in ((q, "q"), (k, "k"), (v, "v"), (decay, "decay"), (state, "state")):
+        _f32(t, nm)
+    H, dk, dv = state.shape[1:]
+    buf = torch.cat([q, k, v], dim=1).contiguous()
+    n, lib = q.shape[0], _lib.load()
+    nb = int(lib.sd_decay_chunks_scratch_bytes(n, entries.shape[0], H, dk, dv)) if cut else 0
+    scratch = torch.empty(nb, dtype=torch.uint8, device=q.device) if nb else None
+    out = torch.empty(n, H * dv, dtype=torch.float32, device=q.device)
+    _lib.check(lib.sd_decay_chunks(buf.data_ptr(), buf.data_ptr() + 4 * H * dk, buf.data_ptr() + 8 * H * dk, buf.shape[1],
+                                   _p(decay), float(q_scale), _p(state), _p(entries), entries.shape[0], n, _p(out), H, dk, dv,
+                                   _p(scratch), nb, _stream()), "sd_decay_chunks")
+    return out
+
+
 def matmul_rows_batched(x, w) -> torch.Tensor:
     """x f32 [M, B, K], w [B, N, K] -> f32 [M, B, N]: product b uses w[b]."""
     _f32(x, "x")
