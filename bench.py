@@ -102,7 +102,8 @@ def parse():
     ap.add_argument("--tp-draft", choices=["replicated", "sharded"], default="replicated",
                     help="the draft whole on every rank (no exchange in its passes), or sharded "
                          "like the target with a vocabulary-parallel head")
-    ap.add_argument("--family", choices=["spec", "puguzen", "naburax", "fepopel", "zopupel", "gufasun"], default="spec",
+    ap.add_argument("--family", choices=["spec", "puguzen", "naburax", "fepopel", "zopupel", "gufasun", "tovapel"],
+                    default="spec",
                     help="spec: the headline speculative-decoding workload (default).  puguzen: prefill and "
                          "decode throughput of the Puguzen decoder family (recurrent and windowed layers) at "
                          "layer sizes of real models, beside a Llama-style decoder of equal size, with the "
@@ -117,9 +118,12 @@ def parse():
                          "the Fepopel family at equal size.  gufasun: the same for the Gufasun family (both "
                          "sublayers on one residual, convolved window attention with a distance bias, matrix "
                          "memories with exponential gates), beside the Puguzen family at equal size and the "
-                         "Naburax family's like kernels")
+                         "Naburax family's like kernels.  tovapel: the same for the Tovapel family (several "
+                         "residual streams, window attention with kept first tokens beside linear attention "
+                         "with a decay per key channel, routed experts with identity experts), beside a Naburax "
+                         "model of attention beside a state-space recurrence at equal size")
     ap.add_argument("--seq-sizes", default="w1024,w2048,w4096",
-                    help="--family puguzen / naburax / fepopel / zopupel / gufasun: sizes to run")
+                    help="--family puguzen / naburax / fepopel / zopupel / gufasun / tovapel: sizes to run")
     return ap.parse_args()
 
 
@@ -1368,8 +1372,167 @@ def main_guf_family(args):
                       "data": "synthetic", "n_gpus": 1, "steps": steps, "warmup": warm, "sizes": results}))
 
 
+# ---------------------------------------------------------------------------------------------
+# --family tovapel
+TOV_STREAMS, TOV_RANK, TOV_TAU, TOV_LIMIT = 4, 16, 16.0, 7.0
+
+
+def _tov_config(sz):
+    """Four layers of both mixers with routed experts (as many with matrices as the Naburax bench model
+    has, and a quarter as many identity experts)."""
+    from vllm_omni_draft_amd.config import ExpertsSpec, LinearSpec, MixerSpec, SeqLayerSpec, SeqModelConfig
+    H, G, D = sz["heads"], sz["kv_heads"], SEQ_HEAD
+    m = MixerSpec("parallel", H, D, D, kv_heads=G, scale=D ** -0.5, softcap=50.0, window=SEQ_WINDOW, keep_first=NAB_KEEP,
+                  qkv_bias=True, qk_head_norm=True, sink=True, head_gate=True,
+                  linear=LinearSpec(heads=H, dim=D, vdim=D, rank=TOV_RANK, tau=TOV_TAU))
+    ex = ExpertsSpec(sz["experts"], sz["top"], sz["eff"], score="softmax", scale_input=False, act="clamped_gate",
+                     limit=TOV_LIMIT, correction=True, identity=sz["experts"] // 4)
+    cfg = SeqModelConfig("tovapel", sz["width"], SEQ_VOCAB, [SeqLayerSpec(m, 0, ex) for _ in range(4)], name="tovapel-bench",
+                         block="streams", tied_head=False, streams=TOV_STREAMS, logit_softcap=30.0)
+    cfg.validate()
+    return cfg
+
+
+def _nab_parallel_config(sz):
+    """The Naburax bench model with attention beside a state-space recurrence in every layer."""
+    cfg = _nab_config(sz)
+    cfg.layers = [cfg.layers[1]] * 4
+    cfg.validate()
+    return cfg
+
+
+def tov_kernel_rooflines(cfg, device, ctx, rows):
+    """The family's own kernels alone at `rows` token rows of one sequence that ends at position
+    ctx, as fep_kernel_rooflines reports them; `like` names the kernel of another family each is
+    set beside."""
+    from vllm_omni_draft_amd import ops
+    m, ex, W, S = cfg.layers[0].mixer, cfg.layers[0].experts, cfg.width, cfg.streams
+    r = m.linear
+    g = torch.Generator(device="cpu").manual_seed(0)
+    rn = lambda *s: torch.randn(*s, generator=g).to(device)
+    bf = lambda *s: torch.randn(*s, generator=g).to(torch.bfloat16).to(device)
+    pages = -(-ctx // ops.PAGE)
+    tables = torch.arange(pages, dtype=torch.int32, device=device).view(1, -1)
+    pos_l = list(range(ctx - rows, ctx))
+    pos = torch.tensor(pos_l, dtype=torch.int32, device=device)
+    slot = torch.zeros(rows, dtype=torch.int32, device=device)
+    ent = torch.tensor([[0, 0, rows, ctx - rows]], dtype=torch.int32, device=device)
+    seen = [min(p + 1, m.window + min(m.keep_first, max(p + 1 - m.window, 0))) for p in pos_l]
+    keys, span = sum(seen), min(ctx, m.window + rows - 1 + m.keep_first)
+    H, G, D = m.heads, m.kv_heads, m.dim
+    out = []
+    kc, vc, q = bf(pages, G, ops.PAGE, D), bf(pages, G, ops.PAGE, D), rn(rows, H * D)
+    sinks, gates = rn(H), rn(rows, H)
+    us = _events(lambda: ops.gated_softmax_attention(q, kc, vc, pos, slot, tables, H, G, D, D, m.scale, m.window,
+                                                     m.keep_first, m.softcap, sinks, gates, ent, bf16_only=True), 5)
+    # (matrix-core work where rows share their keys: priced at the f32 vector peak, like the kernel beside it)
+    out.append(("gated_softmax_attention", "window_softmax_attention (grouped heads)", us,
+                G * 2 * D * 2 * span + rows * H * D * 6, 2.0 * keys * H * 2 * D, F32_VALU_PEAK_TFLOPS))
+    buf = rn(rows, (H + 2 * G) * D)
+    parts = torch.split(buf, [H * D, G * D, G * D], dim=1)
+    bias, qw, kw = [bf(t.shape[1]) for t in parts], bf(D), bf(D)
+    us = _events(lambda: ops.biased_qkv_prep(*parts, bias, G, D, D, qw, kw, 1e-5, kc, vc, pos, slot, tables), 5)
+    out.append(("biased_qkv_prep", "qk_norm_append", us, rows * (8 * H * D + 12 * G * D), 0.0, F32_VALU_PEAK_TFLOPS))
+    Hr, dk, dv, rk = r.heads, r.dim, r.vdim, r.rank
+    buf2 = rn(rows, Hr * (2 * dk + 2 * dv) + rk)
+    sq, sk, sv, sg, a1 = torch.split(buf2, [Hr * dk, Hr * dk, Hr * dv, Hr * dv, rk], dim=1)
+    a2, ab, w = bf(Hr * dk, rk), rn(Hr * dk) + 3, bf(dv)
+    state = torch.zeros(1, Hr, dk, dv, device=device)
+    flops = rows * Hr * dk * dv * 5.0
+    if rows == 1:
+        us = _events(lambda: ops.decay_step_rows(sq, sk, sv, sg, a1, a2, ab, r.tau, state, w, 1e-5, pos, slot,
+                                                 q_scale=dk ** -0.5), 5)
+        out.append(("decay_step_rows (decays and read-out included)", "decay_scan_rows", us,
+                    4 * (2 * Hr * dk + 3 * Hr * dv + 2 * Hr * dk * dv) + 2 * Hr * dk * rk, flops, F32_VALU_PEAK_TFLOPS))
+        us = _events(lambda: ops.biased_qkv_prep(*parts, bias, G, D, D, qw, kw, 1e-5, kc, vc, pos, slot, tables,
+                                                 step=(sq, sk, sv, sg, a1, a2, ab, r.tau, state, w, dk ** -0.5)), 5)
+        out.append(("biased_qkv_prep with decay_step_rows (as a decoding step runs them)", "decay_scan_rows", us,
+                    4 * (2 * Hr * dk + 3 * Hr * dv + 2 * Hr * dk * dv) + 2 * Hr * dk * rk + 8 * H * D + 12 * G * D, flops,
+                    F32_VALU_PEAK_TFLOPS))
+    else:
+        ac = a1.contiguous()
+        us = _events(lambda: ops.low_rank_decay(ac, a2, ab, r.tau), 5)
+        out.append(("low_rank_decay", "ssd_steps", us, rows * 4 * (Hr * dk + rk), rows * Hr * dk * rk * 2.0,
+                    F32_VALU_PEAK_TFLOPS))
+        dec = ops.low_rank_decay(ac, a2, ab, r.tau)
+        scr = ops.decay_chunks_scratch(rows, 1, Hr, dk, dv, device)
+        us = _events(lambda: ops.decay_chunks(sq, sk, sv, dec, state, ent, q_scale=dk ** -0.5, scratch=scr), 5)
+        out.append(("decay_chunks", "decay_scan_rows", us, 4 * (rows * Hr * (3 * dk + 2 * dv) + 2 * Hr * dk * dv), flops,
+                    F32_VALU_PEAK_TFLOPS))
+    x, a, b = rn(rows, S, W), rn(rows, W), rn(rows, W)
+    wa, wb, wn, mix, outf, cin = bf(W), bf(W), bf(W), rn(S, S) * 0.1, rn(S), rn(S)
+    us = _events(lambda: ops.streams_residual(x, a=a, b=b, w_a=wa, w_b=wb, mix=mix, out=outf, in_=cin, w_next=wn, bf16=True), 5)
+    out.append(("streams_residual (two normed results)", "postnorm_residual", us, rows * W * (8 * S + 8 + 2), 0.0,
+                F32_VALU_PEAK_TFLOPS))
+    E, top, F = ex.experts, ex.top, ex.ff
+    h = rn(rows, W)
+    wr, corr = bf(ex.outputs, W), rn(ex.outputs) * 0.01
+    us = _events(lambda: ops.moe_route_rows_corrected(h, wr, corr, top), 5)
+    out.append(("moe_route_rows_corrected", "moe_route_rows", us, rows * 4 * W + 2 * ex.outputs * W,
+                2.0 * rows * ex.outputs * W, F32_VALU_PEAK_TFLOPS))
+    us = _events(lambda: ops.moe_route_rows(h, wr, top, "softmax"), 5)
+    out.append(("moe_route_rows (like kernel, same sizes)", "", us, rows * 4 * W + 2 * ex.outputs * W,
+                2.0 * rows * ex.outputs * W, F32_VALU_PEAK_TFLOPS))
+    gu = (torch.randn(E, 2 * F, W, generator=g) * W ** -0.5).to(torch.bfloat16).to(device)
+    dn = (torch.randn(E, W, F, generator=g) * F ** -0.5).to(torch.bfloat16).to(device)
+    sel_e = torch.stack([torch.randperm(E, generator=g)[:top] for _ in range(rows)]).to(torch.int32).to(device)
+    sel_w = torch.rand(rows, top, generator=g).to(device)
+    used = min(E, rows * top)
+    nbytes = 2 * used * 3 * F * W + 4 * rows * W * (1 + top) + 2 * rows * top * F * 2
+    us = _events(lambda: ops.moe_experts_clamped(h, sel_e, sel_w, gu, dn, ex.limit), 5)
+    out.append(("moe_experts_clamped (no identity chosen; wrapper's fill included)", "moe_experts", us, nbytes,
+                2.0 * rows * top * 3 * F * W, BF16_MFMA_PEAK_TFLOPS))
+    # the like kernels of other families at the same sizes
+    us = _events(lambda: ops.window_softmax_attention(q, kc, vc, pos, slot, tables, H, G, D, D, m.window, m.keep_first,
+                                                      m.scale), 5)
+    out.append(("window_softmax_attention (grouped heads; like kernel)", "", us, G * 2 * D * 2 * span + rows * H * D * 8,
+                2.0 * keys * H * 2 * D, F32_VALU_PEAK_TFLOPS))
+    dec1 = torch.rand(rows, Hr * dk, generator=g).to(device) * 0.1 + 0.9
+    us = _events(lambda: ops.decay_scan(sq.contiguous(), sk.contiguous(), sv.contiguous(), dec1, state, ent, Hr, dk, dv), 5)
+    out.append(("decay_scan (decay per channel; like kernel, wrapper copies included)", "", us,
+                4 * (rows * Hr * (3 * dk + 2 * dv) + 2 * Hr * dk * dv), flops, F32_VALU_PEAK_TFLOPS))
+    x1 = rn(rows, W)
+    us = _events(lambda: ops.postnorm_residual(x1, a, wa, 1e-5, b=b, sb=1.0), 5)
+    out.append(("postnorm_residual (like kernel)", "", us, rows * W * 16, 0.0, F32_VALU_PEAK_TFLOPS))
+    us = _events(lambda: ops.moe_experts(h, sel_e, sel_w, gu, dn, scale_input=False), 5)
+    out.append(("moe_experts (like kernel)", "", us, nbytes, 2.0 * rows * top * 3 * F * W, BF16_MFMA_PEAK_TFLOPS))
+    res = []
+    for name, like, us, nbytes, flops, peak in out:
+        floor_us = max(nbytes / (HBM_PEAK_GBS * 1e3), flops / (peak * 1e6))
+        res.append({"kernel": name, "like": like, "rows": rows, "ctx": ctx, "avg_us": round(us, 2),
+                    "min_bytes": int(nbytes), "flops": int(flops), "achieved_gbs": round(nbytes / us * 1e-3, 1),
+                    "achieved_tflops": round(flops / us * 1e-6, 2), "roofline_us": round(floor_us, 2),
+                    "times_roofline": round(us / floor_us, 1)})
+    return res
+
+
+def main_tov_family(args):
+    """Prefill and decode throughput of the Tovapel family beside a Naburax model of attention beside a
+    state-space recurrence at equal width, heads, window and experts (both bf16, seeded random weights),
+    one JSON line."""
+    if not torch.cuda.is_available():
+        raise SystemExit("bench.py needs a GPU (there is no CPU path)")
+    device = torch.device("cuda", 0)
+    P, B, steps, warm = args.prompt_len, 4, args.steps, args.warmup
+    results = []
+    for name in args.seq_sizes.split(","):
+        sz = NAB_SIZES[name]
+        cfg, ncfg = _tov_config(sz), _nab_parallel_config(sz)
+        mine = _run_seq_engine(cfg, device, P, B, steps, warm)
+        kern = tov_kernel_rooflines(cfg, device, P, 1) + tov_kernel_rooflines(cfg, device, P, min(P, 1024))
+        other = _run_seq_engine(ncfg, device, P, B, steps, warm)
+        results.append({"size": name, **sz, "layers": [l.mixer.kind for l in cfg.layers], "head_dim": SEQ_HEAD,
+                        "streams": TOV_STREAMS, "rank": TOV_RANK, "window": SEQ_WINDOW, "keep_first": NAB_KEEP,
+                        "prompt_len": P, "decode_batch": B, "tovapel": mine, "naburax_equal_size": other, "kernels": kern})
+    print(json.dumps({"metric": "tovapel_family_throughput", "unit": "tokens/s", "dtype": "bf16",
+                      "data": "synthetic", "n_gpus": 1, "steps": steps, "warmup": warm, "sizes": results}))
+
+
 def main():
     args = parse()
+    if args.family == "tovapel":
+        main_tov_family(args)
+        return
     if args.family == "gufasun":
         main_guf_family(args)
         return

@@ -24,7 +24,7 @@ template <> __device__ __forceinline__ void st_f<bf16_t>(bf16_t* p, float v) { *
 
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ float log_sigmoid_f(float z) {
-  return z >= 0.f ? -log1pf(expf(-z)) : z - log1pf(expf(z));
+  return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
 }
 
 // Sums of two numbers over a workgroup of up to 16 waves (butterfly inside each wave, then the waves in
@@ -79,7 +79,7 @@ template <int N> __device__ __forceinline__ void st_pack(bf16_t* p, const Pack<N
 template <typename T, int V, int SM>
 __global__ __launch_bounds__(1024) void streams_kernel(sd_streams_update g, int W, float eps, int round) {
   extern __shared__ float row[];   // [W]
-  __shared__ float red[32];
+  __shared__ float red[32], f_mix[SM * SM], f_out[SM], f_in[SM];
   const int i = blockIdx.x, r = g.rows ? g.rows[i] : i, S = g.streams, np = W / V, nthr = blockDim.x, tid = threadIdx.x;
   float* xr = g.x + (size_t)r * S * W;
   const bool enter = g.tokens != nullptr, pair = g.b != nullptr;
@@ -131,13 +131,23 @@ __global__ __launch_bounds__(1024) void streams_kernel(sd_streams_update g, int 
     return y;
   };
   const bool mine = tid < np;
-  Pack<V> x0[SM], a0, b0, wn;
+  Pack<V> x0[SM], a0, b0, wn, wa0, wb0;
   if (mine) {
     load_x(tid * V, x0);
     if (g.a) a0 = load_a(tid * V);
-    if (pair) b0 = ld_pack<V>(g.b + (size_t)r * g.lda + tid * V);
+    if (pair) {
+      b0 = ld_pack<V>(g.b + (size_t)r * g.lda + tid * V);
+      wa0 = ld_pack<V>((const T*)g.w_a + tid * V);
+      wb0 = ld_pack<V>((const T*)g.w_b + tid * V);
+    }
     if (g.w_next) wn = ld_pack<V>((const T*)g.w_next + tid * V);
   }
+  for (int c = tid; c < SM * SM; c += nthr) f_mix[c] = g.a && c / SM < S && c % SM < S ? g.mix[c / SM * S + c % SM] : 0.f;
+  if (tid < SM) {
+    f_out[tid] = g.a && tid < S ? g.out[tid] : 0.f;
+    f_in[tid] = tid < S ? (g.in ? g.in[tid] : 1.f) : 0.f;
+  }
+  if (!pair) __syncthreads();      // (a pair's sums wait for all threads anyway)
   float ra = 1.f, rb = 0.f;
   if (pair) {
     float sa = 0.f, sb = 0.f;
@@ -167,7 +177,8 @@ __global__ __launch_bounds__(1024) void streams_kernel(sd_streams_update g, int 
       y = p == tid ? a0 : load_a(c);
       if (pair) {
         const Pack<V> b = p == tid ? b0 : ld_pack<V>(g.b + (size_t)r * g.lda + c);
-        const Pack<V> wa = ld_pack<V>((const T*)g.w_a + c), wb = ld_pack<V>((const T*)g.w_b + c);
+        const Pack<V> wa = p == tid ? wa0 : ld_pack<V>((const T*)g.w_a + c);
+        const Pack<V> wb = p == tid ? wb0 : ld_pack<V>((const T*)g.w_b + c);
 #pragma unroll
         for (int k = 0; k < V; ++k) y.v[k] = 0.5f * (y.v[k] * ra * wa.v[k] + b.v[k] * rb * wb.v[k]);
       }
@@ -180,13 +191,13 @@ __global__ __launch_bounds__(1024) void streams_kernel(sd_streams_update g, int 
       if (t < S) {
         Pack<V> n = xs[t];
         if (g.a) {
-          const float ot = g.out[t];
+          const float ot = f_out[t];
 #pragma unroll
           for (int k = 0; k < V; ++k) n.v[k] = 0.f;
 #pragma unroll
           for (int s = 0; s < SM; ++s)
             if (s < S) {
-              const float m = g.mix[s * S + t];
+              const float m = f_mix[s * SM + t];
 #pragma unroll
               for (int k = 0; k < V; ++k) n.v[k] = fmaf(m, xs[s].v[k], n.v[k]);
             }
@@ -194,7 +205,7 @@ __global__ __launch_bounds__(1024) void streams_kernel(sd_streams_update g, int 
           for (int k = 0; k < V; ++k) n.v[k] = fmaf(ot, y.v[k], n.v[k]);
         }
         if ((g.a || enter) && !g.rows) st_pack<V>(xr + (size_t)t * W + c, n);
-        const float in = g.in ? g.in[t] : 1.f;
+        const float in = f_in[t];
 #pragma unroll
         for (int k = 0; k < V; ++k) {
           sum.v[k] += n.v[k];
@@ -228,11 +239,12 @@ template <typename T, int V>
 void launch_streams(const sd_streams_update& g, int n, int W, float eps, int round, hipStream_t st) {
   int nthr = (W / V + 63) / 64 * 64;
   if (nthr > 1024) nthr = 1024;
+  const int nthr1 = W >= 1024 ? 1024 : (W + 63) / 64 * 64;
   const size_t lds = sizeof(float) * W;
   if (g.streams <= 2) streams_kernel<T, V, 2><<<n, nthr, lds, st>>>(g, W, eps, round);
   else if (g.streams <= 4) streams_kernel<T, V, 4><<<n, nthr, lds, st>>>(g, W, eps, round);
-  else if (g.streams <= 8) streams_kernel<T, V, 8><<<n, nthr, lds, st>>>(g, W, eps, round);
-  else streams_kernel<T, V, 16><<<n, nthr, lds, st>>>(g, W, eps, round);
+  else if (g.streams <= 8) streams_kernel<T, 1, 8><<<n, nthr1, lds, st>>>(g, W, eps, round);   // (registers)
+  else streams_kernel<T, 1, 16><<<n, nthr1, lds, st>>>(g, W, eps, round);
 }
 
 // z = cap tanh(z / cap), in place
@@ -264,50 +276,66 @@ struct QkvArgs {
 };
 constexpr int kUnitRegs = 8;    // channels per lane at most: a head has up to 512
 // One head of a row, by one wave: units 0 .. H-1 query heads (bias, norm, in place), then G key heads
-// (bias, norm, appended), then G value heads (bias, appended).
-template <typename T>
-__device__ __forceinline__ void qkv_unit(const QkvArgs& g, int r, int unit) {
+// (bias, norm, appended), then G value heads (bias, appended).  NC: channels per lane (loads run unguarded, on channels clamped into the head).
+template <typename T, int NC>
+__device__ __forceinline__ void head_prep(const float* __restrict__ src, const T* __restrict__ bias,
+                                          const T* __restrict__ w, int d, float eps, float* q_dst, T* c_dst) {
   const int lane = threadIdx.x & 63;
-  const bool is_q = unit < g.H, is_v = unit >= g.H + g.G;
-  const int head = is_q ? unit : (is_v ? unit - g.H - g.G : unit - g.H), d = is_v ? g.dv : g.dk;
-  const float* src = (is_q ? g.q : (is_v ? g.v : g.k)) + (size_t)r * g.ld + (size_t)head * d;
-  const T* bias = (const T*)(is_q ? g.q_bias : (is_v ? g.v_bias : g.k_bias));
-  float val[kUnitRegs], ss = 0.f;
+  float val[NC], wt[NC], bs[NC], ss = 0.f;
 #pragma unroll
-  for (int k = 0; k < kUnitRegs; ++k) {
+  for (int k = 0; k < NC; ++k) {
+    const int c = lane + 64 * k < d ? lane + 64 * k : d - 1;
+    val[k] = src[c];
+    bs[k] = bias ? ld_f(bias + c) : 0.f;
+    wt[k] = w ? ld_f(w + c) : 1.f;
+  }
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    val[k] += bs[k];
+    if (lane + 64 * k < d) ss = fmaf(val[k], val[k], ss);
+  }
+  const float rstd = w ? 1.f / sqrtf(wave_sum(ss) / (float)d + eps) : 1.f;
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
     const int c = lane + 64 * k;
     if (c < d) {
-      val[k] = src[c];
-      if (bias) val[k] += ld_f(bias + (size_t)head * d + c);
-      ss = fmaf(val[k], val[k], ss);
-    }
-  }
-  float rstd = 1.f;
-  const T* w = nullptr;
-  if (!is_v) {
-    w = (const T*)(is_q ? g.q_w : g.k_w);
-    rstd = 1.f / sqrtf(wave_sum(ss) / (float)d + g.eps);
-  }
-  T* dst = nullptr;
-  if (!is_q) {
-    const int pos = g.row_pos[r];
-    const int pg = g.block_tables[(size_t)g.row_slot[r] * g.max_blocks + pos / g.page];
-    dst = (T*)(is_v ? g.v_cache : g.k_cache) + (((size_t)pg * g.G + head) * g.page + pos % g.page) * d;
-  }
-  float* qdst = g.q + (size_t)r * g.ld + (size_t)head * d;
-#pragma unroll
-  for (int k = 0; k < kUnitRegs; ++k) {
-    const int c = lane + 64 * k;
-    if (c < d) {
-      const float o = w ? val[k] * rstd * ld_f(w + c) : val[k];
-      if (is_q) qdst[c] = o;
-      else st_f(dst + c, o);
+      const float o = val[k] * rstd * wt[k];
+      if (q_dst) q_dst[c] = o;
+      else st_f(c_dst + c, o);
     }
   }
 }
+template <typename T, int NC>
+__device__ __forceinline__ void qkv_unit_nc(const QkvArgs& g, int r, int unit) {
+  if (unit < g.H) {
+    float* q = g.q + (size_t)r * g.ld + (size_t)unit * g.dk;
+    head_prep<T, NC>(q, g.q_bias ? (const T*)g.q_bias + (size_t)unit * g.dk : nullptr, (const T*)g.q_w, g.dk, g.eps, q, nullptr);
+    return;
+  }
+  const int pos = g.row_pos[r];
+  const int pg = g.block_tables[(size_t)g.row_slot[r] * g.max_blocks + pos / g.page];
+  unit -= g.H;
+  if (unit < g.G) {
+    head_prep<T, NC>(g.k + (size_t)r * g.ld + (size_t)unit * g.dk,
+                     g.k_bias ? (const T*)g.k_bias + (size_t)unit * g.dk : nullptr, (const T*)g.k_w, g.dk, g.eps, nullptr,
+                     (T*)g.k_cache + (((size_t)pg * g.G + unit) * g.page + pos % g.page) * g.dk);
+    return;
+  }
+  unit -= g.G;
+  head_prep<T, NC>(g.v + (size_t)r * g.ld + (size_t)unit * g.dv,
+                   g.v_bias ? (const T*)g.v_bias + (size_t)unit * g.dv : nullptr, (const T*)nullptr, g.dv, g.eps, nullptr,
+                   (T*)g.v_cache + (((size_t)pg * g.G + unit) * g.page + pos % g.page) * g.dv);
+}
+template <typename T>
+__device__ __forceinline__ void qkv_unit(const QkvArgs& g, int r, int unit) {
+  const int d = g.dk > g.dv ? g.dk : g.dv;
+  if (d <= 64) qkv_unit_nc<T, 1>(g, r, unit);
+  else if (d <= 128) qkv_unit_nc<T, 2>(g, r, unit);
+  else qkv_unit_nc<T, kUnitRegs>(g, r, unit);
+}
 template <typename T>
 __global__ __launch_bounds__(256) void qkv_prep_kernel(QkvArgs g) {
-  const int unit = blockIdx.y * 4 + (threadIdx.x >> 6);
+  const int unit = blockIdx.y * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   if (unit < g.H + 2 * g.G) qkv_unit<T>(g, blockIdx.x, unit);
 }
 
@@ -316,8 +344,19 @@ __global__ __launch_bounds__(256) void qkv_prep_kernel(QkvArgs g) {
 template <typename T>
 __device__ __forceinline__ float low_rank_decay(const float* a1, const T* a2, int rank, float b, float inv_tau) {
   float z = 0.f;
-#pragma unroll 8
-  for (int j = 0; j < rank; ++j) z = fmaf(a1[j], ld_f(a2 + j), z);
+  constexpr int U = 16;            // loads in flight, on indices clamped into the row
+  for (int j0 = 0; j0 < rank; j0 += U) {
+    float x[U], w[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int j = j0 + u < rank ? j0 + u : rank - 1;
+      x[u] = a1[j];
+      w[u] = ld_f(a2 + j);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (j0 + u < rank) z = fmaf(x[u], w[u], z);
+  }
   return expf(log_sigmoid_f(z + b) * inv_tau);
 }
 // A thread per channel, kDecayRows rows per workgroup; the rows' a1 in LDS, the channel's a2 row in
@@ -328,25 +367,42 @@ __global__ __launch_bounds__(256) void low_rank_decay_kernel(const float* __rest
                                                             const T* __restrict__ a2, const float* __restrict__ bias,
                                                             int rank, float inv_tau, float* __restrict__ out, int n_rows,
                                                             int n_cols) {
-  extern __shared__ float as[];   // [kDecayRows][rank]
+  extern __shared__ float as[];   // [kDecayRows][RK, or rank]
   const int r0 = blockIdx.x * kDecayRows, nr = n_rows - r0 < kDecayRows ? n_rows - r0 : kDecayRows;
-  for (int i = threadIdx.x; i < nr * rank; i += 256) as[i] = a1[(size_t)(r0 + i / rank) * ld + i % rank];
+  constexpr bool regs = RK > 0;
+  const int lda = regs ? RK : rank;
+  for (int i = threadIdx.x; i < nr * lda; i += 256) {
+    const int j = i % lda;
+    as[i] = j < rank ? a1[(size_t)(r0 + i / lda) * ld + j] : 0.f;
+  }
   const int c = blockIdx.y * 256 + threadIdx.x, cc = c < n_cols ? c : n_cols - 1;
   const T* w = a2 + (size_t)cc * rank;
   float wr[RK > 0 ? RK : 1];
   if constexpr (RK > 0) {
+    if (rank % 4 == 0) {           // (a row is then aligned to four elements, like the matrix)
 #pragma unroll
-    for (int j = 0; j < RK; ++j) wr[j] = j < rank ? ld_f(w + j) : 0.f;
+      for (int j = 0; j < RK; j += 4) {
+        const Pack<4> p = ld_pack<4>(w + (j < rank ? j : 0));
+#pragma unroll
+        for (int k = 0; k < 4; ++k) wr[j + k] = j < rank ? p.v[k] : 0.f;
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < RK; ++j) {
+        const float v = ld_f(w + (j < rank ? j : 0));
+        wr[j] = j < rank ? v : 0.f;
+      }
+    }
   }
   const float b = bias[cc];
   __syncthreads();
   if (c >= n_cols) return;
+#pragma unroll 4
   for (int i = 0; i < nr; ++i) {
     float z = 0.f;
     if constexpr (RK > 0) {
 #pragma unroll
-      for (int j = 0; j < RK; ++j)
-        if (j < rank) z = fmaf(as[i * rank + j], wr[j], z);
+      for (int j = 0; j < RK; ++j) z = fmaf(as[i * RK + j], wr[j], z);   // (zeros behind the rank)
     } else {
       for (int j = 0; j < rank; ++j) z = fmaf(as[i * rank + j], ld_f(w + j), z);
     }
@@ -373,7 +429,7 @@ __global__ __launch_bounds__(1024) void decay_step_kernel(StepArgs a, QkvArgs g,
   const sd_decay_step& s = a.s;
   const int r = blockIdx.y, h = blockIdx.x, H = s.heads, dk = s.dim, dv = s.vdim, tid = threadIdx.x;
   if (h >= H) {
-    const int unit = (h - H) * (blockDim.x >> 6) + (tid >> 6);
+    const int unit = (h - H) * (blockDim.x >> 6) + __builtin_amdgcn_readfirstlane(tid >> 6);
     if (with_qkv && unit < g.H + 2 * g.G) qkv_unit<T>(g, r, unit);
     return;
   }
@@ -451,8 +507,8 @@ __global__ __launch_bounds__(1024) void decay_step_kernel(StepArgs a, QkvArgs g,
 //   S  <- diag(P_last) S + (k_s R_s)^T v_s
 // Every factor is a product of decays, at most one: nothing is divided, however strong the decay.  The
 // inner sums of a block are formed channel by channel with running products.  A wave owns 16 value
-// columns (two such sets); its part of S lives in accumulators, whose layout is that of the right
-// operand of q S as it is (the key channels of an MFMA step in the order the accumulators hold them).
+// columns; its part of S lives in accumulators, whose layout is that of the right operand of q S as it is
+// (the key channels of an MFMA step in the order the accumulators hold them).
 //
 // A long portion is cut into chunks of tokens that run side by side: every chunk's own sum from a zero
 // state (kSums), the states at the chunks' starts (chunk_carry_kernel, chunk after chunk), then the
@@ -475,6 +531,7 @@ struct ChunkArgs {
 constexpr int kBlock = 16;       // tokens of a block
 constexpr int kBlockCols = 128;  // value columns per workgroup
 constexpr int kTokLd = kBlock + 4;
+constexpr int kChunkThreads = 512;
 
 // The portion and the first row (inside it) of the n-th group of `per` rows over all portions.
 __device__ __forceinline__ bool nth_group(const int32_t* entries, int n_entries, int per, int n, int* e, int* first) {
@@ -492,12 +549,12 @@ __device__ __forceinline__ bool nth_group(const int32_t* entries, int n_entries,
 // Up to 16 rows of up to COLS columns on their way from memory to LDS, V columns a piece.
 template <int COLS, int V>
 struct BlockRows {
-  static constexpr int PIECES = kBlock * COLS / V, N = (PIECES + 255) / 256;
+  static constexpr int PIECES = kBlock * COLS / V, N = (PIECES + kChunkThreads - 1) / kChunkThreads;
   Pack<V> v[N];
   __device__ __forceinline__ void load(const float* src, int64_t ld, int rows, int cols) {
 #pragma unroll
     for (int u = 0; u < N; ++u) {
-      const int idx = threadIdx.x + 256 * u, t = idx / (COLS / V), c = idx % (COLS / V) * V;
+      const int idx = threadIdx.x + kChunkThreads * u, t = idx / (COLS / V), c = idx % (COLS / V) * V;
       v[u] = ld_pack<V>(src + (size_t)(t < rows ? t : rows - 1) * ld + (c < cols ? c : cols - V));
     }
   }
@@ -505,8 +562,8 @@ struct BlockRows {
   __device__ __forceinline__ void store(float* dst, int ldd, int rows, int cols, float f, float pad) {
 #pragma unroll
     for (int u = 0; u < N; ++u) {
-      const int idx = threadIdx.x + 256 * u, t = idx / (COLS / V), c = idx % (COLS / V) * V;
-      if (PIECES % 256 != 0 && idx >= PIECES) continue;
+      const int idx = threadIdx.x + kChunkThreads * u, t = idx / (COLS / V), c = idx % (COLS / V) * V;
+      if (PIECES % kChunkThreads != 0 && idx >= PIECES) continue;
       Pack<V> p;
 #pragma unroll
       for (int e = 0; e < V; ++e) p.v[e] = t < rows && c < cols ? v[u].v[e] * f : pad;
@@ -521,7 +578,7 @@ constexpr size_t decay_chunk_lds() {
                           (size_t)kBlock * (kBlockCols + 4) + (size_t)kBlock * kTokLd);
 }
 template <int DKP, int V, int MODE>   // keys of up to DKP channels
-__global__ __launch_bounds__(256) void decay_chunk_kernel(ChunkArgs g) {
+__global__ __launch_bounds__(kChunkThreads, DKP <= 128 ? 4 : 2) void decay_chunk_kernel(ChunkArgs g) {
   extern __shared__ float lds[];
   constexpr int LDK = DKP + 4, LDV = kBlockCols + 4, KT = DKP / 16;
   float* qs = lds;                     // [16][LDK]
@@ -559,26 +616,21 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(ChunkArgs g) {
     rv.load(g.v + row * g.ld + (size_t)h * dv + c0, g.ld, n, cols);
   };
   fetch(0);
-  f32x4 S[2][KT];
+  const int c = 16 * wave + col;       // this wave's columns of the state; rows 16 * kt + 4 * quad + i
+  const bool works = 16 * wave < cols;
+  f32x4 S[KT];
 #pragma unroll
-  for (int u = 0; u < 2; ++u)
-#pragma unroll
-    for (int kt = 0; kt < KT; ++kt) S[u][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
-  // this wave's columns of the state: 16 * (wave + 4 * u) + col; rows 16 * kt + 4 * quad + i
+  for (int kt = 0; kt < KT; ++kt) S[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
   if (MODE == kReads || (MODE == kWhole && kept)) {
-    const float* s0 = MODE == kReads ? g.cs + at * dv + c0 : slot_state;
+    const float* s0 = (MODE == kReads ? g.cs + at * dv + c0 : slot_state) + (c < cols ? c : cols - 1);
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const int c = 16 * (wave + 4 * u) + col;
+    for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
-      for (int kt = 0; kt < KT; ++kt)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int k = 16 * kt + 4 * quad + i;
-          const float s = s0[(size_t)(k < dk ? k : dk - 1) * dv + (c < cols ? c : cols - 1)];
-          S[u][kt][i] = k < dk && c < cols ? s : 0.f;
-        }
-    }
+      for (int i = 0; i < 4; ++i) {
+        const int k = 16 * kt + 4 * quad + i;
+        const float s = s0[(size_t)(k < dk ? k : dk - 1) * dv];
+        S[kt][i] = k < dk && c < cols ? s : 0.f;
+      }
   }
   float run = 1.f;                     // kSums: product of the chunk's decays, thread < DKP a channel
   for (int t0 = 0; t0 < nt; t0 += kBlock) {
@@ -590,137 +642,134 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(ChunkArgs g) {
     rv.store(vs, LDV, n, cols, 1.f, 0.f);
     __syncthreads();
     if (t0 + kBlock < nt) fetch(t0 + kBlock);
-    // products of decays, a thread per channel: the first half of the threads forward, the others backward
-    if (DKP > 128 || tid < 128) {
-      const int c = tid;
-      if (c < DKP) {
-        float p = 1.f;
+    // products of decays, a thread per channel: forward, and (other threads) backward
+    if (tid < DKP) {
+      float d[kBlock], p = 1.f;
+#pragma unroll
+      for (int t = 0; t < kBlock; ++t) d[t] = ds[t * LDK + tid];
+      if constexpr (MODE != kSums) {
+        float q[kBlock];
+#pragma unroll
+        for (int t = 0; t < kBlock; ++t) q[t] = qs[t * LDK + tid];
 #pragma unroll
         for (int t = 0; t < kBlock; ++t) {
-          p *= ds[t * LDK + c];
-          if constexpr (MODE != kSums) qp[t * LDK + c] = qs[t * LDK + c] * p;
+          p *= d[t];
+          qp[t * LDK + tid] = q[t] * p;
         }
-        tot[c] = p;
-        run *= p;
-      }
-    }
-    if (DKP > 128 || tid >= 128) {
-      const int c = DKP > 128 ? tid : tid - 128;
-      if (c < DKP) {
-        float p = 1.f, w[kBlock];
+      } else {
 #pragma unroll
-        for (int t = kBlock - 1; t >= 0; --t) {
-          w[t] = ks[t * LDK + c] * p;
-          p *= ds[t * LDK + c];
-        }
-#pragma unroll
-        for (int t = 0; t < kBlock; t += 4)
-          *reinterpret_cast<f32x4*>(kr + c * kTokLd + t) = f32x4{w[t], w[t + 1], w[t + 2], w[t + 3]};
+        for (int t = 0; t < kBlock; ++t) p *= d[t];
       }
+      tot[tid] = p;
+      run *= p;
+    } else if (tid < 2 * DKP) {
+      const int ch = tid - DKP;
+      float d[kBlock], w[kBlock], p = 1.f;
+#pragma unroll
+      for (int t = 0; t < kBlock; ++t) {
+        d[t] = ds[t * LDK + ch];
+        w[t] = ks[t * LDK + ch];
+      }
+#pragma unroll
+      for (int t = kBlock - 1; t >= 0; --t) {
+        w[t] *= p;
+        p *= d[t];
+      }
+#pragma unroll
+      for (int t = 0; t < kBlock; t += 4)
+        *reinterpret_cast<f32x4*>(kr + ch * kTokLd + t) = f32x4{w[t], w[t + 1], w[t + 2], w[t + 3]};
     }
     if constexpr (MODE != kSums) {
-      // inner sums: this wave's tokens s = wave, wave + 4, ..; a lane per channel; then 64 sums over 64
+      // inner sums: this wave's tokens s = wave and wave + 8; a lane per channel; then 32 sums over 64
       // lanes, halving the number of values a lane holds at every exchange
-      float a[64];
+      float a[32];
 #pragma unroll
-      for (int i = 0; i < 64; ++i) a[i] = 0.f;
+      for (int i = 0; i < 32; ++i) a[i] = 0.f;
 #pragma unroll
       for (int c1 = 0; c1 < (DKP + 63) / 64; ++c1) {
-        const int c = lane + 64 * c1;
-        if (DKP >= 64 || lane < DKP) {
-          float w[4];
+        const int ch = DKP >= 64 ? lane + 64 * c1 : (lane < DKP ? lane : DKP - 1);
+        float d[kBlock], q[kBlock], w[2];
 #pragma unroll
-          for (int j = 0; j < 4; ++j) w[j] = ks[(wave + 4 * j) * LDK + c];
-#pragma unroll
-          for (int t = 0; t < kBlock; ++t) {
-            const float d = ds[t * LDK + c], q = qs[t * LDK + c];
-#pragma unroll
-            for (int j = 0; j < 4; ++j) {
-              const int s = wave + 4 * j;
-              if (t > s) w[j] *= d;
-              if (t >= s) a[16 * j + t] = fmaf(q, w[j], a[16 * j + t]);
-            }
-          }
+        for (int t = 0; t < kBlock; ++t) {
+          d[t] = ds[t * LDK + ch];
+          q[t] = qs[t * LDK + ch];
         }
+#pragma unroll
+        for (int j = 0; j < 2; ++j) w[j] = ks[(wave + 8 * j) * LDK + ch];
+        if (DKP < 64 && lane >= DKP) w[0] = w[1] = 0.f;
+#pragma unroll
+        for (int j = 0; j < 2; ++j)
+#pragma unroll
+          for (int t = 8 * j; t < kBlock; ++t) {
+            const int dt = t - 8 * j;   // (against the wave's number, which is below 8)
+            w[j] *= dt > 7 || dt > wave ? d[t] : 1.f;
+            a[16 * j + t] = fmaf(dt > 7 || dt >= wave ? q[t] : 0.f, w[j], a[16 * j + t]);
+          }
       }
 #pragma unroll
-      for (int b = 0; b < 6; ++b) {
-        const int half = 32 >> b;
+      for (int b = 0; b < 5; ++b) {
+        const int half = 16 >> b;
         const bool up = (lane >> b) & 1;
 #pragma unroll
         for (int i = 0; i < half; ++i) {
-          const float give = up ? a[i] : a[i + half], hold = up ? a[i + half] : a[i];
-          a[i] = hold + __shfl_xor(give, 1 << b, SD_WAVE);
+          const float lo = a[i], hi = a[i + half];
+          a[i] = (up ? hi : lo) + __shfl_xor(up ? lo : hi, 1 << b, SD_WAVE);
         }
       }
-      const int idx = (int)(__brev((unsigned)lane) >> 26);       // the value that this lane is left with
-      as[(idx & 15) * kTokLd + wave + 4 * (idx >> 4)] = a[0];
+      a[0] += __shfl_xor(a[0], 32, SD_WAVE);
+      const int idx = (int)(__brev((unsigned)lane) >> 27);       // the value that this lane is left with
+      if (lane < 32) as[(idx & 15) * kTokLd + wave + 8 * (idx >> 4)] = a[0];
     }
     __syncthreads();
-    f32x4 vv[2];
+    if (!works) continue;
+    f32x4 vv;
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) vv[u][i] = vs[(4 * quad + i) * LDV + 16 * (wave + 4 * u) + col];
-    const bool two = 16 * (wave + 4) < cols;                     // (whether the second set has columns)
+    for (int i = 0; i < 4; ++i) vv[i] = vs[(4 * quad + i) * LDV + c];
     if constexpr (MODE != kSums) {
-      f32x4 o[2];
-      o[0] = o[1] = f32x4{0.f, 0.f, 0.f, 0.f};
+      f32x4 o = {0.f, 0.f, 0.f, 0.f}, o2 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kt = 0; kt < KT; ++kt) {
         const f32x4 a = *reinterpret_cast<const f32x4*>(qp + col * LDK + 16 * kt + 4 * quad);
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          o[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], S[0][kt][i], o[0], 0, 0, 0);
-          if (two) o[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], S[1][kt][i], o[1], 0, 0, 0);
+          f32x4& acc = i & 1 ? o2 : o;
+          acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], S[kt][i], acc, 0, 0, 0);
         }
       }
       const f32x4 a = *reinterpret_cast<const f32x4*>(as + col * kTokLd + 4 * quad);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        o[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], vv[0][i], o[0], 0, 0, 0);
-        if (two) o[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], vv[1][i], o[1], 0, 0, 0);
+        f32x4& acc = i & 1 ? o2 : o;
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], vv[i], acc, 0, 0, 0);
       }
+      o += o2;
 #pragma unroll
-      for (int u = 0; u < 2; ++u)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int t = 4 * quad + i, c = 16 * (wave + 4 * u) + col;
-          if (t < n && c < cols) g.out[(size_t)(row0 + t0 + t) * H * dv + (size_t)h * dv + c0 + c] = o[u][i];
-        }
+      for (int i = 0; i < 4; ++i) {
+        const int t = 4 * quad + i;
+        if (t < n && c < cols) g.out[(size_t)(row0 + t0 + t) * H * dv + (size_t)h * dv + c0 + c] = o[i];
+      }
     }
     if (MODE != kReads || t0 + kBlock < nt) {
 #pragma unroll
+      for (int kt = 0; kt < KT; ++kt) S[kt] *= *reinterpret_cast<const f32x4*>(tot + 16 * kt + 4 * quad);
+#pragma unroll
       for (int kt = 0; kt < KT; ++kt) {
-        const f32x4 f = *reinterpret_cast<const f32x4*>(tot + 16 * kt + 4 * quad);
         const f32x4 a = *reinterpret_cast<const f32x4*>(kr + (16 * kt + col) * kTokLd + 4 * quad);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          S[0][kt][i] *= f[i];
-          S[1][kt][i] *= f[i];
-        }
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          S[0][kt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], vv[0][i], S[0][kt], 0, 0, 0);
-          if (two) S[1][kt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], vv[1][i], S[1][kt], 0, 0, 0);
-        }
+        for (int i = 0; i < 4; ++i) S[kt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], vv[i], S[kt], 0, 0, 0);
       }
     }
   }
   if constexpr (MODE != kReads) {
     float* dst = MODE == kSums ? g.cs + at * dv + c0 : slot_state;
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const int c = 16 * (wave + 4 * u) + col;
+    for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
-      for (int kt = 0; kt < KT; ++kt)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int k = 16 * kt + 4 * quad + i;
-          if (k < dk && c < cols) dst[(size_t)k * dv + c] = S[u][kt][i];
-        }
-    }
-    if (MODE == kSums && blockIdx.z == 0 && tid < DKP && tid < dk && (DKP > 128 || tid < 128)) g.ct[at + tid] = run;
+      for (int i = 0; i < 4; ++i) {
+        const int k = 16 * kt + 4 * quad + i;
+        if (k < dk && c < cols) dst[(size_t)k * dv + c] = S[kt][i];
+      }
+    if (MODE == kSums && blockIdx.z == 0 && tid < dk) g.ct[at + tid] = run;
   }
 }
 
@@ -771,11 +820,11 @@ hipError_t launch_decay_chunks(const ChunkArgs& c, size_t nc, hipStream_t st) {
   constexpr size_t lds = decay_chunk_lds<DKP>();
   const unsigned z = (c.dv + kBlockCols - 1) / kBlockCols;
   if (nc == 0) {
-    decay_chunk_kernel<DKP, V, kWhole><<<dim3(c.n_entries, c.H, z), 256, lds, st>>>(c);
+    decay_chunk_kernel<DKP, V, kWhole><<<dim3(c.n_entries, c.H, z), kChunkThreads, lds, st>>>(c);
   } else {
-    decay_chunk_kernel<DKP, V, kSums><<<dim3((unsigned)nc, c.H, z), 256, lds, st>>>(c);
+    decay_chunk_kernel<DKP, V, kSums><<<dim3((unsigned)nc, c.H, z), kChunkThreads, lds, st>>>(c);
     chunk_carry_kernel<<<dim3((c.dk * c.dv + 255) / 256, c.H, c.n_entries), 256, 0, st>>>(c);
-    decay_chunk_kernel<DKP, V, kReads><<<dim3((unsigned)nc, c.H, z), 256, lds, st>>>(c);
+    decay_chunk_kernel<DKP, V, kReads><<<dim3((unsigned)nc, c.H, z), kChunkThreads, lds, st>>>(c);
   }
   return hipGetLastError();
 }
@@ -897,8 +946,9 @@ extern "C" int sd_low_rank_decay(const float* a1, int64_t ld, const void* a2, co
   SD_REQUIRE(a1 && a2 && a2_bias && out && n_rows >= 1 && n_cols >= 1 && rank >= 1 && ld >= rank && tau > 0.f,
              SD_ERR_INVALID, "sd_low_rank_decay: bad argument");
   SD_REQUIRE(rank <= 1536, SD_ERR_UNSUPPORTED, "sd_low_rank_decay: rank %d above 1536", rank);
+  SD_REQUIRE(sd_aligned16(a2), SD_ERR_INVALID, "sd_low_rank_decay: a2 unaligned");
   const dim3 grid((n_rows + kDecayRows - 1) / kDecayRows, (n_cols + 255) / 256);
-  const size_t lds = sizeof(float) * kDecayRows * rank;
+  const size_t lds = sizeof(float) * kDecayRows * (rank <= 16 ? 16 : (rank <= 64 ? 64 : rank));
   hipStream_t st = (hipStream_t)stream;
 #define SD_GO(T)                                                                                                        \
   do {                                                                                                                  \

@@ -1710,11 +1710,22 @@ def streams_residual(x, *, tokens=None, embed=None, a=None, n_a=1, sel=None, inp
     return (hb if bf16 else h), copy
 
 
-def _decay_step(buf, sizes, a2, a2_bias, tau, q_scale, state, norm_w, y):
-    """The sd_decay_step over buf [rows, ld], which stacks q, k, v, gate, a1 at column `sizes` starts."""
+def _side_by_side(*parts):
+    """(addresses, row stride, what must stay alive) of f32 matrices whose rows are equally far apart: column
+    slices of one buffer as they are, others copied into one."""
+    ld = parts[0].stride(0)
+    if not all(t.dtype == torch.float32 and t.stride(1) == 1 and t.stride(0) == ld for t in parts) \
+            or len({t.untyped_storage().data_ptr() for t in parts}) > 1:
+        buf = torch.cat(parts, dim=1).contiguous()
+        parts = torch.split(buf, [t.shape[1] for t in parts], dim=1)
+        ld = buf.shape[1]
+    return [t.data_ptr() for t in parts], ld, parts
+
+
+def _decay_step(p, ld, a2, a2_bias, tau, q_scale, state, norm_w, y):
+    """The sd_decay_step over q, k, v, gate, a1 at the addresses p."""
     H, dk, dv = state.shape[1:]
-    p = [buf.data_ptr() + 4 * s for s in sizes]
-    return _lib.DecayStep(q=p[0], k=p[1], v=p[2], a1=p[4], gate=p[3], ld=buf.shape[1], a2=_p(a2), a2_bias=_p(a2_bias),
+    return _lib.DecayStep(q=p[0], k=p[1], v=p[2], a1=p[4], gate=p[3], ld=ld, a2=_p(a2), a2_bias=_p(a2_bias),
                           rank=a2.shape[1], tau=float(tau), q_scale=float(q_scale), state=_p(state), norm_w=_p(norm_w),
                           y=_p(y), y_bf16=None, ldy=H * dv, heads=H, dim=dk, vdim=dv)
 
@@ -1722,12 +1733,9 @@ def _decay_step(buf, sizes, a2, a2_bias, tau, q_scale, state, norm_w, y):
 def decay_step_rows(q, k, v, gate, a1, a2, a2_bias, tau, state, norm_w, eps, row_pos, row_slot, q_scale=1.0):
     """Linear attention with decays, rows alone in their entries: f32 [rows, H*dv]; state f32 [slots, H, dk, dv]
     moves on.  q, k [rows, H*dk], v, gate [rows, H*dv], a1 [rows, rank], a2 [H*dk, rank]."""
-    buf = torch.cat([q, k, v, gate, a1], dim=1).contiguous()
-    at = [0]
-    for t in (q, k, v, gate):
-        at.append(at[-1] + t.shape[1])
+    p, ld, _keep = _side_by_side(q, k, v, gate, a1)
     y = torch.empty(q.shape[0], v.shape[1], dtype=torch.float32, device=q.device)
-    s = _decay_step(buf, at, a2, a2_bias, tau, q_scale, state, norm_w, y)
+    s = _decay_step(p, ld, a2, a2_bias, tau, q_scale, state, norm_w, y)
     _lib.check(_lib.load().sd_decay_step_rows(C.byref(s), _wkind(a2, "a2"), float(eps), _p(row_pos), _p(row_slot), q.shape[0],
                                               _stream()), "sd_decay_step_rows")
     return y
@@ -1736,26 +1744,23 @@ def decay_step_rows(q, k, v, gate, a1, a2, a2_bias, tau, state, norm_w, eps, row
 def biased_qkv_prep(q, k, v, biases, G, dk, dv, q_norm_w, k_norm_w, eps, k_cache, v_cache, row_pos, row_slot,
                     block_tables, step=None):
     """sd_biased_qkv_prep on q f32 [rows, H*dk], k [rows, G*dk], v [rows, G*dv]; biases: (q, k, v), each may be
-    None.  Returns the prepared q; keys and values go to the caches.  step: the arguments of
+    None.  Returns the prepared q (in place where q, k, v are columns of one buffer); keys and values go to
+    the caches.  step: the arguments of
     decay_step_rows up to norm_w (and q_scale), whose result is then returned too."""
-    buf = torch.cat([q, k, v], dim=1).contiguous()
-    nq, nk, ld = q.shape[1], k.shape[1], buf.shape[1]
+    p, ld, parts = _side_by_side(q, k, v)
+    nq = q.shape[1]
     y, s = None, None
     if step is not None:
         sq, sk, sv, gate, a1, a2, a2_bias, tau, state, norm_w, q_scale = step
-        buf2 = torch.cat([sq, sk, sv, gate, a1], dim=1).contiguous()
-        at = [0]
-        for t in (sq, sk, sv, gate):
-            at.append(at[-1] + t.shape[1])
+        sp, sld, _keep = _side_by_side(sq, sk, sv, gate, a1)
         y = torch.empty(q.shape[0], sv.shape[1], dtype=torch.float32, device=q.device)
-        s = _decay_step(buf2, at, a2, a2_bias, tau, q_scale, state, norm_w, y)
+        s = _decay_step(sp, sld, a2, a2_bias, tau, q_scale, state, norm_w, y)
     _lib.check(_lib.load().sd_biased_qkv_prep(
-        buf.data_ptr(), buf.data_ptr() + 4 * nq, buf.data_ptr() + 4 * (nq + nk), ld, _p(biases[0]), _p(biases[1]),
+        p[0], p[1], p[2], ld, _p(biases[0]), _p(biases[1]),
         _p(biases[2]), nq // dk, G, dk, dv, _p(q_norm_w), _p(k_norm_w), _wkind(q_norm_w, "q_norm_w"), float(eps), _p(k_cache),
         _p(v_cache), _p(row_pos), _p(row_slot), _p(block_tables), block_tables.shape[1], PAGE, q.shape[0],
         C.byref(s) if s is not None else None, _stream()), "sd_biased_qkv_prep")
-    out = buf[:, :nq].contiguous()
-    return out if step is None else (out, y)
+    return parts[0] if step is None else (parts[0], y)
 
 
 def low_rank_decay(a1, a2, a2_bias, tau) -> torch.Tensor:
@@ -1768,19 +1773,25 @@ def low_rank_decay(a1, a2, a2_bias, tau) -> torch.Tensor:
     return out
 
 
-def decay_chunks(q, k, v, decay, state, entries, q_scale=1.0, cut=True) -> torch.Tensor:
+def decay_chunks_scratch(n_rows, n_entries, H, dk, dv, device="cuda"):
+    """The scratch of decay_chunks' cut form, or None where it needs none."""
+    n = int(_lib.load().sd_decay_chunks_scratch_bytes(n_rows, n_entries, H, dk, dv))
+    return torch.empty(n, dtype=torch.uint8, device=device) if n else None
+
+
+def decay_chunks(q, k, v, decay, state, entries, q_scale=1.0, cut=True, scratch=None) -> torch.Tensor:
     """The recurrence with decays per key channel over portions: q, k, decay f32 [rows, H*dk], v [rows, H*dv], state
     f32 [slots, H, dk, dv] (moves on) -> f32 [rows, H*dv].  cut=False: every portion in one go."""
-    for t, nm in ((q, "q"), (k, "k"), (v, "v"), (decay, "decay"), (state, "state")):
+    for t, nm in ((decay, "decay"), (state, "state")):
         _f32(t, nm)
     H, dk, dv = state.shape[1:]
-    buf = torch.cat([q, k, v], dim=1).contiguous()
+    p, ld, _keep = _side_by_side(q, k, v)
     n, lib = q.shape[0], _lib.load()
-    nb = int(lib.sd_decay_chunks_scratch_bytes(n, entries.shape[0], H, dk, dv)) if cut else 0
-    scratch = torch.empty(nb, dtype=torch.uint8, device=q.device) if nb else None
+    if scratch is None and cut:
+        scratch = decay_chunks_scratch(n, entries.shape[0], H, dk, dv, q.device)
+    nb = scratch.numel() if scratch is not None else 0
     out = torch.empty(n, H * dv, dtype=torch.float32, device=q.device)
-    _lib.check(lib.sd_decay_chunks(buf.data_ptr(), buf.data_ptr() + 4 * H * dk, buf.data_ptr() + 8 * H * dk, buf.shape[1],
-                                   _p(decay), float(q_scale), _p(state), _p(entries), entries.shape[0], n, _p(out), H, dk, dv,
+    _lib.check(lib.sd_decay_chunks(*p, ld, _p(decay), float(q_scale), _p(state), _p(entries), entries.shape[0], n, _p(out), H, dk, dv,
                                    _p(scratch), nb, _stream()), "sd_decay_chunks")
     return out
 
