@@ -154,7 +154,7 @@ def read_streams(x, w_in):
 
 
 def update_streams(x, y, mix, out):
-    """All streams at once from the old ones; mix is indexed [from, to]."""
+    """x_t <- sum_s mix[s, t] x_s + out_t y for every t, x on the right as it was."""
     return torch.einsum("nsw,st->ntw", x, mix.to(F64)) + out.to(F64)[None, :, None] * y[:, None, :]
 
 

@@ -203,6 +203,7 @@ class DecoderModel:
 # ---------------------------------------------------------------------------------------------
 _MIX_KIND = {"retention": 0, "gla": 1, "attention": 2, "latent_attention": 3, "parallel": 4, "softmax_attention": 5,
              "mlstm": 6}
+_MIX_SOFTMAX_DECAY = 7   # a "parallel" mixer whose right side is linear attention
 _EXPERT_ACT = {"silu": 0, "relu2": 1, "clamped_gate": 2}
 
 
@@ -272,7 +273,7 @@ class SeqModel:
             if cfg.block == "streams":
                 r, ex = m.linear, spec.experts
                 layers[i] = _lib.SeqLayer(
-                    kind=7, block=4, heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, ff=spec.ff,
+                    kind=_MIX_SOFTMAX_DECAY, block=4, heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, ff=spec.ff,
                     ff_act={"relu": 0, "silu": 1}[spec.ff_act], q_scale=r.dim ** -0.5, score_scale=m.scale,
                     window=m.window or 0x7fffffff, keep_first=m.keep_first, softcap=m.softcap, sinks=_ptr(t.sinks),
                     head_gate=int(m.head_gate), norm_w=_ptr(t.norm_w), norm2_w=_ptr(t.norm2_w),
